@@ -33,7 +33,8 @@ def _compiled(src):
     -Rpass-analysis=kernel-resource-usage, once per file and test session."""
     with tempfile.TemporaryDirectory() as td:
         asm = os.path.join(td, "k.s")
-        r = subprocess.run([HIPCC, "--offload-arch=gfx950", "-O3", "-std=c++17", "-fPIC", "--cuda-device-only", "-S", os.path.join(CSRC, src), "-o", asm,
+        r = subprocess.run([HIPCC, "--offload-arch=gfx950", "-O3", "-std=c++17", "-fPIC", "-Xclang", "-target-feature", "-Xclang",
+                            "-packed-fp32-ops", "--cuda-device-only", "-S", os.path.join(CSRC, src), "-o", asm,
                             "-Rpass-analysis=kernel-resource-usage"], capture_output=True, text=True)
         assert r.returncode == 0, r.stderr[-2000:]
         text = open(asm).read()

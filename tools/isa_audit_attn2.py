@@ -26,7 +26,7 @@ def regs_of(tok):
 def main():
     with tempfile.TemporaryDirectory() as td:
         asm = os.path.join(td, "k.s")
-        r = subprocess.run(["/opt/rocm/bin/hipcc", "--offload-arch=gfx950", "-O3", "-std=c++17", "--cuda-device-only", "-I" + CSRC,
+        r = subprocess.run(["/opt/rocm/bin/hipcc", "--offload-arch=gfx950", "-O3", "-std=c++17", "-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops", "--cuda-device-only", "-I" + CSRC,
                             "-I" + os.path.join(ROOT, "include"), "-S", os.path.join(CSRC, "lm_kernels.hip"), "-o", asm], capture_output=True, text=True)
         if r.returncode:
             sys.exit(r.stderr[-2000:])
