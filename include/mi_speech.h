@@ -236,6 +236,30 @@ mis_status mis_lm_reset(mis_tts*, int batch, int max_context);
 mis_status mis_lm_prefill(mis_tts*, const int32_t* prompt_ids, const int32_t* prompt_lens, int batch, int max_context,
                           float* logits_out, float* hidden_out);
 mis_status mis_lm_forward(mis_tts*, const int32_t* ids, const uint8_t* active, float* logits_out);
+/* ---- language models by architecture.  config.json with an "architecture" entry describes the model layer by layer ("layers": per layer the
+ * mixer with its sizes, the feed-forward, optionally another layer whose tensors it shares); the engine serves "Rugunex" (parallel blocks
+ * with layer scale, latent attention under a sliding window, squared-ReLU feed-forward).  The handle is the mis_tts of this section: rows,
+ * caches, mis_lm_reset / prefill / forward, the sampler and the generate loop are shared. */
+enum { MIS_COMPUTE_BF16 = 0, MIS_COMPUTE_F32 = 1 };  /* MIS_COMPUTE_F32: every product and activation in float32 */
+/* chosen by config.json; directories without "architecture" load as the Llama family (bf16 only, no codec) */
+mis_status mis_lm_load(const char* model_dir, int compute, int device, mis_tts** out);
+/* the same from the text of config.json; tensors follow with mis_tts_set_tensor, then mis_tts_finalize */
+mis_status mis_lm_create(const char* config_json, int compute, int device, mis_tts** out);
+int32_t    mis_lm_vocab_size(const mis_tts*);
+int32_t    mis_lm_hidden_size(const mis_tts*);
+int32_t    mis_lm_num_layers(const mis_tts*);
+/* step function (models described layer by layer): the next counts[i] tokens of batch row rows[i], i < n_entries, tokens concatenated in entry
+ * order.  Rows start at position 0 after mis_lm_reset.  want: places in the concatenated tokens; logits_out f32 [n_want][vocab] (host).
+ * residual_out (nullable, host): f32 [layers][tokens][hidden], the residual stream behind every layer. */
+mis_status mis_lm_extend(mis_tts*, const int32_t* rows, const int32_t* counts, int n_entries, const int32_t* tokens, const int32_t* want, int n_want,
+                         float* logits_out, float* residual_out);
+/* rows a prompt pass computes at once (default 4096) */
+mis_status mis_lm_set_prefill_rows(mis_tts*, int rows);
+/* generate loop without a codec: tokens_out int32 [batch][max_tokens], n_tokens [batch] (up to and including stop_id; stop_id < 0: none) */
+mis_status mis_lm_generate(mis_tts*, const int32_t* prompt_ids, const int32_t* prompt_lens, int batch, const mis_gen_params* params, int stop_id,
+                           int32_t* tokens_out, int32_t* n_tokens);
+mis_status mis_lm_generate_stream(mis_tts*, const int32_t* prompt_ids, const int32_t* prompt_lens, int batch, const mis_gen_params* params, int stop_id,
+                                  mis_event_cb on_event, void* user, const volatile int* cancel_flag);
 /* same, also returning model.norm(h) of the fed token: hidden_out f32 [batch, hidden_size] (Soprano decodes these,
  * Soprano.swift:254-275); either output may be NULL */
 mis_status mis_lm_forward_hidden(mis_tts*, const int32_t* ids, const uint8_t* active, float* logits_out, float* hidden_out);

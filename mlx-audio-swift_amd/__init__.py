@@ -13,6 +13,8 @@ the Swift shim a maintainer would add):
     soprano.SopranoModel   <-> class SopranoModel : SpeechGenerationModel  (MLXAudioTTS/Models/Soprano/Soprano.swift)
     qwen3tts.Qwen3TTSModel <-> class Qwen3TTSModel : SpeechGenerationModel  (MLXAudioTTS/Models/Qwen3TTS/Qwen3TTS.swift)
     stt.WhisperModel       <-> class WhisperModel : STTGenerationModel   (MLXAudioSTT/Models/Whisper/WhisperModel.swift)
+    lm.BlockLanguageModel      language models described layer by layer in config.json (token generation, step function)
+    registry.load_model    <-> TTS.loadModel                      (MLXAudioTTS/TTSModel.swift)
     dsp.*                  <-> computeMelSpectrogram (MLXAudioCore/DSP.swift) / WhisperAudio.encoderFeatures
     generation.*           <-> AudioGeneration / AudioGenerationInfo / AudioGenerationError /
                                GenerateParameters                (MLXAudioCore/Generation/GenerationTypes.swift)
@@ -30,6 +32,8 @@ from .orpheus import deinterleave, parse_output  # noqa: F401
 from .soprano import SopranoModel, SopranoConfiguration  # noqa: F401
 from .qwen3tts import (Qwen3TTSModel, Qwen3TTSConfiguration, Qwen3TTSDecoderConfiguration, Qwen3TTSGenerateParameters,  # noqa: F401
                        PreparedPrompt)
+from .lm import BlockLanguageModel, BlockModelConfiguration  # noqa: F401
+from .registry import load_model  # noqa: F401
 from . import dsp  # noqa: F401
 from .stt import WhisperModel, WhisperConfig, STTGenerateParameters, STTOutput  # noqa: F401
 

@@ -9,6 +9,9 @@ _HERE = os.path.dirname(os.path.abspath(__file__))
 # MIS_LIB_PATH: load a diagnostics build of the same library instead (e.g. `make timing`, tools/attn_phases.py)
 LIB_PATH = os.environ.get("MIS_LIB_PATH") or os.path.join(_HERE, "libmi_speech.so")
 
+# `make lm`: the token engines alone.  load_language_models() falls back on it (and builds it) where the whole library has not been built.
+LM_LIB_PATH = os.path.join(_HERE, "libmi_speech_lm.so")
+
 MIS_OK = 0
 STATUS_NAMES = {0: "ok", 1: "modelNotInitialized", 2: "generationFailed", 3: "invalidInput",
                 4: "audioDecodingFailed", 5: "audioEncodingFailed", 6: "cancelled", 7: "device"}
@@ -169,6 +172,15 @@ SYMBOLS = {
     "mis_tts_destroy": (None, [_P]),
     "mis_lm_reset": (C.c_int, [_P, C.c_int, C.c_int]),
     "mis_lm_forward": (C.c_int, [_P, _P, _P, _P]),
+    "mis_lm_load": (C.c_int, [C.c_char_p, C.c_int, C.c_int, C.POINTER(_P)]),
+    "mis_lm_create": (C.c_int, [C.c_char_p, C.c_int, C.c_int, C.POINTER(_P)]),
+    "mis_lm_vocab_size": (C.c_int32, [_P]),
+    "mis_lm_hidden_size": (C.c_int32, [_P]),
+    "mis_lm_num_layers": (C.c_int32, [_P]),
+    "mis_lm_extend": (C.c_int, [_P, _P, _P, C.c_int, _P, _P, C.c_int, _P, _P]),
+    "mis_lm_set_prefill_rows": (C.c_int, [_P, C.c_int]),
+    "mis_lm_generate": (C.c_int, [_P, _P, _P, C.c_int, C.POINTER(GenParamsC), C.c_int, _P, _P]),
+    "mis_lm_generate_stream": (C.c_int, [_P, _P, _P, C.c_int, C.POINTER(GenParamsC), C.c_int, EVENT_CB, _P, _P]),
     "mis_lm_forward_hidden": (C.c_int, [_P, _P, _P, _P, _P]),
     "mis_sample_logits": (C.c_int, [C.c_int, _P, C.c_int, C.c_int, _P, _P, C.c_int, C.POINTER(GenParamsC), C.c_int,
                                     C.c_int, C.c_int, _P]),
@@ -290,11 +302,30 @@ DEBUG_SYMBOLS = {
     "mis_debug_token_engine": (C.c_int, [_P, _P, C.c_int, C.c_int, C.c_int, _P, C.c_int, _P, _P, _P, _P, C.POINTER(C.c_double)]),
 }
 
+# what libmi_speech_lm.so serves
+LM_SYMBOLS = ["mis_last_error", "mis_abi_version", "mis_free", "mis_device_count", "mis_tts_load", "mis_tts_create", "mis_tts_set_tensor",
+              "mis_tts_init_synthetic", "mis_tts_finalize", "mis_tts_destroy", "mis_tts_last_timing", "mis_sample_logits"] + \
+    [n for n in SYMBOLS if n.startswith("mis_lm_")]
+
 _lib = None
 
 
 class MisLibraryMissing(RuntimeError):
     pass
+
+
+def _bind(path, names, preload_torch=True):
+    if preload_torch:
+        try:        # if torch is installed, let ITS bundled ROCm runtime load first (one libamdhip64 per process)
+            import torch  # noqa: F401
+        except Exception:
+            pass
+    l = C.CDLL(path)
+    table = {**SYMBOLS, **DEBUG_SYMBOLS}
+    for name in names:
+        fn = getattr(l, name)          # AttributeError if the ABI lost a symbol
+        fn.restype, fn.argtypes = table[name]
+    return l
 
 
 def lib():
@@ -305,16 +336,28 @@ def lib():
             raise MisLibraryMissing(
                 f"{LIB_PATH} not found: build it with `python -c 'import __graft_entry__ as g; g.build()'` "
                 "(hipcc --offload-arch=gfx950). There is no CPU fallback.")
-        try:        # if torch is installed, let ITS bundled ROCm runtime load first (one libamdhip64 per process)
-            import torch  # noqa: F401
-        except Exception:
-            pass
-        l = C.CDLL(LIB_PATH)
-        for name, (res, args) in list(SYMBOLS.items()) + list(DEBUG_SYMBOLS.items()):
-            fn = getattr(l, name)          # AttributeError if the ABI lost a symbol
-            fn.restype = res
-            fn.argtypes = args
-        _lib = l
+        _lib = _bind(LIB_PATH, list(SYMBOLS) + list(DEBUG_SYMBOLS))
+    return _lib
+
+
+def load_language_models(build: bool = True):
+    """The library for a process that only runs language models (command line tools): the whole library where it is built, else the
+    language-model build of it, compiled here when missing.  No torch in the process: nothing to load before the library."""
+    global _lib
+    if _lib is None:
+        if os.path.exists(LIB_PATH):
+            _lib = _bind(LIB_PATH, list(SYMBOLS) + list(DEBUG_SYMBOLS), preload_torch=False)
+        else:
+            if build:
+                import subprocess
+                import sys
+                r = subprocess.run(["make", "-C", os.path.join(_HERE, "csrc"), "-j8", "lm"], stdout=subprocess.PIPE, stderr=subprocess.STDOUT, text=True)
+                if r.returncode != 0:
+                    sys.stderr.write(r.stdout[-8000:])
+                    raise MisLibraryMissing("hipcc build of libmi_speech_lm.so failed")
+            if not os.path.exists(LM_LIB_PATH):
+                raise MisLibraryMissing(f"{LM_LIB_PATH} not found")
+            _lib = _bind(LM_LIB_PATH, LM_SYMBOLS, preload_torch=False)
     return _lib
 
 

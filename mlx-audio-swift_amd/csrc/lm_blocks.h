@@ -1,0 +1,99 @@
+// lm_blocks.h - language models described layer by layer (config.json "layers"): weights, caches, the decode step and the prompt pass.  The
+// engine around it - handles, batch rows, positions, sampler, generate loop, captured graphs - is lm_engine.hip's.
+#pragma once
+#include <deque>
+#include <map>
+#include <memory>
+#include <set>
+#include "lm_latent.h"
+
+// ---- configuration
+struct LatentMixerSpec { int heads = 0, dim = 0, rot_dim = 0, vdim = 0, kv_rank = 0, window = 0; float scale = 1.0f; RotarySpec rot; };
+struct BlockSpec { LatentMixerSpec mix; int ff = 0 /* 0: no feed-forward */; int weights_of = -1; };
+struct BlockModelSpec {
+    std::string architecture;
+    int width = 0, vocab = 0;
+    float eps = 1e-6f, logit_scale = 1.0f, softcap = 0.0f;
+    std::vector<BlockSpec> layers;
+};
+// architectures this engine serves, by config.json "architecture"
+bool block_architecture_known(const std::string& name);
+BlockModelSpec parse_block_model(const JsonValue& cfg);
+
+// ---- one request's share of a prompt pass
+struct PassEntry { int seq, pos0, n; };
+
+// Device state of the batch rows, owned by the engine
+struct BlockRows { const int32_t* ids; const uint8_t* active; int32_t *pos_cur, *pos_next; };
+
+class LmBlocks {
+public:
+    LmBlocks(const BlockModelSpec& spec, bool f32);
+    const BlockModelSpec spec;
+    const bool f32;                     // 32-bit mode: float32 operands, caches and GEMMs (weights stay bf16, exact in float32)
+    int d, dp, V, Vpad, L;
+
+    // weights: `src` bf16 row-major on the device; throws on an unknown name or a wrong shape
+    void set_tensor(const std::string& name, const bf16_t* src, const std::vector<int64_t>& shape, hipStream_t s);
+    std::vector<std::pair<std::string, std::vector<int64_t>>> tensor_list() const;      // every tensor the configuration implies
+    void init_synthetic(uint64_t seed, hipStream_t s);
+    void finalize() const;              // throws when a tensor is missing
+
+    // caches and step buffers for `batch` rows of up to Smax positions
+    void reset(int batch, int Smax, hipStream_t s);
+    // one token of every active row (captured in the engine's decode graph); leaves the final norm of every row as the head's operand
+    void enqueue_step(const BlockRows& r, hipStream_t s);
+    void enqueue_head(hipStream_t s);   // logits of the batch rows: float32 [Mpad][Vpad]
+    float* logits() { return logits_.p; }
+    // tokens of several requests at their positions, in chunks of at most pass_rows rows.  want: places in `tokens` whose logits go to
+    // logits_out [n_want][V] (host); residual_out (host, nullable): [L][tokens][d].  last_rows: leave the final norm of every entry's
+    // last token as operand row `seq` of the head (what enqueue_step leaves).
+    void pass(const std::vector<PassEntry>& entries, const std::vector<int32_t>& tokens, const std::vector<int32_t>& want, float* logits_out,
+              float* residual_out, bool last_rows, hipStream_t s);
+    void final_norm_rows(float* out, int rows, hipStream_t s);     // the head's operand as float32 [rows][d] (host or device)
+    int pass_rows = 4096;
+    double weight_bytes_per_step() const, cache_bytes_per_key() const;
+
+private:
+    struct Weights {                    // one set per layer that owns tensors
+        DevBuf<bf16_t> w1;              // packed [(Nqkv + ffp) / 16][dp / 32]: q | latent | rotary key | up
+        DevBuf<bf16_t> c_norm, norm1, ls1, ls2;
+        DevBuf<bf16_t> uk_t;            // packed per head [Rp / 16][np / 32]  (absorbed form)
+        DevBuf<bf16_t> ukv;             // packed [(H np + H vp) / 16][Rp / 32] (expanded form; its value part serves the absorbed form too)
+        DevBuf<bf16_t> wo, wdown;       // packed [dp / 16][Ko / 32], [dp / 16][ffp / 32]
+    };
+    struct Layer { LatentDims D; int owner, ffp, Nqkv, Ko, S_attn = 1, S_o = 1, S_down = 1, rope = 0; };
+    std::vector<Layer> layers_;
+    std::vector<std::unique_ptr<Weights>> w_;
+    std::set<std::string> loaded_;
+    DevBuf<bf16_t> emb_, g_embed_, g_final_, head_;
+    struct Rope { RotarySpec spec; DevBuf<float> cs, sn; };
+    std::deque<Rope> ropes_;
+    DevBuf<bf16_t> stage_, place_;
+
+    int batch_ = 0, Mpad_ = 0, Smax_ = 0, rope_len_ = 0;
+    std::vector<std::unique_ptr<DevBuf<uint8_t>>> cache_;
+    // step buffers; bf16 ones hold float32 in the 32-bit mode (sized in bytes)
+    DevBuf<float> x_, qkv_, part_o_, part_d_, attn_part_, attn_ml_, logits_;
+    DevBuf<uint8_t> h_, act_, q_, olat_;
+    std::map<int, DevBuf<uint8_t>> attn_;          // per H v: the columns up to the K padding stay zero
+    // pass buffers
+    DevBuf<float> px_, pqkv_, plog_;
+    DevBuf<uint8_t> ph_, pact_, pq_, polat_, phead_;
+    DevBuf<bf16_t> pkv_;
+    std::map<int, DevBuf<uint8_t>> pattn_;
+    std::map<int, size_t> pattn_rows_;
+    DevBuf<int32_t> pids_, pseq_, ppos_, pkey_, pwant_;
+    DevBuf<LatentTile> ptiles_;
+
+    int esz() const { return f32 ? 4 : 2; }
+    const Weights& W(int li) const { return *w_[layers_[li].owner]; }
+    void place(const bf16_t* src, int64_t N, int64_t K, int part1, int part2, int g_out, int off2, int Np, int Kp, hipStream_t s);
+    Operand operand(void* p, int ld, int rows_padded, bool packed) const;
+    LatentRows latent_rows(int li, const float* qkv, void* q, bool expanded, const RowTable& rows) const;
+    const bf16_t* norm_after(int li) const { return li + 1 < L ? W(li + 1).norm1.p : g_final_.p; }
+    void step_layer(int li, const BlockRows& r, hipStream_t s);
+    void pass_layer(int li, int M, const RowTable& rows, int n_tiles, int Mk, hipStream_t s);
+    void absorbed_attention(int li, const float* qkv, void* q, void* olat, const Operand& out, const RowTable& rows, int M, int S, hipStream_t s);
+    void head_rows(const void* operand, bool packed, int rows, int rows_padded, float* out, hipStream_t s);
+};

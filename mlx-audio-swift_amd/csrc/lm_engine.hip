@@ -11,6 +11,7 @@
 #include "common.h"
 #include "kernels.h"
 #include "lm_kernels.h"
+#include "lm_blocks.h"
 
 #include <math.h>
 #include <string.h>
@@ -22,6 +23,8 @@
 #define ORPHEUS_END_OF_SPEECH 128258
 
 struct mis_tts {
+    std::unique_ptr<LmBlocks> blocks;      // a model described layer by layer (lm_blocks.h) instead of the Llama chain below; null: the Llama chain
+    std::vector<int32_t> blk_pos;          // host mirror of pos_next (block models)
     int device = 0;
     hipStream_t stream = nullptr;
     mis_lm_config cfg{};
@@ -131,6 +134,29 @@ extern "C" mis_status mis_tts_create(const mis_lm_config* cfg, mis_snac* codec, 
     if (c->cfg.qk_norm) c->qknorm.alloc((size_t)2 * c->L * D);
     c->use_graph = getenv("MIS_NO_GRAPH") == nullptr;
     *out = c;
+    MIS_API_END
+}
+
+// The handle of a block model: same rows, positions, sampler, graphs and generate loop; weights, caches and the kernel chain are LmBlocks'.
+static mis_tts* create_block_model(const BlockModelSpec& spec, bool f32, int device) {
+    int n = 0;
+    HIP_CHECK(hipGetDeviceCount(&n));
+    MIS_REQUIRE(device >= 0 && device < n, MIS_ERR_DEVICE, "device %d not available (%d GPUs visible)", device, n);
+    HIP_CHECK(hipSetDevice(device));
+    std::unique_ptr<mis_tts> c(new mis_tts());
+    c->device = device;
+    c->blocks.reset(new LmBlocks(spec, f32));
+    c->d = spec.width; c->L = c->blocks->L; c->V = spec.vocab; c->Vpad = c->blocks->Vpad;
+    c->cfg.hidden_size = c->d; c->cfg.num_hidden_layers = c->L; c->cfg.vocab_size = c->V; c->cfg.rms_norm_eps = spec.eps;
+    HIP_CHECK(hipStreamCreateWithFlags(&c->stream, hipStreamNonBlocking));
+    c->use_graph = getenv("MIS_NO_GRAPH") == nullptr;
+    return c.release();
+}
+extern "C" mis_status mis_lm_create(const char* config_json, int compute, int device, mis_tts** out) {
+    MIS_API_BEGIN
+    MIS_REQUIRE(config_json && out, MIS_ERR_INVALID_INPUT, "null argument");
+    MIS_REQUIRE(compute == MIS_COMPUTE_BF16 || compute == MIS_COMPUTE_F32, MIS_ERR_INVALID_INPUT, "unknown compute type");
+    *out = create_block_model(parse_block_model(json_parse(config_json)), compute == MIS_COMPUTE_F32, device);
     MIS_API_END
 }
 
@@ -259,6 +285,19 @@ extern "C" mis_status mis_tts_set_tensor(mis_tts* c, const char* name_, const vo
     MIS_REQUIRE(!c->finalized, MIS_ERR_INVALID_INPUT, "set_tensor after finalize");
     MIS_REQUIRE(dtype == MIS_F32 || dtype == MIS_F16 || dtype == MIS_BF16, MIS_ERR_INVALID_INPUT, "unsupported dtype");
     std::string name = name_;
+    if (c->blocks) {
+        HIP_CHECK(hipSetDevice(c->device));
+        size_t n = 1;
+        for (int i = 0; i < ndim; ++i) { MIS_REQUIRE(shape[i] > 0, MIS_ERR_INVALID_INPUT, "bad shape"); n *= (size_t)shape[i]; }
+        const size_t esz = dtype == MIS_F32 ? 4 : 2;
+        c->raw_staging.alloc(n * esz);
+        c->staging.alloc(n);
+        HIP_CHECK(hipMemcpyAsync(c->raw_staging.p, data, n * esz, hipMemcpyDefault, c->stream));
+        launch_convert_to_bf16(c->raw_staging.p, dtype, c->staging.p, n, c->stream);
+        c->blocks->set_tensor(name, c->staging.p, std::vector<int64_t>(shape, shape + ndim), c->stream);
+        HIP_CHECK(hipStreamSynchronize(c->stream));
+        return MIS_OK;
+    }
     if (name.find("rotary_emb.inv_freq") != std::string::npos) return MIS_OK;      // sanitize, LlamaTTS.swift:584-586
     if (name == "lm_head.weight" && c->cfg.tie_word_embeddings) return MIS_OK;     // :588-590
     HIP_CHECK(hipSetDevice(c->device));
@@ -324,6 +363,7 @@ extern "C" mis_status mis_tts_set_tensor_quantized(mis_tts* c, const char* name_
     MIS_API_BEGIN
     MIS_REQUIRE(c && name_ && wq && scales && biases, MIS_ERR_INVALID_INPUT, "null argument");
     MIS_REQUIRE(!c->finalized, MIS_ERR_INVALID_INPUT, "set_tensor after finalize");
+    MIS_REQUIRE(!c->blocks, MIS_ERR_INVALID_INPUT, "quantised tensors are not supported for this architecture");
     set_quantized_any(c, name_, wq, scales, biases, sb_dtype, N, K, group_size, bits);
     MIS_API_END
 }
@@ -349,7 +389,7 @@ __global__ void k_synth_quant(uint32_t* __restrict__ wq, bf16_t* __restrict__ sc
 }
 extern "C" mis_status mis_tts_init_synthetic_quantized(mis_tts* c, uint64_t seed, int bits) {
     MIS_API_BEGIN
-    MIS_REQUIRE(c && !c->finalized && (bits == 4 || bits == 8), MIS_ERR_INVALID_INPUT, "bad argument");
+    MIS_REQUIRE(c && !c->finalized && !c->blocks && (bits == 4 || bits == 8), MIS_ERR_INVALID_INPUT, "bad argument");
     HIP_CHECK(hipSetDevice(c->device));
     hipStream_t s = c->stream;
     const int d = c->d, ff = c->ff, HD = c->H * c->D, KD = c->Hkv * c->D;
@@ -398,6 +438,7 @@ extern "C" mis_status mis_tts_init_synthetic(mis_tts* c, uint64_t seed) {
     MIS_REQUIRE(c && !c->finalized, MIS_ERR_INVALID_INPUT, "bad handle");
     HIP_CHECK(hipSetDevice(c->device));
     hipStream_t s = c->stream;
+    if (c->blocks) { c->blocks->init_synthetic(seed, s); return MIS_OK; }
     const int d = c->d, ff = c->ff, HD = c->H * c->D, KD = c->Hkv * c->D;
     const uint64_t base = seed * 100000ull;
     size_t big = std::max((size_t)c->V * d, (size_t)ff * d);
@@ -439,6 +480,12 @@ extern "C" mis_status mis_tts_finalize(mis_tts* c) {
     MIS_API_BEGIN
     MIS_REQUIRE(c && !c->finalized, MIS_ERR_INVALID_INPUT, "bad handle");
     HIP_CHECK(hipSetDevice(c->device));
+    if (c->blocks) {
+        c->blocks->finalize();
+        c->staging.release(); c->raw_staging.release();
+        c->finalized = true;
+        return MIS_OK;
+    }
     // update(parameters:verify:.all), LlamaTTS.swift:971: every parameter must be present
     std::vector<std::string> want = {"model.embed_tokens.weight", "model.norm.weight"};
     if (!c->cfg.tie_word_embeddings) want.push_back("lm_head.weight");
@@ -538,6 +585,15 @@ static void lm_reset(mis_tts* c, int batch, int max_context) {
     if (regraph) destroy_graphs(c);
     bool new_tables = Smax != c->Smax;
     c->batch = batch; c->Mpad = Mpad; c->Smax = Smax;
+    if (c->blocks) {
+        c->blocks->reset(batch, Smax, s);
+        c->blk_pos.assign(batch, 0);
+        c->ids.alloc(Mpad); c->pos_cur.alloc(Mpad); c->pos_next.alloc(Mpad); c->active.alloc(Mpad);
+        c->ids.zero(s); c->pos_cur.zero(s); c->pos_next.zero(s); c->active.zero(s);
+        c->e_buf.alloc((size_t)Mpad * c->Vpad);
+        HIP_CHECK(hipStreamSynchronize(s));
+        return;
+    }
     const int d = c->d, HD = c->H * c->D;
     c->ksb_part = 4;                                     // split-K roles and gate+up: the four waves of a block share an item's K range
     c->ksb_gu = 4;
@@ -655,6 +711,7 @@ static void gemm_down(mis_tts* c, size_t li, hipStream_t s) {
 // table/rows/ids: embedding source override (composite engines feed input embeddings as a [rows][d] table)
 static void enqueue_layers(mis_tts* c, const bf16_t* table = nullptr, int table_rows = 0, const int32_t* ids = nullptr) {
     hipStream_t s = c->stream;
+    if (c->blocks) { c->blocks->enqueue_step(BlockRows{c->ids.p, c->active.p, c->pos_cur.p, c->pos_next.p}, s); return; }
     const int d = c->d, Mpad = c->Mpad;
     const float eps = c->cfg.rms_norm_eps;
     launch_embed_rmsnorm(table ? table : c->emb.p, ids ? ids : c->ids.p, c->active.p, c->pos_cur.p, c->pos_next.p, c->norms.p,
@@ -685,6 +742,7 @@ static void enqueue_layers(mis_tts* c, const bf16_t* table = nullptr, int table_
     }
 }
 static void enqueue_lm_head(mis_tts* c, const bf16_t* head = nullptr) {
+    if (c->blocks) { c->blocks->enqueue_head(c->stream); return; }
     if (!head && c->q_head.on) {
         launch_gemm_skinny_q(c->q_head.bits, EPI_BF16, c->qa_head.R, c->qa_head.ksb, c->q_head.q.p, c->q_head.sb.p, c->x.p, c->logits.p, c->Vpad / 16, c->d / 64, 1, c->Vpad,
                              c->Mpad, c->stream);
@@ -904,6 +962,74 @@ static void prefill_batched(mis_tts* c, const int32_t* prompt_mat_dev, const int
     HIP_CHECK(hipStreamSynchronize(s));                                      // pn / pc are host stack memory
 }
 
+// ---- block models: tokens of several rows at their positions (prompts, portions of prompts); the rows' positions move behind them
+static void blocks_pass(mis_tts* c, const std::vector<PassEntry>& entries, const std::vector<int32_t>& tokens, const std::vector<int32_t>& want, float* logits_out,
+                        float* residual_out, bool last_rows) {
+    c->blocks->pass(entries, tokens, want, logits_out, residual_out, last_rows, c->stream);
+    for (auto& e : entries) c->blk_pos[e.seq] = e.pos0 + e.n;
+    std::vector<int32_t> cur(c->blk_pos);
+    for (auto& p : cur) p = std::max(p - 1, 0);
+    HIP_CHECK(hipMemcpyAsync(c->pos_next.p, c->blk_pos.data(), (size_t)c->batch * 4, hipMemcpyHostToDevice, c->stream));
+    HIP_CHECK(hipMemcpyAsync(c->pos_cur.p, cur.data(), (size_t)c->batch * 4, hipMemcpyHostToDevice, c->stream));
+    HIP_CHECK(hipStreamSynchronize(c->stream));
+}
+static void blocks_prefill(mis_tts* c, const std::vector<int32_t>& flat, const std::vector<int32_t>& lens) {
+    std::vector<PassEntry> entries;
+    for (int b = 0; b < (int)lens.size(); ++b) entries.push_back(PassEntry{b, 0, lens[b]});
+    blocks_pass(c, entries, flat, {}, nullptr, nullptr, true);
+}
+
+// The step function of a block model: entry i = counts[i] next tokens of batch row rows[i] (after mis_lm_reset every row stands at position 0).
+// One token each: the decode step's chain; otherwise the prompt pass.
+extern "C" mis_status mis_lm_extend(mis_tts* c, const int32_t* rows, const int32_t* counts, int n_entries, const int32_t* tokens, const int32_t* want, int n_want,
+                                    float* logits_out, float* residual_out) {
+    MIS_API_BEGIN
+    MIS_REQUIRE(c && rows && counts && tokens && n_entries >= 1 && n_want >= 0 && (n_want == 0 || (want && logits_out)), MIS_ERR_INVALID_INPUT, "bad argument");
+    MIS_REQUIRE(c->blocks, MIS_ERR_INVALID_INPUT, "mis_lm_extend serves models described layer by layer");
+    MIS_REQUIRE(c->finalized && c->batch > 0, MIS_ERR_NOT_INITIALIZED, "call mis_lm_reset first");
+    HIP_CHECK(hipSetDevice(c->device));
+    hipStream_t s = c->stream;
+    std::vector<PassEntry> entries;
+    std::set<int32_t> seen;
+    size_t total = 0;
+    bool single = true;
+    for (int i = 0; i < n_entries; ++i) {
+        MIS_REQUIRE(rows[i] >= 0 && rows[i] < c->batch && seen.insert(rows[i]).second, MIS_ERR_INVALID_INPUT, "bad or repeated batch row %d", rows[i]);
+        MIS_REQUIRE(counts[i] >= 1 && c->blk_pos[rows[i]] + counts[i] <= c->Smax, MIS_ERR_INVALID_INPUT, "row %d exceeds max_context %d", rows[i], c->Smax);
+        entries.push_back(PassEntry{rows[i], c->blk_pos[rows[i]], counts[i]});
+        total += counts[i];
+        single = single && counts[i] == 1;
+    }
+    std::vector<int32_t> toks(tokens, tokens + total), wv(want, want + n_want);
+    for (auto t : toks) MIS_REQUIRE(t >= 0 && t < c->V, MIS_ERR_INVALID_INPUT, "token %d outside the vocabulary", t);
+    for (auto w : wv) MIS_REQUIRE(w >= 0 && (size_t)w < total, MIS_ERR_INVALID_INPUT, "wanted place %d outside the tokens", w);
+    if (!single || residual_out) {
+        blocks_pass(c, entries, toks, wv, logits_out, residual_out, false);
+        return MIS_OK;
+    }
+    std::vector<int32_t> ids(c->batch, 0);
+    std::vector<uint8_t> act(c->batch, 0);
+    for (int i = 0; i < n_entries; ++i) { ids[rows[i]] = toks[i]; act[rows[i]] = 1; ++c->blk_pos[rows[i]]; }
+    HIP_CHECK(hipMemcpyAsync(c->ids.p, ids.data(), (size_t)c->batch * 4, hipMemcpyHostToDevice, s));
+    HIP_CHECK(hipMemcpyAsync(c->active.p, act.data(), c->batch, hipMemcpyHostToDevice, s));
+    enqueue_layers(c);
+    if (n_want) {
+        enqueue_lm_head(c);
+        for (int k = 0; k < n_want; ++k)
+            HIP_CHECK(hipMemcpyAsync(logits_out + (size_t)k * c->V, c->blocks->logits() + (size_t)rows[wv[k]] * c->Vpad, (size_t)c->V * 4, hipMemcpyDeviceToHost, s));
+    }
+    HIP_CHECK(hipGetLastError());
+    HIP_CHECK(hipStreamSynchronize(s));
+    MIS_API_END
+}
+// rows a prompt pass computes at once (bounds its activation memory; longer prompts run in several passes)
+extern "C" mis_status mis_lm_set_prefill_rows(mis_tts* c, int rows) {
+    MIS_API_BEGIN
+    MIS_REQUIRE(c && c->blocks && rows >= 1, MIS_ERR_INVALID_INPUT, "bad argument");
+    c->blocks->pass_rows = rows;
+    MIS_API_END
+}
+
 extern "C" mis_status mis_lm_reset(mis_tts* c, int batch, int max_context) {
     MIS_API_BEGIN
     MIS_REQUIRE(c, MIS_ERR_INVALID_INPUT, "null handle");
@@ -962,6 +1088,17 @@ extern "C" mis_status mis_lm_forward_hidden(mis_tts* c, const int32_t* ids, cons
     HIP_CHECK(hipMemcpyAsync(c->ids.p, ids, c->batch * 4, hipMemcpyDefault, s));
     HIP_CHECK(hipMemcpyAsync(c->active.p, act.data(), c->batch, hipMemcpyHostToDevice, s));
     enqueue_layers(c);
+    if (c->blocks) {
+        for (int b = 0; b < c->batch; ++b) c->blk_pos[b] += act[b] ? 1 : 0;
+        if (hidden_out) c->blocks->final_norm_rows(hidden_out, c->batch, s);
+        if (logits_out) {
+            enqueue_lm_head(c);
+            HIP_CHECK(hipMemcpy2DAsync(logits_out, (size_t)c->V * 4, c->blocks->logits(), (size_t)c->Vpad * 4, (size_t)c->V * 4, c->batch, hipMemcpyDefault, s));
+        }
+        HIP_CHECK(hipGetLastError());
+        HIP_CHECK(hipStreamSynchronize(s));
+        return MIS_OK;
+    }
     if (hidden_out) {
         size_t n = (size_t)c->batch * c->d;
         c->logits_f32.alloc(std::max(n, c->logits_f32.n));
@@ -1006,6 +1143,16 @@ extern "C" mis_status mis_lm_prefill(mis_tts* c, const int32_t* prompt_ids, cons
     HIP_CHECK(hipMemcpy(flat.data(), prompt_ids, total * 4, hipMemcpyDefault));
     for (auto t : flat) MIS_REQUIRE(t >= 0 && t < c->V, MIS_ERR_INVALID_INPUT, "prompt token %d outside the vocabulary", t);
     lm_reset(c, batch, std::max(max_context, Lmax + 1));
+    if (c->blocks) {
+        blocks_prefill(c, flat, lens);
+        if (hidden_out) c->blocks->final_norm_rows(hidden_out, batch, s);
+        if (logits_out) {
+            enqueue_lm_head(c);
+            HIP_CHECK(hipMemcpy2DAsync(logits_out, (size_t)c->V * 4, c->blocks->logits(), (size_t)c->Vpad * 4, (size_t)c->V * 4, batch, hipMemcpyDefault, s));
+        }
+        HIP_CHECK(hipStreamSynchronize(s));
+        return MIS_OK;
+    }
     std::vector<int32_t> pm((size_t)batch * Lmax, 0);
     {
         size_t off = 0;
@@ -1169,10 +1316,10 @@ __global__ void k_collect_hidden(const bf16_t* __restrict__ x, const uint8_t* __
     if (!prefill && threadIdx.x == 0) hid_count[b] = slot + 1;
 }
 
-struct HiddenMode {            // Soprano: collect model.norm(h) per step instead of decoding SNAC frames
+struct HiddenMode {            // no codec behind the loop: Soprano collects model.norm(h) per step; a text model (hidden null) only its tokens
     bool on = false;
     int stop_id = -1;
-    DevBuf<float>* hidden = nullptr;      // [batch][max_tokens + 1][d]
+    DevBuf<float>* hidden = nullptr;      // [batch][max_tokens + 1][d], or null
     std::vector<int32_t> n_hidden;
 };
 
@@ -1188,7 +1335,8 @@ static void run_generate_attempt(mis_tts* c, const int32_t* prompt_ids, const in
                                  bool want_tokens, mis_event_cb cb, void* user, const volatile int* cancel, GenOutputs& out,
                                  HiddenMode* hm, bool multi_launch_only, std::vector<int32_t>& emitted) {
     MIS_REQUIRE(c && c->finalized, MIS_ERR_NOT_INITIALIZED, "model not initialized");
-    const bool hidden_mode = hm && hm->on;
+    const bool hidden_mode = hm && hm->on, collect_hidden = hidden_mode && hm->hidden;
+    MIS_REQUIRE(!c->blocks || (hidden_mode && !collect_hidden), MIS_ERR_INVALID_INPUT, "this architecture generates tokens (mis_lm_generate)");
     MIS_REQUIRE(hidden_mode || c->codec, MIS_ERR_NOT_INITIALIZED, "SNAC model not loaded");            // LlamaTTS.swift:672-674
     MIS_REQUIRE(prompt_ids && prompt_lens && gp, MIS_ERR_INVALID_INPUT, "null argument");
     MIS_REQUIRE(batch >= 1 && batch <= 64, MIS_ERR_INVALID_INPUT, "batch per GPU must be 1..64");
@@ -1265,9 +1413,10 @@ static void run_generate_attempt(mis_tts* c, const int32_t* prompt_ids, const in
         c->samp_l32.alloc((size_t)c->Mpad * c->Vpad);
         sp.penalty_flavor = 1; sp.top_p = 1.0f; sp.logits32 = c->samp_l32.p;
     }
+    if (c->blocks) { sp.logits32 = c->blocks->logits(); sp.f32_input = 1; }   // the head's float32 logits are sampled as they are
     DevBuf<int32_t> hid_count;
     int64_t hid_rows = max_tokens + 1;
-    if (hidden_mode) {
+    if (collect_hidden) {
         hm->hidden->alloc((size_t)batch * hid_rows * c->d);
         hid_count.alloc(batch);
         std::vector<int32_t> ones_i(batch, 1);           // slot 0 = last prompt token (Soprano.swift:824-825)
@@ -1288,14 +1437,14 @@ static void run_generate_attempt(mis_tts* c, const int32_t* prompt_ids, const in
                       c->a_qkv.R, c->a_qkv.ksb, c->a_qkv.U, c->a_o.R, c->a_o.ksb, c->a_o.U, c->a_down.R, c->a_down.ksb, c->a_down.U,
                       c->a_head.R, c->a_head.ksb, c->a_head.U, c->r_gu, c->ksb_gu, c->qa_gu.R, c->qa_gu.ksb, c->qa_head.R, c->qa_head.ksb};
         mix(ints, sizeof(ints));
-        const void* hp[] = {hidden_mode ? (const void*)hm->hidden->p : nullptr, hidden_mode ? (const void*)hid_count.p : nullptr};
+        const void* hp[] = {collect_hidden ? (const void*)hm->hidden->p : nullptr, collect_hidden ? (const void*)hid_count.p : nullptr};
         mix(hp, sizeof(hp));
         if (key != c->graph_key) destroy_graphs(c);
         c->graph_key = key;
     }
 
     auto collect = [&](int prefill) {
-        if (hidden_mode)
+        if (collect_hidden)
             hipLaunchKernelGGL(k_collect_hidden, dim3(batch), dim3(256), 0, s, c->x.p, c->active.p, hid_count.p, hm->hidden->p,
                                hid_rows, c->d, c->Mpad / 16, prefill);
     };
@@ -1324,7 +1473,8 @@ static void run_generate_attempt(mis_tts* c, const int32_t* prompt_ids, const in
     auto t_host0 = std::chrono::steady_clock::now();
     HIP_CHECK(hipEventRecord(ev[0], s));
     // ---- prefill: Lmax steps of the ragged, left-padded batch (prefill :711)
-    if (prefill_batched_ok(c, Lmax)) {
+    if (c->blocks) blocks_prefill(c, flat, lens);
+    else if (prefill_batched_ok(c, Lmax)) {
         prefill_batched(c, c->prompt_mat.p, c->prompt_lens.p, lens, Lmax);
         collect(1);
     } else {
@@ -1393,9 +1543,11 @@ static void run_generate_attempt(mis_tts* c, const int32_t* prompt_ids, const in
     }
 
     if (hidden_mode) {
-        hm->n_hidden.resize(batch);
         out.n_tokens.resize(batch);
-        HIP_CHECK(hipMemcpyAsync(hm->n_hidden.data(), hid_count.p, batch * 4, hipMemcpyDeviceToHost, s));
+        if (collect_hidden) {
+            hm->n_hidden.resize(batch);
+            HIP_CHECK(hipMemcpyAsync(hm->n_hidden.data(), hid_count.p, batch * 4, hipMemcpyDeviceToHost, s));
+        }
         HIP_CHECK(hipMemcpyAsync(out.n_tokens.data(), c->n_gen.p, batch * 4, hipMemcpyDeviceToHost, s));
         if (want_tokens) {
             out.tokens.resize((size_t)batch * max_tokens);
@@ -1403,14 +1555,16 @@ static void run_generate_attempt(mis_tts* c, const int32_t* prompt_ids, const in
             HIP_CHECK(hipMemcpyAsync(out.tokens.data(), c->tokens_out.p, out.tokens.size() * 4, hipMemcpyDeviceToHost, s));
         }
         HIP_CHECK(hipStreamSynchronize(s));
-        // the graphs reference hid_count / hidden: never reuse them after this call
-        destroy_graphs(c);
-        c->graph_key = 0;
+        if (collect_hidden) {                                // the graphs reference hid_count / hidden: never reuse them after this call
+            destroy_graphs(c);
+            c->graph_key = 0;
+        }
         c->timing.prefill_ms = ms_between(ev[0], ev[1]);
         c->timing.decode_ms = ms_between(ev[1], ev[2]);
         c->timing.codec_ms = 0;
         c->timing.steps = steps;
         c->timing.step_ms_avg = steps ? c->timing.decode_ms / steps : 0;
+        c->timing.hbm_bytes_per_step = c->blocks ? c->blocks->weight_bytes_per_step() : 0;
         for (auto& e2 : ev) (void)hipEventDestroy(e2);
         return;
     }
@@ -1611,6 +1765,48 @@ extern "C" mis_status mis_tts_generate_device(mis_tts* c, const int32_t* prompt_
     MIS_API_END
 }
 
+// Token generation without a codec behind it: the prompts' continuations as ids (stop_id < 0: none).  tokens_out [batch][max_tokens], n_tokens
+// [batch]: ids of every row up to and including stop_id.  Serves every architecture of the engine.
+extern "C" mis_status mis_lm_generate(mis_tts* c, const int32_t* prompt_ids, const int32_t* prompt_lens, int batch, const mis_gen_params* params, int stop_id,
+                                      int32_t* tokens_out, int32_t* n_tokens) {
+    MIS_API_BEGIN
+    MIS_REQUIRE(c && tokens_out && n_tokens, MIS_ERR_INVALID_INPUT, "null argument");
+    default_params_check(params);
+    GenOutputs out;
+    HiddenMode hm;
+    hm.on = true; hm.stop_id = stop_id;
+    run_generate(c, prompt_ids, prompt_lens, batch, params, nullptr, nullptr, 0, true, nullptr, nullptr, nullptr, out, &hm);
+    memcpy(tokens_out, out.tokens.data(), out.tokens.size() * 4);
+    for (int b = 0; b < batch; ++b) n_tokens[b] = out.n_tokens[b];
+    MIS_API_END
+}
+// The same with .token events while the loop runs and one .info per row behind it
+extern "C" mis_status mis_lm_generate_stream(mis_tts* c, const int32_t* prompt_ids, const int32_t* prompt_lens, int batch, const mis_gen_params* params, int stop_id,
+                                             mis_event_cb on_event, void* user, const volatile int* cancel_flag) {
+    MIS_API_BEGIN
+    MIS_REQUIRE(c && on_event, MIS_ERR_INVALID_INPUT, "null argument");
+    default_params_check(params);
+    GenOutputs out;
+    HiddenMode hm;
+    hm.on = true; hm.stop_id = stop_id;
+    run_generate(c, prompt_ids, prompt_lens, batch, params, nullptr, nullptr, 0, false, on_event, user, cancel_flag, out, &hm);
+    std::vector<int32_t> lens(batch);
+    HIP_CHECK(hipMemcpy(lens.data(), prompt_lens, (size_t)batch * 4, hipMemcpyDefault));
+    for (int b = 0; b < batch; ++b) {
+        mis_gen_info info{};
+        info.prompt_token_count = lens[b];
+        info.generation_token_count = out.n_tokens[b];
+        info.prefill_time = c->timing.prefill_ms * 1e-3;
+        info.generate_time = c->timing.decode_ms * 1e-3;
+        info.tokens_per_second = info.generate_time > 0 ? out.n_tokens[b] / info.generate_time : 0;
+        size_t free_b = 0, total_b = 0;
+        (void)hipMemGetInfo(&free_b, &total_b);
+        info.peak_memory_gb = (double)(total_b - free_b) / 1e9;
+        on_event(user, b, MIS_EVENT_INFO, &info, 1);
+    }
+    MIS_API_END
+}
+
 // Upper bound of the audio one row can decode to.  parseOutput (LlamaTTS.swift:749-752) keeps everything after the LAST
 // start-of-speech marker - or the whole sequence, prompt included, when the prompt carries none - so the prompt length counts.
 static int64_t max_pcm_per_row(mis_tts* c, const mis_gen_params* p, const int32_t* prompt_lens, int batch) {
@@ -1703,7 +1899,7 @@ extern "C" mis_status mis_tts_last_timing(mis_tts* c, mis_tts_timing* out) {
 
 extern "C" mis_status mis_tts_time_gemm(mis_tts* c, int which, int batch, int iters, double* avg_ms, double* bytes) {
     MIS_API_BEGIN
-    MIS_REQUIRE(c && avg_ms && bytes && iters >= 1, MIS_ERR_INVALID_INPUT, "bad argument");
+    MIS_REQUIRE(c && !c->blocks && avg_ms && bytes && iters >= 1, MIS_ERR_INVALID_INPUT, "bad argument");
     MIS_REQUIRE(c->finalized, MIS_ERR_NOT_INITIALIZED, "model not finalized");
     static const int attn_ctx = std::max(1, env_int("MIS_TIME_ATTN_CTX", 368));      // mean context of the C3 workload
     if (c->batch != batch || (which == 5 && c->Smax < attn_ctx + 1)) lm_reset(c, batch, which == 5 ? attn_ctx + 1 : 64);
@@ -1780,6 +1976,8 @@ extern "C" mis_status mis_tts_load(const char* model_dir, mis_snac* codec, int d
         MIS_REQUIRE(model_dir && out, MIS_ERR_INVALID_INPUT, "null argument");
         std::string dir = model_dir;
         JsonValue j = json_parse(read_text_file(dir + "/config.json"));
+        if (const JsonValue* arch = j.get("architecture"))
+            if (arch->type == JsonValue::STR && block_architecture_known(arch->str)) return mis_lm_load(model_dir, MIS_COMPUTE_BF16, device, out);
         mis_lm_config cf{};
         cf.hidden_size = (int)j.number_or("hidden_size", 0);
         cf.num_hidden_layers = (int)j.number_or("num_hidden_layers", 0);
@@ -1860,6 +2058,39 @@ extern "C" mis_status mis_tts_load(const char* model_dir, mis_snac* codec, int d
         return MIS_ERR_GENERATION_FAILED;
     }
 }
+
+// A language model of any architecture the engine serves, chosen by config.json: "architecture" names a model described layer by layer
+// (compute: bf16 or true float32); everything else is the Llama family (bf16).
+extern "C" mis_status mis_lm_load(const char* model_dir, int compute, int device, mis_tts** out) {
+    mis_tts* c = nullptr;
+    MIS_API_BEGIN
+    MIS_REQUIRE(model_dir && out, MIS_ERR_INVALID_INPUT, "null argument");
+    const std::string dir = model_dir;
+    const JsonValue j = json_parse(read_text_file(dir + "/config.json"));
+    const JsonValue* arch = j.get("architecture");
+    if (!(arch && arch->type == JsonValue::STR && block_architecture_known(arch->str))) {
+        MIS_REQUIRE(compute == MIS_COMPUTE_BF16, MIS_ERR_INVALID_INPUT, "this architecture runs in bf16 only");
+        return mis_tts_load(model_dir, nullptr, device, out);
+    }
+    c = create_block_model(parse_block_model(j), compute == MIS_COMPUTE_F32, device);
+    try {
+        for (auto& path : list_safetensors(dir)) {
+            SafeTensorFile f;
+            f.open(path);
+            for (auto& e : f.entries) {
+                const mis_status st = mis_tts_set_tensor(c, e.name.c_str(), e.data, dtype_from_safetensors(e.dtype), e.shape.data(), (int)e.shape.size());
+                if (st != MIS_OK) { mis_tts_destroy(c); return st; }
+            }
+        }
+        const mis_status st = mis_tts_finalize(c);
+        if (st != MIS_OK) { mis_tts_destroy(c); return st; }
+    } catch (...) { mis_tts_destroy(c); throw; }
+    *out = c;
+    MIS_API_END
+}
+extern "C" int32_t mis_lm_vocab_size(const mis_tts* c) { return c ? c->V : 0; }
+extern "C" int32_t mis_lm_hidden_size(const mis_tts* c) { return c ? c->d : 0; }
+extern "C" int32_t mis_lm_num_layers(const mis_tts* c) { return c ? c->L : 0; }
 
 // ---------------------------------------------------------------------------- diagnostics
 // Cost of a dependent kernel boundary on this machine: a hipGraph of n trivial kernels (mode 0: one

@@ -7,7 +7,10 @@ __host__ __device__ __forceinline__ size_t xpk_index(int m, int k, int MT) {
     return ((((size_t)(k >> 5) * MT + (m >> 4)) * 64) + (((k & 31) >> 3) << 4) + (m & 15)) * 8 + (k & 7);
 }
 
-enum { EPI_PARTIAL = 0, EPI_BF16 = 1, EPI_SILU_MUL = 2, EPI_GELU_PACKED = 3, EPI_SILU_PACKED = 4 };
+enum { EPI_PARTIAL = 0, EPI_BF16 = 1, EPI_SILU_MUL = 2, EPI_GELU_PACKED = 3, EPI_SILU_PACKED = 4,
+       EPI_SPLIT_RELU2 = 5,      // tiles below GemmExtra::split: float32 sums; the others: T(relu(y)^2) in the packed layout (out2)
+       EPI_SOFTCAP = 6 };        // float32: cap tanh(scale y / cap) (cap <= 0: scale y)
+struct GemmExtra { void* out2 = nullptr; int split = 0; float scale = 1.0f, cap = 0.0f; };
 
 void launch_convert_to_bf16(const void* src, int dtype, bf16_t* dst, size_t n, hipStream_t s);
 // MLX affine-quantised matrix (uint32 words, per-group scales / biases of dtype sb_dtype = mis_dtype) -> bf16 [N][K]
@@ -31,7 +34,7 @@ void launch_reduce_residual_rmsnorm(const float* slabs, int S, int Mpad, int N, 
 // in the packed fragment layout (it is the next GEMM's X operand).  EPI_SILU_PACKED: h = T(xW+b), T(h * T(sigmoid(h))) packed.
 // ksb = 2: 128-thread blocks, two waves per item.  U: k-tiles per register buffer (0: 4, or 3 at R = 4); R = 4 is built for <= 32 rows.
 void launch_gemm_skinny(int epi, int R, int ksb, const bf16_t* Wp, const bf16_t* X, void* out, int NT, int KT, int S,
-                        int N_out, int Mpad, hipStream_t s, const bf16_t* bias = nullptr, int U = 0);
+                        int N_out, int Mpad, hipStream_t s, const bf16_t* bias = nullptr, int U = 0, const GemmExtra& ex = GemmExtra());
 // The same GEMM with the residual add + LayerNorm / RMSNorm glue in its prologue (<= 16 rows, K <= 1280; see k_gemm_skinny_norm): X is rebuilt per
 // block from the producer's S_in split-K slabs [S_in][16][K] and the residual stream h_in [16][K]; h_new is written to h_out (!= h_in).
 // ln_bias == nullptr: RMSNorm.  R = 2, eight waves per item.
@@ -49,8 +52,13 @@ void launch_pack_qweight(int bits, const uint32_t* wq, const bf16_t* scales, con
                          int tile_stride, int tile_offset, hipStream_t s);
 
 // batched prefill (lm_prefill.hip): M = positions x rows
-enum { PF_F32 = 0, PF_RESID = 1, PF_SILU = 2 };
-void launch_gemm_pf(int epi, const bf16_t* X, const bf16_t* Wp, void* C, int M, int N, int K, hipStream_t s);
+enum { PF_F32 = 0, PF_RESID = 1, PF_SILU = 2,
+       PF_SPLIT_RELU2 = 3,       // tiles below PfExtra::split: float32 [M][ldc]; the others: T(relu(y)^2) bf16 row-major [M][ld2] at out2
+       PF_SCALED_ADD = 4,        // float32 C[M][ldc] += ls[n] * y
+       PF_ROWS_BF16 = 5,         // bf16 row-major [M][ldc]; rows of X gathered: row m at X + xrow[m] * ldx
+       PF_SOFTCAP = 6 };         // float32 [M][ldc]: cap tanh(scale y / cap)
+struct PfExtra { int ldx = 0; const int32_t* xrow = nullptr; int ldc = 0; void* out2 = nullptr; int split = 0, ld2 = 0; const bf16_t* ls = nullptr; float scale = 1.0f, cap = 0.0f; };
+void launch_gemm_pf(int epi, const bf16_t* X, const bf16_t* Wp, void* C, int M, int N, int K, hipStream_t s, const PfExtra& ex = PfExtra());
 void launch_pf_embed_rmsnorm(const bf16_t* emb, const int32_t* prompt, const int32_t* lens, int Lmax, int t0, int Tc, int batch, int Mpad, int vocab,
                              const bf16_t* wnorm, bf16_t* h, bf16_t* x, int32_t* pos_tab, uint8_t* act_tab, int d, float eps, hipStream_t s);
 void launch_pf_add_resid(bf16_t* h, const float* part, size_t n, hipStream_t s);
@@ -159,6 +167,7 @@ struct SamplerParams {
     int max_tokens;
     unsigned long long* dbg; // diagnostics (null in the product): [16] s_memtime stamps of block (0, 0) of the one-launch sampler
     // host side only (sampler_resolve): which kernels the launcher may pick - fixed per generate call and hashed into the graph key
+    int f32_input;           // 1: logits32 already holds the model's float32 logits (`logits` unused)
     int path_resolved;       // 0: launch_sampler reads MIS_SAMPLER_WIDE / MIS_SAMPLER_SPIN itself, per launch (stand-alone entry point)
     int force_multi;         // 1: the multi-launch kernels whatever the range (shared device, recovery after a time-out, MIS_SAMPLER_WIDE)
     int spin;                // polls per row barrier of the one-launch sampler before it gives up

@@ -631,9 +631,33 @@ __device__ __forceinline__ float gelu_erf(float x) { return 0.5f * x * (1.0f + e
 template <int MT, int R, int EPI>
 __device__ __forceinline__ void gemm_epilogue(const f32x4_t (&acc)[R][MT], void* __restrict__ out, int ntg, int ks,
                                               int NT, int N_out, int Mpad, int lane, int mt_only,
-                                              const bf16_t* __restrict__ bias) {
+                                              const bf16_t* __restrict__ bias, const GemmExtra& ex = GemmExtra()) {
     const int nl = (lane >> 4) * 4, ml = lane & 15;
-    if (EPI == EPI_PARTIAL) {
+    if constexpr (EPI == EPI_SPLIT_RELU2 || EPI == EPI_SOFTCAP) {
+#pragma unroll
+        for (int r = 0; r < R; ++r) {
+            const int tile = ntg * R + r;
+            if (tile >= NT) continue;
+#pragma unroll
+            for (int mt = 0; mt < MT; ++mt) {
+                if (mt_only >= 0 && mt != mt_only) continue;
+                float v[4] = {acc[r][mt][0], acc[r][mt][1], acc[r][mt][2], acc[r][mt][3]};
+                if (EPI == EPI_SPLIT_RELU2 && tile >= ex.split) {
+                    uint16_t res[4];
+#pragma unroll
+                    for (int e = 0; e < 4; ++e) { const float t = fmaxf(v[e], 0.0f); res[e] = f32_to_bf16(t * t); }
+                    *reinterpret_cast<uint2*>((bf16_t*)ex.out2 + xpk_index(mt * 16 + ml, (tile - ex.split) * 16 + nl, MT)) =
+                        make_uint2((uint32_t)res[0] | ((uint32_t)res[1] << 16), (uint32_t)res[2] | ((uint32_t)res[3] << 16));
+                    continue;
+                }
+                if (EPI == EPI_SOFTCAP) {
+#pragma unroll
+                    for (int e = 0; e < 4; ++e) { const float t = v[e] * ex.scale; v[e] = ex.cap > 0.0f ? ex.cap * tanhf(t / ex.cap) : t; }
+                }
+                *reinterpret_cast<float4*>(reinterpret_cast<float*>(out) + ((size_t)mt * 16 + ml) * N_out + tile * 16 + nl) = make_float4(v[0], v[1], v[2], v[3]);
+            }
+        }
+    } else if (EPI == EPI_PARTIAL) {
         float* o = reinterpret_cast<float*>(out);
 #pragma unroll
         for (int r = 0; r < R; ++r) {
@@ -725,7 +749,7 @@ __device__ __forceinline__ void gemm_epilogue(const f32x4_t (&acc)[R][MT], void*
 template <int MT, int R, int EPI, int KSB, int U>
 __global__ void __launch_bounds__((KSB == 1 ? 4 : KSB) * 64, 2) k_gemm_skinny(const bf16_t* __restrict__ Wp, const bf16_t* __restrict__ X,
                                                      void* __restrict__ out, int NT, int KT, int S, int n_items,
-                                                     int N_out, int Mpad, const bf16_t* __restrict__ bias) {
+                                                     int N_out, int Mpad, const bf16_t* __restrict__ bias, GemmExtra ex) {
     static_assert(EPI != EPI_SILU_MUL || (R & 1) == 0, "silu-mul epilogue pairs a gate tile with an up tile");
     // k-tiles per register buffer: 4 at R <= 2; 3 or 2 at four n-tiles per wave (4 would spill: 2 x 4 x (4 + 2) fragments + 32 accumulators)
     constexpr int GU = U;
@@ -834,7 +858,7 @@ __global__ void __launch_bounds__((KSB == 1 ? 4 : KSB) * 64, 2) k_gemm_skinny(co
 #undef GEMM_MATH_TAIL
 
     if (KSB == 1) {
-        gemm_epilogue<MT, R, EPI>(acc, out, ntg, ks, NT, N_out, Mpad, lane, -1, bias);
+        gemm_epilogue<MT, R, EPI>(acc, out, ntg, ks, NT, N_out, Mpad, lane, -1, bias, ex);
     } else {
         __shared__ float4 red[KSB][R * MT][64];
 #pragma unroll
@@ -857,20 +881,20 @@ __global__ void __launch_bounds__((KSB == 1 ? 4 : KSB) * 64, 2) k_gemm_skinny(co
                 for (int m2 = 0; m2 < MT; ++m2)
                     if (m2 == mt) acc[r][m2] = (f32x4_t){s0.x, s0.y, s0.z, s0.w};
             }
-            gemm_epilogue<MT, R, EPI>(acc, out, ntg, ks, NT, N_out, Mpad, lane, mt, bias);
+            gemm_epilogue<MT, R, EPI>(acc, out, ntg, ks, NT, N_out, Mpad, lane, mt, bias, ex);
         }
     }
 }
 
 template <int MT>
 static void launch_gemm_mt(int epi, int R, int ksb, int U, const bf16_t* Wp, const bf16_t* X, void* out, int NT, int KT, int S,
-                           int N_out, int Mpad, const bf16_t* bias, hipStream_t s) {
+                           int N_out, int Mpad, const bf16_t* bias, hipStream_t s, const GemmExtra& ex) {
     int n_items = ((NT + R - 1) / R) * S;
     dim3 grid(ksb == 1 ? (n_items + 3) / 4 : n_items), block((ksb == 1 ? 4 : ksb) * 64);
 #define GEMM_CASE(E, RR, KS, UU)                                                                              \
     if (epi == E && R == RR && ksb == KS && U == UU) {                                                        \
         hipLaunchKernelGGL((k_gemm_skinny<MT, RR, E, KS, UU>), grid, block, 0, s, Wp, X, out, NT, KT, S, n_items, \
-                           N_out, Mpad, bias);                                                                    \
+                           N_out, Mpad, bias, ex);                                                                \
         return;                                                                                               \
     }
     GEMM_CASE(EPI_PARTIAL, 1, 1, 4)
@@ -891,7 +915,11 @@ static void launch_gemm_mt(int epi, int R, int ksb, int U, const bf16_t* Wp, con
         GEMM_CASE(EPI_BF16, 4, 4, 3)
         GEMM_CASE(EPI_BF16, 4, 4, 2)
         GEMM_CASE(EPI_BF16, 4, 2, 3)
+        GEMM_CASE(EPI_SPLIT_RELU2, 4, 4, 3)
+        GEMM_CASE(EPI_SOFTCAP, 4, 4, 3)
     }
+    GEMM_CASE(EPI_SPLIT_RELU2, 2, 4, 4)
+    GEMM_CASE(EPI_SOFTCAP, 2, 4, 4)
     GEMM_CASE(EPI_GELU_PACKED, 2, 4, 4)
     GEMM_CASE(EPI_GELU_PACKED, 1, 4, 4)
     GEMM_CASE(EPI_BF16, 1, 4, 4)
@@ -902,14 +930,14 @@ static void launch_gemm_mt(int epi, int R, int ksb, int U, const bf16_t* Wp, con
 }
 
 void launch_gemm_skinny(int epi, int R, int ksb, const bf16_t* Wp, const bf16_t* X, void* out, int NT, int KT, int S,
-                        int N_out, int Mpad, hipStream_t s, const bf16_t* bias, int U) {
+                        int N_out, int Mpad, hipStream_t s, const bf16_t* bias, int U, const GemmExtra& ex) {
     MIS_REQUIRE(epi == EPI_PARTIAL || S == 1, MIS_ERR_GENERATION_FAILED, "split-K needs the partial epilogue");
     if (U <= 0) U = R >= 4 ? 3 : GEMM_U;
     switch (Mpad / 16) {
-        case 1: launch_gemm_mt<1>(epi, R, ksb, U, Wp, X, out, NT, KT, S, N_out, Mpad, bias, s); break;
-        case 2: launch_gemm_mt<2>(epi, R, ksb, U, Wp, X, out, NT, KT, S, N_out, Mpad, bias, s); break;
-        case 3: launch_gemm_mt<3>(epi, R, ksb, U, Wp, X, out, NT, KT, S, N_out, Mpad, bias, s); break;
-        case 4: launch_gemm_mt<4>(epi, R, ksb, U, Wp, X, out, NT, KT, S, N_out, Mpad, bias, s); break;
+        case 1: launch_gemm_mt<1>(epi, R, ksb, U, Wp, X, out, NT, KT, S, N_out, Mpad, bias, s, ex); break;
+        case 2: launch_gemm_mt<2>(epi, R, ksb, U, Wp, X, out, NT, KT, S, N_out, Mpad, bias, s, ex); break;
+        case 3: launch_gemm_mt<3>(epi, R, ksb, U, Wp, X, out, NT, KT, S, N_out, Mpad, bias, s, ex); break;
+        case 4: launch_gemm_mt<4>(epi, R, ksb, U, Wp, X, out, NT, KT, S, N_out, Mpad, bias, s, ex); break;
         default: throw MisError(MIS_ERR_INVALID_INPUT, "batch per GPU must be <= 64");
     }
 }

@@ -1,0 +1,821 @@
+// lm_latent.hip - kernels of the layer-list language models (see lm_latent.h): float32 residual stream, layer-scaled parallel branches,
+// latent attention with a sliding window, rotary tables with YaRN scaling, and the true-float32 GEMM of the 32-bit mode.
+//
+// Latent attention.  A token leaves ONE cache row [c | k_r]: the RMS-normed latent c (R values, shared by all heads) and the rotated key
+// part k_r (r values, shared by all heads).  Two algebraically equal forms are used:
+//   absorbed (decode)   q_lat = W_uk^T q_plain;  score = q_lat . c + q_rot . k_r;  o_lat = sum_j p_j c_j;  out = W_uv o_lat
+//                       - a decode step reads R + r values per cached token whatever the number of heads;
+//   expanded (prompts)  k = W_uk c, v = W_uv c for every key row by one GEMM, then ordinary tiled attention with n + r and v dimensions
+//                       - (n + r + v) instead of (2 R + r) multiplications per (query, key, head).
+// Scores, the softmax and its weights are float32 in both; the weights enter the matrix cores as bf16 hi + lo pairs.
+#include "lm_latent.h"
+#include <math.h>
+
+// ============================================================================ rotary tables (host)
+// Pair i of a rotated vector turns by pos * f_i, f_i = base^(-2 i / dims).  YaRN: a pair that turns more than `fast` times over the original
+// context keeps f_i, one that turns less than `slow` times gets f_i / factor, a linear ramp over the pair index between; both cos and sin
+// are multiplied by 0.1 ln(factor) + 1.
+void rotary_tables_host(const RotarySpec& r, int positions, std::vector<float>& cos_out, std::vector<float>& sin_out) {
+    const int half = r.dims / 2;
+    std::vector<double> f(half);
+    double mag = 1.0;
+    for (int i = 0; i < half; ++i) f[i] = pow(r.base, -2.0 * i / r.dims);
+    if (r.yarn) {
+        auto dim_of_turns = [&](double turns) { return r.dims * log(r.original / (2.0 * M_PI * turns)) / (2.0 * log(r.base)); };
+        const double lo = std::max(floor(dim_of_turns(r.fast)), 0.0), hi = std::min(ceil(dim_of_turns(r.slow)), (double)(r.dims - 1));
+        for (int i = 0; i < half; ++i) {
+            const double ramp = std::min(std::max((i - lo) / std::max(hi - lo, 0.001), 0.0), 1.0);
+            f[i] = f[i] / r.factor * ramp + f[i] * (1.0 - ramp);
+        }
+        mag = 0.1 * log(r.factor) + 1.0;
+    }
+    cos_out.resize((size_t)positions * half);
+    sin_out.resize((size_t)positions * half);
+    for (int p = 0; p < positions; ++p)
+        for (int i = 0; i < half; ++i) {
+            const double a = (double)p * f[i];
+            cos_out[(size_t)p * half + i] = (float)(cos(a) * mag);
+            sin_out[(size_t)p * half + i] = (float)(sin(a) * mag);
+        }
+}
+
+LatentDims latent_dims(int H, int n, int r, int v, int R, int window, int rot_dims, float scale, float eps) {
+    LatentDims D{};
+    D.H = H; D.n = n; D.r = r; D.v = v; D.R = R;
+    D.np = (int)round_up(n, 32); D.rp = (int)round_up(r, 16); D.vp = (int)round_up(v, 16);
+    D.Rp = std::max(128, (int)round_up(R, 64));
+    D.CW = (int)round_up(D.Rp + D.rp, 32);
+    D.DK = (int)round_up(D.np + D.rp, 32);
+    D.window = window; D.rot_dims = rot_dims; D.scale = scale; D.eps = eps;
+    return D;
+}
+
+// ============================================================================ small helpers
+__device__ __forceinline__ float lat_block_sum(float v, float* red) {          // any block of whole waves; every thread gets the total
+    v = wave_sum_dpp(v);
+    if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = v;
+    __syncthreads();
+    const int nw = blockDim.x >> 6;
+    float t = 0.0f;
+    for (int i = 0; i < nw; ++i) t += red[i];
+    __syncthreads();
+    return t;
+}
+__device__ __forceinline__ void load4_bf16(const bf16_t* p, float (&o)[4]) {
+    const uint2 q = *reinterpret_cast<const uint2*>(p);
+    o[0] = bf16_to_f32((bf16_t)(q.x & 0xffffu)); o[1] = bf16_to_f32((bf16_t)(q.x >> 16));
+    o[2] = bf16_to_f32((bf16_t)(q.y & 0xffffu)); o[3] = bf16_to_f32((bf16_t)(q.y >> 16));
+}
+__device__ __forceinline__ uint2 pack4_bf16(const float (&v)[4]) {
+    return make_uint2((uint32_t)f32_to_bf16(v[0]) | ((uint32_t)f32_to_bf16(v[1]) << 16), (uint32_t)f32_to_bf16(v[2]) | ((uint32_t)f32_to_bf16(v[3]) << 16));
+}
+// four consecutive columns k .. k + 3 (k % 4 == 0) of operand row m
+__device__ __forceinline__ void operand_store4(const Operand& h, int m, int k, const float (&v)[4]) {
+    if (h.kind == OPK_F32) *reinterpret_cast<float4*>((float*)h.p + (size_t)m * h.ld + k) = make_float4(v[0], v[1], v[2], v[3]);
+    else {
+        bf16_t* o = (bf16_t*)h.p + (h.kind == OPK_PACKED ? xpk_index(m, k, h.MT) : (size_t)m * h.ld + k);
+        *reinterpret_cast<uint2*>(o) = pack4_bf16(v);
+    }
+}
+__device__ __forceinline__ void operand_store1(const Operand& h, int m, int k, float v) {
+    if (h.kind == OPK_F32) ((float*)h.p)[(size_t)m * h.ld + k] = v;
+    else ((bf16_t*)h.p)[h.kind == OPK_PACKED ? xpk_index(m, k, h.MT) : (size_t)m * h.ld + k] = f32_to_bf16(v);
+}
+
+// ============================================================================ embedding, residual + layer scale + norm
+// CPT groups of four columns per thread; columns of the width padding (d .. dp) hold zeros everywhere (weights, tables, stream)
+template <int CPT>
+__global__ void __launch_bounds__(1024) k_rows_embed_norm2(const bf16_t* __restrict__ emb, const int32_t* __restrict__ ids, int vocab,
+                                                           const bf16_t* __restrict__ g_embed, const bf16_t* __restrict__ g_norm, float* __restrict__ x,
+                                                           Operand h, int d, int dp, float eps, int n_rows, const uint8_t* __restrict__ on,
+                                                           int32_t* __restrict__ pos_cur, int32_t* __restrict__ pos_next) {
+    __shared__ float red[16];
+    const int m = blockIdx.x, tid = threadIdx.x, nth = blockDim.x, nc = dp >> 2;
+    int id = m < n_rows ? ids[m] : 0;
+    if (id < 0 || id >= vocab) id = 0;
+    if (pos_next && tid == 0 && m < n_rows) {
+        const int p = pos_next[m];
+        pos_cur[m] = p;
+        if (on[m]) pos_next[m] = p + 1;
+    }
+    float e[CPT][4], ge[CPT][4], gn[CPT][4], ss = 0.0f;
+#pragma unroll
+    for (int g = 0; g < CPT; ++g) {
+        const int c = tid + g * nth, cc = c < nc ? c : 0;
+        load4_bf16(emb + (size_t)id * dp + 4 * cc, e[g]);
+        load4_bf16(g_embed + 4 * cc, ge[g]);
+        load4_bf16(g_norm + 4 * cc, gn[g]);
+#pragma unroll
+        for (int j = 0; j < 4; ++j) ss += c < nc ? e[g][j] * e[g][j] : 0.0f;
+    }
+    const float inv = 1.0f / sqrtf(lat_block_sum(ss, red) / (float)d + eps);
+    float s2 = 0.0f;
+#pragma unroll
+    for (int g = 0; g < CPT; ++g) {
+        const int c = tid + g * nth;
+#pragma unroll
+        for (int j = 0; j < 4; ++j) { e[g][j] = e[g][j] * inv * ge[g][j]; s2 += c < nc ? e[g][j] * e[g][j] : 0.0f; }
+        if (c < nc) *reinterpret_cast<float4*>(x + (size_t)m * dp + 4 * c) = make_float4(e[g][0], e[g][1], e[g][2], e[g][3]);
+    }
+    const float inv2 = 1.0f / sqrtf(lat_block_sum(s2, red) / (float)d + eps);
+#pragma unroll
+    for (int g = 0; g < CPT; ++g) {
+        const int c = tid + g * nth;
+        float o[4];
+#pragma unroll
+        for (int j = 0; j < 4; ++j) o[j] = e[g][j] * inv2 * gn[g][j];
+        if (c < nc) operand_store4(h, m, 4 * c, o);
+    }
+}
+
+// SG >= number of slabs of either branch (clamped, unconditional loads: one round trip); SG = 0: no slabs, the stream is only normed
+template <int CPT, int SG>
+__global__ void __launch_bounds__(1024) k_scaled_residual_norm(ScaledSlabs A, ScaledSlabs B, int slab_rows, float* __restrict__ x, const int32_t* __restrict__ row_of,
+                                                               const bf16_t* __restrict__ g_norm, Operand h, int d, int dp, float eps) {
+    __shared__ float red[16];
+    const int m = blockIdx.x, tid = threadIdx.x, nth = blockDim.x, nc = dp >> 2;
+    const size_t xr = (size_t)(row_of ? row_of[m] : m) * dp;
+    float v[CPT][4], gn[CPT][4], ss = 0.0f;
+#pragma unroll
+    for (int g = 0; g < CPT; ++g) {
+        const int c = tid + g * nth, cc = c < nc ? c : 0;
+        const float4 t = *reinterpret_cast<const float4*>(x + xr + 4 * cc);
+        v[g][0] = t.x; v[g][1] = t.y; v[g][2] = t.z; v[g][3] = t.w;
+        load4_bf16(g_norm + 4 * cc, gn[g]);
+    }
+    if constexpr (SG > 0) {
+#pragma unroll
+        for (int br = 0; br < 2; ++br) {
+            const ScaledSlabs& P = br ? B : A;
+            if (P.S == 0) continue;                              // uniform
+            float4 sl[CPT][SG];
+            float ls[CPT][4];
+#pragma unroll
+            for (int g = 0; g < CPT; ++g) {
+                const int c = tid + g * nth, cc = c < nc ? c : 0;
+#pragma unroll
+                for (int j = 0; j < SG; ++j)
+                    sl[g][j] = *reinterpret_cast<const float4*>(P.p + ((size_t)(j < P.S ? j : P.S - 1) * slab_rows + m) * dp + 4 * cc);
+                load4_bf16(P.ls + 4 * cc, ls[g]);
+            }
+#pragma unroll
+            for (int g = 0; g < CPT; ++g) {
+                float a[4] = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+                for (int j = 0; j < SG; ++j) {                   // slab order 0, 1, 2, ...: deterministic
+                    const bool live = j < P.S;
+                    a[0] += live ? sl[g][j].x : 0.0f; a[1] += live ? sl[g][j].y : 0.0f; a[2] += live ? sl[g][j].z : 0.0f; a[3] += live ? sl[g][j].w : 0.0f;
+                }
+#pragma unroll
+                for (int j = 0; j < 4; ++j) v[g][j] += ls[g][j] * a[j];
+            }
+        }
+#pragma unroll
+        for (int g = 0; g < CPT; ++g) {
+            const int c = tid + g * nth;
+            if (c < nc) *reinterpret_cast<float4*>(x + xr + 4 * c) = make_float4(v[g][0], v[g][1], v[g][2], v[g][3]);
+        }
+    }
+#pragma unroll
+    for (int g = 0; g < CPT; ++g)
+#pragma unroll
+        for (int j = 0; j < 4; ++j) ss += tid + g * nth < nc ? v[g][j] * v[g][j] : 0.0f;
+    const float inv = 1.0f / sqrtf(lat_block_sum(ss, red) / (float)d + eps);
+#pragma unroll
+    for (int g = 0; g < CPT; ++g) {
+        const int c = tid + g * nth;
+        float o[4];
+#pragma unroll
+        for (int j = 0; j < 4; ++j) o[j] = v[g][j] * inv * gn[g][j];
+        if (c < nc) operand_store4(h, m, 4 * c, o);
+    }
+}
+
+static int row_cpt(int dp) { const int nc = dp / 4; return nc <= 1024 ? (nc >= 512 ? 2 : 1) : (nc <= 2048 ? 2 : 4); }
+static int row_threads(int dp, int cpt) { return (int)round_up(cdiv(dp / 4, cpt), 64); }
+static void row_check(int dp) { MIS_REQUIRE(dp % 4 == 0 && dp <= 16384, MIS_ERR_INVALID_INPUT, "model width above 16384"); }
+
+void launch_rows_embed_norm2(const bf16_t* emb, const int32_t* ids, int vocab, const bf16_t* g_embed, const bf16_t* g_norm, float* x, const Operand& h,
+                             int d, int dp, float eps, int n_rows, int rows, const uint8_t* on, int32_t* pos_cur, int32_t* pos_next, hipStream_t s) {
+    row_check(dp);
+    const int cpt = row_cpt(dp), nth = row_threads(dp, cpt);
+#define EMB2(C) hipLaunchKernelGGL((k_rows_embed_norm2<C>), dim3(rows), dim3(nth), 0, s, emb, ids, vocab, g_embed, g_norm, x, h, d, dp, eps, n_rows, on, pos_cur, pos_next)
+    if (cpt == 1) EMB2(1); else if (cpt == 2) EMB2(2); else EMB2(4);
+#undef EMB2
+}
+static void residual_norm(const ScaledSlabs& a, const ScaledSlabs& b, int slab_rows, float* x, const int32_t* row_of, const bf16_t* g_norm, const Operand& h,
+                          int d, int dp, float eps, int rows, hipStream_t s) {
+    row_check(dp);
+    const int cpt = row_cpt(dp), nth = row_threads(dp, cpt), S = std::max(a.S, b.S);
+    MIS_REQUIRE(S <= 8, MIS_ERR_GENERATION_FAILED, "more than 8 split-K slabs per branch");
+#define RN(C, G) hipLaunchKernelGGL((k_scaled_residual_norm<C, G>), dim3(rows), dim3(nth), 0, s, a, b, slab_rows, x, row_of, g_norm, h, d, dp, eps)
+#define RNC(C) do { if (S == 0) RN(C, 0); else if (S == 1) RN(C, 1); else if (S == 2) RN(C, 2); else if (S <= 4) RN(C, 4); else RN(C, 8); } while (0)
+    if (cpt == 1) RNC(1); else if (cpt == 2) RNC(2); else RNC(4);
+#undef RNC
+#undef RN
+}
+void launch_scaled_residual_norm(const ScaledSlabs& a, const ScaledSlabs& b, int slab_rows, float* x, const bf16_t* g_norm, const Operand& h, int d, int dp,
+                                 float eps, int rows, hipStream_t s) {
+    residual_norm(a, b, slab_rows, x, nullptr, g_norm, h, d, dp, eps, rows, s);
+}
+void launch_gather_norm(const float* x, const int32_t* row_of, const bf16_t* g_norm, const Operand& h, int d, int dp, float eps, int rows, hipStream_t s) {
+    residual_norm(ScaledSlabs{}, ScaledSlabs{}, 0, const_cast<float*>(x), row_of, g_norm, h, d, dp, eps, rows, s);
+}
+
+// ============================================================================ float32 GEMM (v_mfma_f32_16x16x4_f32)
+// Weight tiles are the bf16 fragments of the other GEMMs: lane q*16 + i holds W[16 nt + i][32 kt + 8 q .. + 8].  Taking element e of every lane
+// as one K = 4 step (k = 8 q + e for q = 0..3) needs no re-layout; the other operand is read as X[m][32 kt + 8 q + e].
+template <int EPI>
+__global__ void __launch_bounds__(256) k_gemm_f32(GemmF32 g) {
+    const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+    const int nt = blockIdx.x * 4 + wave, m0 = blockIdx.y * 64, z = blockIdx.z;
+    if (nt >= g.NT) return;
+    const int li = lane & 15, q = lane >> 4;
+    const bf16_t* wp = g.W + g.wz * z + ((size_t)nt * g.KT * 64 + lane) * 8;
+    const float* xp[4];
+#pragma unroll
+    for (int j = 0; j < 4; ++j) xp[j] = g.X + g.xz * z + (size_t)min(m0 + j * 16 + li, g.M - 1) * g.ldx + q * 8;
+    f32x4_t acc[4];
+#pragma unroll
+    for (int j = 0; j < 4; ++j) acc[j] = (f32x4_t){0.f, 0.f, 0.f, 0.f};
+    for (int kt = 0; kt < g.KT; ++kt) {
+        const bf16x8_t w = *reinterpret_cast<const bf16x8_t*>(wp + (size_t)kt * 512);
+        float wf[8];
+#pragma unroll
+        for (int e = 0; e < 8; ++e) wf[e] = bf16_to_f32((bf16_t)w[e]);
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+            const float4 a = *reinterpret_cast<const float4*>(xp[j] + kt * 32), b = *reinterpret_cast<const float4*>(xp[j] + kt * 32 + 4);
+            const float xf[8] = {a.x, a.y, a.z, a.w, b.x, b.y, b.z, b.w};
+#pragma unroll
+            for (int e = 0; e < 8; ++e) acc[j] = __builtin_amdgcn_mfma_f32_16x16x4f32(wf[e], xf[e], acc[j], 0, 0, 0);
+        }
+    }
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+        const int m = m0 + j * 16 + li;
+        if (m >= g.M) continue;
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+            const int n = nt * 16 + q * 4 + e;
+            if (n >= g.n_valid) continue;
+            float* o = g.out + (size_t)m * g.ldo + g.oz * z + n;
+            const float v = acc[j][e];
+            if (EPI == F32_STORE) *o = v;
+            else if (EPI == F32_RELU2) { const float t = fmaxf(v, 0.0f); *o = t * t; }
+            else if (EPI == F32_ADD_SCALED) *o += bf16_to_f32(g.ls[n]) * v;
+            else { const float t = v * g.scale; *o = g.cap > 0.0f ? g.cap * tanhf(t / g.cap) : t; }
+        }
+    }
+}
+void launch_gemm_f32(const GemmF32& g, hipStream_t s) {
+    MIS_REQUIRE(g.M >= 1 && g.NT >= 1 && g.KT >= 1 && g.ldx % 4 == 0 && g.xz % 4 == 0, MIS_ERR_GENERATION_FAILED, "float32 GEMM: bad shape");
+    dim3 grid(cdiv(g.NT, 4), cdiv(g.M, 64), g.heads);
+    if (g.epi == F32_STORE) hipLaunchKernelGGL((k_gemm_f32<F32_STORE>), grid, dim3(256), 0, s, g);
+    else if (g.epi == F32_RELU2) hipLaunchKernelGGL((k_gemm_f32<F32_RELU2>), grid, dim3(256), 0, s, g);
+    else if (g.epi == F32_ADD_SCALED) hipLaunchKernelGGL((k_gemm_f32<F32_ADD_SCALED>), grid, dim3(256), 0, s, g);
+    else hipLaunchKernelGGL((k_gemm_f32<F32_SOFTCAP>), grid, dim3(256), 0, s, g);
+}
+
+// ============================================================================ projections -> cache row and query rows
+__device__ __forceinline__ void put(float* p, float v) { *p = v; }
+__device__ __forceinline__ void put(bf16_t* p, float v) { *p = f32_to_bf16(v); }
+__device__ __forceinline__ float get(const float* p) { return *p; }
+__device__ __forceinline__ float get(const bf16_t* p) { return bf16_to_f32(*p); }
+
+// element j of a rotated vector of r values whose first rot_dims are rotated pairwise (2 i, 2 i + 1); zero past r
+__device__ __forceinline__ float rotary_at(const float* src, int j, int r, int rot_dims, const float* cs, const float* sn) {
+    if (j >= r) return 0.0f;
+    if (j >= rot_dims) return src[j];
+    const float c = cs[j >> 1], s = sn[j >> 1];
+    return (j & 1) ? src[j] * c + src[j - 1] * s : src[j] * c - src[j + 1] * s;
+}
+
+template <typename T>
+__device__ __forceinline__ void latent_row(const LatentDims& D, const LatentRows& p, int m, float* red) {
+    const int tid = threadIdx.x, nth = blockDim.x, HQ = D.np + D.rp;
+    if (p.rows.on && !p.rows.on[m]) return;                                    // block-uniform
+    const int pos = p.rows.pos[m], seq = p.rows.seq ? p.rows.seq[m] : m;
+    const float* row = p.qkv + (size_t)m * p.ld;
+    const float* craw = row + (size_t)D.H * HQ;
+    const float *cs = p.rope_cos + (size_t)pos * (D.rot_dims / 2), *sn = p.rope_sin + (size_t)pos * (D.rot_dims / 2);
+    float ss = 0.0f;
+    for (int i = tid; i < D.R; i += nth) ss += craw[i] * craw[i];
+    const float inv = 1.0f / sqrtf(lat_block_sum(ss, red) / (float)D.R + D.eps);
+    T* cache = (T*)p.cache + ((size_t)seq * p.Smax + pos) * D.CW;
+    for (int i = tid; i < D.CW; i += nth) {
+        float v = 0.0f;
+        if (i < D.R) v = craw[i] * inv * bf16_to_f32(p.c_norm[i]);
+        else if (i >= D.Rp) v = rotary_at(craw + D.Rp, i - D.Rp, D.r, D.rot_dims, cs, sn);
+        put(cache + i, v);
+    }
+    T* q = (T*)p.q + (size_t)m * D.H * p.q_ld;
+    const int j0 = p.with_plain ? 0 : p.q_rot_off, w = p.q_ld - j0;
+    for (int t = tid; t < D.H * w; t += nth) {
+        const int hd = t / w, j = j0 + (t - hd * w);
+        const float* src = row + (size_t)hd * HQ;
+        put(q + (size_t)hd * p.q_ld + j, j < p.q_rot_off ? src[j] : rotary_at(src + D.np, j - p.q_rot_off, D.r, D.rot_dims, cs, sn));
+    }
+}
+template <typename T>
+__global__ void __launch_bounds__(256) k_latent_rows(LatentDims D, LatentRows p) {
+    __shared__ float red[4];
+    latent_row<T>(D, p, blockIdx.x, red);
+}
+static void latent_rows_check(const LatentDims& D, const LatentRows& p) {
+    MIS_REQUIRE(p.rows.pos && p.Smax >= 1 && D.rot_dims % 2 == 0 && D.rot_dims <= D.r && p.q_rot_off + D.r <= p.q_ld && (!p.with_plain || p.q_rot_off == D.np),
+                MIS_ERR_GENERATION_FAILED, "latent rows: bad layout");
+}
+void launch_latent_rows(const LatentDims& D, const LatentRows& p, int rows, hipStream_t s) {
+    latent_rows_check(D, p);
+    if (p.f32) hipLaunchKernelGGL((k_latent_rows<float>), dim3(rows), dim3(256), 0, s, D, p);
+    else hipLaunchKernelGGL((k_latent_rows<bf16_t>), dim3(rows), dim3(256), 0, s, D, p);
+}
+
+// ---- per-head GEMM of a few rows: A = packed weight tiles of the head, B = rows (converted to bf16 fragments on the fly)
+__device__ __forceinline__ bf16x8_t frag8(const float* p) {
+    const float4 a = *reinterpret_cast<const float4*>(p), b = *reinterpret_cast<const float4*>(p + 4);
+    const float f[8] = {a.x, a.y, a.z, a.w, b.x, b.y, b.z, b.w};
+    bf16x8_t r;
+#pragma unroll
+    for (int e = 0; e < 8; ++e) r[e] = (short)f32_to_bf16(f[e]);
+    return r;
+}
+__device__ __forceinline__ bf16x8_t frag8(const bf16_t* p) { return *reinterpret_cast<const bf16x8_t*>(p); }
+
+// two row tiles (32 rows from m0) x one weight tile over KT k-tiles
+template <typename T>
+__device__ __forceinline__ void head_tile(const T* X, size_t ldx, int m0, int rows, const bf16_t* wt, int KT, f32x4_t (&acc)[2]) {
+    const int lane = threadIdx.x & 63, li = lane & 15, q = lane >> 4;
+    const T* x0 = X + (size_t)min(m0 + li, rows - 1) * ldx + q * 8;
+    const T* x1 = X + (size_t)min(m0 + 16 + li, rows - 1) * ldx + q * 8;
+    acc[0] = acc[1] = (f32x4_t){0.f, 0.f, 0.f, 0.f};
+#pragma unroll 4
+    for (int kt = 0; kt < KT; ++kt) {
+        const bf16x8_t a = *reinterpret_cast<const bf16x8_t*>(wt + ((size_t)kt * 64 + lane) * 8);
+        const bf16x8_t b0 = frag8(x0 + kt * 32), b1 = frag8(x1 + kt * 32);
+        acc[0] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, b0, acc[0], 0, 0, 0);
+        acc[1] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, b1, acc[1], 0, 0, 0);
+    }
+}
+
+// blocks [0, n_abs): q_lat tiles (4 waves = 4 latent tiles of one head, 32 rows); blocks behind: one row each (latent_row)
+__global__ void __launch_bounds__(256) k_latent_absorb(LatentDims D, LatentRows p, const bf16_t* __restrict__ uk_t, int rows, int n_abs, int mblocks) {
+    __shared__ float red[4];
+    if ((int)blockIdx.x >= n_abs) { latent_row<bf16_t>(D, p, blockIdx.x - n_abs, red); return; }
+    const int tb = D.Rp / 64;                                                   // blocks of four latent tiles per head
+    const int mb = blockIdx.x % mblocks, t = blockIdx.x / mblocks;
+    const int hd = t / tb, rt = (t - hd * tb) * 4 + (threadIdx.x >> 6);
+    const int KT = D.np / 32, HQ = D.np + D.rp, m0 = mb * 32;
+    f32x4_t acc[2];
+    head_tile<float>(p.qkv + (size_t)hd * HQ, p.ld, m0, rows, uk_t + ((size_t)hd * (D.Rp / 16) + rt) * KT * 512, KT, acc);
+    const int lane = threadIdx.x & 63;
+#pragma unroll
+    for (int j = 0; j < 2; ++j) {
+        const int m = m0 + j * 16 + (lane & 15);
+        if (m >= rows) continue;
+        const float v[4] = {acc[j][0], acc[j][1], acc[j][2], acc[j][3]};
+        *reinterpret_cast<uint2*>((bf16_t*)p.q + ((size_t)m * D.H + hd) * p.q_ld + rt * 16 + (lane >> 4) * 4) = pack4_bf16(v);
+    }
+}
+void launch_latent_absorb(const LatentDims& D, const LatentRows& p, const bf16_t* uk_t, int rows, hipStream_t s) {
+    latent_rows_check(D, p);
+    MIS_REQUIRE(!p.f32 && !p.with_plain && p.q_rot_off == D.Rp && p.q_ld == D.CW && p.ld % 4 == 0, MIS_ERR_GENERATION_FAILED, "latent absorb: bad layout");
+    const int mblocks = cdiv(rows, 32), n_abs = D.H * (D.Rp / 64) * mblocks;
+    hipLaunchKernelGGL(k_latent_absorb, dim3(n_abs + rows), dim3(256), 0, s, D, p, uk_t, rows, n_abs, mblocks);
+}
+
+// one wave per (head, value tile, 32 rows)
+__global__ void __launch_bounds__(256) k_latent_values(LatentDims D, const bf16_t* __restrict__ o_lat, const bf16_t* __restrict__ uv, size_t uvz, Operand out, int rows) {
+    const int vt = D.vp / 16, item = blockIdx.x * 4 + (threadIdx.x >> 6);
+    if (item >= D.H * vt) return;
+    const int hd = item / vt, t = item - hd * vt, m0 = blockIdx.y * 32, lane = threadIdx.x & 63, KT = D.Rp / 32;
+    f32x4_t acc[2];
+    head_tile<bf16_t>(o_lat + (size_t)hd * D.Rp, (size_t)D.H * D.Rp, m0, rows, uv + uvz * hd + (size_t)t * KT * 512, KT, acc);
+#pragma unroll
+    for (int j = 0; j < 2; ++j) {
+        const int m = m0 + j * 16 + (lane & 15), c = t * 16 + (lane >> 4) * 4;
+        if (m >= rows) continue;
+        if (D.v % 4 == 0) {
+            const float v[4] = {acc[j][0], acc[j][1], acc[j][2], acc[j][3]};
+            if (c < D.v) operand_store4(out, m, hd * D.v + c, v);
+        } else {
+#pragma unroll
+            for (int e = 0; e < 4; ++e) if (c + e < D.v) operand_store1(out, m, hd * D.v + c + e, acc[j][e]);
+        }
+    }
+}
+void launch_latent_values(const LatentDims& D, const bf16_t* o_lat, const bf16_t* uv, size_t uvz, const Operand& out, int rows, hipStream_t s) {
+    hipLaunchKernelGGL(k_latent_values, dim3(cdiv((int64_t)D.H * (D.vp / 16), 4), cdiv(rows, 32)), dim3(256), 0, s, D, o_lat, uv, uvz, out, rows);
+}
+
+// ============================================================================ absorbed attention, any sizes (float32 mode; bf16 sizes past the MFMA kernel)
+#define LAT_OC 8                                   // latent columns per thread: Rp <= 256 * LAT_OC
+template <typename T>
+__global__ void __launch_bounds__(256) k_latent_attn_any(LatentDims D, LatentAttn p) {
+    extern __shared__ float sm[];                  // q [CW] | weights [256] | red [8]
+    float *sq = sm, *sw = sm + D.CW, *red = sw + 256;
+    const int m = blockIdx.x, hd = blockIdx.y, tid = threadIdx.x, lane = tid & 63;
+    T* out = (T*)p.out + ((size_t)m * D.H + hd) * D.Rp;
+    if (p.rows.on && !p.rows.on[m]) { for (int i = tid; i < D.Rp; i += 256) put(out + i, 0.0f); return; }
+    const int pos = p.rows.pos[m], seq = p.rows.seq ? p.rows.seq[m] : m;
+    const int lo = D.window > 0 ? max(0, pos - D.window + 1) : 0;
+    const T* q = (const T*)p.q + ((size_t)m * D.H + hd) * D.CW;
+    const T* cache = (const T*)p.cache + (size_t)seq * p.Smax * D.CW;
+    for (int i = tid; i < D.CW; i += 256) sq[i] = get(q + i);
+    __syncthreads();
+    float mx = -INFINITY, sum = 0.0f, acc[LAT_OC];
+#pragma unroll
+    for (int j = 0; j < LAT_OC; ++j) acc[j] = 0.0f;
+    for (int k0 = lo; k0 <= pos; k0 += 256) {
+        const int key = k0 + tid;
+        float sc = -INFINITY;
+        if (key <= pos) {
+            const T* kr = cache + (size_t)key * D.CW;
+            float a = 0.0f;
+            for (int i = 0; i < D.CW; i += 8) {
+#pragma unroll
+                for (int e = 0; e < 8; ++e) a += sq[i + e] * get(kr + i + e);
+            }
+            sc = a * D.scale;
+        }
+        float cm = wave_max(sc);
+        if (lane == 0) red[tid >> 6] = cm;
+        __syncthreads();
+        cm = fmaxf(fmaxf(red[0], red[1]), fmaxf(red[2], red[3]));
+        const float mn = fmaxf(mx, cm), alpha = expf(mx - mn);
+        const float w = key <= pos ? expf(sc - mn) : 0.0f;
+        sw[tid] = w;
+        const float ws = wave_sum(w);
+        if (lane == 0) red[4 + (tid >> 6)] = ws;
+        __syncthreads();
+        sum = sum * alpha + ((red[4] + red[5]) + (red[6] + red[7]));
+        mx = mn;
+        const int nk = min(256, pos - k0 + 1);
+#pragma unroll
+        for (int j = 0; j < LAT_OC; ++j) {
+            const int c = tid + 256 * j;
+            if (c >= D.Rp) continue;
+            float a = acc[j] * alpha;
+            for (int k = 0; k < nk; ++k) a += sw[k] * get(cache + (size_t)(k0 + k) * D.CW + c);
+            acc[j] = a;
+        }
+        __syncthreads();
+    }
+#pragma unroll
+    for (int j = 0; j < LAT_OC; ++j) {
+        const int c = tid + 256 * j;
+        if (c < D.Rp) put(out + c, acc[j] / sum);
+    }
+}
+
+// ============================================================================ absorbed attention on the matrix cores (decode)
+// Block = 4 waves: one row, one tile of 16 heads, one share of the row's 32-key tiles.  A key tile is read ONCE: each thread fetches 4 keys x 8
+// columns, writes them to LDS as key rows (score operand) and, transposed in registers, as column rows (value operand).  Scores: S^T = K q^T,
+// wave w = (key half w & 1, half w >> 1 of the columns); the halves meet in LDS, every wave then holds the 16 x 32 weights as the A operand
+// of its own quarter of the latent columns.  The next tile's loads are in flight during all of it (barriers wait for LDS only).
+#define LAT_KT 32
+#define LAT_VS 36                                  // LDS stride of a transposed column (32 keys + 4)
+__device__ __forceinline__ void lds_barrier() { asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory"); }
+__device__ __forceinline__ bf16x8_t lds_frag(const bf16_t* p) {       // 8 values, 8-byte aligned
+    union { uint2 u[2]; bf16x8_t v; } r;
+    r.u[0] = reinterpret_cast<const uint2*>(p)[0];
+    r.u[1] = reinterpret_cast<const uint2*>(p)[1];
+    return r.v;
+}
+// 4 keys x 8 columns -> column e: the four keys packed
+__device__ __forceinline__ uint2 column_of(const uint4 (&r)[4], int e) {
+    const uint32_t a[4] = {r[0].x, r[0].y, r[0].z, r[0].w}, b[4] = {r[1].x, r[1].y, r[1].z, r[1].w}, c[4] = {r[2].x, r[2].y, r[2].z, r[2].w},
+                   d[4] = {r[3].x, r[3].y, r[3].z, r[3].w};
+    const int w = e >> 1;
+    if (e & 1) return make_uint2((a[w] >> 16) | (b[w] & 0xffff0000u), (c[w] >> 16) | (d[w] & 0xffff0000u));
+    return make_uint2((a[w] & 0xffffu) | (b[w] << 16), (c[w] & 0xffffu) | (d[w] << 16));
+}
+static size_t latent_decode_lds(const LatentDims& D) {
+    return (size_t)LAT_KT * (D.CW + 8) * 2 + (size_t)D.Rp * LAT_VS * 2 + 2 * 16 * 36 * 4;
+}
+// NTW: latent tiles per wave (Rp / 64 <= NTW); NST: staging rounds (CW <= 256 NST); QF: query fragments per wave (CW / 32 <= 2 QF)
+template <int NTW, int NST, int QF>
+__global__ void __launch_bounds__(256, 2) k_latent_attn_decode(LatentDims D, LatentAttn p, int rows) {
+    extern __shared__ __attribute__((aligned(16))) uint8_t lds[];
+    const int KS = D.CW + 8;
+    bf16_t* sk = reinterpret_cast<bf16_t*>(lds);                                // [32][CW + 8]
+    bf16_t* sv = sk + (size_t)LAT_KT * KS;                                      // [Rp][LAT_VS]
+    float* sc = reinterpret_cast<float*>(sv + (size_t)D.Rp * LAT_VS);           // [2][16][36]
+    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, li = lane & 15, lq = lane >> 4;
+    const int m = blockIdx.x / p.S, sp = blockIdx.x - m * p.S, h0 = blockIdx.y * 16;
+    const bool on = !p.rows.on || p.rows.on[m];
+    const int pos = on ? p.rows.pos[m] : 0, seq = p.rows.seq ? p.rows.seq[m] : m;
+    const int lo = D.window > 0 ? max(0, pos - D.window + 1) : 0;
+    const int nt = on ? (pos - lo + LAT_KT) / LAT_KT : 0;
+    const int t0 = (int)((long long)nt * sp / p.S), t1 = (int)((long long)nt * (sp + 1) / p.S);
+    const bf16_t* cache = (const bf16_t*)p.cache + (size_t)seq * p.Smax * D.CW;
+    const int nch = D.CW >> 3, CT = D.CW >> 5;
+    int chunk[NST], kg[NST];
+#pragma unroll
+    for (int i = 0; i < NST; ++i) {
+        const int task = tid + 256 * i;
+        kg[i] = task / nch;
+        chunk[i] = task - kg[i] * nch;
+    }
+    uint4 st[NST][4];
+    auto fetch = [&](int t) {
+#pragma unroll
+        for (int i = 0; i < NST; ++i)
+#pragma unroll
+            for (int k = 0; k < 4; ++k) {
+                const int key = min(lo + t * LAT_KT + 4 * min(kg[i], 7) + k, pos);      // (rounds past the tile read a valid row and are not stored)
+                st[i][k] = *reinterpret_cast<const uint4*>(cache + (size_t)key * D.CW + chunk[i] * 8);
+            }
+    };
+    // this wave's half of the query columns: heads past H read head H - 1 and are dropped at the end
+    const int half = wave >> 1, kt0 = half ? (CT + 1) / 2 : 0, kt1 = half ? CT : (CT + 1) / 2;
+    bf16x8_t qf[QF];
+    {
+        const bf16_t* q = (const bf16_t*)p.q + ((size_t)m * D.H + min(h0 + li, D.H - 1)) * D.CW + lq * 8;
+#pragma unroll
+        for (int i = 0; i < QF; ++i) qf[i] = *reinterpret_cast<const bf16x8_t*>(q + min(kt0 + i, CT - 1) * 32);
+    }
+    f32x4_t o[NTW];
+#pragma unroll
+    for (int i = 0; i < NTW; ++i) o[i] = (f32x4_t){0.f, 0.f, 0.f, 0.f};
+    float mx = -INFINITY, ls = 0.0f;                                            // of head li; ls: this lane's keys only
+    if (t0 < t1) fetch(t0);
+    for (int t = t0; t < t1; ++t) {
+#pragma unroll
+        for (int i = 0; i < NST; ++i)
+            if (kg[i] < 8) {
+#pragma unroll
+                for (int k = 0; k < 4; ++k) *reinterpret_cast<uint4*>(sk + (size_t)(4 * kg[i] + k) * KS + chunk[i] * 8) = st[i][k];
+                if (chunk[i] * 8 < D.Rp) {
+#pragma unroll
+                    for (int e = 0; e < 8; ++e) *reinterpret_cast<uint2*>(sv + (size_t)(chunk[i] * 8 + e) * LAT_VS + 4 * kg[i]) = column_of(st[i], e);
+                }
+            }
+        if (t + 1 < t1) fetch(t + 1);
+        lds_barrier();
+        f32x4_t s = (f32x4_t){0.f, 0.f, 0.f, 0.f};
+        {
+            const bf16_t* kr = sk + (size_t)((wave & 1) * 16 + li) * KS + lq * 8;
+#pragma unroll
+            for (int i = 0; i < QF; ++i)
+                if (kt0 + i < kt1) s = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*reinterpret_cast<const bf16x8_t*>(kr + (kt0 + i) * 32), qf[i], s, 0, 0, 0);
+        }
+        *reinterpret_cast<float4*>(sc + ((size_t)half * 16 + li) * 36 + (wave & 1) * 16 + lq * 4) = make_float4(s[0], s[1], s[2], s[3]);
+        lds_barrier();
+        float w[8];
+        {
+            const float *a = sc + (size_t)li * 36 + lq * 8, *b = a + 16 * 36;
+            float tm = -INFINITY;
+#pragma unroll
+            for (int e = 0; e < 8; ++e) {
+                w[e] = (a[e] + b[e]) * D.scale;
+                if (lo + t * LAT_KT + lq * 8 + e > pos) w[e] = -INFINITY;
+                tm = fmaxf(tm, w[e]);
+            }
+            tm = fmaxf(tm, __shfl_xor(tm, 16, 64));
+            tm = fmaxf(tm, __shfl_xor(tm, 32, 64));
+            const float mn = fmaxf(mx, tm), alpha = __expf(mx - mn);
+            float add = 0.0f;
+#pragma unroll
+            for (int e = 0; e < 8; ++e) { w[e] = __expf(w[e] - mn); add += w[e]; }
+            ls = ls * alpha + add;
+            mx = mn;
+#pragma unroll
+            for (int e = 0; e < 4; ++e) {
+                const float ah = __shfl(alpha, lq * 4 + e, 64);                 // head of accumulator row e
+#pragma unroll
+                for (int i = 0; i < NTW; ++i) o[i][e] *= ah;
+            }
+        }
+        bf16x8_t ph, pl;
+#pragma unroll
+        for (int e = 0; e < 8; ++e) {
+            const bf16_t hi = f32_to_bf16(w[e]);
+            ph[e] = (short)hi;
+            pl[e] = (short)f32_to_bf16(w[e] - bf16_to_f32(hi));
+        }
+#pragma unroll
+        for (int i = 0; i < NTW; ++i) {
+            const int tile = i * 4 + wave;
+            if (tile * 16 >= D.Rp) continue;                                    // wave-uniform
+            const bf16x8_t v = lds_frag(sv + (size_t)(tile * 16 + li) * LAT_VS + lq * 8);
+            o[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(ph, v, o[i], 0, 0, 0);
+            o[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(pl, v, o[i], 0, 0, 0);
+        }
+        lds_barrier();                                                          // everyone is done with sk / sv / sc
+    }
+    ls += __shfl_xor(ls, 16, 64);
+    ls += __shfl_xor(ls, 32, 64);
+    const int Hp = gridDim.y * 16;
+    if (p.S > 1 && wave == 0 && lq == 0) {
+        float* ml = p.ml + (((size_t)sp * rows + m) * Hp + h0 + li) * 2;
+        ml[0] = mx; ml[1] = ls;
+    }
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+        const int hd = h0 + lq * 4 + e;
+        const float l = __shfl(ls, lq * 4 + e, 64), inv = l > 0.0f ? 1.0f / l : 0.0f;
+#pragma unroll
+        for (int i = 0; i < NTW; ++i) {
+            const int c = (i * 4 + wave) * 16 + li;
+            if (c >= D.Rp) continue;
+            if (p.S > 1) p.part[(((size_t)sp * rows + m) * Hp + hd) * D.Rp + c] = o[i][e];
+            else if (hd < D.H) ((bf16_t*)p.out)[((size_t)m * D.H + hd) * D.Rp + c] = f32_to_bf16(o[i][e] * inv);
+        }
+    }
+}
+// the shares of a row meet: one block per (row, head), two columns per thread
+__global__ void __launch_bounds__(256) k_latent_combine(LatentDims D, LatentAttn p, int rows, int Hp) {
+    const int m = blockIdx.x, hd = blockIdx.y;
+    float mx = -INFINITY;
+    for (int s = 0; s < p.S; ++s) mx = fmaxf(mx, p.ml[(((size_t)s * rows + m) * Hp + hd) * 2]);
+    const int c = threadIdx.x * 2;
+    float a0 = 0.0f, a1 = 0.0f, l = 0.0f;
+    for (int s = 0; s < p.S; ++s) {
+        const float* ml = p.ml + (((size_t)s * rows + m) * Hp + hd) * 2;
+        const float w = ml[1] > 0.0f ? __expf(ml[0] - mx) : 0.0f;              // (an empty share holds sum 0)
+        const float2 v = *reinterpret_cast<const float2*>(p.part + (((size_t)s * rows + m) * Hp + hd) * D.Rp + c);
+        l += w * ml[1];
+        a0 += w * v.x; a1 += w * v.y;
+    }
+    const float inv = l > 0.0f ? 1.0f / l : 0.0f;
+    *reinterpret_cast<uint32_t*>((bf16_t*)p.out + ((size_t)m * D.H + hd) * D.Rp + c) = (uint32_t)f32_to_bf16(a0 * inv) | ((uint32_t)f32_to_bf16(a1 * inv) << 16);
+}
+
+bool latent_attn_mfma_ok(const LatentDims& D) { return D.Rp <= 512 && D.CW <= (D.Rp <= 128 ? 256 : D.Rp <= 256 ? 512 : 768); }
+// shares per row: about two blocks per CU, at least two key tiles each
+int latent_attn_splits(const LatentDims& D, int rows, int Smax) {
+    if (!latent_attn_mfma_ok(D)) return 1;
+    const int keys = D.window > 0 ? std::min(D.window, Smax) : Smax, tiles = cdiv(keys, LAT_KT), blocks = rows * cdiv(D.H, 16);
+    return std::max(1, std::min(std::min(cdiv(384, blocks), tiles / 2), 16));
+}
+void launch_latent_attn_absorbed(const LatentDims& D, const LatentAttn& p, int rows, hipStream_t s) {
+    MIS_REQUIRE(p.rows.pos && p.q && p.cache && p.out && rows >= 1, MIS_ERR_GENERATION_FAILED, "latent attention: null operand");
+    if (p.f32 || !latent_attn_mfma_ok(D)) {
+        MIS_REQUIRE(D.Rp <= 256 * LAT_OC, MIS_ERR_INVALID_INPUT, "latent size above 2048");
+        const size_t sm = (size_t)(D.CW + 256 + 8) * 4;
+        if (p.f32) hipLaunchKernelGGL((k_latent_attn_any<float>), dim3(rows, D.H), dim3(256), sm, s, D, p);
+        else hipLaunchKernelGGL((k_latent_attn_any<bf16_t>), dim3(rows, D.H), dim3(256), sm, s, D, p);
+        return;
+    }
+    MIS_REQUIRE(p.S == 1 || (p.part && p.ml), MIS_ERR_GENERATION_FAILED, "latent attention: no scratch for the key shares");
+    const dim3 grid(rows * p.S, cdiv(D.H, 16));
+    const size_t sm = latent_decode_lds(D);
+#define LAT_GO(A, B, C)                                                                                                                    \
+    do {                                                                                                                                   \
+        static const hipError_t attr = hipFuncSetAttribute((const void*)k_latent_attn_decode<A, B, C>, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024); \
+        HIP_CHECK(attr);                                                                                                                   \
+        hipLaunchKernelGGL((k_latent_attn_decode<A, B, C>), grid, dim3(256), sm, s, D, p, rows);                                           \
+    } while (0)
+    if (D.Rp <= 128) LAT_GO(2, 1, 4);
+    else if (D.Rp <= 256) LAT_GO(4, 2, 8);
+    else LAT_GO(8, 3, 12);
+#undef LAT_GO
+    if (p.S > 1) hipLaunchKernelGGL(k_latent_combine, dim3(rows, D.H), dim3(D.Rp / 2), 0, s, D, p, rows, (int)grid.y * 16);
+}
+
+// ============================================================================ expanded attention on the matrix cores (prompts)
+// Block = one tile of up to 64 queries of one sequence, one head; wave w owns 16 queries.  Key tiles of 32: key rows [plain | rotary] and transposed
+// values go through LDS, fetched one tile ahead.  S^T = K q^T with the key rows permuted (A row i of half f = key 8 (i >> 2) + (i & 3) + 4 f),
+// so that a lane's eight scores are eight consecutive keys of ITS query: the weights are the next MFMA's A operand without leaving registers.
+template <int KT, int VT>
+__global__ void __launch_bounds__(256, 2) k_latent_attn_prefill(LatentDims D, LatentPrefill p) {
+    extern __shared__ __attribute__((aligned(16))) uint8_t lds[];
+    const int KS = D.DK + 8;
+    bf16_t* sk = reinterpret_cast<bf16_t*>(lds);                                // [32][DK + 8]
+    bf16_t* sv = sk + (size_t)LAT_KT * KS;                                      // [vp][LAT_VS]
+    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, li = lane & 15, lq = lane >> 4, hd = blockIdx.x;
+    const LatentTile T = p.tiles[blockIdx.y];
+    const int q_last = T.pos0 + T.n - 1;
+    const int k_lo = D.window > 0 ? max(T.kpos0, T.pos0 - D.window + 1) : T.kpos0;
+    const int ntile = (q_last - k_lo + LAT_KT) / LAT_KT;
+    const int kt_n = D.DK >> 5, vt_n = D.vp >> 4;
+    constexpr int NK = KT / 2;                                                  // staging rounds of the key rows: 32 DK / 8 / 256 <= KT / 2
+    const int nch = D.DK >> 3, nplain = D.np >> 3, nrot = (D.np + D.rp) >> 3, nv = D.vp >> 3;
+    int kkey[NK], kch[NK];
+#pragma unroll
+    for (int i = 0; i < NK; ++i) { const int t = tid + 256 * i; kkey[i] = t / nch; kch[i] = t - kkey[i] * nch; }
+    const int vkg = tid / nv, vch = tid - vkg * nv;                             // 8 groups of 4 keys x vp / 8 chunks (vp <= 256)
+    const bf16_t* kplain = p.kv + (size_t)hd * D.np;
+    const bf16_t* vals = p.kv + (size_t)D.H * D.np + (size_t)hd * D.vp;
+    const bf16_t* crot = p.cache + (size_t)T.seq * p.Smax * D.CW + D.Rp;
+    uint4 sk_r[NK], sv_r[4];
+    auto fetch = [&](int t) {
+        const int k0 = k_lo + t * LAT_KT;
+#pragma unroll
+        for (int i = 0; i < NK; ++i) {
+            const int key = min(k0 + min(kkey[i], LAT_KT - 1), q_last);
+            const int c = kch[i];
+            const bf16_t* src = c < nplain ? kplain + (size_t)(T.krow0 + key - T.kpos0) * p.ldkv + c * 8
+                                           : crot + (size_t)key * D.CW + (c < nrot ? c - nplain : 0) * 8;
+            sk_r[i] = *reinterpret_cast<const uint4*>(src);
+            if (c >= nrot) sk_r[i] = make_uint4(0, 0, 0, 0);
+        }
+#pragma unroll
+        for (int k = 0; k < 4; ++k) {
+            const int key = min(k0 + 4 * min(vkg, 7) + k, q_last);
+            sv_r[k] = *reinterpret_cast<const uint4*>(vals + (size_t)(T.krow0 + key - T.kpos0) * p.ldkv + vch * 8);
+        }
+    };
+    const int wq0 = wave * 16, qi = wq0 + li;                                   // this lane's query of the tile
+    const int qpos = T.pos0 + min(qi, T.n - 1);
+    const bool w_on = wq0 < T.n;
+    const int w_first = T.pos0 + wq0, w_last = T.pos0 + min(wq0 + 15, T.n - 1);
+    bf16x8_t qf[KT];
+    {
+        const bf16_t* q = p.q + ((size_t)(T.row0 + min(qi, T.n - 1)) * D.H + hd) * D.DK + lq * 8;
+#pragma unroll
+        for (int i = 0; i < KT; ++i) qf[i] = *reinterpret_cast<const bf16x8_t*>(q + min(i, kt_n - 1) * 32);
+    }
+    f32x4_t o[VT];
+#pragma unroll
+    for (int i = 0; i < VT; ++i) o[i] = (f32x4_t){0.f, 0.f, 0.f, 0.f};
+    float mx = -INFINITY, ls = 0.0f;
+    const int perm = 8 * (li >> 2) + (li & 3);
+    fetch(0);
+    for (int t = 0; t < ntile; ++t) {
+        const int k0 = k_lo + t * LAT_KT;
+#pragma unroll
+        for (int i = 0; i < NK; ++i)
+            if (kkey[i] < LAT_KT) *reinterpret_cast<uint4*>(sk + (size_t)kkey[i] * KS + kch[i] * 8) = sk_r[i];
+        if (vkg < 8) {
+#pragma unroll
+            for (int e = 0; e < 8; ++e) *reinterpret_cast<uint2*>(sv + (size_t)(vch * 8 + e) * LAT_VS + 4 * vkg) = column_of(sv_r, e);
+        }
+        if (t + 1 < ntile) fetch(t + 1);
+        lds_barrier();
+        if (w_on && k0 <= w_last && (D.window <= 0 || k0 + LAT_KT - 1 > w_first - D.window)) {            // wave-uniform: some key is seen
+            f32x4_t s[2];
+#pragma unroll
+            for (int f = 0; f < 2; ++f) {
+                s[f] = (f32x4_t){0.f, 0.f, 0.f, 0.f};
+                const bf16_t* kr = sk + (size_t)(perm + 4 * f) * KS + lq * 8;
+#pragma unroll
+                for (int i = 0; i < KT; ++i)
+                    if (i < kt_n) s[f] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*reinterpret_cast<const bf16x8_t*>(kr + i * 32), qf[i], s[f], 0, 0, 0);
+            }
+            float w[8], tm = -INFINITY;
+#pragma unroll
+            for (int e = 0; e < 8; ++e) {
+                const int key = k0 + 8 * lq + e;
+                const bool seen = key <= qpos && (D.window <= 0 || key > qpos - D.window);
+                w[e] = seen ? s[e >> 2][e & 3] * D.scale : -INFINITY;
+                tm = fmaxf(tm, w[e]);
+            }
+            tm = fmaxf(tm, __shfl_xor(tm, 16, 64));
+            tm = fmaxf(tm, __shfl_xor(tm, 32, 64));
+            const float mn = fmaxf(mx, tm), base = mn == -INFINITY ? 0.0f : mn;  // a query may see none of this tile's keys yet
+            const float alpha = __expf(mx - base);
+            float add = 0.0f;
+#pragma unroll
+            for (int e = 0; e < 8; ++e) { w[e] = __expf(w[e] - base); add += w[e]; }
+            ls = ls * alpha + add;
+            mx = mn;
+#pragma unroll
+            for (int e = 0; e < 4; ++e) {
+                const float aq = __shfl(alpha, lq * 4 + e, 64);
+#pragma unroll
+                for (int i = 0; i < VT; ++i) o[i][e] *= aq;
+            }
+            bf16x8_t ph, pl;
+#pragma unroll
+            for (int e = 0; e < 8; ++e) {
+                const bf16_t hi = f32_to_bf16(w[e]);
+                ph[e] = (short)hi;
+                pl[e] = (short)f32_to_bf16(w[e] - bf16_to_f32(hi));
+            }
+#pragma unroll
+            for (int i = 0; i < VT; ++i) {
+                if (i >= vt_n) continue;
+                const bf16x8_t v = lds_frag(sv + (size_t)(i * 16 + li) * LAT_VS + lq * 8);
+                o[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(ph, v, o[i], 0, 0, 0);
+                o[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(pl, v, o[i], 0, 0, 0);
+            }
+        }
+        lds_barrier();
+    }
+    ls += __shfl_xor(ls, 16, 64);
+    ls += __shfl_xor(ls, 32, 64);
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+        const int q = wq0 + lq * 4 + e;
+        const float inv = 1.0f / __shfl(ls, lq * 4 + e, 64);
+        if (q >= T.n) continue;
+        bf16_t* out = p.out + (size_t)(T.row0 + q) * p.ldo + (size_t)hd * D.v;
+#pragma unroll
+        for (int i = 0; i < VT; ++i) {
+            const int c = i * 16 + li;
+            if (c < D.v) out[c] = f32_to_bf16(o[i][e] * inv);
+        }
+    }
+}
+bool latent_prefill_mfma_ok(const LatentDims& D) { return D.DK <= 256 && D.vp <= 256; }
+void launch_latent_attn_prefill(const LatentDims& D, const LatentPrefill& p, hipStream_t s) {
+    MIS_REQUIRE(latent_prefill_mfma_ok(D) && p.n_tiles >= 1 && p.ldkv % 8 == 0, MIS_ERR_GENERATION_FAILED, "latent prompt attention: unsupported sizes");
+    const dim3 grid(D.H, p.n_tiles);
+    const size_t sm = (size_t)LAT_KT * (D.DK + 8) * 2 + (size_t)D.vp * LAT_VS * 2;
+    if (D.DK <= 128 && D.vp <= 128) hipLaunchKernelGGL((k_latent_attn_prefill<4, 8>), grid, dim3(256), sm, s, D, p);
+    else if (D.DK <= 192 && D.vp <= 128) hipLaunchKernelGGL((k_latent_attn_prefill<6, 8>), grid, dim3(256), sm, s, D, p);
+    else hipLaunchKernelGGL((k_latent_attn_prefill<8, 16>), grid, dim3(256), sm, s, D, p);
+}

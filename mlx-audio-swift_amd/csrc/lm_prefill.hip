@@ -109,6 +109,7 @@ struct PfGemmParams {
     const bf16_t* Wp;     // packed [NT][KT][64][8]
     void* C;              // PF_F32: float [M][N]; PF_RESID: bf16 h [M][N] (read-modify-write); PF_SILU: bf16 act [M][N/2]
     int M, N, K;          // N = rows of W (PF_SILU: 2 * ff, gate / up tiles interleaved)
+    PfExtra ex;           // the epilogues of layer-list models (lm_blocks.hip)
 };
 
 template <int EPI>
@@ -135,7 +136,9 @@ __global__ void __launch_bounds__(256, 2) k_gemm_pf(PfGemmParams p) {
         wsrc[q] = p.Wp + ((size_t)nt * KT + ktl) * 512 + lane * 8;
         const int r = (wave * 4 + q) * 8 + (lane >> 3);
         const int chunk = (lane & 7) ^ ((r >> 1) & 7);
-        xsrc[q] = p.X + (size_t)min(m0 + r, p.M - 1) * p.K + chunk * 8;
+        const int xm = min(m0 + r, p.M - 1);
+        if constexpr (EPI == PF_ROWS_BF16) xsrc[q] = p.X + (size_t)p.ex.xrow[xm] * p.ex.ldx + chunk * 8;
+        else xsrc[q] = p.X + (size_t)xm * p.K + chunk * 8;
     }
     auto stage = [&](int buf, int ks) {                  // k-step ks covers k-tiles 2 ks, 2 ks + 1 = columns 64 ks .. +64
 #pragma unroll
@@ -207,7 +210,33 @@ __global__ void __launch_bounds__(256, 2) k_gemm_pf(PfGemmParams p) {
                 const int tile = (n0 >> 4) + wn * 4 + i;
                 if (tile >= NT) continue;
                 const int n = tile * 16 + nl;
-                if (EPI == PF_F32) {
+                if constexpr (EPI >= PF_SPLIT_RELU2) {
+                    float v[4] = {acc[i][j][0], acc[i][j][1], acc[i][j][2], acc[i][j][3]};
+                    float* c32 = reinterpret_cast<float*>(p.C) + (size_t)m * p.ex.ldc + n;
+                    if (EPI == PF_ROWS_BF16 || (EPI == PF_SPLIT_RELU2 && tile >= p.ex.split)) {
+                        uint16_t res[4];
+#pragma unroll
+                        for (int e = 0; e < 4; ++e) {
+                            if (EPI == PF_SPLIT_RELU2) { const float t = fmaxf(v[e], 0.0f); v[e] = t * t; }
+                            res[e] = f32_to_bf16(v[e]);
+                        }
+                        bf16_t* o = EPI == PF_ROWS_BF16 ? reinterpret_cast<bf16_t*>(p.C) + (size_t)m * p.ex.ldc + n
+                                                        : reinterpret_cast<bf16_t*>(p.ex.out2) + (size_t)m * p.ex.ld2 + (n - p.ex.split * 16);
+                        *reinterpret_cast<uint2*>(o) = make_uint2((uint32_t)res[0] | ((uint32_t)res[1] << 16), (uint32_t)res[2] | ((uint32_t)res[3] << 16));
+                    } else if (EPI == PF_SCALED_ADD) {
+                        const uint2 lw = *reinterpret_cast<const uint2*>(p.ex.ls + n);
+                        const float l[4] = {bf16_to_f32((bf16_t)(lw.x & 0xffffu)), bf16_to_f32((bf16_t)(lw.x >> 16)), bf16_to_f32((bf16_t)(lw.y & 0xffffu)),
+                                            bf16_to_f32((bf16_t)(lw.y >> 16))};
+                        const float4 o = *reinterpret_cast<const float4*>(c32);
+                        *reinterpret_cast<float4*>(c32) = make_float4(o.x + l[0] * v[0], o.y + l[1] * v[1], o.z + l[2] * v[2], o.w + l[3] * v[3]);
+                    } else {
+                        if (EPI == PF_SOFTCAP) {
+#pragma unroll
+                            for (int e = 0; e < 4; ++e) { const float t = v[e] * p.ex.scale; v[e] = p.ex.cap > 0.0f ? p.ex.cap * tanhf(t / p.ex.cap) : t; }
+                        }
+                        *reinterpret_cast<float4*>(c32) = make_float4(v[0], v[1], v[2], v[3]);
+                    }
+                } else if (EPI == PF_F32) {
                     *reinterpret_cast<float4*>(reinterpret_cast<float*>(p.C) + (size_t)m * p.N + n) =
                         make_float4(acc[i][j][0], acc[i][j][1], acc[i][j][2], acc[i][j][3]);
                 } else {
@@ -230,14 +259,20 @@ __global__ void __launch_bounds__(256, 2) k_gemm_pf(PfGemmParams p) {
     }
 }
 
-void launch_gemm_pf(int epi, const bf16_t* X, const bf16_t* Wp, void* C, int M, int N, int K, hipStream_t s) {
+void launch_gemm_pf(int epi, const bf16_t* X, const bf16_t* Wp, void* C, int M, int N, int K, hipStream_t s, const PfExtra& ex) {
     MIS_REQUIRE(K % PF_BK == 0 && K >= 2 * PF_BK && N % 16 == 0 && M >= 1, MIS_ERR_GENERATION_FAILED, "prefill GEMM: K must be a multiple of 64");
     MIS_REQUIRE(epi != PF_SILU || N % 32 == 0, MIS_ERR_GENERATION_FAILED, "prefill GEMM: gate / up tiles come in pairs");
-    PfGemmParams p{X, Wp, C, M, N, K};
+    MIS_REQUIRE(epi < PF_SPLIT_RELU2 || (ex.ldc % 4 == 0 && (epi != PF_ROWS_BF16 || (ex.xrow && ex.ldx % 8 == 0))), MIS_ERR_GENERATION_FAILED,
+                "prefill GEMM: bad row strides");
+    PfGemmParams p{X, Wp, C, M, N, K, ex};
     dim3 grid(cdiv(N, PF_BN), cdiv(M, PF_BM)), block(256);
     if (epi == PF_F32) hipLaunchKernelGGL((k_gemm_pf<PF_F32>), grid, block, 0, s, p);
     else if (epi == PF_RESID) hipLaunchKernelGGL((k_gemm_pf<PF_RESID>), grid, block, 0, s, p);
     else if (epi == PF_SILU) hipLaunchKernelGGL((k_gemm_pf<PF_SILU>), grid, block, 0, s, p);
+    else if (epi == PF_SPLIT_RELU2) hipLaunchKernelGGL((k_gemm_pf<PF_SPLIT_RELU2>), grid, block, 0, s, p);
+    else if (epi == PF_SCALED_ADD) hipLaunchKernelGGL((k_gemm_pf<PF_SCALED_ADD>), grid, block, 0, s, p);
+    else if (epi == PF_ROWS_BF16) hipLaunchKernelGGL((k_gemm_pf<PF_ROWS_BF16>), grid, block, 0, s, p);
+    else if (epi == PF_SOFTCAP) hipLaunchKernelGGL((k_gemm_pf<PF_SOFTCAP>), grid, block, 0, s, p);
     else throw MisError(MIS_ERR_GENERATION_FAILED, "unknown prefill GEMM epilogue");
 }
 void launch_pf_embed_rmsnorm(const bf16_t* emb, const int32_t* prompt, const int32_t* lens, int Lmax, int t0, int Tc, int batch, int Mpad, int vocab,

@@ -129,7 +129,7 @@ __global__ void __launch_bounds__(64) k_samp_prepare(SamplerParams p) {
     SamplerScratch* sc = p.scratch + b;
     for (int i = tid; i < 256; i += 64) { sc->hist1[i] = 0; sc->hist2[i] = 0; }
     if (row_skipped(p, b)) return;
-    if (p.logits32) {                                   // Soprano flavour: the processed logits are float32
+    if (p.logits32 && !p.f32_input) {                   // Soprano flavour: the processed logits are float32
         const bf16_t* src = p.logits + (size_t)b * p.Vpad;
         float* dst = p.logits32 + (size_t)b * p.Vpad;
         for (int i = tid; i < p.vocab; i += 64) dst[i] = bf16_to_f32(src[i]);
@@ -144,10 +144,10 @@ __global__ void __launch_bounds__(64) k_samp_prepare(SamplerParams p) {
             bool first = (id >= 0 && id < p.vocab);
             for (int j = 0; j < t; ++j) first = first && (win[j] != id);
             if (first) {
-                float l = bf16_to_f32(logits[id]);
+                float l = p.f32_input ? p.logits32[(size_t)b * p.Vpad + id] : bf16_to_f32(logits[id]);
                 float v;
                 if (p.penalty_flavor == 0) {
-                    float pen = bf16_round_f32(p.penalty);        // scalar weakly typed to bf16
+                    float pen = p.f32_input ? p.penalty : bf16_round_f32(p.penalty);        // scalar weakly typed to the logits' type
                     v = (l < 0.0f) ? l * pen : __fdiv_rn(l, pen);
                 } else {
                     // Soprano applyRepetitionPenalty (Soprano.swift:888-901): float32, once PER OCCURRENCE in the window
