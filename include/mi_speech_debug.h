@@ -46,6 +46,11 @@ int32_t mis_debug_sampler_failures(void);
 mis_status mis_debug_token_engine(mis_tts* lm, const int32_t* prompt, int n_prompt, int n_new, int xcds, const mis_gen_params* sampling,
                                   int stop_id, int32_t* next_tokens, float* logits_out, float* hidden_out, int32_t* counts, double* ms_out);
 
+/* rotary tables of the layer-list models: cos / sin f32 [positions][dims / 2] (host memory; no device involved).  yarn = 0: factor / original /
+ * fast / slow unused */
+mis_status mis_debug_rotary_tables(int dims, double base, int yarn, double factor, double original, double fast, double slow, int positions,
+                                   float* cos_out, float* sin_out);
+
 #ifdef __cplusplus
 }
 #endif

@@ -170,6 +170,8 @@ std::vector<std::pair<std::string, std::vector<int64_t>>> LmBlocks::tensor_list(
 void LmBlocks::set_tensor(const std::string& name, const bf16_t* src, const std::vector<int64_t>& shape, hipStream_t s) {
     static const std::vector<int64_t> none;
     const std::vector<int64_t>* want = nullptr;
+    for (int i = 0; i < L; ++i)                                                // the second layer scale of a layer without feed-forward scales nothing
+        if (layers_[i].owner == i && !layers_[i].ffp && name == "l" + std::to_string(i) + ".ls2") return;
     const auto list = tensor_list();
     for (auto& t : list) if (t.first == name) want = &t.second;
     MIS_REQUIRE(want, MIS_ERR_INVALID_INPUT, "unexpected tensor %s", name.c_str());

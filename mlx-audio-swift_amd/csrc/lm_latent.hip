@@ -39,6 +39,18 @@ void rotary_tables_host(const RotarySpec& r, int positions, std::vector<float>& 
         }
 }
 
+extern "C" mis_status mis_debug_rotary_tables(int dims, double base, int yarn, double factor, double original, double fast, double slow, int positions,
+                                              float* cos_out, float* sin_out) {
+    MIS_API_BEGIN
+    MIS_REQUIRE(dims >= 2 && dims % 2 == 0 && positions >= 1 && cos_out && sin_out, MIS_ERR_INVALID_INPUT, "bad argument");
+    RotarySpec r{dims, base, yarn != 0, factor, original, fast, slow};
+    std::vector<float> c, s;
+    rotary_tables_host(r, positions, c, s);
+    std::copy(c.begin(), c.end(), cos_out);
+    std::copy(s.begin(), s.end(), sin_out);
+    MIS_API_END
+}
+
 LatentDims latent_dims(int H, int n, int r, int v, int R, int window, int rot_dims, float scale, float eps) {
     LatentDims D{};
     D.H = H; D.n = n; D.r = r; D.v = v; D.R = R;
