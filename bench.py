@@ -345,6 +345,60 @@ def self_spawn(args):
     return subprocess.run(cmd, env=env).returncode
 
 
+LATENT_SIZES = {
+    # a 3B-class and a small model, each as Rugunex (latent attention, squared-ReLU feed-forward) and as the Llama chain of equal width, heads,
+    # feed-forward width, depth and vocabulary
+    "3b": dict(width=3072, layers=28, heads=24, kv_heads=8, dim=128, rot_dim=64, vdim=128, kv_rank=512, ff=8192, vocab=32768),
+    "small": dict(width=1024, layers=24, heads=16, kv_heads=8, dim=64, rot_dim=32, vdim=64, kv_rank=256, ff=4096, vocab=32768),
+}
+
+
+def latent_config(z, window):
+    mx = dict(heads=z["heads"], dim=z["dim"], rot_dim=z["rot_dim"], vdim=z["vdim"], kv_rank=z["kv_rank"], mask=dict(size=window),
+              scale=(z["dim"] + z["rot_dim"]) ** -0.5,
+              rot=dict(base=500000.0, dims=z["rot_dim"], scaling=dict(factor=8.0, original=4096, fast=32.0, slow=1.0)))
+    return dict(architecture="Rugunex", width=z["width"], vocab=z["vocab"], norm=dict(eps=1e-6), logit_scale=1.0, logit_softcap=30.0,
+                layers=[dict(type="latent_attention", mixer=mx, mlp=dict(kind="dense", ff=z["ff"]))] * z["layers"])
+
+
+def latent_lm_bench(args):
+    """--latent-lm: prefill and decode throughput of the Rugunex design (random weights) beside the Llama chain at equal size; one JSON line per
+    (size, batch, prompt).  Greedy generation through the same loop for both; prefill and decode are timed by the engine with HIP events."""
+    import ctypes as C
+    import mlx_audio_swift_amd as mas
+    L = mas._lib.lib()
+    window, new = args.latent_window, args.latent_new
+    cases = [tuple(int(x) for x in c.split("x")) for c in args.latent_cases.split(",")]
+    for name in args.latent_sizes.split(","):
+        z = LATENT_SIZES[name]
+        for kind in args.latent_models.split(","):
+            if kind == "rugunex":
+                m = mas.BlockLanguageModel.synthetic(latent_config(z, window))
+            else:
+                m = mas.LlamaTTSModel.synthetic(mas.LlamaTTSConfiguration(
+                    hidden_size=z["width"], num_hidden_layers=z["layers"], intermediate_size=z["ff"], num_attention_heads=z["heads"],
+                    num_key_value_heads=z["kv_heads"], head_dim=z["vdim"], vocab_size=z["vocab"], rope_theta=500000.0, rope_plain=True, tie_word_embeddings=False))
+            for batch, prompt in cases:
+                rng = np.random.default_rng(1)
+                flat = rng.integers(0, z["vocab"], batch * prompt).astype(np.int32)
+                lens = np.full(batch, prompt, np.int32)
+                gp = mas.GenerateParameters(max_tokens=new, temperature=0.0, repetition_penalty=1.0, repetition_context_size=0).to_c()
+                toks, n = np.zeros((batch, new), np.int32), np.zeros(batch, np.int32)
+                best = None
+                for it in range(args.warmup + args.steps):
+                    if L.mis_lm_generate(m._h, flat.ctypes.data, lens.ctypes.data, batch, C.byref(gp), -1, toks.ctypes.data, n.ctypes.data) != 0:
+                        raise RuntimeError(mas._lib.last_error())
+                    t = m.last_timing()
+                    if it >= args.warmup:
+                        cur = (t["prefill_ms"], t["decode_ms"] / t["steps"])
+                        best = cur if best is None else (min(best[0], cur[0]), min(best[1], cur[1]))
+                print(json.dumps({"bench": "latent-lm", "size": name, "model": kind, "batch": batch, "prompt": prompt, "new_tokens": new,
+                                  "window": window if kind == "rugunex" else None, "prefill_ms": round(best[0], 3),
+                                  "prefill_tokens_per_s": round(batch * prompt / best[0] * 1e3), "decode_step_ms": round(best[1], 4),
+                                  "decode_tokens_per_s": round(batch / best[1] * 1e3), "dtype": "bf16", "data": "synthetic"}), flush=True)
+            m.close()
+
+
 def main():
     ap = argparse.ArgumentParser()
     ap.add_argument("--gpus", type=int, default=1)
@@ -352,7 +406,16 @@ def main():
     ap.add_argument("--warmup", type=int, default=1)
     ap.add_argument("--no-cpu-baseline", action="store_true")
     ap.add_argument("--no-secondary", action="store_true", help="skip the secondary configurations (Whisper / Soprano / Qwen3-TTS) after the timed region")
+    ap.add_argument("--latent-lm", action="store_true", help="instead of the headline workload: the Rugunex design beside the Llama chain at equal size")
+    ap.add_argument("--latent-sizes", default="3b,small")
+    ap.add_argument("--latent-cases", default="1x512,32x512,4x2048", help="batch x prompt, comma separated")
+    ap.add_argument("--latent-models", default="rugunex,llama")
+    ap.add_argument("--latent-window", type=int, default=4096)
+    ap.add_argument("--latent-new", type=int, default=128)
     args = ap.parse_args()
+    if args.latent_lm:
+        latent_lm_bench(args)
+        return
     if args.gpus > 1 and "WORLD_SIZE" not in os.environ:
         raise SystemExit(self_spawn(args))
 

@@ -62,7 +62,7 @@ private:
         DevBuf<bf16_t> ukv;             // packed [(H np + H vp) / 16][Rp / 32] (expanded form; its value part serves the absorbed form too)
         DevBuf<bf16_t> wo, wdown;       // packed [dp / 16][Ko / 32], [dp / 16][ffp / 32]
     };
-    struct Layer { LatentDims D; int owner, ffp, Nqkv, Ko, S_attn = 1, S_o = 1, S_down = 1, rope = 0; };
+    struct Layer { LatentDims D; int owner, ffp, Nqkv, Ko, shares = 1, s1 = 1, s2 = 0, rope = 0; };
     std::vector<Layer> layers_;
     std::vector<std::unique_ptr<Weights>> w_;
     std::set<std::string> loaded_;
@@ -74,7 +74,8 @@ private:
     int batch_ = 0, Mpad_ = 0, Smax_ = 0, rope_len_ = 0;
     std::vector<std::unique_ptr<DevBuf<uint8_t>>> cache_;
     // step buffers; bf16 ones hold float32 in the 32-bit mode (sized in bytes)
-    DevBuf<float> x_, qkv_, part_o_, part_d_, attn_part_, attn_ml_, logits_;
+    DevBuf<float> x_, qkv_, part_, share_ml_, logits_;
+    DevBuf<bf16_t> share_;
     DevBuf<uint8_t> h_, act_, q_, olat_;
     std::map<int, DevBuf<uint8_t>> attn_;          // per H v: the columns up to the K padding stay zero
     // pass buffers
@@ -94,6 +95,7 @@ private:
     const bf16_t* norm_after(int li) const { return li + 1 < L ? W(li + 1).norm1.p : g_final_.p; }
     void step_layer(int li, const BlockRows& r, hipStream_t s);
     void pass_layer(int li, int M, const RowTable& rows, int n_tiles, int Mk, hipStream_t s);
-    void absorbed_attention(int li, const float* qkv, void* q, void* olat, const Operand& out, const RowTable& rows, int M, int S, hipStream_t s);
+    // shares > 0 (decode, bf16): the keys of a row in that many shares on the matrix cores; 0: the kernels for any sizes
+    void absorbed_attention(int li, const float* qkv, void* q, void* olat, const Operand& out, const RowTable& rows, int M, int shares, hipStream_t s);
     void head_rows(const void* operand, bool packed, int rows, int rows_padded, float* out, hipStream_t s);
 };

@@ -3,8 +3,8 @@
 //
 // Decode step, per layer (bf16): ONE weight-streaming GEMM for everything that reads the layer's norm - queries, latent, rotary key (float32
 // sums) and the feed-forward's up rows (relu^2 in the epilogue, packed for the down projection) -> latent row + absorbed queries (one launch)
-// -> attention over the latent cache (-> meeting of the key shares) -> values -> the two projections back to the width as split-K slabs ->
-// x += ls1 sum + ls2 sum, norm for the next layer.  The residual stream, scores, norms and rotations are float32.
+// -> attention over the latent cache in shares of keys -> shares weighted, values -> both projections back to the width as split-K slabs of ONE
+// launch -> x += ls1 sum + ls2 sum, norm for the next layer.  The residual stream, scores, norms and rotations are float32.
 // Prompt pass: rows = tokens of all requests, (sequence, position) per row; k_gemm_pf GEMMs, keys and values expanded from the latent
 // cache for the chunk's keys and the window before it, both projections added to the stream in their epilogues.
 #include <math.h>
@@ -269,32 +269,31 @@ void LmBlocks::reset(int batch, int Smax, hipStream_t s) {
     }
     if (same) return;                                                          // (a cache row is written before it is read: nothing to clear)
     cache_.resize(L);
-    size_t n_qkv = 0, n_act = 0, n_q = 0, n_ol = 0, n_part = 0, n_ml = 0, s_o = 1, s_d = 1;
-    const int max_s = dp > 8192 ? 4 : 8;
+    size_t n_qkv = 0, n_act = 0, n_q = 0, n_ol = 0, n_share = 0, n_ml = 0, n_slab = 2;
+    const int max_s = dp > 8192 ? 4 : 8;                                       // slabs the residual kernel takes
     for (int i = 0; i < L; ++i) {
         Layer& l = layers_[i];
         const LatentDims& D = l.D;
         if (!cache_[i]) cache_[i].reset(new DevBuf<uint8_t>());
         cache_[i]->alloc((size_t)batch * Smax * D.CW * esz());
-        l.S_attn = f32 ? 1 : latent_attn_splits(D, batch, Smax);
-        l.S_o = f32 ? 1 : std::min(max_s, gemm_choose_split(dp / 16 / 2, l.Ko / 32, 4, max_s));
-        l.S_down = f32 || !l.ffp ? 1 : std::min(max_s, gemm_choose_split(dp / 16 / 2, l.ffp / 32, 4, max_s));
+        l.shares = !f32 && latent_decode_mfma_ok(D) ? latent_decode_shares(D, batch, Smax) : 0;
+        l.s1 = 1; l.s2 = l.ffp ? 1 : 0;
+        if (!f32) gemm_choose_dual_split(dp / 16 / 2, l.Ko / 32, l.ffp / 32, 4, max_s, &l.s1, &l.s2);
         n_qkv = std::max(n_qkv, (size_t)l.Nqkv); n_act = std::max(n_act, (size_t)l.ffp);
-        n_q = std::max(n_q, (size_t)D.H * D.CW); n_ol = std::max(n_ol, (size_t)D.H * D.Rp);
-        if (l.S_attn > 1) {
-            const size_t rows = (size_t)l.S_attn * batch * round_up(D.H, 16);
-            n_part = std::max(n_part, rows * D.Rp); n_ml = std::max(n_ml, rows * 2);
-        }
-        s_o = std::max(s_o, (size_t)l.S_o); s_d = std::max(s_d, (size_t)l.S_down);
+        n_q = std::max(n_q, (size_t)D.H * D.CW);
+        if (!l.shares) n_ol = std::max(n_ol, (size_t)D.H * D.Rp);
+        n_share = std::max(n_share, (size_t)l.shares * batch * D.H * D.Rp);
+        n_ml = std::max(n_ml, (size_t)l.shares * batch * D.H * 2);
+        n_slab = std::max(n_slab, (size_t)(l.s1 + l.s2));
         DevBuf<uint8_t>& at = attn_[D.H * D.v];
         at.alloc((size_t)Mpad_ * l.Ko * esz());
         at.zero(s);
     }
     x_.alloc((size_t)Mpad_ * dp); h_.alloc((size_t)Mpad_ * dp * esz());
     qkv_.alloc((size_t)Mpad_ * n_qkv); act_.alloc((size_t)Mpad_ * std::max<size_t>(n_act, 1) * esz());
-    q_.alloc((size_t)Mpad_ * n_q * esz()); olat_.alloc((size_t)Mpad_ * n_ol * esz());
-    part_o_.alloc(s_o * Mpad_ * dp); part_d_.alloc(s_d * Mpad_ * dp);
-    attn_part_.alloc(n_part); attn_ml_.alloc(n_ml);
+    q_.alloc((size_t)Mpad_ * n_q * esz()); olat_.alloc((size_t)Mpad_ * std::max<size_t>(n_ol, 1) * esz());
+    part_.alloc(n_slab * Mpad_ * dp);
+    share_.alloc(n_share); share_ml_.alloc(n_ml);
     logits_.alloc((size_t)Mpad_ * Vpad);
     x_.zero(s); h_.zero(s); qkv_.zero(s); act_.zero(s); q_.zero(s); olat_.zero(s); logits_.zero(s);
 }
@@ -314,7 +313,7 @@ LatentRows LmBlocks::latent_rows(int li, const float* qkv, void* q, bool expande
 }
 
 // projections in qkv -> cache rows, absorbed queries, latent sums, values (operand of the output projection)
-void LmBlocks::absorbed_attention(int li, const float* qkv, void* q, void* olat, const Operand& out, const RowTable& rows, int M, int S, hipStream_t s) {
+void LmBlocks::absorbed_attention(int li, const float* qkv, void* q, void* olat, const Operand& out, const RowTable& rows, int M, int shares, hipStream_t s) {
     const Layer& l = layers_[li];
     const LatentDims& D = l.D;
     const Weights& w = W(li);
@@ -329,8 +328,15 @@ void LmBlocks::absorbed_attention(int li, const float* qkv, void* q, void* olat,
         launch_gemm_f32(g, s);
     } else launch_latent_absorb(D, lr, w.uk_t.p, M, s);
     LatentAttn a{};
-    a.q = q; a.cache = cache_[li]->p; a.Smax = Smax_; a.rows = rows; a.out = olat; a.f32 = f32 ? 1 : 0; a.S = S; a.part = attn_part_.p; a.ml = attn_ml_.p;
-    launch_latent_attn_absorbed(D, a, M, s);
+    a.q = q; a.cache = cache_[li]->p; a.Smax = Smax_; a.rows = rows; a.out = olat; a.f32 = f32 ? 1 : 0;
+    if (shares > 0) {
+        LatentShares sh;
+        sh.S = shares; sh.part = share_.p; sh.ml = share_ml_.p;
+        launch_latent_attn_decode(D, a, sh, M, s);
+        launch_latent_share_values(D, sh, uv, uvz, out, M, s);
+        return;
+    }
+    launch_latent_attn_any(D, a, M, s);
     if (f32) {
         GemmF32 g{};
         g.X = (const float*)olat; g.ldx = D.H * D.Rp; g.xz = D.Rp; g.W = uv; g.wz = uvz;
@@ -360,16 +366,17 @@ void LmBlocks::step_layer(int li, const BlockRows& r, hipStream_t s) {
         GemmExtra ex; ex.out2 = act_.p; ex.split = l.Nqkv / 16;
         launch_gemm_skinny(EPI_SPLIT_RELU2, wide ? 4 : 2, 4, w.w1.p, (const bf16_t*)h_.p, qkv_.p, NT, dp / 32, 1, l.Nqkv, Mpad_, s, nullptr, 0, ex);
     }
-    absorbed_attention(li, qkv_.p, q_.p, olat_.p, operand(at, l.Ko, Mpad_, true), rows, batch_, l.S_attn, s);
+    absorbed_attention(li, qkv_.p, q_.p, olat_.p, operand(at, l.Ko, Mpad_, true), rows, batch_, l.shares, s);
+    const size_t slab = (size_t)Mpad_ * dp;
     if (f32) {
-        launch_gemm_f32(gemm32(at, l.Ko, w.wo.p, part_o_.p, dp, batch_, dp, l.Ko, F32_STORE), s);
-        if (l.ffp) launch_gemm_f32(gemm32(act_.p, l.ffp, w.wdown.p, part_d_.p, dp, batch_, dp, l.ffp, F32_STORE), s);
-    } else {
-        launch_gemm_skinny(EPI_PARTIAL, 2, 4, w.wo.p, (const bf16_t*)at, part_o_.p, dp / 16, l.Ko / 32, l.S_o, dp, Mpad_, s);
-        if (l.ffp) launch_gemm_skinny(EPI_PARTIAL, 2, 4, w.wdown.p, (const bf16_t*)act_.p, part_d_.p, dp / 16, l.ffp / 32, l.S_down, dp, Mpad_, s);
-    }
-    ScaledSlabs o{part_o_.p, l.S_o, w.ls1.p}, f{part_d_.p, l.ffp ? l.S_down : 0, w.ls2.p};
-    launch_scaled_residual_norm(o, f, Mpad_, x_.p, norm_after(li), operand(h_.p, dp, Mpad_, true), d, dp, spec.eps, f32 ? batch_ : Mpad_, s);
+        launch_gemm_f32(gemm32(at, l.Ko, w.wo.p, part_.p, dp, batch_, dp, l.Ko, F32_STORE), s);
+        if (l.ffp) launch_gemm_f32(gemm32(act_.p, l.ffp, w.wdown.p, part_.p + slab, dp, batch_, dp, l.ffp, F32_STORE), s);
+    } else if (l.ffp) {
+        GemmExtra ex; ex.w2 = w.wdown.p; ex.x2 = (const bf16_t*)act_.p; ex.kt2 = l.ffp / 32; ex.s1 = l.s1;
+        launch_gemm_skinny(EPI_DUAL, 2, 4, w.wo.p, (const bf16_t*)at, part_.p, dp / 16, l.Ko / 32, l.s1 + l.s2, dp, Mpad_, s, nullptr, 0, ex);
+    } else launch_gemm_skinny(EPI_PARTIAL, 2, 4, w.wo.p, (const bf16_t*)at, part_.p, dp / 16, l.Ko / 32, l.s1, dp, Mpad_, s);
+    const ScaledSlabs sl{part_.p, l.s1, l.s2, w.ls1.p, w.ls2.p};
+    launch_scaled_residual_norm(sl, Mpad_, x_.p, norm_after(li), operand(h_.p, dp, Mpad_, true), d, dp, spec.eps, f32 ? batch_ : Mpad_, s);
 }
 void LmBlocks::enqueue_step(const BlockRows& r, hipStream_t s) {
     launch_rows_embed_norm2(emb_.p, r.ids, V, g_embed_.p, W(0).norm1.p, x_.p, operand(h_.p, dp, Mpad_, true), d, dp, spec.eps, batch_, Mpad_, r.active, r.pos_cur,
@@ -415,7 +422,7 @@ void LmBlocks::pass_layer(int li, int M, const RowTable& rows, int n_tiles, int 
         a.q = (const bf16_t*)pq_.p; a.kv = pkv_.p; a.ldkv = Nkv; a.cache = (const bf16_t*)cache_[li]->p; a.Smax = Smax_; a.tiles = ptiles_.p; a.n_tiles = n_tiles;
         a.out = (bf16_t*)at; a.ldo = l.Ko;
         launch_latent_attn_prefill(D, a, s);
-    } else absorbed_attention(li, pqkv_.p, pq_.p, polat_.p, operand(at, l.Ko, 0, false), rows, M, 1, s);
+    } else absorbed_attention(li, pqkv_.p, pq_.p, polat_.p, operand(at, l.Ko, 0, false), rows, M, 0, s);
     if (f32) {
         GemmF32 g = gemm32(at, l.Ko, w.wo.p, px_.p, dp, M, dp, l.Ko, F32_ADD_SCALED);
         g.ls = w.ls1.p;

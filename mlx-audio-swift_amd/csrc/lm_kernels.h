@@ -9,8 +9,14 @@ __host__ __device__ __forceinline__ size_t xpk_index(int m, int k, int MT) {
 
 enum { EPI_PARTIAL = 0, EPI_BF16 = 1, EPI_SILU_MUL = 2, EPI_GELU_PACKED = 3, EPI_SILU_PACKED = 4,
        EPI_SPLIT_RELU2 = 5,      // tiles below GemmExtra::split: float32 sums; the others: T(relu(y)^2) in the packed layout (out2)
-       EPI_SOFTCAP = 6 };        // float32: cap tanh(scale y / cap) (cap <= 0: scale y)
-struct GemmExtra { void* out2 = nullptr; int split = 0; float scale = 1.0f, cap = 0.0f; };
+       EPI_SOFTCAP = 6,          // float32: cap tanh(scale y / cap) (cap <= 0: scale y)
+       EPI_DUAL = 7 };           // two products of one output width in one launch: slabs [0, s1) = X W^T, slabs [s1, S) = x2 w2^T (kt2 k-tiles)
+struct GemmExtra {
+    void* out2 = nullptr; int split = 0; float scale = 1.0f, cap = 0.0f;
+    const bf16_t *w2 = nullptr, *x2 = nullptr; int kt2 = 0, s1 = 0;
+};
+// slabs of the two products of an EPI_DUAL launch (s1 + s2 <= s_max; kt2 = 0: no second product)
+void gemm_choose_dual_split(int items, int kt1, int kt2, int ksb, int s_max, int* s1, int* s2);
 
 void launch_convert_to_bf16(const void* src, int dtype, bf16_t* dst, size_t n, hipStream_t s);
 // MLX affine-quantised matrix (uint32 words, per-group scales / biases of dtype sb_dtype = mis_dtype) -> bf16 [N][K]

@@ -657,7 +657,7 @@ __device__ __forceinline__ void gemm_epilogue(const f32x4_t (&acc)[R][MT], void*
                 *reinterpret_cast<float4*>(reinterpret_cast<float*>(out) + ((size_t)mt * 16 + ml) * N_out + tile * 16 + nl) = make_float4(v[0], v[1], v[2], v[3]);
             }
         }
-    } else if (EPI == EPI_PARTIAL) {
+    } else if (EPI == EPI_PARTIAL || EPI == EPI_DUAL) {
         float* o = reinterpret_cast<float*>(out);
 #pragma unroll
         for (int r = 0; r < R; ++r) {
@@ -757,7 +757,13 @@ __global__ void __launch_bounds__((KSB == 1 ? 4 : KSB) * 64, 2) k_gemm_skinny(co
     const int item = (KSB == 1) ? blockIdx.x * 4 + wave : blockIdx.x;
     if (item >= n_items) return;                      // (KSB == 1: a wave of the last block may have no item)
     const int ntg = item / S, ks = item - ntg * S;
-    int kt0 = (int)(((long long)KT * ks) / S), kt1 = (int)(((long long)KT * (ks + 1)) / S);
+    int kq = ks, Sq = S;                              // slab of its product (EPI_DUAL: two products share the launch; block-uniform)
+    if constexpr (EPI == EPI_DUAL) {
+        static_assert(EPI != EPI_DUAL || KSB > 1, "the two products of a dual launch need block-wide items");
+        if (ks >= ex.s1) { Wp = ex.w2; X = ex.x2; KT = ex.kt2; kq = ks - ex.s1; Sq = S - ex.s1; }
+        else Sq = ex.s1;
+    }
+    int kt0 = (int)(((long long)KT * kq) / Sq), kt1 = (int)(((long long)KT * (kq + 1)) / Sq);
     if (KSB > 1) {                                    // this wave's quarter of the item's K range
         int len = kt1 - kt0;
         int a = kt0 + (int)(((long long)len * wave) / KSB), b = kt0 + (int)(((long long)len * (wave + 1)) / KSB);
@@ -918,6 +924,9 @@ static void launch_gemm_mt(int epi, int R, int ksb, int U, const bf16_t* Wp, con
         GEMM_CASE(EPI_SPLIT_RELU2, 4, 4, 3)
         GEMM_CASE(EPI_SOFTCAP, 4, 4, 3)
     }
+    if constexpr (MT <= 2) { GEMM_CASE(EPI_DUAL, 4, 4, 2) GEMM_CASE(EPI_DUAL, 4, 2, 2) }
+    GEMM_CASE(EPI_DUAL, 2, 4, 4)
+    GEMM_CASE(EPI_DUAL, 2, 2, 4)
     GEMM_CASE(EPI_SPLIT_RELU2, 2, 4, 4)
     GEMM_CASE(EPI_SOFTCAP, 2, 4, 4)
     GEMM_CASE(EPI_GELU_PACKED, 2, 4, 4)
@@ -931,7 +940,8 @@ static void launch_gemm_mt(int epi, int R, int ksb, int U, const bf16_t* Wp, con
 
 void launch_gemm_skinny(int epi, int R, int ksb, const bf16_t* Wp, const bf16_t* X, void* out, int NT, int KT, int S,
                         int N_out, int Mpad, hipStream_t s, const bf16_t* bias, int U, const GemmExtra& ex) {
-    MIS_REQUIRE(epi == EPI_PARTIAL || S == 1, MIS_ERR_GENERATION_FAILED, "split-K needs the partial epilogue");
+    MIS_REQUIRE(epi == EPI_PARTIAL || epi == EPI_DUAL || S == 1, MIS_ERR_GENERATION_FAILED, "split-K needs the partial epilogue");
+    MIS_REQUIRE(epi != EPI_DUAL || (ex.s1 >= 1 && ex.s1 < S && ex.w2 && ex.x2 && ex.kt2 >= 1), MIS_ERR_GENERATION_FAILED, "dual GEMM: second product missing");
     if (U <= 0) U = R >= 4 ? 3 : GEMM_U;
     switch (Mpad / 16) {
         case 1: launch_gemm_mt<1>(epi, R, ksb, U, Wp, X, out, NT, KT, S, N_out, Mpad, bias, s, ex); break;
@@ -1166,6 +1176,22 @@ int gemm_choose_split(int items, int KT, int ksb, int s_max) {
         if (cost < best_cost * (1.0 - 1e-9)) { best_cost = cost; best = S; }
     }
     return best;
+}
+
+// the same cost for two products that share a launch: every block streams one slab's share of one product
+void gemm_choose_dual_split(int items, int kt1, int kt2, int ksb, int s_max, int* s1, int* s2) {
+    if (kt2 <= 0) { *s1 = std::max(1, std::min(s_max, gemm_choose_split(items, kt1, ksb, s_max))); *s2 = 0; return; }
+    static const int n_cu = [] { int dev = 0; hipDeviceProp_t prop{}; return (hipGetDevice(&dev) == hipSuccess && hipGetDeviceProperties(&prop, dev) == hipSuccess && prop.multiProcessorCount > 0) ? prop.multiProcessorCount : 256; }();
+    const int U = 4;
+    double best = 1e30;
+    *s1 = *s2 = 1;
+    for (int a = 1; a < s_max && a <= std::max(1, kt1 / (2 * ksb)); ++a)
+        for (int b = 1; a + b <= s_max && b <= std::max(1, kt2 / (2 * ksb)); ++b) {
+            auto wave_tiles = [&](int kt, int s) { const int kw = (kt + s * ksb - 1) / (s * ksb); return (kw + U - 1) / U * U; };
+            const long blocks = (long)items * (a + b);
+            const double cost = (double)((blocks + n_cu - 1) / n_cu) * std::max(wave_tiles(kt1, a), wave_tiles(kt2, b)) * (1.0 + 0.01 * (a + b));
+            if (cost < best * (1.0 - 1e-9)) { best = cost; *s1 = a; *s2 = b; }
+        }
 }
 
 // ============================================================================ decode attention

@@ -29,10 +29,11 @@ struct RowTable { const int32_t* seq = nullptr; const int32_t* pos = nullptr; co
 // x = rms(E[id]) * g_embed (float32 residual), operand = rms(x) * g_norm.  pos_cur / pos_next non-null: the decode step's position advance.
 void launch_rows_embed_norm2(const bf16_t* emb, const int32_t* ids, int vocab, const bf16_t* g_embed, const bf16_t* g_norm, float* x, const Operand& h,
                              int d, int dp, float eps, int n_rows, int rows, const uint8_t* on, int32_t* pos_cur, int32_t* pos_next, hipStream_t s);
-// x += lsA * sum(slabsA) + lsB * sum(slabsB); operand = rms(x) * g_norm.  Slabs [S][slab_rows][dp] float32, added in slab order; S = 0: branch absent.
-struct ScaledSlabs { const float* p = nullptr; int S = 0; const bf16_t* ls = nullptr; };
-void launch_scaled_residual_norm(const ScaledSlabs& a, const ScaledSlabs& b, int slab_rows, float* x, const bf16_t* g_norm, const Operand& h, int d, int dp,
-                                 float eps, int rows, hipStream_t s);
+// x += ls1 * sum(slabs 0 .. s1 - 1) + ls2 * sum(slabs s1 .. s1 + s2 - 1); operand = rms(x) * g_norm.  Slabs [s1 + s2][slab_rows][dp] float32 (what an
+// EPI_DUAL launch writes), added in slab order; s2 = 0: one branch.
+struct ScaledSlabs { const float* p = nullptr; int s1 = 0, s2 = 0; const bf16_t *ls1 = nullptr, *ls2 = nullptr; };
+void launch_scaled_residual_norm(const ScaledSlabs& a, int slab_rows, float* x, const bf16_t* g_norm, const Operand& h, int d, int dp, float eps, int rows,
+                                 hipStream_t s);
 // operand row i = rms(x[row_of[i]]) * g_norm (row_of null: i)
 void launch_gather_norm(const float* x, const int32_t* row_of, const bf16_t* g_norm, const Operand& h, int d, int dp, float eps, int rows, hipStream_t s);
 
@@ -83,16 +84,19 @@ struct LatentAttn {
     RowTable rows;
     void* out;                  // [rows][H][Rp] latent sums (bf16, or float32 when f32)
     int f32;
-    // bf16 split over the keys: partial sums [S][rows][Hp][Rp] float32 and (max, sum) pairs [S][rows][Hp][2], Hp = H rounded up to 16
-    int S = 1;
-    float* part = nullptr;
-    float* ml = nullptr;
 };
-bool latent_attn_mfma_ok(const LatentDims& D);
-int latent_attn_splits(const LatentDims& D, int rows, int Smax);
-void launch_latent_attn_absorbed(const LatentDims& D, const LatentAttn& p, int rows, hipStream_t s);
+// any sizes, either element type
+void launch_latent_attn_any(const LatentDims& D, const LatentAttn& p, int rows, hipStream_t s);
 // values of the latent sums: operand[m][h v + j] = sum_R o_lat[m][h] W_uv[h][j]  (bf16; uv: packed per head, head stride uvz)
 void launch_latent_values(const LatentDims& D, const bf16_t* o_lat, const bf16_t* uv, size_t uvz, const Operand& out, int rows, hipStream_t s);
+
+// decode, bf16, matrix cores: every row's keys in S shares.  A share leaves its normalised latent sums (bf16) and (max, sum) of its scores; the
+// second launch weights the shares and applies the values.
+struct LatentShares { int S = 1; bf16_t* part = nullptr; float* ml = nullptr; };      // part [S][rows][H][Rp], ml [S][rows][H][2]
+bool latent_decode_mfma_ok(const LatentDims& D);
+int latent_decode_shares(const LatentDims& D, int rows, int Smax);
+void launch_latent_attn_decode(const LatentDims& D, const LatentAttn& p, const LatentShares& sh, int rows, hipStream_t s);
+void launch_latent_share_values(const LatentDims& D, const LatentShares& sh, const bf16_t* uv, size_t uvz, const Operand& out, int rows, hipStream_t s);
 
 // prompt pass, bf16: keys and values expanded by a GEMM into kv [key rows][H np | H vp]; one block per (tile of queries of one sequence, head)
 struct LatentTile { int32_t row0, n, seq, pos0, krow0, kpos0; };     // n <= LATENT_QT queries from pos0; key row of position p: krow0 + p - kpos0

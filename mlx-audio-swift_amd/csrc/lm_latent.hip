@@ -140,50 +140,43 @@ __global__ void __launch_bounds__(1024) k_rows_embed_norm2(const bf16_t* __restr
     }
 }
 
-// SG >= number of slabs of either branch (clamped, unconditional loads: one round trip); SG = 0: no slabs, the stream is only normed
+// SG >= s1 + s2 (clamped, unconditional loads: one round trip for everything the row needs); SG = 0: no slabs, the stream is only normed
 template <int CPT, int SG>
-__global__ void __launch_bounds__(1024) k_scaled_residual_norm(ScaledSlabs A, ScaledSlabs B, int slab_rows, float* __restrict__ x, const int32_t* __restrict__ row_of,
+__global__ void __launch_bounds__(1024) k_scaled_residual_norm(ScaledSlabs A, int slab_rows, float* __restrict__ x, const int32_t* __restrict__ row_of,
                                                                const bf16_t* __restrict__ g_norm, Operand h, int d, int dp, float eps) {
     __shared__ float red[16];
     const int m = blockIdx.x, tid = threadIdx.x, nth = blockDim.x, nc = dp >> 2;
     const size_t xr = (size_t)(row_of ? row_of[m] : m) * dp;
     float v[CPT][4], gn[CPT][4], ss = 0.0f;
+    float4 sl[CPT][SG ? SG : 1];
+    float l1[CPT][4], l2[CPT][4];
 #pragma unroll
     for (int g = 0; g < CPT; ++g) {
         const int c = tid + g * nth, cc = c < nc ? c : 0;
         const float4 t = *reinterpret_cast<const float4*>(x + xr + 4 * cc);
         v[g][0] = t.x; v[g][1] = t.y; v[g][2] = t.z; v[g][3] = t.w;
         load4_bf16(g_norm + 4 * cc, gn[g]);
+        if constexpr (SG > 0) {
+            const int S = A.s1 + A.s2;
+#pragma unroll
+            for (int j = 0; j < SG; ++j) sl[g][j] = *reinterpret_cast<const float4*>(A.p + ((size_t)(j < S ? j : S - 1) * slab_rows + m) * dp + 4 * cc);
+            load4_bf16(A.ls1 + 4 * cc, l1[g]);
+            load4_bf16((A.s2 ? A.ls2 : A.ls1) + 4 * cc, l2[g]);
+        }
     }
     if constexpr (SG > 0) {
 #pragma unroll
-        for (int br = 0; br < 2; ++br) {
-            const ScaledSlabs& P = br ? B : A;
-            if (P.S == 0) continue;                              // uniform
-            float4 sl[CPT][SG];
-            float ls[CPT][4];
-#pragma unroll
-            for (int g = 0; g < CPT; ++g) {
-                const int c = tid + g * nth, cc = c < nc ? c : 0;
-#pragma unroll
-                for (int j = 0; j < SG; ++j)
-                    sl[g][j] = *reinterpret_cast<const float4*>(P.p + ((size_t)(j < P.S ? j : P.S - 1) * slab_rows + m) * dp + 4 * cc);
-                load4_bf16(P.ls + 4 * cc, ls[g]);
-            }
-#pragma unroll
-            for (int g = 0; g < CPT; ++g) {
-                float a[4] = {0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-                for (int j = 0; j < SG; ++j) {                   // slab order 0, 1, 2, ...: deterministic
-                    const bool live = j < P.S;
-                    a[0] += live ? sl[g][j].x : 0.0f; a[1] += live ? sl[g][j].y : 0.0f; a[2] += live ? sl[g][j].z : 0.0f; a[3] += live ? sl[g][j].w : 0.0f;
-                }
-#pragma unroll
-                for (int j = 0; j < 4; ++j) v[g][j] += ls[g][j] * a[j];
-            }
-        }
-#pragma unroll
         for (int g = 0; g < CPT; ++g) {
+            float a[4] = {0.f, 0.f, 0.f, 0.f}, b[4] = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+            for (int j = 0; j < SG; ++j) {                       // slab order 0, 1, 2, ...: deterministic
+                const bool first = j < A.s1, second = !first && j < A.s1 + A.s2;
+                const float f[4] = {sl[g][j].x, sl[g][j].y, sl[g][j].z, sl[g][j].w};
+#pragma unroll
+                for (int e = 0; e < 4; ++e) { a[e] += first ? f[e] : 0.0f; b[e] += second ? f[e] : 0.0f; }
+            }
+#pragma unroll
+            for (int e = 0; e < 4; ++e) v[g][e] += l1[g][e] * a[e] + l2[g][e] * b[e];
             const int c = tid + g * nth;
             if (c < nc) *reinterpret_cast<float4*>(x + xr + 4 * c) = make_float4(v[g][0], v[g][1], v[g][2], v[g][3]);
         }
@@ -215,23 +208,23 @@ void launch_rows_embed_norm2(const bf16_t* emb, const int32_t* ids, int vocab, c
     if (cpt == 1) EMB2(1); else if (cpt == 2) EMB2(2); else EMB2(4);
 #undef EMB2
 }
-static void residual_norm(const ScaledSlabs& a, const ScaledSlabs& b, int slab_rows, float* x, const int32_t* row_of, const bf16_t* g_norm, const Operand& h,
-                          int d, int dp, float eps, int rows, hipStream_t s) {
+static void residual_norm(const ScaledSlabs& a, int slab_rows, float* x, const int32_t* row_of, const bf16_t* g_norm, const Operand& h, int d, int dp,
+                          float eps, int rows, hipStream_t s) {
     row_check(dp);
-    const int cpt = row_cpt(dp), nth = row_threads(dp, cpt), S = std::max(a.S, b.S);
-    MIS_REQUIRE(S <= 8, MIS_ERR_GENERATION_FAILED, "more than 8 split-K slabs per branch");
-#define RN(C, G) hipLaunchKernelGGL((k_scaled_residual_norm<C, G>), dim3(rows), dim3(nth), 0, s, a, b, slab_rows, x, row_of, g_norm, h, d, dp, eps)
-#define RNC(C) do { if (S == 0) RN(C, 0); else if (S == 1) RN(C, 1); else if (S == 2) RN(C, 2); else if (S <= 4) RN(C, 4); else RN(C, 8); } while (0)
+    const int cpt = row_cpt(dp), nth = row_threads(dp, cpt), S = a.s1 + a.s2;
+    MIS_REQUIRE(S <= (cpt == 4 ? 4 : 8), MIS_ERR_GENERATION_FAILED, "too many split-K slabs");
+#define RN(C, G) hipLaunchKernelGGL((k_scaled_residual_norm<C, G>), dim3(rows), dim3(nth), 0, s, a, slab_rows, x, row_of, g_norm, h, d, dp, eps)
+#define RNC(C) do { if (S == 0) RN(C, 0); else if (S <= 2) RN(C, 2); else if (S <= 4) RN(C, 4); else RN(C, C == 4 ? 4 : 8); } while (0)
     if (cpt == 1) RNC(1); else if (cpt == 2) RNC(2); else RNC(4);
 #undef RNC
 #undef RN
 }
-void launch_scaled_residual_norm(const ScaledSlabs& a, const ScaledSlabs& b, int slab_rows, float* x, const bf16_t* g_norm, const Operand& h, int d, int dp,
-                                 float eps, int rows, hipStream_t s) {
-    residual_norm(a, b, slab_rows, x, nullptr, g_norm, h, d, dp, eps, rows, s);
+void launch_scaled_residual_norm(const ScaledSlabs& a, int slab_rows, float* x, const bf16_t* g_norm, const Operand& h, int d, int dp, float eps, int rows,
+                                 hipStream_t s) {
+    residual_norm(a, slab_rows, x, nullptr, g_norm, h, d, dp, eps, rows, s);
 }
 void launch_gather_norm(const float* x, const int32_t* row_of, const bf16_t* g_norm, const Operand& h, int d, int dp, float eps, int rows, hipStream_t s) {
-    residual_norm(ScaledSlabs{}, ScaledSlabs{}, 0, const_cast<float*>(x), row_of, g_norm, h, d, dp, eps, rows, s);
+    residual_norm(ScaledSlabs{}, 0, const_cast<float*>(x), row_of, g_norm, h, d, dp, eps, rows, s);
 }
 
 // ============================================================================ float32 GEMM (v_mfma_f32_16x16x4_f32)
@@ -295,12 +288,20 @@ __device__ __forceinline__ void put(bf16_t* p, float v) { *p = f32_to_bf16(v); }
 __device__ __forceinline__ float get(const float* p) { return *p; }
 __device__ __forceinline__ float get(const bf16_t* p) { return bf16_to_f32(*p); }
 
-// element j of a rotated vector of r values whose first rot_dims are rotated pairwise (2 i, 2 i + 1); zero past r
-__device__ __forceinline__ float rotary_at(const float* src, int j, int r, int rot_dims, const float* cs, const float* sn) {
-    if (j >= r) return 0.0f;
-    if (j >= rot_dims) return src[j];
-    const float c = cs[j >> 1], s = sn[j >> 1];
-    return (j & 1) ? src[j] * c + src[j - 1] * s : src[j] * c - src[j + 1] * s;
+__device__ __forceinline__ void put4(float* p, const float (&v)[4]) { *reinterpret_cast<float4*>(p) = make_float4(v[0], v[1], v[2], v[3]); }
+__device__ __forceinline__ void put4(bf16_t* p, const float (&v)[4]) { *reinterpret_cast<uint2*>(p) = pack4_bf16(v); }
+
+// columns j .. j + 3 (j % 4 == 0) of a rotary part: pairs (2 i, 2 i + 1) below rot_dims are turned, the others pass (padding columns hold zeros)
+__device__ __forceinline__ void rotary4(const float* src, int j, int rot_dims, const float* cs, const float* sn, float (&o)[4]) {
+    const float4 t = *reinterpret_cast<const float4*>(src + j);
+    o[0] = t.x; o[1] = t.y; o[2] = t.z; o[3] = t.w;
+#pragma unroll
+    for (int k = 0; k < 2; ++k)
+        if (j + 2 * k < rot_dims) {
+            const float c = cs[(j >> 1) + k], s = sn[(j >> 1) + k], u = o[2 * k], v = o[2 * k + 1];
+            o[2 * k] = u * c - v * s;
+            o[2 * k + 1] = v * c + u * s;
+        }
 }
 
 template <typename T>
@@ -309,24 +310,35 @@ __device__ __forceinline__ void latent_row(const LatentDims& D, const LatentRows
     if (p.rows.on && !p.rows.on[m]) return;                                    // block-uniform
     const int pos = p.rows.pos[m], seq = p.rows.seq ? p.rows.seq[m] : m;
     const float* row = p.qkv + (size_t)m * p.ld;
-    const float* craw = row + (size_t)D.H * HQ;
+    const float* craw = row + (size_t)D.H * HQ;                                 // [latent Rp | rotary key rp], padding columns zero
     const float *cs = p.rope_cos + (size_t)pos * (D.rot_dims / 2), *sn = p.rope_sin + (size_t)pos * (D.rot_dims / 2);
     float ss = 0.0f;
-    for (int i = tid; i < D.R; i += nth) ss += craw[i] * craw[i];
+    for (int i = tid * 4; i < D.Rp; i += nth * 4) {
+        const float4 t = *reinterpret_cast<const float4*>(craw + i);
+        ss += t.x * t.x + t.y * t.y + t.z * t.z + t.w * t.w;
+    }
+    // query rows (independent of the latent's norm)
+    T* q = (T*)p.q + (size_t)m * D.H * p.q_ld;
+    const int j0 = p.with_plain ? 0 : p.q_rot_off, w = (p.q_ld - j0) >> 2;
+    for (int t = tid; t < D.H * w; t += nth) {
+        const int hd = t / w, j = j0 + (t - hd * w) * 4, jr = j - p.q_rot_off;
+        const float* src = row + (size_t)hd * HQ;
+        float o[4] = {0.f, 0.f, 0.f, 0.f};
+        if (jr < 0) { const float4 f = *reinterpret_cast<const float4*>(src + j); o[0] = f.x; o[1] = f.y; o[2] = f.z; o[3] = f.w; }
+        else if (jr < D.rp) rotary4(src + D.np, jr, D.rot_dims, cs, sn, o);
+        put4(q + (size_t)hd * p.q_ld + j, o);
+    }
     const float inv = 1.0f / sqrtf(lat_block_sum(ss, red) / (float)D.R + D.eps);
     T* cache = (T*)p.cache + ((size_t)seq * p.Smax + pos) * D.CW;
-    for (int i = tid; i < D.CW; i += nth) {
-        float v = 0.0f;
-        if (i < D.R) v = craw[i] * inv * bf16_to_f32(p.c_norm[i]);
-        else if (i >= D.Rp) v = rotary_at(craw + D.Rp, i - D.Rp, D.r, D.rot_dims, cs, sn);
-        put(cache + i, v);
-    }
-    T* q = (T*)p.q + (size_t)m * D.H * p.q_ld;
-    const int j0 = p.with_plain ? 0 : p.q_rot_off, w = p.q_ld - j0;
-    for (int t = tid; t < D.H * w; t += nth) {
-        const int hd = t / w, j = j0 + (t - hd * w);
-        const float* src = row + (size_t)hd * HQ;
-        put(q + (size_t)hd * p.q_ld + j, j < p.q_rot_off ? src[j] : rotary_at(src + D.np, j - p.q_rot_off, D.r, D.rot_dims, cs, sn));
+    for (int i = tid * 4; i < D.CW; i += nth * 4) {
+        float o[4] = {0.f, 0.f, 0.f, 0.f};
+        if (i < D.Rp) {
+            const float4 t = *reinterpret_cast<const float4*>(craw + i);
+            float g[4];
+            load4_bf16(p.c_norm + i, g);
+            o[0] = t.x * inv * g[0]; o[1] = t.y * inv * g[1]; o[2] = t.z * inv * g[2]; o[3] = t.w * inv * g[3];
+        } else if (i < D.Rp + D.rp) rotary4(craw + D.Rp, i - D.Rp, D.rot_dims, cs, sn, o);
+        put4(cache + i, o);
     }
 }
 template <typename T>
@@ -355,19 +367,27 @@ __device__ __forceinline__ bf16x8_t frag8(const float* p) {
 }
 __device__ __forceinline__ bf16x8_t frag8(const bf16_t* p) { return *reinterpret_cast<const bf16x8_t*>(p); }
 
-// two row tiles (32 rows from m0) x one weight tile over KT k-tiles
+// two row tiles (32 rows from m0) x one weight tile over KT k-tiles, four k-tiles requested at a time
 template <typename T>
 __device__ __forceinline__ void head_tile(const T* X, size_t ldx, int m0, int rows, const bf16_t* wt, int KT, f32x4_t (&acc)[2]) {
     const int lane = threadIdx.x & 63, li = lane & 15, q = lane >> 4;
     const T* x0 = X + (size_t)min(m0 + li, rows - 1) * ldx + q * 8;
     const T* x1 = X + (size_t)min(m0 + 16 + li, rows - 1) * ldx + q * 8;
     acc[0] = acc[1] = (f32x4_t){0.f, 0.f, 0.f, 0.f};
-#pragma unroll 4
-    for (int kt = 0; kt < KT; ++kt) {
-        const bf16x8_t a = *reinterpret_cast<const bf16x8_t*>(wt + ((size_t)kt * 64 + lane) * 8);
-        const bf16x8_t b0 = frag8(x0 + kt * 32), b1 = frag8(x1 + kt * 32);
-        acc[0] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, b0, acc[0], 0, 0, 0);
-        acc[1] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, b1, acc[1], 0, 0, 0);
+    for (int k0 = 0; k0 < KT; k0 += 4) {
+        bf16x8_t a[4], b0[4], b1[4];
+#pragma unroll
+        for (int u = 0; u < 4; ++u) {
+            const int kt = min(k0 + u, KT - 1);
+            a[u] = *reinterpret_cast<const bf16x8_t*>(wt + ((size_t)kt * 64 + lane) * 8);
+            b0[u] = frag8(x0 + kt * 32); b1[u] = frag8(x1 + kt * 32);
+        }
+#pragma unroll
+        for (int u = 0; u < 4; ++u) {
+            if (k0 + u >= KT) continue;
+            acc[0] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a[u], b0[u], acc[0], 0, 0, 0);
+            acc[1] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a[u], b1[u], acc[1], 0, 0, 0);
+        }
     }
 }
 
@@ -482,10 +502,11 @@ __global__ void __launch_bounds__(256) k_latent_attn_any(LatentDims D, LatentAtt
 }
 
 // ============================================================================ absorbed attention on the matrix cores (decode)
-// Block = 4 waves: one row, one tile of 16 heads, one share of the row's 32-key tiles.  A key tile is read ONCE: each thread fetches 4 keys x 8
-// columns, writes them to LDS as key rows (score operand) and, transposed in registers, as column rows (value operand).  Scores: S^T = K q^T,
-// wave w = (key half w & 1, half w >> 1 of the columns); the halves meet in LDS, every wave then holds the 16 x 32 weights as the A operand
-// of its own quarter of the latent columns.  The next tile's loads are in flight during all of it (barriers wait for LDS only).
+// Block = one row, HT tiles of 16 heads (four waves each), one share of the row's 32-key tiles.  A key tile is read ONCE: each thread fetches
+// 4 keys x 8 columns, writes them to LDS as key rows (score operand) and, transposed in registers, as column rows (value operand).  Scores:
+// S^T = K q^T, wave w of a head tile = (key half w & 1, half w >> 1 of the columns); the halves meet in LDS, every wave then holds the 16 x 32
+// weights as the A operand of its own quarter of the latent columns.  The next tile's loads are in flight during all of it (barriers wait for
+// LDS only).  A share leaves its normalised sums as bf16 and its (max, sum); k_latent_share_values weights the shares.
 #define LAT_KT 32
 #define LAT_VS 36                                  // LDS stride of a transposed column (32 keys + 4)
 __device__ __forceinline__ void lds_barrier() { asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory"); }
@@ -503,43 +524,40 @@ __device__ __forceinline__ uint2 column_of(const uint4 (&r)[4], int e) {
     if (e & 1) return make_uint2((a[w] >> 16) | (b[w] & 0xffff0000u), (c[w] >> 16) | (d[w] & 0xffff0000u));
     return make_uint2((a[w] & 0xffffu) | (b[w] << 16), (c[w] & 0xffffu) | (d[w] << 16));
 }
-static size_t latent_decode_lds(const LatentDims& D) {
-    return (size_t)LAT_KT * (D.CW + 8) * 2 + (size_t)D.Rp * LAT_VS * 2 + 2 * 16 * 36 * 4;
+static size_t latent_decode_lds(const LatentDims& D, int HT) {
+    return (size_t)LAT_KT * (D.CW + 8) * 2 + (size_t)D.Rp * LAT_VS * 2 + (size_t)HT * 2 * 16 * 36 * 4;
 }
-// NTW: latent tiles per wave (Rp / 64 <= NTW); NST: staging rounds (CW <= 256 NST); QF: query fragments per wave (CW / 32 <= 2 QF)
-template <int NTW, int NST, int QF>
-__global__ void __launch_bounds__(256, 2) k_latent_attn_decode(LatentDims D, LatentAttn p, int rows) {
+// NTW: latent tiles per wave (Rp / 64 <= NTW); NST: staging rounds (CW <= 256 HT NST); QF: query fragments per wave (CW / 32 <= 2 QF)
+template <int NTW, int NST, int QF, int HT>
+__global__ void __launch_bounds__(256 * HT, 2) k_latent_attn_decode(LatentDims D, LatentAttn p, LatentShares sh, int rows) {
     extern __shared__ __attribute__((aligned(16))) uint8_t lds[];
     const int KS = D.CW + 8;
     bf16_t* sk = reinterpret_cast<bf16_t*>(lds);                                // [32][CW + 8]
     bf16_t* sv = sk + (size_t)LAT_KT * KS;                                      // [Rp][LAT_VS]
-    float* sc = reinterpret_cast<float*>(sv + (size_t)D.Rp * LAT_VS);           // [2][16][36]
-    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, li = lane & 15, lq = lane >> 4;
-    const int m = blockIdx.x / p.S, sp = blockIdx.x - m * p.S, h0 = blockIdx.y * 16;
+    const int tid = threadIdx.x, lane = tid & 63, wave = (tid >> 6) & 3, ht = tid >> 8, li = lane & 15, lq = lane >> 4;
+    float* sc = reinterpret_cast<float*>(sv + (size_t)D.Rp * LAT_VS) + (size_t)ht * 2 * 16 * 36;        // [2][16][36]
+    const int m = blockIdx.x / sh.S, sp = blockIdx.x - m * sh.S, h0 = (blockIdx.y * HT + ht) * 16;
     const bool on = !p.rows.on || p.rows.on[m];
     const int pos = on ? p.rows.pos[m] : 0, seq = p.rows.seq ? p.rows.seq[m] : m;
     const int lo = D.window > 0 ? max(0, pos - D.window + 1) : 0;
     const int nt = on ? (pos - lo + LAT_KT) / LAT_KT : 0;
-    const int t0 = (int)((long long)nt * sp / p.S), t1 = (int)((long long)nt * (sp + 1) / p.S);
+    const int t0 = (int)((long long)nt * sp / sh.S), t1 = (int)((long long)nt * (sp + 1) / sh.S);
     const bf16_t* cache = (const bf16_t*)p.cache + (size_t)seq * p.Smax * D.CW;
     const int nch = D.CW >> 3, CT = D.CW >> 5;
-    int chunk[NST], kg[NST];
-#pragma unroll
-    for (int i = 0; i < NST; ++i) {
-        const int task = tid + 256 * i;
-        kg[i] = task / nch;
-        chunk[i] = task - kg[i] * nch;
-    }
+    const int kg = tid & 7;                                                     // four keys 4 kg .. of the tile; eight lanes share a 16-byte column chunk
     uint4 st[NST][4];
     auto fetch = [&](int t) {
 #pragma unroll
-        for (int i = 0; i < NST; ++i)
+        for (int i = 0; i < NST; ++i) {
+            const int chunk = min((tid >> 3) + 32 * HT * i, nch - 1);           // (rounds past the row read its last chunk and are not stored)
 #pragma unroll
             for (int k = 0; k < 4; ++k) {
-                const int key = min(lo + t * LAT_KT + 4 * min(kg[i], 7) + k, pos);      // (rounds past the tile read a valid row and are not stored)
-                st[i][k] = *reinterpret_cast<const uint4*>(cache + (size_t)key * D.CW + chunk[i] * 8);
+                const int key = min(lo + t * LAT_KT + 4 * kg + k, pos);
+                st[i][k] = *reinterpret_cast<const uint4*>(cache + (size_t)key * D.CW + chunk * 8);
             }
+        }
     };
+    if (t0 < t1) fetch(t0);
     // this wave's half of the query columns: heads past H read head H - 1 and are dropped at the end
     const int half = wave >> 1, kt0 = half ? (CT + 1) / 2 : 0, kt1 = half ? CT : (CT + 1) / 2;
     bf16x8_t qf[QF];
@@ -552,18 +570,19 @@ __global__ void __launch_bounds__(256, 2) k_latent_attn_decode(LatentDims D, Lat
 #pragma unroll
     for (int i = 0; i < NTW; ++i) o[i] = (f32x4_t){0.f, 0.f, 0.f, 0.f};
     float mx = -INFINITY, ls = 0.0f;                                            // of head li; ls: this lane's keys only
-    if (t0 < t1) fetch(t0);
     for (int t = t0; t < t1; ++t) {
 #pragma unroll
-        for (int i = 0; i < NST; ++i)
-            if (kg[i] < 8) {
+        for (int i = 0; i < NST; ++i) {
+            const int chunk = (tid >> 3) + 32 * HT * i;
+            if (chunk < nch) {
 #pragma unroll
-                for (int k = 0; k < 4; ++k) *reinterpret_cast<uint4*>(sk + (size_t)(4 * kg[i] + k) * KS + chunk[i] * 8) = st[i][k];
-                if (chunk[i] * 8 < D.Rp) {
+                for (int k = 0; k < 4; ++k) *reinterpret_cast<uint4*>(sk + (size_t)(4 * kg + k) * KS + chunk * 8) = st[i][k];
+                if (chunk * 8 < D.Rp) {
 #pragma unroll
-                    for (int e = 0; e < 8; ++e) *reinterpret_cast<uint2*>(sv + (size_t)(chunk[i] * 8 + e) * LAT_VS + 4 * kg[i]) = column_of(st[i], e);
+                    for (int e = 0; e < 8; ++e) *reinterpret_cast<uint2*>(sv + (size_t)(chunk * 8 + e) * LAT_VS + 4 * kg) = column_of(st[i], e);
                 }
             }
+        }
         if (t + 1 < t1) fetch(t + 1);
         lds_barrier();
         f32x4_t s = (f32x4_t){0.f, 0.f, 0.f, 0.f};
@@ -593,11 +612,13 @@ __global__ void __launch_bounds__(256, 2) k_latent_attn_decode(LatentDims D, Lat
             for (int e = 0; e < 8; ++e) { w[e] = __expf(w[e] - mn); add += w[e]; }
             ls = ls * alpha + add;
             mx = mn;
+            if (t > t0) {                                                       // (the first tile has nothing to rescale)
 #pragma unroll
-            for (int e = 0; e < 4; ++e) {
-                const float ah = __shfl(alpha, lq * 4 + e, 64);                 // head of accumulator row e
+                for (int e = 0; e < 4; ++e) {
+                    const float ah = __shfl(alpha, lq * 4 + e, 64);             // head of accumulator row e
 #pragma unroll
-                for (int i = 0; i < NTW; ++i) o[i][e] *= ah;
+                    for (int i = 0; i < NTW; ++i) o[i][e] *= ah;
+                }
             }
         }
         bf16x8_t ph, pl;
@@ -619,72 +640,158 @@ __global__ void __launch_bounds__(256, 2) k_latent_attn_decode(LatentDims D, Lat
     }
     ls += __shfl_xor(ls, 16, 64);
     ls += __shfl_xor(ls, 32, 64);
-    const int Hp = gridDim.y * 16;
-    if (p.S > 1 && wave == 0 && lq == 0) {
-        float* ml = p.ml + (((size_t)sp * rows + m) * Hp + h0 + li) * 2;
-        ml[0] = mx; ml[1] = ls;
+    if (wave == 0 && lq == 0 && h0 + li < D.H) {
+        float* ml = sh.ml + (((size_t)sp * rows + m) * D.H + h0 + li) * 2;
+        *reinterpret_cast<float2*>(ml) = make_float2(mx, ls);
     }
+    // normalised rows through LDS (the key rows' place), then 16-byte stores
+    bf16_t* so = sk + (size_t)ht * 16 * (D.Rp + 8);
 #pragma unroll
     for (int e = 0; e < 4; ++e) {
-        const int hd = h0 + lq * 4 + e;
         const float l = __shfl(ls, lq * 4 + e, 64), inv = l > 0.0f ? 1.0f / l : 0.0f;
 #pragma unroll
         for (int i = 0; i < NTW; ++i) {
             const int c = (i * 4 + wave) * 16 + li;
-            if (c >= D.Rp) continue;
-            if (p.S > 1) p.part[(((size_t)sp * rows + m) * Hp + hd) * D.Rp + c] = o[i][e];
-            else if (hd < D.H) ((bf16_t*)p.out)[((size_t)m * D.H + hd) * D.Rp + c] = f32_to_bf16(o[i][e] * inv);
+            if (c < D.Rp) so[(size_t)(lq * 4 + e) * (D.Rp + 8) + c] = f32_to_bf16(o[i][e] * inv);
         }
     }
-}
-// the shares of a row meet: one block per (row, head), two columns per thread
-__global__ void __launch_bounds__(256) k_latent_combine(LatentDims D, LatentAttn p, int rows, int Hp) {
-    const int m = blockIdx.x, hd = blockIdx.y;
-    float mx = -INFINITY;
-    for (int s = 0; s < p.S; ++s) mx = fmaxf(mx, p.ml[(((size_t)s * rows + m) * Hp + hd) * 2]);
-    const int c = threadIdx.x * 2;
-    float a0 = 0.0f, a1 = 0.0f, l = 0.0f;
-    for (int s = 0; s < p.S; ++s) {
-        const float* ml = p.ml + (((size_t)s * rows + m) * Hp + hd) * 2;
-        const float w = ml[1] > 0.0f ? __expf(ml[0] - mx) : 0.0f;              // (an empty share holds sum 0)
-        const float2 v = *reinterpret_cast<const float2*>(p.part + (((size_t)s * rows + m) * Hp + hd) * D.Rp + c);
-        l += w * ml[1];
-        a0 += w * v.x; a1 += w * v.y;
+    lds_barrier();
+    const int rc = D.Rp >> 3;
+    for (int t = tid & 255; t < 16 * rc; t += 256) {
+        const int hr = t / rc, c = t - hr * rc;
+        if (h0 + hr < D.H)
+            *reinterpret_cast<uint4*>(sh.part + (((size_t)sp * rows + m) * D.H + h0 + hr) * D.Rp + c * 8) =
+                *reinterpret_cast<const uint4*>(so + (size_t)hr * (D.Rp + 8) + c * 8);
     }
-    const float inv = l > 0.0f ? 1.0f / l : 0.0f;
-    *reinterpret_cast<uint32_t*>((bf16_t*)p.out + ((size_t)m * D.H + hd) * D.Rp + c) = (uint32_t)f32_to_bf16(a0 * inv) | ((uint32_t)f32_to_bf16(a1 * inv) << 16);
 }
 
-bool latent_attn_mfma_ok(const LatentDims& D) { return D.Rp <= 512 && D.CW <= (D.Rp <= 128 ? 256 : D.Rp <= 256 ? 512 : 768); }
-// shares per row: about two blocks per CU, at least two key tiles each
-int latent_attn_splits(const LatentDims& D, int rows, int Smax) {
-    if (!latent_attn_mfma_ok(D)) return 1;
-    const int keys = D.window > 0 ? std::min(D.window, Smax) : Smax, tiles = cdiv(keys, LAT_KT), blocks = rows * cdiv(D.H, 16);
-    return std::max(1, std::min(std::min(cdiv(384, blocks), tiles / 2), 16));
-}
-void launch_latent_attn_absorbed(const LatentDims& D, const LatentAttn& p, int rows, hipStream_t s) {
-    MIS_REQUIRE(p.rows.pos && p.q && p.cache && p.out && rows >= 1, MIS_ERR_GENERATION_FAILED, "latent attention: null operand");
-    if (p.f32 || !latent_attn_mfma_ok(D)) {
-        MIS_REQUIRE(D.Rp <= 256 * LAT_OC, MIS_ERR_INVALID_INPUT, "latent size above 2048");
-        const size_t sm = (size_t)(D.CW + 256 + 8) * 4;
-        if (p.f32) hipLaunchKernelGGL((k_latent_attn_any<float>), dim3(rows, D.H), dim3(256), sm, s, D, p);
-        else hipLaunchKernelGGL((k_latent_attn_any<bf16_t>), dim3(rows, D.H), dim3(256), sm, s, D, p);
-        return;
+// One block of 16 waves per (head, 16 rows): weights of the shares -> latent sums of the rows (bf16, LDS) -> values.  Wave = (value tile, part of the
+// latent columns); its weight fragments are requested before the shares are read.
+// KF: k-tiles per wave at most; above 8 (value dimensions past 128) the fragments are requested behind the shares (registers).
+template <int KF>
+__global__ void __launch_bounds__(1024) k_latent_share_values(LatentDims D, LatentShares sh, const bf16_t* __restrict__ uv, size_t uvz, Operand out, int rows) {
+    extern __shared__ __attribute__((aligned(16))) uint8_t lds[];
+    bf16_t* so = reinterpret_cast<bf16_t*>(lds);                                // [16][Rp + 8]
+    float4* red = reinterpret_cast<float4*>(lds + (size_t)16 * (D.Rp + 8) * 2); // [16][64]
+    const int hd = blockIdx.x, m0 = blockIdx.y * 16, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, li = lane & 15, lq = lane >> 4;
+    const int vt = D.vp >> 4, KT = D.Rp >> 5, KH = vt <= 4 ? 4 : vt <= 8 ? 2 : 1;
+    const int tile = wave / KH, kh = wave - tile * KH, kt0 = KT * kh / KH, kn = KT * (kh + 1) / KH - kt0;
+    constexpr bool early = KF <= 8;
+    bf16x8_t wf[KF];
+    auto request = [&](int t) {
+        const bf16_t* wp = uv + uvz * hd + ((size_t)min(t, vt - 1) * KT + kt0) * 512 + lane * 8;
+#pragma unroll
+        for (int i = 0; i < KF; ++i) wf[i] = *reinterpret_cast<const bf16x8_t*>(wp + (size_t)min(i, kn - 1) * 512);
+    };
+    if constexpr (early) request(tile);
+    const int rc = D.Rp >> 3;
+    for (int t = tid; t < 16 * rc; t += 1024) {
+        const int r = t / rc, c = t - r * rc, m = min(m0 + r, rows - 1);
+        const float2* ml = reinterpret_cast<const float2*>(sh.ml) + (size_t)m * D.H + hd;
+        const bf16_t* pp = sh.part + ((size_t)m * D.H + hd) * D.Rp + c * 8;
+        const size_t ss = (size_t)rows * D.H;
+        float a[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f}, l = 0.0f, mx = -INFINITY;
+        for (int s0 = 0; s0 < sh.S; s0 += 8) {
+            float2 q[8];
+            bf16x8_t v[8];
+#pragma unroll
+            for (int u = 0; u < 8; ++u) {
+                const int s = min(s0 + u, sh.S - 1);
+                q[u] = ml[ss * s];
+                v[u] = *reinterpret_cast<const bf16x8_t*>(pp + ss * s * D.Rp);
+            }
+            float mn = mx;
+#pragma unroll
+            for (int u = 0; u < 8; ++u) mn = fmaxf(mn, (s0 + u < sh.S && q[u].y > 0.0f) ? q[u].x : -INFINITY);        // (an empty share holds sum 0)
+            const float alpha = mx == -INFINITY ? 0.0f : __expf(mx - mn);
+            l *= alpha;
+#pragma unroll
+            for (int e = 0; e < 8; ++e) a[e] *= alpha;
+#pragma unroll
+            for (int u = 0; u < 8; ++u) {
+                const float w = (s0 + u < sh.S && q[u].y > 0.0f) ? __expf(q[u].x - mn) * q[u].y : 0.0f;
+                l += w;
+#pragma unroll
+                for (int e = 0; e < 8; ++e) a[e] += w * bf16_to_f32((bf16_t)v[u][e]);
+            }
+            mx = mn;
+        }
+        const float inv = l > 0.0f ? 1.0f / l : 0.0f;
+        bf16x8_t o;
+#pragma unroll
+        for (int e = 0; e < 8; ++e) o[e] = (short)f32_to_bf16(a[e] * inv);
+        *reinterpret_cast<bf16x8_t*>(so + (size_t)r * (D.Rp + 8) + c * 8) = o;
     }
-    MIS_REQUIRE(p.S == 1 || (p.part && p.ml), MIS_ERR_GENERATION_FAILED, "latent attention: no scratch for the key shares");
-    const dim3 grid(rows * p.S, cdiv(D.H, 16));
-    const size_t sm = latent_decode_lds(D);
-#define LAT_GO(A, B, C)                                                                                                                    \
-    do {                                                                                                                                   \
-        static const hipError_t attr = hipFuncSetAttribute((const void*)k_latent_attn_decode<A, B, C>, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024); \
-        HIP_CHECK(attr);                                                                                                                   \
-        hipLaunchKernelGGL((k_latent_attn_decode<A, B, C>), grid, dim3(256), sm, s, D, p, rows);                                           \
+    __syncthreads();
+    for (int t0 = 0; t0 < vt; t0 += 16 / KH) {
+        const int vtile = t0 + tile;
+        f32x4_t acc = (f32x4_t){0.f, 0.f, 0.f, 0.f};
+        if (vtile < vt) {
+            if (!early || t0 > 0) request(vtile);                               // (more value tiles than one round of waves)
+#pragma unroll
+            for (int i = 0; i < KF; ++i)
+                if (i < kn)
+                    acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wf[i], *reinterpret_cast<const bf16x8_t*>(so + (size_t)li * (D.Rp + 8) + (kt0 + i) * 32 + lq * 8), acc, 0, 0, 0);
+        }
+        if (KH > 1) {
+            red[wave * 64 + lane] = make_float4(acc[0], acc[1], acc[2], acc[3]);
+            __syncthreads();
+        }
+        const int m = m0 + li, c = vtile * 16 + lq * 4;
+        if (kh == 0 && vtile < vt && m < rows) {
+            float v[4] = {acc[0], acc[1], acc[2], acc[3]};
+            for (int k = 1; k < KH; ++k) {
+                const float4 t = red[(wave + k) * 64 + lane];
+                v[0] += t.x; v[1] += t.y; v[2] += t.z; v[3] += t.w;
+            }
+            if (D.v % 4 == 0) {
+                if (c < D.v) operand_store4(out, m, hd * D.v + c, v);
+            } else {
+#pragma unroll
+                for (int e = 0; e < 4; ++e) if (c + e < D.v) operand_store1(out, m, hd * D.v + c + e, v[e]);
+            }
+        }
+        if (KH > 1 && t0 + 16 / KH < vt) __syncthreads();
+    }
+}
+
+void launch_latent_attn_any(const LatentDims& D, const LatentAttn& p, int rows, hipStream_t s) {
+    MIS_REQUIRE(p.rows.pos && p.q && p.cache && p.out && rows >= 1 && D.Rp <= 256 * LAT_OC, MIS_ERR_GENERATION_FAILED, "latent attention: bad operands");
+    const size_t sm = (size_t)(D.CW + 256 + 8) * 4;
+    if (p.f32) hipLaunchKernelGGL((k_latent_attn_any<float>), dim3(rows, D.H), dim3(256), sm, s, D, p);
+    else hipLaunchKernelGGL((k_latent_attn_any<bf16_t>), dim3(rows, D.H), dim3(256), sm, s, D, p);
+}
+bool latent_decode_mfma_ok(const LatentDims& D) { return D.Rp <= 512 && D.CW <= (D.Rp <= 128 ? 256 : D.Rp <= 256 ? 512 : 768) && D.vp <= 256; }
+// shares per row: about one block per compute unit, one key tile each at least
+int latent_decode_shares(const LatentDims& D, int rows, int Smax) {
+    const char* e = getenv("MIS_LATENT_SHARES");                                // A/B
+    const int keys = D.window > 0 ? std::min(D.window, Smax) : Smax, tiles = cdiv(keys, LAT_KT), blocks = rows * cdiv(D.H, D.H > 16 ? 32 : 16);
+    const int want = e && atoi(e) > 0 ? atoi(e) : cdiv(256, blocks);
+    return std::max(1, std::min(std::min(want, tiles), 32));
+}
+void launch_latent_attn_decode(const LatentDims& D, const LatentAttn& p, const LatentShares& sh, int rows, hipStream_t s) {
+    MIS_REQUIRE(p.rows.pos && p.q && p.cache && sh.part && sh.ml && sh.S >= 1 && rows >= 1 && !p.f32 && latent_decode_mfma_ok(D), MIS_ERR_GENERATION_FAILED,
+                "latent decode attention: bad operands");
+    const int HT = D.H > 16 ? 2 : 1;
+    const dim3 grid(rows * sh.S, cdiv(D.H, 16 * HT));
+    const size_t sm = latent_decode_lds(D, HT);
+#define LAT_GO(A, B, C, T)                                                                                                                                      \
+    do {                                                                                                                                                        \
+        static const hipError_t attr = hipFuncSetAttribute((const void*)k_latent_attn_decode<A, B, C, T>, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024); \
+        HIP_CHECK(attr);                                                                                                                                        \
+        hipLaunchKernelGGL((k_latent_attn_decode<A, B, C, T>), grid, dim3(256 * T), sm, s, D, p, sh, rows);                                                     \
     } while (0)
-    if (D.Rp <= 128) LAT_GO(2, 1, 4);
-    else if (D.Rp <= 256) LAT_GO(4, 2, 8);
-    else LAT_GO(8, 3, 12);
+    if (D.Rp <= 128) { if (HT == 1) LAT_GO(2, 1, 4, 1); else LAT_GO(2, 1, 4, 2); }
+    else if (D.Rp <= 256) { if (HT == 1) LAT_GO(4, 2, 8, 1); else LAT_GO(4, 1, 8, 2); }
+    else { if (HT == 1) LAT_GO(8, 3, 12, 1); else LAT_GO(8, 2, 12, 2); }
 #undef LAT_GO
-    if (p.S > 1) hipLaunchKernelGGL(k_latent_combine, dim3(rows, D.H), dim3(D.Rp / 2), 0, s, D, p, rows, (int)grid.y * 16);
+}
+void launch_latent_share_values(const LatentDims& D, const LatentShares& sh, const bf16_t* uv, size_t uvz, const Operand& out, int rows, hipStream_t s) {
+    const size_t sm = (size_t)16 * (D.Rp + 8) * 2 + 16 * 64 * 16;
+    const int vt = D.vp / 16, KH = vt <= 4 ? 4 : vt <= 8 ? 2 : 1;               // as in the kernel
+    const dim3 grid(D.H, cdiv(rows, 16));
+    if (cdiv(D.Rp / 32, KH) <= 8) hipLaunchKernelGGL((k_latent_share_values<8>), grid, dim3(1024), sm, s, D, sh, uv, uvz, out, rows);
+    else hipLaunchKernelGGL((k_latent_share_values<16>), grid, dim3(1024), sm, s, D, sh, uv, uvz, out, rows);
 }
 
 // ============================================================================ expanded attention on the matrix cores (prompts)

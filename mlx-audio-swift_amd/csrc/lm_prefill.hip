@@ -118,6 +118,7 @@ __global__ void __launch_bounds__(256, 2) k_gemm_pf(PfGemmParams p) {
     __shared__ __attribute__((aligned(1024))) bf16_t Xs[2][PF_BM * PF_BK];
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
     const int n0 = blockIdx.x * PF_BN, m0 = blockIdx.y * PF_BM;
+    if (n0 >= p.N) return;                              // (padding of the grid, see launch_gemm_pf)
     const int wn = wave >> 1, wm = wave & 1;            // wave tile: 64 n x 64 m
     const int NT = p.N >> 4, KT = p.K >> 5;
     f32x4_t acc[4][4];
@@ -265,7 +266,10 @@ void launch_gemm_pf(int epi, const bf16_t* X, const bf16_t* Wp, void* C, int M, 
     MIS_REQUIRE(epi < PF_SPLIT_RELU2 || (ex.ldc % 4 == 0 && (epi != PF_ROWS_BF16 || (ex.xrow && ex.ldx % 8 == 0))), MIS_ERR_GENERATION_FAILED,
                 "prefill GEMM: bad row strides");
     PfGemmParams p{X, Wp, C, M, N, K, ex};
-    dim3 grid(cdiv(N, PF_BN), cdiv(M, PF_BM)), block(256);
+    // column tiles rounded up to the 8 XCDs: blocks are dealt to the XCDs by linear id, so that every row of tiles finds its weight tiles in the
+    // L2 that held them for the row before
+    const int nx = cdiv(N, PF_BN);
+    dim3 grid(nx >= 16 ? (int)round_up(nx, 8) : nx, cdiv(M, PF_BM)), block(256);
     if (epi == PF_F32) hipLaunchKernelGGL((k_gemm_pf<PF_F32>), grid, block, 0, s, p);
     else if (epi == PF_RESID) hipLaunchKernelGGL((k_gemm_pf<PF_RESID>), grid, block, 0, s, p);
     else if (epi == PF_SILU) hipLaunchKernelGGL((k_gemm_pf<PF_SILU>), grid, block, 0, s, p);
