@@ -502,13 +502,17 @@ __global__ void __launch_bounds__(256) k_latent_attn_any(LatentDims D, LatentAtt
 }
 
 // ============================================================================ absorbed attention on the matrix cores (decode)
-// Block = one row, HT tiles of 16 heads (four waves each), one share of the row's 32-key tiles.  A key tile is read ONCE: each thread fetches
-// 4 keys x 8 columns, writes them to LDS as key rows (score operand) and, transposed in registers, as column rows (value operand).  Scores:
-// S^T = K q^T, wave w of a head tile = (key half w & 1, half w >> 1 of the columns); the halves meet in LDS, every wave then holds the 16 x 32
-// weights as the A operand of its own quarter of the latent columns.  The next tile's loads are in flight during all of it (barriers wait for
-// LDS only).  A share leaves its normalised sums as bf16 and its (max, sum); k_latent_share_values weights the shares.
-#define LAT_KT 32
-#define LAT_VS 36                                  // LDS stride of a transposed column (32 keys + 4)
+// Block = one row, HT tiles of 16 heads (four waves each), one share of the row's keys, walked in tiles of 64.  A key is read ONCE: each thread
+// fetches 4 keys x 8 columns, writes them to LDS as key rows (score operand) and, transposed in registers, as column rows (value operand);
+// the next tile's loads are in flight during the rest (barriers wait for LDS only).  Wave w of a head tile scores keys 16 w .. + 15
+// (S^T = K q^T, the whole query in registers), the four maxima meet in LDS, each wave turns ITS scores into weights and leaves them as bf16
+// hi + lo; every wave then multiplies all 64 weights with its own quarter of the latent columns.  A share leaves its normalised sums as bf16
+// and its (max, sum); k_latent_share_values weights the shares.
+#define LAT_KT 32                                  // key tile of the prompt kernel
+#define LAT_VS 36                                  // its LDS stride of a transposed column (32 keys + 4)
+#define LAD_KT 64                                  // key tile of the decode kernel
+#define LAD_VS 68
+#define LAD_PS 72                                  // LDS stride of a head's weights
 __device__ __forceinline__ void lds_barrier() { asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory"); }
 __device__ __forceinline__ bf16x8_t lds_frag(const bf16_t* p) {       // 8 values, 8-byte aligned
     union { uint2 u[2]; bf16x8_t v; } r;
@@ -521,125 +525,137 @@ __device__ __forceinline__ uint2 column_of(const uint4 (&r)[4], int e) {
     const uint32_t a[4] = {r[0].x, r[0].y, r[0].z, r[0].w}, b[4] = {r[1].x, r[1].y, r[1].z, r[1].w}, c[4] = {r[2].x, r[2].y, r[2].z, r[2].w},
                    d[4] = {r[3].x, r[3].y, r[3].z, r[3].w};
     const int w = e >> 1;
-    if (e & 1) return make_uint2((a[w] >> 16) | (b[w] & 0xffff0000u), (c[w] >> 16) | (d[w] & 0xffff0000u));
-    return make_uint2((a[w] & 0xffffu) | (b[w] << 16), (c[w] & 0xffffu) | (d[w] << 16));
+    const uint32_t sel = (e & 1) ? 0x07060302u : 0x05040100u;        // v_perm: high / low halves of two words
+    return make_uint2(__builtin_amdgcn_perm(b[w], a[w], sel), __builtin_amdgcn_perm(d[w], c[w], sel));
 }
 static size_t latent_decode_lds(const LatentDims& D, int HT) {
-    return (size_t)LAT_KT * (D.CW + 8) * 2 + (size_t)D.Rp * LAT_VS * 2 + (size_t)HT * 2 * 16 * 36 * 4;
+    return (size_t)LAD_KT * (D.CW + 8) * 2 + (size_t)D.Rp * LAD_VS * 2 + (size_t)HT * (2 * 16 * LAD_PS * 2 + 4 * 16 * 4);
 }
-// NTW: latent tiles per wave (Rp / 64 <= NTW); NST: staging rounds (CW <= 256 HT NST); QF: query fragments per wave (CW / 32 <= 2 QF)
+// NTW: latent tiles per wave (Rp / 64 <= NTW); NST: staging rounds (CW <= 128 HT NST); QF: query fragments (CW / 32 <= QF)
 template <int NTW, int NST, int QF, int HT>
-__global__ void __launch_bounds__(256 * HT, 2) k_latent_attn_decode(LatentDims D, LatentAttn p, LatentShares sh, int rows) {
+__global__ void __launch_bounds__(256 * HT, HT) k_latent_attn_decode(LatentDims D, LatentAttn p, LatentShares sh, int rows) {
     extern __shared__ __attribute__((aligned(16))) uint8_t lds[];
     const int KS = D.CW + 8;
-    bf16_t* sk = reinterpret_cast<bf16_t*>(lds);                                // [32][CW + 8]
-    bf16_t* sv = sk + (size_t)LAT_KT * KS;                                      // [Rp][LAT_VS]
+    bf16_t* sk = reinterpret_cast<bf16_t*>(lds);                                // [64][CW + 8]
+    bf16_t* sv = sk + (size_t)LAD_KT * KS;                                      // [Rp][LAD_VS]
     const int tid = threadIdx.x, lane = tid & 63, wave = (tid >> 6) & 3, ht = tid >> 8, li = lane & 15, lq = lane >> 4;
-    float* sc = reinterpret_cast<float*>(sv + (size_t)D.Rp * LAT_VS) + (size_t)ht * 2 * 16 * 36;        // [2][16][36]
+    bf16_t* sw = sv + (size_t)D.Rp * LAD_VS + (size_t)ht * 2 * 16 * LAD_PS;     // [hi, lo][16 heads][LAD_PS]
+    float* smx = reinterpret_cast<float*>(sv + (size_t)D.Rp * LAD_VS + (size_t)HT * 2 * 16 * LAD_PS) + ht * 64;      // [4 waves][16 heads]
     const int m = blockIdx.x / sh.S, sp = blockIdx.x - m * sh.S, h0 = (blockIdx.y * HT + ht) * 16;
     const bool on = !p.rows.on || p.rows.on[m];
-    const int pos = on ? p.rows.pos[m] : 0, seq = p.rows.seq ? p.rows.seq[m] : m;
+    const int pos = p.rows.pos[m], seq = p.rows.seq ? p.rows.seq[m] : m;
     const int lo = D.window > 0 ? max(0, pos - D.window + 1) : 0;
-    const int nt = on ? (pos - lo + LAT_KT) / LAT_KT : 0;
-    const int t0 = (int)((long long)nt * sp / sh.S), t1 = (int)((long long)nt * (sp + 1) / sh.S);
+    const int nk = pos - lo + 1, per = ((nk + sh.S - 1) / sh.S + 3) & ~3;
+    const int k0 = lo + sp * per, k1 = on ? min(k0 + per, pos + 1) : k0;        // this share's keys
     const bf16_t* cache = (const bf16_t*)p.cache + (size_t)seq * p.Smax * D.CW;
     const int nch = D.CW >> 3, CT = D.CW >> 5;
-    const int kg = tid & 7;                                                     // four keys 4 kg .. of the tile; eight lanes share a 16-byte column chunk
+    const int kg = tid & 15;                                                    // four keys 4 kg .. of the tile; sixteen lanes share a 16-byte column chunk
     uint4 st[NST][4];
     auto fetch = [&](int t) {
+        const bf16_t* kr[4];
+#pragma unroll
+        for (int k = 0; k < 4; ++k) kr[k] = cache + (size_t)min(t + 4 * kg + k, k1 - 1) * D.CW;
 #pragma unroll
         for (int i = 0; i < NST; ++i) {
-            const int chunk = min((tid >> 3) + 32 * HT * i, nch - 1);           // (rounds past the row read its last chunk and are not stored)
+            const int chunk = min((tid >> 4) + 16 * HT * i, nch - 1);           // (rounds past the row read its last chunk and are not stored)
 #pragma unroll
-            for (int k = 0; k < 4; ++k) {
-                const int key = min(lo + t * LAT_KT + 4 * kg + k, pos);
-                st[i][k] = *reinterpret_cast<const uint4*>(cache + (size_t)key * D.CW + chunk * 8);
-            }
+            for (int k = 0; k < 4; ++k) st[i][k] = *reinterpret_cast<const uint4*>(kr[k] + chunk * 8);
         }
     };
-    if (t0 < t1) fetch(t0);
-    // this wave's half of the query columns: heads past H read head H - 1 and are dropped at the end
-    const int half = wave >> 1, kt0 = half ? (CT + 1) / 2 : 0, kt1 = half ? CT : (CT + 1) / 2;
-    bf16x8_t qf[QF];
+    if (k0 < k1) fetch(k0);
+    bf16x8_t qf[QF];                                                            // heads past H read head H - 1 and are dropped at the end
     {
         const bf16_t* q = (const bf16_t*)p.q + ((size_t)m * D.H + min(h0 + li, D.H - 1)) * D.CW + lq * 8;
 #pragma unroll
-        for (int i = 0; i < QF; ++i) qf[i] = *reinterpret_cast<const bf16x8_t*>(q + min(kt0 + i, CT - 1) * 32);
+        for (int i = 0; i < QF; ++i) qf[i] = *reinterpret_cast<const bf16x8_t*>(q + min(i, CT - 1) * 32);
     }
     f32x4_t o[NTW];
 #pragma unroll
     for (int i = 0; i < NTW; ++i) o[i] = (f32x4_t){0.f, 0.f, 0.f, 0.f};
     float mx = -INFINITY, ls = 0.0f;                                            // of head li; ls: this lane's keys only
-    for (int t = t0; t < t1; ++t) {
+    for (int t = k0; t < k1; t += LAD_KT) {
 #pragma unroll
         for (int i = 0; i < NST; ++i) {
-            const int chunk = (tid >> 3) + 32 * HT * i;
+            const int chunk = (tid >> 4) + 16 * HT * i;
             if (chunk < nch) {
 #pragma unroll
                 for (int k = 0; k < 4; ++k) *reinterpret_cast<uint4*>(sk + (size_t)(4 * kg + k) * KS + chunk * 8) = st[i][k];
                 if (chunk * 8 < D.Rp) {
 #pragma unroll
-                    for (int e = 0; e < 8; ++e) *reinterpret_cast<uint2*>(sv + (size_t)(chunk * 8 + e) * LAT_VS + 4 * kg) = column_of(st[i], e);
+                    for (int e = 0; e < 8; ++e) *reinterpret_cast<uint2*>(sv + (size_t)(chunk * 8 + e) * LAD_VS + 4 * kg) = column_of(st[i], e);
                 }
             }
         }
-        if (t + 1 < t1) fetch(t + 1);
+        if (t + LAD_KT < k1) fetch(t + LAD_KT);
         lds_barrier();
-        f32x4_t s = (f32x4_t){0.f, 0.f, 0.f, 0.f};
+        float w[4], tm = -INFINITY;
         {
-            const bf16_t* kr = sk + (size_t)((wave & 1) * 16 + li) * KS + lq * 8;
+            f32x4_t s0 = (f32x4_t){0.f, 0.f, 0.f, 0.f}, s1 = s0;
+            if (t + wave * 16 < k1) {                                           // wave-uniform
+                const bf16_t* kr = sk + (size_t)(wave * 16 + li) * KS + lq * 8;
 #pragma unroll
-            for (int i = 0; i < QF; ++i)
-                if (kt0 + i < kt1) s = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*reinterpret_cast<const bf16x8_t*>(kr + (kt0 + i) * 32), qf[i], s, 0, 0, 0);
-        }
-        *reinterpret_cast<float4*>(sc + ((size_t)half * 16 + li) * 36 + (wave & 1) * 16 + lq * 4) = make_float4(s[0], s[1], s[2], s[3]);
-        lds_barrier();
-        float w[8];
-        {
-            const float *a = sc + (size_t)li * 36 + lq * 8, *b = a + 16 * 36;
-            float tm = -INFINITY;
+                for (int i = 0; i < QF; i += 2) {
+                    if (i < CT) s0 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*reinterpret_cast<const bf16x8_t*>(kr + i * 32), qf[i], s0, 0, 0, 0);
+                    if (i + 1 < QF && i + 1 < CT) s1 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*reinterpret_cast<const bf16x8_t*>(kr + (i + 1) * 32), qf[i + 1 < QF ? i + 1 : i], s1, 0, 0, 0);
+                }
+            }
 #pragma unroll
-            for (int e = 0; e < 8; ++e) {
-                w[e] = (a[e] + b[e]) * D.scale;
-                if (lo + t * LAT_KT + lq * 8 + e > pos) w[e] = -INFINITY;
+            for (int e = 0; e < 4; ++e) {
+                w[e] = t + wave * 16 + lq * 4 + e < k1 ? (s0[e] + s1[e]) * D.scale : -INFINITY;
                 tm = fmaxf(tm, w[e]);
             }
-            tm = fmaxf(tm, __shfl_xor(tm, 16, 64));
-            tm = fmaxf(tm, __shfl_xor(tm, 32, 64));
-            const float mn = fmaxf(mx, tm), alpha = __expf(mx - mn);
+        }
+        tm = fmaxf(tm, __shfl_xor(tm, 16, 64));
+        tm = fmaxf(tm, __shfl_xor(tm, 32, 64));
+        if (lq == 0) smx[wave * 16 + li] = tm;
+        lds_barrier();
+        const float mn = fmaxf(mx, fmaxf(fmaxf(smx[li], smx[16 + li]), fmaxf(smx[32 + li], smx[48 + li]))), alpha = __expf(mx - mn);
+        mx = mn;
+        {
             float add = 0.0f;
+            uint16_t hi[4], lw[4];
 #pragma unroll
-            for (int e = 0; e < 8; ++e) { w[e] = __expf(w[e] - mn); add += w[e]; }
+            for (int e = 0; e < 4; ++e) {
+                w[e] = __expf(w[e] - mn);
+                add += w[e];
+                hi[e] = f32_to_bf16(w[e]);
+                lw[e] = f32_to_bf16(w[e] - bf16_to_f32(hi[e]));
+            }
             ls = ls * alpha + add;
-            mx = mn;
-            if (t > t0) {                                                       // (the first tile has nothing to rescale)
+            bf16_t* pw = sw + (size_t)li * LAD_PS + wave * 16 + lq * 4;
+            *reinterpret_cast<uint2*>(pw) = make_uint2((uint32_t)hi[0] | ((uint32_t)hi[1] << 16), (uint32_t)hi[2] | ((uint32_t)hi[3] << 16));
+            *reinterpret_cast<uint2*>(pw + 16 * LAD_PS) = make_uint2((uint32_t)lw[0] | ((uint32_t)lw[1] << 16), (uint32_t)lw[2] | ((uint32_t)lw[3] << 16));
+        }
+        if (t > k0 && __any(alpha != 1.0f)) {                                   // (the first tile has nothing to rescale)
 #pragma unroll
-                for (int e = 0; e < 4; ++e) {
-                    const float ah = __shfl(alpha, lq * 4 + e, 64);             // head of accumulator row e
+            for (int e = 0; e < 4; ++e) {
+                const float ah = __shfl(alpha, lq * 4 + e, 64);                 // head of accumulator row e
 #pragma unroll
-                    for (int i = 0; i < NTW; ++i) o[i][e] *= ah;
-                }
+                for (int i = 0; i < NTW; ++i) o[i][e] *= ah;
             }
         }
-        bf16x8_t ph, pl;
+        lds_barrier();
 #pragma unroll
-        for (int e = 0; e < 8; ++e) {
-            const bf16_t hi = f32_to_bf16(w[e]);
-            ph[e] = (short)hi;
-            pl[e] = (short)f32_to_bf16(w[e] - bf16_to_f32(hi));
-        }
+        for (int ks = 0; ks < 2; ++ks) {
+            if (t + 32 * ks >= k1) continue;                                    // uniform
+            const bf16x8_t ph = *reinterpret_cast<const bf16x8_t*>(sw + (size_t)li * LAD_PS + ks * 32 + lq * 8),
+                           pl = *reinterpret_cast<const bf16x8_t*>(sw + (size_t)(16 + li) * LAD_PS + ks * 32 + lq * 8);
 #pragma unroll
-        for (int i = 0; i < NTW; ++i) {
-            const int tile = i * 4 + wave;
-            if (tile * 16 >= D.Rp) continue;                                    // wave-uniform
-            const bf16x8_t v = lds_frag(sv + (size_t)(tile * 16 + li) * LAT_VS + lq * 8);
-            o[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(ph, v, o[i], 0, 0, 0);
-            o[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(pl, v, o[i], 0, 0, 0);
+            for (int i = 0; i < NTW; ++i) {
+                const int tile = i * 4 + wave;
+                if (tile * 16 >= D.Rp) continue;                                // wave-uniform
+                const bf16x8_t v = lds_frag(sv + (size_t)(tile * 16 + li) * LAD_VS + ks * 32 + lq * 8);
+                o[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(ph, v, o[i], 0, 0, 0);
+                o[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(pl, v, o[i], 0, 0, 0);
+            }
         }
-        lds_barrier();                                                          // everyone is done with sk / sv / sc
+        lds_barrier();                                                          // everyone is done with the tile
     }
     ls += __shfl_xor(ls, 16, 64);
     ls += __shfl_xor(ls, 32, 64);
+    if (lq == 0) smx[wave * 16 + li] = ls;
+    lds_barrier();
+    ls = (smx[li] + smx[16 + li]) + (smx[32 + li] + smx[48 + li]);
     if (wave == 0 && lq == 0 && h0 + li < D.H) {
         float* ml = sh.ml + (((size_t)sp * rows + m) * D.H + h0 + li) * 2;
         *reinterpret_cast<float2*>(ml) = make_float2(mx, ls);
@@ -665,85 +681,75 @@ __global__ void __launch_bounds__(256 * HT, 2) k_latent_attn_decode(LatentDims D
     }
 }
 
-// One block of 16 waves per (head, 16 rows): weights of the shares -> latent sums of the rows (bf16, LDS) -> values.  Wave = (value tile, part of the
-// latent columns); its weight fragments are requested before the shares are read.
-// KF: k-tiles per wave at most; above 8 (value dimensions past 128) the fragments are requested behind the shares (registers).
-template <int KF>
-__global__ void __launch_bounds__(1024) k_latent_share_values(LatentDims D, LatentShares sh, const bf16_t* __restrict__ uv, size_t uvz, Operand out, int rows) {
+// One block of 8 waves per (head, 8 rows): weights of the shares -> latent sums of the rows (bf16, LDS) -> values.  A wave owns every eighth value
+// tile; its weight fragments are requested before the shares are read.
+#define LSV_KF 16                                  // k-tiles (Rp <= 512)
+#define LSV_ROWS 8
+__global__ void __launch_bounds__(512) k_latent_share_values(LatentDims D, LatentShares sh, const bf16_t* __restrict__ uv, size_t uvz, Operand out, int rows) {
     extern __shared__ __attribute__((aligned(16))) uint8_t lds[];
-    bf16_t* so = reinterpret_cast<bf16_t*>(lds);                                // [16][Rp + 8]
-    float4* red = reinterpret_cast<float4*>(lds + (size_t)16 * (D.Rp + 8) * 2); // [16][64]
-    const int hd = blockIdx.x, m0 = blockIdx.y * 16, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, li = lane & 15, lq = lane >> 4;
-    const int vt = D.vp >> 4, KT = D.Rp >> 5, KH = vt <= 4 ? 4 : vt <= 8 ? 2 : 1;
-    const int tile = wave / KH, kh = wave - tile * KH, kt0 = KT * kh / KH, kn = KT * (kh + 1) / KH - kt0;
-    constexpr bool early = KF <= 8;
-    bf16x8_t wf[KF];
+    bf16_t* so = reinterpret_cast<bf16_t*>(lds);                                // [LSV_ROWS][Rp + 8]
+    const int hd = blockIdx.x, m0 = blockIdx.y * LSV_ROWS, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, li = lane & 15, lq = lane >> 4;
+    const int vt = D.vp >> 4, KT = D.Rp >> 5;
+    bf16x8_t wf[LSV_KF];
     auto request = [&](int t) {
-        const bf16_t* wp = uv + uvz * hd + ((size_t)min(t, vt - 1) * KT + kt0) * 512 + lane * 8;
+        const bf16_t* wp = uv + uvz * hd + (size_t)min(t, vt - 1) * KT * 512 + lane * 8;
 #pragma unroll
-        for (int i = 0; i < KF; ++i) wf[i] = *reinterpret_cast<const bf16x8_t*>(wp + (size_t)min(i, kn - 1) * 512);
+        for (int i = 0; i < LSV_KF; ++i) wf[i] = *reinterpret_cast<const bf16x8_t*>(wp + (size_t)min(i, KT - 1) * 512);
     };
-    if constexpr (early) request(tile);
+    request(wave);
     const int rc = D.Rp >> 3;
-    for (int t = tid; t < 16 * rc; t += 1024) {
-        const int r = t / rc, c = t - r * rc, m = min(m0 + r, rows - 1);
-        const float2* ml = reinterpret_cast<const float2*>(sh.ml) + (size_t)m * D.H + hd;
-        const bf16_t* pp = sh.part + ((size_t)m * D.H + hd) * D.Rp + c * 8;
-        const size_t ss = (size_t)rows * D.H;
-        float a[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f}, l = 0.0f, mx = -INFINITY;
-        for (int s0 = 0; s0 < sh.S; s0 += 8) {
-            float2 q[8];
-            bf16x8_t v[8];
+    for (int t = tid; t < LSV_ROWS * rc; t += 512) {
+        const int r = t / rc, c = t - r * rc, m = m0 + r;
+        bf16x8_t o = {0, 0, 0, 0, 0, 0, 0, 0};
+        if (m < rows) {
+            const float2* ml = reinterpret_cast<const float2*>(sh.ml) + (size_t)m * D.H + hd;
+            const bf16_t* pp = sh.part + ((size_t)m * D.H + hd) * D.Rp + c * 8;
+            const size_t ss = (size_t)rows * D.H;
+            float a[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f}, l = 0.0f, mx = -INFINITY;
+            for (int s0 = 0; s0 < sh.S; s0 += 8) {
+                float2 q[8];
+                bf16x8_t v[8];
 #pragma unroll
-            for (int u = 0; u < 8; ++u) {
-                const int s = min(s0 + u, sh.S - 1);
-                q[u] = ml[ss * s];
-                v[u] = *reinterpret_cast<const bf16x8_t*>(pp + ss * s * D.Rp);
+                for (int u = 0; u < 8; ++u) {
+                    const int s = min(s0 + u, sh.S - 1);
+                    q[u] = ml[ss * s];
+                    v[u] = *reinterpret_cast<const bf16x8_t*>(pp + ss * s * D.Rp);
+                }
+                float mn = mx;
+#pragma unroll
+                for (int u = 0; u < 8; ++u) mn = fmaxf(mn, (s0 + u < sh.S && q[u].y > 0.0f) ? q[u].x : -INFINITY);        // (an empty share holds sum 0)
+                const float alpha = mx == -INFINITY ? 0.0f : __expf(mx - mn);
+                l *= alpha;
+#pragma unroll
+                for (int e = 0; e < 8; ++e) a[e] *= alpha;
+#pragma unroll
+                for (int u = 0; u < 8; ++u) {
+                    const float w = (s0 + u < sh.S && q[u].y > 0.0f) ? __expf(q[u].x - mn) * q[u].y : 0.0f;
+                    l += w;
+#pragma unroll
+                    for (int e = 0; e < 8; ++e) a[e] += w * bf16_to_f32((bf16_t)v[u][e]);
+                }
+                mx = mn;
             }
-            float mn = mx;
+            const float inv = l > 0.0f ? 1.0f / l : 0.0f;
 #pragma unroll
-            for (int u = 0; u < 8; ++u) mn = fmaxf(mn, (s0 + u < sh.S && q[u].y > 0.0f) ? q[u].x : -INFINITY);        // (an empty share holds sum 0)
-            const float alpha = mx == -INFINITY ? 0.0f : __expf(mx - mn);
-            l *= alpha;
-#pragma unroll
-            for (int e = 0; e < 8; ++e) a[e] *= alpha;
-#pragma unroll
-            for (int u = 0; u < 8; ++u) {
-                const float w = (s0 + u < sh.S && q[u].y > 0.0f) ? __expf(q[u].x - mn) * q[u].y : 0.0f;
-                l += w;
-#pragma unroll
-                for (int e = 0; e < 8; ++e) a[e] += w * bf16_to_f32((bf16_t)v[u][e]);
-            }
-            mx = mn;
+            for (int e = 0; e < 8; ++e) o[e] = (short)f32_to_bf16(a[e] * inv);
         }
-        const float inv = l > 0.0f ? 1.0f / l : 0.0f;
-        bf16x8_t o;
-#pragma unroll
-        for (int e = 0; e < 8; ++e) o[e] = (short)f32_to_bf16(a[e] * inv);
         *reinterpret_cast<bf16x8_t*>(so + (size_t)r * (D.Rp + 8) + c * 8) = o;
     }
     __syncthreads();
-    for (int t0 = 0; t0 < vt; t0 += 16 / KH) {
-        const int vtile = t0 + tile;
-        f32x4_t acc = (f32x4_t){0.f, 0.f, 0.f, 0.f};
-        if (vtile < vt) {
-            if (!early || t0 > 0) request(vtile);                               // (more value tiles than one round of waves)
+    for (int vtile = wave; vtile < vt; vtile += 8) {                            // (no barrier inside)
+        if (vtile >= 8) request(vtile);
+        f32x4_t a0 = (f32x4_t){0.f, 0.f, 0.f, 0.f}, a1 = a0;
+        const bf16_t* xr = so + (size_t)(li & (LSV_ROWS - 1)) * (D.Rp + 8) + lq * 8;       // columns 8 .. 15 of the product repeat the rows, unused
 #pragma unroll
-            for (int i = 0; i < KF; ++i)
-                if (i < kn)
-                    acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wf[i], *reinterpret_cast<const bf16x8_t*>(so + (size_t)li * (D.Rp + 8) + (kt0 + i) * 32 + lq * 8), acc, 0, 0, 0);
-        }
-        if (KH > 1) {
-            red[wave * 64 + lane] = make_float4(acc[0], acc[1], acc[2], acc[3]);
-            __syncthreads();
+        for (int i = 0; i < LSV_KF; i += 2) {
+            if (i < KT) a0 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wf[i], *reinterpret_cast<const bf16x8_t*>(xr + i * 32), a0, 0, 0, 0);
+            if (i + 1 < KT) a1 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wf[i + 1], *reinterpret_cast<const bf16x8_t*>(xr + (i + 1) * 32), a1, 0, 0, 0);
         }
         const int m = m0 + li, c = vtile * 16 + lq * 4;
-        if (kh == 0 && vtile < vt && m < rows) {
-            float v[4] = {acc[0], acc[1], acc[2], acc[3]};
-            for (int k = 1; k < KH; ++k) {
-                const float4 t = red[(wave + k) * 64 + lane];
-                v[0] += t.x; v[1] += t.y; v[2] += t.z; v[3] += t.w;
-            }
+        if (li < LSV_ROWS && m < rows) {
+            const float v[4] = {a0[0] + a1[0], a0[1] + a1[1], a0[2] + a1[2], a0[3] + a1[3]};
             if (D.v % 4 == 0) {
                 if (c < D.v) operand_store4(out, m, hd * D.v + c, v);
             } else {
@@ -751,7 +757,6 @@ __global__ void __launch_bounds__(1024) k_latent_share_values(LatentDims D, Late
                 for (int e = 0; e < 4; ++e) if (c + e < D.v) operand_store1(out, m, hd * D.v + c + e, v[e]);
             }
         }
-        if (KH > 1 && t0 + 16 / KH < vt) __syncthreads();
     }
 }
 
@@ -761,13 +766,15 @@ void launch_latent_attn_any(const LatentDims& D, const LatentAttn& p, int rows, 
     if (p.f32) hipLaunchKernelGGL((k_latent_attn_any<float>), dim3(rows, D.H), dim3(256), sm, s, D, p);
     else hipLaunchKernelGGL((k_latent_attn_any<bf16_t>), dim3(rows, D.H), dim3(256), sm, s, D, p);
 }
-bool latent_decode_mfma_ok(const LatentDims& D) { return D.Rp <= 512 && D.CW <= (D.Rp <= 128 ? 256 : D.Rp <= 256 ? 512 : 768) && D.vp <= 256; }
-// shares per row: about one block per compute unit, one key tile each at least
+bool latent_decode_mfma_ok(const LatentDims& D) {
+    return D.Rp <= 512 && D.CW <= (D.Rp <= 128 ? 256 : D.Rp <= 256 ? 512 : 640) && latent_decode_lds(D, D.H > 16 ? 2 : 1) <= 160 * 1024;
+}
+// shares per row: at most one block per compute unit (a block fills one), at least 32 keys each
 int latent_decode_shares(const LatentDims& D, int rows, int Smax) {
     const char* e = getenv("MIS_LATENT_SHARES");                                // A/B
-    const int keys = D.window > 0 ? std::min(D.window, Smax) : Smax, tiles = cdiv(keys, LAT_KT), blocks = rows * cdiv(D.H, D.H > 16 ? 32 : 16);
-    const int want = e && atoi(e) > 0 ? atoi(e) : cdiv(256, blocks);
-    return std::max(1, std::min(std::min(want, tiles), 32));
+    const int keys = D.window > 0 ? std::min(D.window, Smax) : Smax, blocks = rows * cdiv(D.H, D.H > 16 ? 32 : 16);
+    const int want = e && atoi(e) > 0 ? atoi(e) : std::max(1, 256 / blocks);
+    return std::max(1, std::min(std::min(want, cdiv(keys, 32)), 32));
 }
 void launch_latent_attn_decode(const LatentDims& D, const LatentAttn& p, const LatentShares& sh, int rows, hipStream_t s) {
     MIS_REQUIRE(p.rows.pos && p.q && p.cache && sh.part && sh.ml && sh.S >= 1 && rows >= 1 && !p.f32 && latent_decode_mfma_ok(D), MIS_ERR_GENERATION_FAILED,
@@ -781,17 +788,14 @@ void launch_latent_attn_decode(const LatentDims& D, const LatentAttn& p, const L
         HIP_CHECK(attr);                                                                                                                                        \
         hipLaunchKernelGGL((k_latent_attn_decode<A, B, C, T>), grid, dim3(256 * T), sm, s, D, p, sh, rows);                                                     \
     } while (0)
-    if (D.Rp <= 128) { if (HT == 1) LAT_GO(2, 1, 4, 1); else LAT_GO(2, 1, 4, 2); }
-    else if (D.Rp <= 256) { if (HT == 1) LAT_GO(4, 2, 8, 1); else LAT_GO(4, 1, 8, 2); }
-    else { if (HT == 1) LAT_GO(8, 3, 12, 1); else LAT_GO(8, 2, 12, 2); }
+    if (D.Rp <= 128) { if (HT == 1) LAT_GO(2, 2, 8, 1); else LAT_GO(2, 1, 8, 2); }
+    else if (D.Rp <= 256) { if (HT == 1) LAT_GO(4, 4, 16, 1); else LAT_GO(4, 2, 16, 2); }
+    else { if (HT == 1) LAT_GO(8, 5, 20, 1); else LAT_GO(8, 3, 20, 2); }
 #undef LAT_GO
 }
 void launch_latent_share_values(const LatentDims& D, const LatentShares& sh, const bf16_t* uv, size_t uvz, const Operand& out, int rows, hipStream_t s) {
-    const size_t sm = (size_t)16 * (D.Rp + 8) * 2 + 16 * 64 * 16;
-    const int vt = D.vp / 16, KH = vt <= 4 ? 4 : vt <= 8 ? 2 : 1;               // as in the kernel
-    const dim3 grid(D.H, cdiv(rows, 16));
-    if (cdiv(D.Rp / 32, KH) <= 8) hipLaunchKernelGGL((k_latent_share_values<8>), grid, dim3(1024), sm, s, D, sh, uv, uvz, out, rows);
-    else hipLaunchKernelGGL((k_latent_share_values<16>), grid, dim3(1024), sm, s, D, sh, uv, uvz, out, rows);
+    MIS_REQUIRE(D.Rp <= 32 * LSV_KF, MIS_ERR_GENERATION_FAILED, "latent values: latent size above 512");
+    hipLaunchKernelGGL(k_latent_share_values, dim3(D.H, cdiv(rows, LSV_ROWS)), dim3(512), (size_t)LSV_ROWS * (D.Rp + 8) * 2, s, D, sh, uv, uvz, out, rows);
 }
 
 // ============================================================================ expanded attention on the matrix cores (prompts)
