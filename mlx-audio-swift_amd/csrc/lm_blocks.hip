@@ -364,7 +364,7 @@ void LmBlocks::step_layer(int li, const BlockRows& r, hipStream_t s) {
         const int NT = (l.Nqkv + l.ffp) / 16;
         const bool wide = Mpad_ <= 32 && NT / 4 >= 192;                        // four n-tiles per wave where the launch still fills the chip
         GemmExtra ex; ex.out2 = act_.p; ex.split = l.Nqkv / 16;
-        launch_gemm_skinny(EPI_SPLIT_RELU2, wide ? 4 : 2, 4, w.w1.p, (const bf16_t*)h_.p, qkv_.p, NT, dp / 32, 1, l.Nqkv, Mpad_, s, nullptr, 0, ex);
+        launch_gemm_skinny(EPI_SPLIT_RELU2, wide ? 4 : 2, wide ? 2 : 4, w.w1.p, (const bf16_t*)h_.p, qkv_.p, NT, dp / 32, 1, l.Nqkv, Mpad_, s, nullptr, wide ? 2 : 4, ex);
     }
     absorbed_attention(li, qkv_.p, q_.p, olat_.p, operand(at, l.Ko, Mpad_, true), rows, batch_, l.shares, s);
     const size_t slab = (size_t)Mpad_ * dp;
@@ -373,7 +373,7 @@ void LmBlocks::step_layer(int li, const BlockRows& r, hipStream_t s) {
         if (l.ffp) launch_gemm_f32(gemm32(act_.p, l.ffp, w.wdown.p, part_.p + slab, dp, batch_, dp, l.ffp, F32_STORE), s);
     } else if (l.ffp) {
         GemmExtra ex; ex.w2 = w.wdown.p; ex.x2 = (const bf16_t*)act_.p; ex.kt2 = l.ffp / 32; ex.s1 = l.s1;
-        launch_gemm_skinny(EPI_DUAL, 2, 4, w.wo.p, (const bf16_t*)at, part_.p, dp / 16, l.Ko / 32, l.s1 + l.s2, dp, Mpad_, s, nullptr, 0, ex);
+        launch_gemm_skinny(EPI_DUAL, 2, l.ffp / 32 >= 64 ? 2 : 4, w.wo.p, (const bf16_t*)at, part_.p, dp / 16, l.Ko / 32, l.s1 + l.s2, dp, Mpad_, s, nullptr, 0, ex);
     } else launch_gemm_skinny(EPI_PARTIAL, 2, 4, w.wo.p, (const bf16_t*)at, part_.p, dp / 16, l.Ko / 32, l.s1, dp, Mpad_, s);
     const ScaledSlabs sl{part_.p, l.s1, l.s2, w.ls1.p, w.ls2.p};
     launch_scaled_residual_norm(sl, Mpad_, x_.p, norm_after(li), operand(h_.p, dp, Mpad_, true), d, dp, spec.eps, f32 ? batch_ : Mpad_, s);

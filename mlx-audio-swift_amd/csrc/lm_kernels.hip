@@ -921,10 +921,9 @@ static void launch_gemm_mt(int epi, int R, int ksb, int U, const bf16_t* Wp, con
         GEMM_CASE(EPI_BF16, 4, 4, 3)
         GEMM_CASE(EPI_BF16, 4, 4, 2)
         GEMM_CASE(EPI_BF16, 4, 2, 3)
-        GEMM_CASE(EPI_SPLIT_RELU2, 4, 4, 3)
+        GEMM_CASE(EPI_SPLIT_RELU2, 4, 2, 2)
         GEMM_CASE(EPI_SOFTCAP, 4, 4, 3)
     }
-    if constexpr (MT <= 2) { GEMM_CASE(EPI_DUAL, 4, 4, 2) GEMM_CASE(EPI_DUAL, 4, 2, 2) }
     GEMM_CASE(EPI_DUAL, 2, 4, 4)
     GEMM_CASE(EPI_DUAL, 2, 2, 4)
     GEMM_CASE(EPI_SPLIT_RELU2, 2, 4, 4)

@@ -503,30 +503,25 @@ __global__ void __launch_bounds__(256) k_latent_attn_any(LatentDims D, LatentAtt
 
 // ============================================================================ absorbed attention on the matrix cores (decode)
 // Block = one row, HT tiles of 16 heads (four waves each), one share of the row's keys, walked in tiles of 64.  A key is read ONCE: each thread
-// fetches 4 keys x 8 columns, writes them to LDS as key rows (score operand) and, transposed in registers, as column rows (value operand);
-// the next tile's loads are in flight during the rest (barriers wait for LDS only).  Wave w of a head tile scores keys 16 w .. + 15
+// fetches 4 keys (kg, kg + 16, kg + 32, kg + 48) x 8 columns, writes them to LDS as key rows (score operand) and, transposed in registers, as
+// column rows (value operand; key kg + 16 k at place 4 kg + k); the next tile's loads are in flight during the rest (barriers wait for LDS
+// only).  The queries come through LDS too: a wave needs a head tile's whole query, four times what the block has to fetch.  Wave w of a head tile scores keys 16 w .. + 15
 // (S^T = K q^T, the whole query in registers), the four maxima meet in LDS, each wave turns ITS scores into weights and leaves them as bf16
 // hi + lo; every wave then multiplies all 64 weights with its own quarter of the latent columns.  A share leaves its normalised sums as bf16
 // and its (max, sum); k_latent_share_values weights the shares.
 #define LAT_KT 32                                  // key tile of the prompt kernel
-#define LAT_VS 36                                  // its LDS stride of a transposed column (32 keys + 4)
+#define LAT_VS 40                                  // its LDS stride of a transposed column (32 keys + 8)
 #define LAD_KT 64                                  // key tile of the decode kernel
-#define LAD_VS 68
+#define LAD_VS 72
 #define LAD_PS 72                                  // LDS stride of a head's weights
 __device__ __forceinline__ void lds_barrier() { asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory"); }
-__device__ __forceinline__ bf16x8_t lds_frag(const bf16_t* p) {       // 8 values, 8-byte aligned
-    union { uint2 u[2]; bf16x8_t v; } r;
-    r.u[0] = reinterpret_cast<const uint2*>(p)[0];
-    r.u[1] = reinterpret_cast<const uint2*>(p)[1];
-    return r.v;
-}
+__device__ __forceinline__ bf16x8_t lds_frag(const bf16_t* p) { return *reinterpret_cast<const bf16x8_t*>(p); }
 // 4 keys x 8 columns -> column e: the four keys packed
-__device__ __forceinline__ uint2 column_of(const uint4 (&r)[4], int e) {
-    const uint32_t a[4] = {r[0].x, r[0].y, r[0].z, r[0].w}, b[4] = {r[1].x, r[1].y, r[1].z, r[1].w}, c[4] = {r[2].x, r[2].y, r[2].z, r[2].w},
-                   d[4] = {r[3].x, r[3].y, r[3].z, r[3].w};
+typedef uint32_t u32x4_t __attribute__((ext_vector_type(4)));
+__device__ __forceinline__ uint2 column_of(const u32x4_t (&r)[4], int e) {
     const int w = e >> 1;
     const uint32_t sel = (e & 1) ? 0x07060302u : 0x05040100u;        // v_perm: high / low halves of two words
-    return make_uint2(__builtin_amdgcn_perm(b[w], a[w], sel), __builtin_amdgcn_perm(d[w], c[w], sel));
+    return make_uint2(__builtin_amdgcn_perm(r[1][w], r[0][w], sel), __builtin_amdgcn_perm(r[3][w], r[2][w], sel));
 }
 static size_t latent_decode_lds(const LatentDims& D, int HT) {
     return (size_t)LAD_KT * (D.CW + 8) * 2 + (size_t)D.Rp * LAD_VS * 2 + (size_t)HT * (2 * 16 * LAD_PS * 2 + 4 * 16 * 4);
@@ -541,67 +536,91 @@ __global__ void __launch_bounds__(256 * HT, HT) k_latent_attn_decode(LatentDims 
     const int tid = threadIdx.x, lane = tid & 63, wave = (tid >> 6) & 3, ht = tid >> 8, li = lane & 15, lq = lane >> 4;
     bf16_t* sw = sv + (size_t)D.Rp * LAD_VS + (size_t)ht * 2 * 16 * LAD_PS;     // [hi, lo][16 heads][LAD_PS]
     float* smx = reinterpret_cast<float*>(sv + (size_t)D.Rp * LAD_VS + (size_t)HT * 2 * 16 * LAD_PS) + ht * 64;      // [4 waves][16 heads]
-    const int m = blockIdx.x / sh.S, sp = blockIdx.x - m * sh.S, h0 = (blockIdx.y * HT + ht) * 16;
+    const int sp = blockIdx.x / rows, m = blockIdx.x - sp * rows, h0 = (blockIdx.y * HT + ht) * 16;       // (a row's shares on one XCD where rows % 8 == 0)
     const bool on = !p.rows.on || p.rows.on[m];
     const int pos = p.rows.pos[m], seq = p.rows.seq ? p.rows.seq[m] : m;
     const int lo = D.window > 0 ? max(0, pos - D.window + 1) : 0;
     const int nk = pos - lo + 1, per = ((nk + sh.S - 1) / sh.S + 3) & ~3;
-    const int k0 = lo + sp * per, k1 = on ? min(k0 + per, pos + 1) : k0;        // this share's keys
+    const int k0 = lo + sp * per, k1 = on ? min(k0 + per, pos + 1) : k0;        // this share's keys, in equal tiles of at most LAD_KT
+    const int KT = ((per + (per + LAD_KT - 1) / LAD_KT - 1) / ((per + LAD_KT - 1) / LAD_KT) + 3) & ~3;
     const bf16_t* cache = (const bf16_t*)p.cache + (size_t)seq * p.Smax * D.CW;
     const int nch = D.CW >> 3, CT = D.CW >> 5;
-    const int kg = tid & 15;                                                    // four keys 4 kg .. of the tile; sixteen lanes share a 16-byte column chunk
-    uint4 st[NST][4];
+    const int kg = tid & 15;                                                    // sixteen lanes share a 16-byte column chunk
+    u32x4_t st[NST][4];
     auto fetch = [&](int t) {
         const bf16_t* kr[4];
 #pragma unroll
-        for (int k = 0; k < 4; ++k) kr[k] = cache + (size_t)min(t + 4 * kg + k, k1 - 1) * D.CW;
-#pragma unroll
-        for (int i = 0; i < NST; ++i) {
-            const int chunk = min((tid >> 4) + 16 * HT * i, nch - 1);           // (rounds past the row read its last chunk and are not stored)
-#pragma unroll
-            for (int k = 0; k < 4; ++k) st[i][k] = *reinterpret_cast<const uint4*>(kr[k] + chunk * 8);
-        }
-    };
-    if (k0 < k1) fetch(k0);
-    bf16x8_t qf[QF];                                                            // heads past H read head H - 1 and are dropped at the end
-    {
-        const bf16_t* q = (const bf16_t*)p.q + ((size_t)m * D.H + min(h0 + li, D.H - 1)) * D.CW + lq * 8;
-#pragma unroll
-        for (int i = 0; i < QF; ++i) qf[i] = *reinterpret_cast<const bf16x8_t*>(q + min(i, CT - 1) * 32);
-    }
-    f32x4_t o[NTW];
-#pragma unroll
-    for (int i = 0; i < NTW; ++i) o[i] = (f32x4_t){0.f, 0.f, 0.f, 0.f};
-    float mx = -INFINITY, ls = 0.0f;                                            // of head li; ls: this lane's keys only
-    for (int t = k0; t < k1; t += LAD_KT) {
+        for (int k = 0; k < 4; ++k) kr[k] = cache + (size_t)min(t + kg + 16 * k, k1 - 1) * D.CW;
 #pragma unroll
         for (int i = 0; i < NST; ++i) {
             const int chunk = (tid >> 4) + 16 * HT * i;
             if (chunk < nch) {
 #pragma unroll
-                for (int k = 0; k < 4; ++k) *reinterpret_cast<uint4*>(sk + (size_t)(4 * kg + k) * KS + chunk * 8) = st[i][k];
+                for (int k = 0; k < 4; ++k) st[i][k] = __builtin_nontemporal_load(reinterpret_cast<const u32x4_t*>(kr[k] + chunk * 8));   // read once per step
+            }
+        }
+    };
+    bf16x8_t qf[QF];                                                            // heads past H read head H - 1 and are dropped at the end
+    {
+        constexpr int NQ = (QF * 4 * 16 + 255) / 256;                           // 16-byte chunks per thread: 16 HT rows x CW / 8 over 256 HT threads
+        const bf16_t* q = (const bf16_t*)p.q + (size_t)m * D.H * D.CW;
+        const int hb = blockIdx.y * HT * 16;
+        u32x4_t qr[NQ];
+#pragma unroll
+        for (int i = 0; i < NQ; ++i) {
+            const int t = min(tid + 256 * HT * i, 16 * HT * nch - 1), r = t / nch, c = t - r * nch;
+            qr[i] = *reinterpret_cast<const u32x4_t*>(q + (size_t)min(hb + r, D.H - 1) * D.CW + c * 8);
+        }
+        __builtin_amdgcn_sched_barrier(0);                                      // loads return in order: the queries are not to wait for the keys
+        if (k0 < k1) fetch(k0);
+        __builtin_amdgcn_sched_barrier(0);
+#pragma unroll
+        for (int i = 0; i < NQ; ++i) {
+            const int t = tid + 256 * HT * i, r = t / nch, c = t - r * nch;
+            if (t < 16 * HT * nch) *reinterpret_cast<u32x4_t*>(sk + (size_t)r * KS + c * 8) = qr[i];
+        }
+        lds_barrier();
+#pragma unroll
+        for (int i = 0; i < QF; ++i) {                                          // fragments past the row are zero: the products below need no guards
+            const bf16x8_t f = *reinterpret_cast<const bf16x8_t*>(sk + (size_t)(ht * 16 + li) * KS + min(i, CT - 1) * 32 + lq * 8);
+            qf[i] = i < CT ? f : (bf16x8_t){0, 0, 0, 0, 0, 0, 0, 0};
+        }
+        lds_barrier();
+    }
+    f32x4_t o[NTW];
+#pragma unroll
+    for (int i = 0; i < NTW; ++i) o[i] = (f32x4_t){0.f, 0.f, 0.f, 0.f};
+    float mx = -INFINITY, ls = 0.0f;                                            // of head li; ls: this lane's keys only
+    for (int t = k0; t < k1; t += KT) {
+        const int te = min(t + KT, k1);                                         // end of the tile's keys
+#pragma unroll
+        for (int i = 0; i < NST; ++i) {
+            const int chunk = (tid >> 4) + 16 * HT * i;
+            if (chunk < nch) {
+#pragma unroll
+                for (int k = 0; k < 4; ++k) *reinterpret_cast<u32x4_t*>(sk + (size_t)(kg + 16 * k) * KS + chunk * 8) = st[i][k];
                 if (chunk * 8 < D.Rp) {
 #pragma unroll
                     for (int e = 0; e < 8; ++e) *reinterpret_cast<uint2*>(sv + (size_t)(chunk * 8 + e) * LAD_VS + 4 * kg) = column_of(st[i], e);
                 }
             }
         }
-        if (t + LAD_KT < k1) fetch(t + LAD_KT);
+        if (te < k1) fetch(te);
         lds_barrier();
         float w[4], tm = -INFINITY;
         {
             f32x4_t s0 = (f32x4_t){0.f, 0.f, 0.f, 0.f}, s1 = s0;
-            if (t + wave * 16 < k1) {                                           // wave-uniform
+            if (t + wave * 16 < te) {                                           // wave-uniform
                 const bf16_t* kr = sk + (size_t)(wave * 16 + li) * KS + lq * 8;
 #pragma unroll
                 for (int i = 0; i < QF; i += 2) {
-                    if (i < CT) s0 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*reinterpret_cast<const bf16x8_t*>(kr + i * 32), qf[i], s0, 0, 0, 0);
-                    if (i + 1 < QF && i + 1 < CT) s1 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*reinterpret_cast<const bf16x8_t*>(kr + (i + 1) * 32), qf[i + 1 < QF ? i + 1 : i], s1, 0, 0, 0);
+                    s0 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*reinterpret_cast<const bf16x8_t*>(kr + min(i, CT - 1) * 32), qf[i], s0, 0, 0, 0);
+                    s1 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*reinterpret_cast<const bf16x8_t*>(kr + min(i + 1, CT - 1) * 32), qf[i + 1], s1, 0, 0, 0);
                 }
             }
 #pragma unroll
             for (int e = 0; e < 4; ++e) {
-                w[e] = t + wave * 16 + lq * 4 + e < k1 ? (s0[e] + s1[e]) * D.scale : -INFINITY;
+                w[e] = t + wave * 16 + lq * 4 + e < te ? (s0[e] + s1[e]) * D.scale : -INFINITY;
                 tm = fmaxf(tm, w[e]);
             }
         }
@@ -613,40 +632,33 @@ __global__ void __launch_bounds__(256 * HT, HT) k_latent_attn_decode(LatentDims 
         mx = mn;
         {
             float add = 0.0f;
-            uint16_t hi[4], lw[4];
+            bf16_t* pw = sw + (size_t)li * LAD_PS + lq * 16 + wave;             // key 16 wave + kg at place 4 kg + wave, kg = 4 lq + e
 #pragma unroll
             for (int e = 0; e < 4; ++e) {
                 w[e] = __expf(w[e] - mn);
                 add += w[e];
-                hi[e] = f32_to_bf16(w[e]);
-                lw[e] = f32_to_bf16(w[e] - bf16_to_f32(hi[e]));
+                const bf16_t hi = f32_to_bf16(w[e]);
+                pw[4 * e] = hi;
+                pw[16 * LAD_PS + 4 * e] = f32_to_bf16(w[e] - bf16_to_f32(hi));
             }
             ls = ls * alpha + add;
-            bf16_t* pw = sw + (size_t)li * LAD_PS + wave * 16 + lq * 4;
-            *reinterpret_cast<uint2*>(pw) = make_uint2((uint32_t)hi[0] | ((uint32_t)hi[1] << 16), (uint32_t)hi[2] | ((uint32_t)hi[3] << 16));
-            *reinterpret_cast<uint2*>(pw + 16 * LAD_PS) = make_uint2((uint32_t)lw[0] | ((uint32_t)lw[1] << 16), (uint32_t)lw[2] | ((uint32_t)lw[3] << 16));
         }
         if (t > k0 && __any(alpha != 1.0f)) {                                   // (the first tile has nothing to rescale)
 #pragma unroll
-            for (int e = 0; e < 4; ++e) {
-                const float ah = __shfl(alpha, lq * 4 + e, 64);                 // head of accumulator row e
-#pragma unroll
-                for (int i = 0; i < NTW; ++i) o[i][e] *= ah;
-            }
+            for (int i = 0; i < NTW; ++i) o[i] *= alpha;                        // accumulator column = head li
         }
         lds_barrier();
 #pragma unroll
         for (int ks = 0; ks < 2; ++ks) {
-            if (t + 32 * ks >= k1) continue;                                    // uniform
+            if (ks == 1 && t + 8 >= te) continue;                               // (places 32 .. hold keys kg >= 8: none of them in the share; uniform)
             const bf16x8_t ph = *reinterpret_cast<const bf16x8_t*>(sw + (size_t)li * LAD_PS + ks * 32 + lq * 8),
                            pl = *reinterpret_cast<const bf16x8_t*>(sw + (size_t)(16 + li) * LAD_PS + ks * 32 + lq * 8);
 #pragma unroll
             for (int i = 0; i < NTW; ++i) {
-                const int tile = i * 4 + wave;
-                if (tile * 16 >= D.Rp) continue;                                // wave-uniform
+                const int tile = min(i * 4 + wave, (D.Rp >> 4) - 1);            // (tiles past the latent repeat its last one and are not stored)
                 const bf16x8_t v = lds_frag(sv + (size_t)(tile * 16 + li) * LAD_VS + ks * 32 + lq * 8);
-                o[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(ph, v, o[i], 0, 0, 0);
-                o[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(pl, v, o[i], 0, 0, 0);
+                o[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(v, ph, o[i], 0, 0, 0);        // rows: latent columns, columns: heads
+                o[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(v, pl, o[i], 0, 0, 0);
             }
         }
         lds_barrier();                                                          // everyone is done with the tile
@@ -660,24 +672,25 @@ __global__ void __launch_bounds__(256 * HT, HT) k_latent_attn_decode(LatentDims 
         float* ml = sh.ml + (((size_t)sp * rows + m) * D.H + h0 + li) * 2;
         *reinterpret_cast<float2*>(ml) = make_float2(mx, ls);
     }
-    // normalised rows through LDS (the key rows' place), then 16-byte stores
-    bf16_t* so = sk + (size_t)ht * 16 * (D.Rp + 8);
-#pragma unroll
-    for (int e = 0; e < 4; ++e) {
-        const float l = __shfl(ls, lq * 4 + e, 64), inv = l > 0.0f ? 1.0f / l : 0.0f;
+    // normalised rows through LDS (the key rows' place), then whole rows
+    {
+        const float inv = ls > 0.0f ? 1.0f / ls : 0.0f;
+        const int OS = D.Rp + 8;
+        bf16_t* so = sk + (size_t)ht * 16 * OS;
 #pragma unroll
         for (int i = 0; i < NTW; ++i) {
-            const int c = (i * 4 + wave) * 16 + li;
-            if (c < D.Rp) so[(size_t)(lq * 4 + e) * (D.Rp + 8) + c] = f32_to_bf16(o[i][e] * inv);
+            const int c = (i * 4 + wave) * 16 + lq * 4;
+            const float v[4] = {o[i][0] * inv, o[i][1] * inv, o[i][2] * inv, o[i][3] * inv};
+            if (c < D.Rp) *reinterpret_cast<uint2*>(so + (size_t)li * OS + c) = pack4_bf16(v);
         }
-    }
-    lds_barrier();
-    const int rc = D.Rp >> 3;
-    for (int t = tid & 255; t < 16 * rc; t += 256) {
-        const int hr = t / rc, c = t - hr * rc;
-        if (h0 + hr < D.H)
-            *reinterpret_cast<uint4*>(sh.part + (((size_t)sp * rows + m) * D.H + h0 + hr) * D.Rp + c * 8) =
-                *reinterpret_cast<const uint4*>(so + (size_t)hr * (D.Rp + 8) + c * 8);
+        lds_barrier();
+        bf16_t* out = sh.part + ((size_t)sp * rows + m) * D.H * D.Rp;
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {                                           // wave w: heads 4 w .. of its tile, a row per step
+            const int hd = h0 + wave * 4 + r;
+            if (hd < D.H && lane * 8 < D.Rp)
+                *reinterpret_cast<u32x4_t*>(out + (size_t)hd * D.Rp + lane * 8) = *reinterpret_cast<const u32x4_t*>(so + (size_t)(wave * 4 + r) * OS + lane * 8);
+        }
     }
 }
 
@@ -744,8 +757,9 @@ __global__ void __launch_bounds__(512) k_latent_share_values(LatentDims D, Laten
         const bf16_t* xr = so + (size_t)(li & (LSV_ROWS - 1)) * (D.Rp + 8) + lq * 8;       // columns 8 .. 15 of the product repeat the rows, unused
 #pragma unroll
         for (int i = 0; i < LSV_KF; i += 2) {
-            if (i < KT) a0 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wf[i], *reinterpret_cast<const bf16x8_t*>(xr + i * 32), a0, 0, 0, 0);
-            if (i + 1 < KT) a1 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wf[i + 1], *reinterpret_cast<const bf16x8_t*>(xr + (i + 1) * 32), a1, 0, 0, 0);
+            const bf16x8_t zero = {0, 0, 0, 0, 0, 0, 0, 0};                     // (fragments past the latent: nothing)
+            a0 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(i < KT ? wf[i] : zero, *reinterpret_cast<const bf16x8_t*>(xr + min(i, KT - 1) * 32), a0, 0, 0, 0);
+            a1 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(i + 1 < KT ? wf[i + 1] : zero, *reinterpret_cast<const bf16x8_t*>(xr + min(i + 1, KT - 1) * 32), a1, 0, 0, 0);
         }
         const int m = m0 + li, c = vtile * 16 + lq * 4;
         if (li < LSV_ROWS && m < rows) {
@@ -767,7 +781,7 @@ void launch_latent_attn_any(const LatentDims& D, const LatentAttn& p, int rows, 
     else hipLaunchKernelGGL((k_latent_attn_any<bf16_t>), dim3(rows, D.H), dim3(256), sm, s, D, p);
 }
 bool latent_decode_mfma_ok(const LatentDims& D) {
-    return D.Rp <= 512 && D.CW <= (D.Rp <= 128 ? 256 : D.Rp <= 256 ? 512 : 640) && latent_decode_lds(D, D.H > 16 ? 2 : 1) <= 160 * 1024;
+    return D.Rp <= 512 && D.CW <= (D.Rp <= 128 ? 256 : D.Rp <= 256 ? 512 : 576) && latent_decode_lds(D, D.H > 16 ? 2 : 1) <= 160 * 1024;
 }
 // shares per row: at most one block per compute unit (a block fills one), at least 32 keys each
 int latent_decode_shares(const LatentDims& D, int rows, int Smax) {
@@ -790,7 +804,7 @@ void launch_latent_attn_decode(const LatentDims& D, const LatentAttn& p, const L
     } while (0)
     if (D.Rp <= 128) { if (HT == 1) LAT_GO(2, 2, 8, 1); else LAT_GO(2, 1, 8, 2); }
     else if (D.Rp <= 256) { if (HT == 1) LAT_GO(4, 4, 16, 1); else LAT_GO(4, 2, 16, 2); }
-    else { if (HT == 1) LAT_GO(8, 5, 20, 1); else LAT_GO(8, 3, 20, 2); }
+    else { if (HT == 1) LAT_GO(8, 5, 18, 1); else LAT_GO(8, 3, 18, 2); }
 #undef LAT_GO
 }
 void launch_latent_share_values(const LatentDims& D, const LatentShares& sh, const bf16_t* uv, size_t uvz, const Operand& out, int rows, hipStream_t s) {
@@ -819,11 +833,11 @@ __global__ void __launch_bounds__(256, 2) k_latent_attn_prefill(LatentDims D, La
     int kkey[NK], kch[NK];
 #pragma unroll
     for (int i = 0; i < NK; ++i) { const int t = tid + 256 * i; kkey[i] = t / nch; kch[i] = t - kkey[i] * nch; }
-    const int vkg = tid / nv, vch = tid - vkg * nv;                             // 8 groups of 4 keys x vp / 8 chunks (vp <= 256)
+    const int vkg = tid & 7, vch = tid >> 3;                                    // 8 groups of 4 keys x vp / 8 chunks (vp <= 256)
     const bf16_t* kplain = p.kv + (size_t)hd * D.np;
     const bf16_t* vals = p.kv + (size_t)D.H * D.np + (size_t)hd * D.vp;
     const bf16_t* crot = p.cache + (size_t)T.seq * p.Smax * D.CW + D.Rp;
-    uint4 sk_r[NK], sv_r[4];
+    u32x4_t sk_r[NK], sv_r[4];
     auto fetch = [&](int t) {
         const int k0 = k_lo + t * LAT_KT;
 #pragma unroll
@@ -832,13 +846,13 @@ __global__ void __launch_bounds__(256, 2) k_latent_attn_prefill(LatentDims D, La
             const int c = kch[i];
             const bf16_t* src = c < nplain ? kplain + (size_t)(T.krow0 + key - T.kpos0) * p.ldkv + c * 8
                                            : crot + (size_t)key * D.CW + (c < nrot ? c - nplain : 0) * 8;
-            sk_r[i] = *reinterpret_cast<const uint4*>(src);
-            if (c >= nrot) sk_r[i] = make_uint4(0, 0, 0, 0);
+            sk_r[i] = *reinterpret_cast<const u32x4_t*>(src);
+            if (c >= nrot) sk_r[i] = (u32x4_t){0, 0, 0, 0};
         }
 #pragma unroll
         for (int k = 0; k < 4; ++k) {
-            const int key = min(k0 + 4 * min(vkg, 7) + k, q_last);
-            sv_r[k] = *reinterpret_cast<const uint4*>(vals + (size_t)(T.krow0 + key - T.kpos0) * p.ldkv + vch * 8);
+            const int key = min(k0 + 4 * vkg + k, q_last);
+            sv_r[k] = *reinterpret_cast<const u32x4_t*>(vals + (size_t)(T.krow0 + key - T.kpos0) * p.ldkv + min(vch, nv - 1) * 8);
         }
     };
     const int wq0 = wave * 16, qi = wq0 + li;                                   // this lane's query of the tile
@@ -849,7 +863,10 @@ __global__ void __launch_bounds__(256, 2) k_latent_attn_prefill(LatentDims D, La
     {
         const bf16_t* q = p.q + ((size_t)(T.row0 + min(qi, T.n - 1)) * D.H + hd) * D.DK + lq * 8;
 #pragma unroll
-        for (int i = 0; i < KT; ++i) qf[i] = *reinterpret_cast<const bf16x8_t*>(q + min(i, kt_n - 1) * 32);
+        for (int i = 0; i < KT; ++i) {                                          // fragments past the row are zero: no guards below
+            const bf16x8_t f = *reinterpret_cast<const bf16x8_t*>(q + min(i, kt_n - 1) * 32);
+            qf[i] = i < kt_n ? f : (bf16x8_t){0, 0, 0, 0, 0, 0, 0, 0};
+        }
     }
     f32x4_t o[VT];
 #pragma unroll
@@ -861,8 +878,8 @@ __global__ void __launch_bounds__(256, 2) k_latent_attn_prefill(LatentDims D, La
         const int k0 = k_lo + t * LAT_KT;
 #pragma unroll
         for (int i = 0; i < NK; ++i)
-            if (kkey[i] < LAT_KT) *reinterpret_cast<uint4*>(sk + (size_t)kkey[i] * KS + kch[i] * 8) = sk_r[i];
-        if (vkg < 8) {
+            if (kkey[i] < LAT_KT) *reinterpret_cast<u32x4_t*>(sk + (size_t)kkey[i] * KS + kch[i] * 8) = sk_r[i];
+        if (vch < nv) {
 #pragma unroll
             for (int e = 0; e < 8; ++e) *reinterpret_cast<uint2*>(sv + (size_t)(vch * 8 + e) * LAT_VS + 4 * vkg) = column_of(sv_r, e);
         }
@@ -876,7 +893,7 @@ __global__ void __launch_bounds__(256, 2) k_latent_attn_prefill(LatentDims D, La
                 const bf16_t* kr = sk + (size_t)(perm + 4 * f) * KS + lq * 8;
 #pragma unroll
                 for (int i = 0; i < KT; ++i)
-                    if (i < kt_n) s[f] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*reinterpret_cast<const bf16x8_t*>(kr + i * 32), qf[i], s[f], 0, 0, 0);
+                    s[f] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*reinterpret_cast<const bf16x8_t*>(kr + min(i, kt_n - 1) * 32), qf[i], s[f], 0, 0, 0);
             }
             float w[8], tm = -INFINITY;
 #pragma unroll
@@ -910,8 +927,7 @@ __global__ void __launch_bounds__(256, 2) k_latent_attn_prefill(LatentDims D, La
             }
 #pragma unroll
             for (int i = 0; i < VT; ++i) {
-                if (i >= vt_n) continue;
-                const bf16x8_t v = lds_frag(sv + (size_t)(i * 16 + li) * LAT_VS + lq * 8);
+                const bf16x8_t v = lds_frag(sv + (size_t)(min(i, vt_n - 1) * 16 + li) * LAT_VS + lq * 8);        // (tiles past the values are not stored)
                 o[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(ph, v, o[i], 0, 0, 0);
                 o[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(pl, v, o[i], 0, 0, 0);
             }
