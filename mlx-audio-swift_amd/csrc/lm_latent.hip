@@ -523,15 +523,20 @@ __device__ __forceinline__ uint2 column_of(const u32x4_t (&r)[4], int e) {
     const uint32_t sel = (e & 1) ? 0x07060302u : 0x05040100u;        // v_perm: high / low halves of two words
     return make_uint2(__builtin_amdgcn_perm(r[1][w], r[0][w], sel), __builtin_amdgcn_perm(r[3][w], r[2][w], sel));
 }
+// LDS layouts of the decode kernel, free of bank conflicts for its writes (a wave: 8 keys x 8 chunks) and its fragment reads (16 rows, one chunk):
+// a key row is an odd number of 128-byte halves long and its 16-byte chunks are exchanged within groups of 8 by the row's number / 2; the
+// 8-byte places of a column row are exchanged in groups of four by the column's number / 16
+__host__ __device__ __forceinline__ int lad_key_stride(int CW) { const int k = (CW + 63) / 64 * 64; return k % 128 ? k : k + 64; }
+__device__ __forceinline__ int lad_key_at(int row, int chunk, int KS) { return row * KS + ((chunk & ~7) | ((chunk ^ (row >> 1)) & 7)) * 8; }
 static size_t latent_decode_lds(const LatentDims& D, int HT) {
-    return (size_t)LAD_KT * (D.CW + 8) * 2 + (size_t)D.Rp * LAD_VS * 2 + (size_t)HT * (2 * 16 * LAD_PS * 2 + 4 * 16 * 4);
+    return (size_t)LAD_KT * lad_key_stride(D.CW) * 2 + (size_t)D.Rp * LAD_VS * 2 + (size_t)HT * (2 * 16 * LAD_PS * 2 + 4 * 16 * 4);
 }
 // NTW: latent tiles per wave (Rp / 64 <= NTW); NST: staging rounds (CW <= 128 HT NST); QF: query fragments (CW / 32 <= QF)
 template <int NTW, int NST, int QF, int HT>
 __global__ void __launch_bounds__(256 * HT, HT) k_latent_attn_decode(LatentDims D, LatentAttn p, LatentShares sh, int rows) {
     extern __shared__ __attribute__((aligned(16))) uint8_t lds[];
-    const int KS = D.CW + 8;
-    bf16_t* sk = reinterpret_cast<bf16_t*>(lds);                                // [64][CW + 8]
+    const int KS = lad_key_stride(D.CW);
+    bf16_t* sk = reinterpret_cast<bf16_t*>(lds);                                // [64][KS]
     bf16_t* sv = sk + (size_t)LAD_KT * KS;                                      // [Rp][LAD_VS]
     const int tid = threadIdx.x, lane = tid & 63, wave = (tid >> 6) & 3, ht = tid >> 8, li = lane & 15, lq = lane >> 4;
     bf16_t* sw = sv + (size_t)D.Rp * LAD_VS + (size_t)ht * 2 * 16 * LAD_PS;     // [hi, lo][16 heads][LAD_PS]
@@ -545,7 +550,7 @@ __global__ void __launch_bounds__(256 * HT, HT) k_latent_attn_decode(LatentDims 
     const int KT = ((per + (per + LAD_KT - 1) / LAD_KT - 1) / ((per + LAD_KT - 1) / LAD_KT) + 3) & ~3;
     const bf16_t* cache = (const bf16_t*)p.cache + (size_t)seq * p.Smax * D.CW;
     const int nch = D.CW >> 3, CT = D.CW >> 5;
-    const int kg = tid & 15;                                                    // sixteen lanes share a 16-byte column chunk
+    const int kg = ((tid >> 3) & 7) + 8 * ((tid >> 6) & 1), ch0 = (tid & 7) + 8 * (tid >> 7);        // a load of a wave: 8 keys x 128 bytes
     u32x4_t st[NST][4];
     auto fetch = [&](int t) {
         const bf16_t* kr[4];
@@ -553,7 +558,7 @@ __global__ void __launch_bounds__(256 * HT, HT) k_latent_attn_decode(LatentDims 
         for (int k = 0; k < 4; ++k) kr[k] = cache + (size_t)min(t + kg + 16 * k, k1 - 1) * D.CW;
 #pragma unroll
         for (int i = 0; i < NST; ++i) {
-            const int chunk = (tid >> 4) + 16 * HT * i;
+            const int chunk = ch0 + 16 * HT * i;
             if (chunk < nch) {
 #pragma unroll
                 for (int k = 0; k < 4; ++k) st[i][k] = __builtin_nontemporal_load(reinterpret_cast<const u32x4_t*>(kr[k] + chunk * 8));   // read once per step
@@ -577,12 +582,12 @@ __global__ void __launch_bounds__(256 * HT, HT) k_latent_attn_decode(LatentDims 
 #pragma unroll
         for (int i = 0; i < NQ; ++i) {
             const int t = tid + 256 * HT * i, r = t / nch, c = t - r * nch;
-            if (t < 16 * HT * nch) *reinterpret_cast<u32x4_t*>(sk + (size_t)r * KS + c * 8) = qr[i];
+            if (t < 16 * HT * nch) *reinterpret_cast<u32x4_t*>(sk + lad_key_at(r, c, KS)) = qr[i];
         }
         lds_barrier();
 #pragma unroll
         for (int i = 0; i < QF; ++i) {                                          // fragments past the row are zero: the products below need no guards
-            const bf16x8_t f = *reinterpret_cast<const bf16x8_t*>(sk + (size_t)(ht * 16 + li) * KS + min(i, CT - 1) * 32 + lq * 8);
+            const bf16x8_t f = *reinterpret_cast<const bf16x8_t*>(sk + lad_key_at(ht * 16 + li, min(i, CT - 1) * 4 + lq, KS));
             qf[i] = i < CT ? f : (bf16x8_t){0, 0, 0, 0, 0, 0, 0, 0};
         }
         lds_barrier();
@@ -595,13 +600,13 @@ __global__ void __launch_bounds__(256 * HT, HT) k_latent_attn_decode(LatentDims 
         const int te = min(t + KT, k1);                                         // end of the tile's keys
 #pragma unroll
         for (int i = 0; i < NST; ++i) {
-            const int chunk = (tid >> 4) + 16 * HT * i;
+            const int chunk = ch0 + 16 * HT * i;
             if (chunk < nch) {
 #pragma unroll
-                for (int k = 0; k < 4; ++k) *reinterpret_cast<u32x4_t*>(sk + (size_t)(kg + 16 * k) * KS + chunk * 8) = st[i][k];
+                for (int k = 0; k < 4; ++k) *reinterpret_cast<u32x4_t*>(sk + lad_key_at(kg + 16 * k, chunk, KS)) = st[i][k];
                 if (chunk * 8 < D.Rp) {
 #pragma unroll
-                    for (int e = 0; e < 8; ++e) *reinterpret_cast<uint2*>(sv + (size_t)(chunk * 8 + e) * LAD_VS + 4 * kg) = column_of(st[i], e);
+                    for (int e = 0; e < 8; ++e) *reinterpret_cast<uint2*>(sv + (size_t)(chunk * 8 + e) * LAD_VS + 4 * (kg ^ (4 * ((chunk >> 1) & 3)))) = column_of(st[i], e);
                 }
             }
         }
@@ -611,11 +616,11 @@ __global__ void __launch_bounds__(256 * HT, HT) k_latent_attn_decode(LatentDims 
         {
             f32x4_t s0 = (f32x4_t){0.f, 0.f, 0.f, 0.f}, s1 = s0;
             if (t + wave * 16 < te) {                                           // wave-uniform
-                const bf16_t* kr = sk + (size_t)(wave * 16 + li) * KS + lq * 8;
+                const bf16_t *kr = sk + lad_key_at(wave * 16 + li, lq, KS), *kr1 = sk + lad_key_at(wave * 16 + li, 4 + lq, KS);
 #pragma unroll
-                for (int i = 0; i < QF; i += 2) {
-                    s0 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*reinterpret_cast<const bf16x8_t*>(kr + min(i, CT - 1) * 32), qf[i], s0, 0, 0, 0);
-                    s1 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*reinterpret_cast<const bf16x8_t*>(kr + min(i + 1, CT - 1) * 32), qf[i + 1], s1, 0, 0, 0);
+                for (int i = 0; i < QF; i += 2) {                               // (past the row: its first fragments again, times zero)
+                    s0 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*reinterpret_cast<const bf16x8_t*>(kr + (i < CT ? i * 32 : 0)), qf[i], s0, 0, 0, 0);
+                    s1 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*reinterpret_cast<const bf16x8_t*>(kr1 + (i + 1 < CT ? i * 32 : 0)), qf[i + 1], s1, 0, 0, 0);
                 }
             }
 #pragma unroll
@@ -656,7 +661,7 @@ __global__ void __launch_bounds__(256 * HT, HT) k_latent_attn_decode(LatentDims 
 #pragma unroll
             for (int i = 0; i < NTW; ++i) {
                 const int tile = min(i * 4 + wave, (D.Rp >> 4) - 1);            // (tiles past the latent repeat its last one and are not stored)
-                const bf16x8_t v = lds_frag(sv + (size_t)(tile * 16 + li) * LAD_VS + ks * 32 + lq * 8);
+                const bf16x8_t v = lds_frag(sv + (size_t)(tile * 16 + li) * LAD_VS + ((ks * 4 + lq) ^ (2 * (tile & 3))) * 8);
                 o[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(v, ph, o[i], 0, 0, 0);        // rows: latent columns, columns: heads
                 o[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(v, pl, o[i], 0, 0, 0);
             }
