@@ -89,6 +89,13 @@ struct PinnedBuf {
     T* release() { T* q = p; p = nullptr; return q; }
 };
 
+// Synchronous copies of the generate paths.  hipMemcpy works on the legacy default stream, and any use of that stream while ANOTHER thread captures
+// a graph (two replicas of a group generating at once) invalidates the capture; the per-thread stream does not take part in it.
+static inline hipError_t copy_now(void* dst, const void* src, size_t n, hipMemcpyKind kind) {
+    const hipError_t e = hipMemcpyAsync(dst, src, n, kind, hipStreamPerThread);
+    return e != hipSuccess ? e : hipStreamSynchronize(hipStreamPerThread);
+}
+
 static inline size_t round_up(size_t a, size_t b) { return (a + b - 1) / b * b; }
 static inline int cdiv(int64_t a, int64_t b) { return (int)((a + b - 1) / b); }
 

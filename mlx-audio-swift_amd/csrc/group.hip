@@ -205,11 +205,11 @@ struct HostPrompts { std::vector<int32_t> lens, flat; std::vector<size_t> off; }
 HostPrompts fetch_prompts(const int32_t* prompt_ids, const int32_t* prompt_lens, int batch) {
     HostPrompts h;
     h.lens.resize(batch);
-    HIP_CHECK(hipMemcpy(h.lens.data(), prompt_lens, (size_t)batch * 4, hipMemcpyDefault));
+    HIP_CHECK(copy_now(h.lens.data(), prompt_lens, (size_t)batch * 4, hipMemcpyDefault));
     h.off.assign(batch + 1, 0);
     for (int b = 0; b < batch; ++b) { MIS_REQUIRE(h.lens[b] >= 1, MIS_ERR_INVALID_INPUT, "empty prompt in row %d", b); h.off[b + 1] = h.off[b] + h.lens[b]; }
     h.flat.resize(h.off[batch]);
-    HIP_CHECK(hipMemcpy(h.flat.data(), prompt_ids, h.off[batch] * 4, hipMemcpyDefault));
+    HIP_CHECK(copy_now(h.flat.data(), prompt_ids, h.off[batch] * 4, hipMemcpyDefault));
     return h;
 }
 }   // namespace

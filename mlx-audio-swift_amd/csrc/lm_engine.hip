@@ -1076,12 +1076,12 @@ extern "C" mis_status mis_lm_forward_hidden(mis_tts* c, const int32_t* ids, cons
     std::vector<uint8_t> act(c->batch, 1);
     if (active) {
         std::vector<uint8_t> tmp(c->batch);
-        HIP_CHECK(hipMemcpy(tmp.data(), active, c->batch, hipMemcpyDefault));
+        HIP_CHECK(copy_now(tmp.data(), active, c->batch, hipMemcpyDefault));
         act = tmp;
     }
     {   // context overflow check on the host mirror of pos_next
         std::vector<int32_t> pn(c->batch);
-        HIP_CHECK(hipMemcpy(pn.data(), c->pos_next.p, c->batch * 4, hipMemcpyDeviceToHost));
+        HIP_CHECK(copy_now(pn.data(), c->pos_next.p, c->batch * 4, hipMemcpyDeviceToHost));
         for (int b = 0; b < c->batch; ++b)
             MIS_REQUIRE(!act[b] || pn[b] < c->Smax, MIS_ERR_INVALID_INPUT, "row %d exceeds max_context %d", b, c->Smax);
     }
@@ -1132,7 +1132,7 @@ extern "C" mis_status mis_lm_prefill(mis_tts* c, const int32_t* prompt_ids, cons
     HIP_CHECK(hipSetDevice(c->device));
     hipStream_t s = c->stream;
     std::vector<int32_t> lens(batch);
-    HIP_CHECK(hipMemcpy(lens.data(), prompt_lens, batch * 4, hipMemcpyDefault));
+    HIP_CHECK(copy_now(lens.data(), prompt_lens, batch * 4, hipMemcpyDefault));
     int Lmax = 0;
     size_t total = 0;
     for (int b = 0; b < batch; ++b) {
@@ -1140,7 +1140,7 @@ extern "C" mis_status mis_lm_prefill(mis_tts* c, const int32_t* prompt_ids, cons
         Lmax = std::max(Lmax, lens[b]); total += lens[b];
     }
     std::vector<int32_t> flat(total);
-    HIP_CHECK(hipMemcpy(flat.data(), prompt_ids, total * 4, hipMemcpyDefault));
+    HIP_CHECK(copy_now(flat.data(), prompt_ids, total * 4, hipMemcpyDefault));
     for (auto t : flat) MIS_REQUIRE(t >= 0 && t < c->V, MIS_ERR_INVALID_INPUT, "prompt token %d outside the vocabulary", t);
     lm_reset(c, batch, std::max(max_context, Lmax + 1));
     if (c->blocks) {
@@ -1348,7 +1348,7 @@ static void run_generate_attempt(mis_tts* c, const int32_t* prompt_ids, const in
     hipStream_t s = c->stream;
     const int max_tokens = gp->max_tokens > 0 ? gp->max_tokens : 1200;
     std::vector<int32_t> lens(batch);
-    HIP_CHECK(hipMemcpy(lens.data(), prompt_lens, batch * 4, hipMemcpyDefault));
+    HIP_CHECK(copy_now(lens.data(), prompt_lens, batch * 4, hipMemcpyDefault));
     int Lmax = 0;
     size_t total = 0;
     for (int b = 0; b < batch; ++b) {
@@ -1357,7 +1357,7 @@ static void run_generate_attempt(mis_tts* c, const int32_t* prompt_ids, const in
         total += lens[b];
     }
     std::vector<int32_t> flat(total);
-    HIP_CHECK(hipMemcpy(flat.data(), prompt_ids, total * 4, hipMemcpyDefault));
+    HIP_CHECK(copy_now(flat.data(), prompt_ids, total * 4, hipMemcpyDefault));
     for (auto t : flat) MIS_REQUIRE(t >= 0 && t < c->V, MIS_ERR_INVALID_INPUT, "prompt token %d outside the vocabulary", t);
     const int ctx = std::max(gp->repetition_context, 0);
     const int all_stride = Lmax + max_tokens;
@@ -1791,7 +1791,7 @@ extern "C" mis_status mis_lm_generate_stream(mis_tts* c, const int32_t* prompt_i
     hm.on = true; hm.stop_id = stop_id;
     run_generate(c, prompt_ids, prompt_lens, batch, params, nullptr, nullptr, 0, false, on_event, user, cancel_flag, out, &hm);
     std::vector<int32_t> lens(batch);
-    HIP_CHECK(hipMemcpy(lens.data(), prompt_lens, (size_t)batch * 4, hipMemcpyDefault));
+    HIP_CHECK(copy_now(lens.data(), prompt_lens, (size_t)batch * 4, hipMemcpyDefault));
     for (int b = 0; b < batch; ++b) {
         mis_gen_info info{};
         info.prompt_token_count = lens[b];
@@ -1812,7 +1812,7 @@ extern "C" mis_status mis_lm_generate_stream(mis_tts* c, const int32_t* prompt_i
 static int64_t max_pcm_per_row(mis_tts* c, const mis_gen_params* p, const int32_t* prompt_lens, int batch) {
     MIS_REQUIRE(prompt_lens && batch >= 1, MIS_ERR_INVALID_INPUT, "null argument");
     std::vector<int32_t> lens(batch);
-    HIP_CHECK(hipMemcpy(lens.data(), prompt_lens, (size_t)batch * 4, hipMemcpyDefault));
+    HIP_CHECK(copy_now(lens.data(), prompt_lens, (size_t)batch * 4, hipMemcpyDefault));
     int lmax = 0;
     for (int b = 0; b < batch; ++b) lmax = std::max(lmax, lens[b]);
     int mt = p->max_tokens > 0 ? p->max_tokens : 1200;
@@ -1837,7 +1837,8 @@ extern "C" mis_status mis_tts_generate(mis_tts* c, const int32_t* prompt_ids, co
     int64_t longest = 0;
     for (int b = 0; b < batch; ++b) longest = std::max(longest, out.pcm_lens[b]);
     PinnedBuf<float> host((size_t)batch * std::max<int64_t>(longest, 1));
-    HIP_CHECK(hipMemcpy2D(host.p, (size_t)longest * 4, pcm.p, (size_t)cap * 4, (size_t)longest * 4, batch, hipMemcpyDeviceToHost));
+    HIP_CHECK(hipMemcpy2DAsync(host.p, (size_t)longest * 4, pcm.p, (size_t)cap * 4, (size_t)longest * 4, batch, hipMemcpyDeviceToHost, c->stream));
+    HIP_CHECK(hipStreamSynchronize(c->stream));
     if (tokens_out) {
         PinnedBuf<int32_t> th(out.tokens.size() + 1);
         memcpy(th.p, out.tokens.data(), out.tokens.size() * 4);
@@ -1864,7 +1865,7 @@ extern "C" mis_status mis_tts_generate_stream(mis_tts* c, const int32_t* prompt_
     GenOutputs out;
     run_generate(c, prompt_ids, prompt_lens, batch, params, snac_noise, pcm.p, cap, false, on_event, user, cancel_flag, out);
     std::vector<int32_t> lens(batch);
-    HIP_CHECK(hipMemcpy(lens.data(), prompt_lens, batch * 4, hipMemcpyDefault));
+    HIP_CHECK(copy_now(lens.data(), prompt_lens, batch * 4, hipMemcpyDefault));
     std::vector<float> host;
     for (int b = 0; b < batch; ++b) {
         mis_gen_info info{};
@@ -1878,7 +1879,7 @@ extern "C" mis_status mis_tts_generate_stream(mis_tts* c, const int32_t* prompt_
         info.peak_memory_gb = (double)(total_b - free_b) / 1e9;
         on_event(user, b, MIS_EVENT_INFO, &info, 1);                         // .info, LlamaTTS.swift:893-901
         host.resize((size_t)std::max<int64_t>(out.pcm_lens[b], 1));
-        HIP_CHECK(hipMemcpy(host.data(), pcm.p + (size_t)b * cap, (size_t)out.pcm_lens[b] * 4, hipMemcpyDeviceToHost));
+        HIP_CHECK(copy_now(host.data(), pcm.p + (size_t)b * cap, (size_t)out.pcm_lens[b] * 4, hipMemcpyDeviceToHost));
         on_event(user, b, MIS_EVENT_AUDIO, host.data(), out.pcm_lens[b]);   // ONE final .audio, :904
     }
     MIS_API_END

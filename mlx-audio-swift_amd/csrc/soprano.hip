@@ -439,7 +439,7 @@ static void soprano_generate_impl(mis_soprano* c, const int32_t* prompt_ids, con
         const char* e = getenv("MIS_TOKEN_ENGINE");
         const int xcds = e ? atoi(e) : 4;
         int32_t len0 = 0;
-        if (batch == 1) HIP_CHECK(hipMemcpy(&len0, prompt_lens, 4, hipMemcpyDefault));
+        if (batch == 1) HIP_CHECK(copy_now(&len0, prompt_lens, 4, hipMemcpyDefault));
         const bool one_row_request = batch == 1 && (c->group_batch == 0 || c->group_batch == 1);
         if (one_row_request && !tts_internal_shared_device(c->lm) && (xcds == 1 || xcds == 2 || xcds == 4 || xcds == 8) &&
             token_engine_supports(c->lm) && len0 >= 1 &&

@@ -1132,7 +1132,7 @@ void token_engine_run(mis_tts* lm, const TokenEngineRequest& rq, TokenEngineResu
     hipStream_t s = v.stream;
     out.n_announced = 0;
     std::vector<int32_t> hp(rq.n_prompt);
-    HIP_CHECK(hipMemcpy(hp.data(), rq.prompt, (size_t)rq.n_prompt * 4, hipMemcpyDefault));
+    HIP_CHECK(copy_now(hp.data(), rq.prompt, (size_t)rq.n_prompt * 4, hipMemcpyDefault));
     for (int t : hp) MIS_REQUIRE(t >= 0 && t < v.V, MIS_ERR_INVALID_INPUT, "prompt token %d outside the vocabulary", t);
     // The prompt, all but its last position, through the launch chain's batched prefill (one [positions x 1] pass: ~1 ms where the engine
     // walks 0.24 ms per position); its K/V are imported below and the engine starts at the last prompt position.
@@ -1236,30 +1236,30 @@ void token_engine_run(mis_tts* lm, const TokenEngineRequest& rq, TokenEngineResu
     float ms = 0;
     HIP_CHECK(hipEventElapsedTime(&ms, ev.e0, ev.e1));
     unsigned failed = 0;
-    HIP_CHECK(hipMemcpy(&failed, sc.sync.p + 32, 4, hipMemcpyDeviceToHost));
+    HIP_CHECK(copy_now(&failed, sc.sync.p + 32, 4, hipMemcpyDeviceToHost));
     MIS_REQUIRE(!failed, MIS_ERR_GENERATION_FAILED, "token engine: an edge timed out (its workers were not co-resident)");
     if (cancelled || (rq.cancel && *rq.cancel)) throw MisError(MIS_ERR_CANCELLED, "generation cancelled");
     drain();
     int32_t done[2] = {0, 0};
-    HIP_CHECK(hipMemcpy(done, sc.done.p, 8, hipMemcpyDeviceToHost));
+    HIP_CHECK(copy_now(done, sc.done.p, 8, hipMemcpyDeviceToHost));
     out.n_positions = done[0]; out.n_sampled = done[1]; out.ms = ms; out.head_from = head_from;
     out.next_tokens.assign(n_total, 0);
-    HIP_CHECK(hipMemcpy(out.next_tokens.data(), sc.tokd.p, (size_t)n_total * 4, hipMemcpyDeviceToHost));
+    HIP_CHECK(copy_now(out.next_tokens.data(), sc.tokd.p, (size_t)n_total * 4, hipMemcpyDeviceToHost));
     for (int t = 0; t < n_total; ++t) {
         MIS_REQUIRE(out.next_tokens[t] == tok_host[t], MIS_ERR_GENERATION_FAILED, "token engine: the host-visible id row differs from the device's at position %d", t);
         if (out.next_tokens[t] < 0) out.next_tokens[t] = 0;
     }
     if (rq.want_logits) {
         out.logits.assign((size_t)std::max(head_until - head_from, 1) * v.V, 0.f);
-        HIP_CHECK(hipMemcpy(out.logits.data(), d_logits.p, out.logits.size() * 4, hipMemcpyDeviceToHost));
+        HIP_CHECK(copy_now(out.logits.data(), d_logits.p, out.logits.size() * 4, hipMemcpyDeviceToHost));
     }
     if (rq.want_hidden && !rq.hidden_dev) {
         out.hidden.assign((size_t)n_rows * S::d, 0.f);
-        HIP_CHECK(hipMemcpy(out.hidden.data(), d_hidden.p, out.hidden.size() * 4, hipMemcpyDeviceToHost));
+        HIP_CHECK(copy_now(out.hidden.data(), d_hidden.p, out.hidden.size() * 4, hipMemcpyDeviceToHost));
     }
     if (stamp_env) {
         u64 st[32];
-        HIP_CHECK(hipMemcpy(st, d_dbg.p, sizeof(st), hipMemcpyDeviceToHost));
+        HIP_CHECK(copy_now(st, d_dbg.p, sizeof(st), hipMemcpyDeviceToHost));
         static const char* names[20] = {"layer start", "qkv: red ready", "published", "q|k|v polled in", "barrier", "q/k-norm + RoPE", "scores",
                                         "softmax + P.V", "o: red ready", "published", "h polled in", "barrier", "gate|up: red ready", "published",
                                         "act polled in", "barrier", "down: red ready", "published", "h polled in", "barrier"};

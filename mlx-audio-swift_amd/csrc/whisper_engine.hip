@@ -475,7 +475,7 @@ extern "C" mis_status mis_whisper_encode(mis_whisper* c, const float* features, 
     DevBuf<float> f;
     size_t n = (size_t)batch * 3000 * c->nmel;
     f.alloc(n);
-    HIP_CHECK(hipMemcpy(f.p, features, n * 4, hipMemcpyDefault));
+    HIP_CHECK(copy_now(f.p, features, n * 4, hipMemcpyDefault));
     whisper_encode_device(c, f.p, batch);
     if (enc_out) {
         size_t ne = (size_t)batch * 1500 * c->d;
@@ -483,7 +483,7 @@ extern "C" mis_status mis_whisper_encode(mis_whisper* c, const float* features, 
         o.alloc(ne);
         hipLaunchKernelGGL(k_bf16_to_f32_flat, dim3((unsigned)((ne + 255) / 256)), dim3(256), 0, c->stream, c->enc_out.p, o.p, ne);
         HIP_CHECK(hipStreamSynchronize(c->stream));
-        HIP_CHECK(hipMemcpy(enc_out, o.p, ne * 4, hipMemcpyDefault));
+        HIP_CHECK(copy_now(enc_out, o.p, ne * 4, hipMemcpyDefault));
     }
     MIS_API_END
 }
@@ -590,9 +590,9 @@ extern "C" mis_status mis_whisper_decoder_forward(mis_whisper* c, const int32_t*
     HIP_CHECK(hipSetDevice(c->device));
     hipStream_t s = c->stream;
     std::vector<uint8_t> act(c->batch, 1);
-    if (active) HIP_CHECK(hipMemcpy(act.data(), active, c->batch, hipMemcpyDefault));
+    if (active) HIP_CHECK(copy_now(act.data(), active, c->batch, hipMemcpyDefault));
     std::vector<int32_t> pn(c->batch);
-    HIP_CHECK(hipMemcpy(pn.data(), c->pos_next.p, c->batch * 4, hipMemcpyDeviceToHost));
+    HIP_CHECK(copy_now(pn.data(), c->pos_next.p, c->batch * 4, hipMemcpyDeviceToHost));
     for (int b = 0; b < c->batch; ++b)
         MIS_REQUIRE(!act[b] || pn[b] < c->cfg.max_target_positions, MIS_ERR_INVALID_INPUT, "row %d exceeds max_target_positions", b);
     HIP_CHECK(hipMemcpyAsync(c->ids.p, tokens, c->batch * 4, hipMemcpyDefault, s));
@@ -626,20 +626,21 @@ static void whisper_generate_impl(mis_whisper* c, const float* pcm, const int64_
     // ---- features (WhisperAudio.encoderFeatures) on the device, then the encoder
     const int64_t W = 480000;
     std::vector<int64_t> hl(batch, stride);
-    if (lens) HIP_CHECK(hipMemcpy(hl.data(), lens, batch * sizeof(int64_t), hipMemcpyDefault));
+    if (lens) HIP_CHECK(copy_now(hl.data(), lens, batch * sizeof(int64_t), hipMemcpyDefault));
     DevBuf<float> padded, feats;
     padded.alloc((size_t)batch * W);
     feats.alloc((size_t)batch * 3000 * c->nmel);
-    HIP_CHECK(hipMemset(padded.p, 0, (size_t)batch * W * 4));
+    HIP_CHECK(hipMemsetAsync(padded.p, 0, (size_t)batch * W * 4, hipStreamPerThread));
     for (int b = 0; b < batch; ++b) {
         int64_t n = std::min<int64_t>(std::min<int64_t>(hl[b], stride), W);
-        if (n > 0) HIP_CHECK(hipMemcpy(padded.p + (size_t)b * W, pcm + (size_t)b * stride, (size_t)n * 4, hipMemcpyDefault));
+        if (n > 0) HIP_CHECK(copy_now(padded.p + (size_t)b * W, pcm + (size_t)b * stride, (size_t)n * 4, hipMemcpyDefault));
     }
+    HIP_CHECK(hipStreamSynchronize(hipStreamPerThread));
     whisper_features_device(c->device, padded.p, batch, c->nmel, feats.p, s);
     whisper_encode_device(c, feats.p, batch);
     // ---- prompt prefill, one token per step (same prompt for every row)
     std::vector<int32_t> prompt(n_prompt);
-    HIP_CHECK(hipMemcpy(prompt.data(), prompt_ids, n_prompt * 4, hipMemcpyDefault));
+    HIP_CHECK(copy_now(prompt.data(), prompt_ids, n_prompt * 4, hipMemcpyDefault));
     // maxTokens = max(1, min(maxTokens, maxTargetPositions - prompt - 1))   (:222-226)
     int max_tokens = std::max(1, std::min(sp->max_tokens > 0 ? sp->max_tokens : c->cfg.max_target_positions,
                                           c->cfg.max_target_positions - n_prompt - 1));
@@ -740,8 +741,8 @@ static void whisper_generate_impl(mis_whisper* c, const float* pcm, const int64_
         MIS_REQUIRE(attempt(true), MIS_ERR_GENERATION_FAILED, "sampler: time-out flag raised on the multi-launch path");
     }
     std::vector<int32_t> ng(batch), toks((size_t)batch * max_tokens);
-    HIP_CHECK(hipMemcpy(ng.data(), c->n_gen.p, batch * 4, hipMemcpyDeviceToHost));
-    HIP_CHECK(hipMemcpy(toks.data(), c->tokens_out.p, toks.size() * 4, hipMemcpyDeviceToHost));
+    HIP_CHECK(copy_now(ng.data(), c->n_gen.p, batch * 4, hipMemcpyDeviceToHost));
+    HIP_CHECK(copy_now(toks.data(), c->tokens_out.p, toks.size() * 4, hipMemcpyDeviceToHost));
     if (tokens_out) {
         PinnedBuf<int32_t> th(toks.size() + 1);
         memcpy(th.p, toks.data(), toks.size() * 4);

@@ -46,6 +46,12 @@ def middle():
                                                         dict(mixer=mixer(heads=2, dim=160, rot_dim=62, vdim=64, kv_rank=200, window=70))])
 
 
+def many():
+    """More heads than one attention block takes; more value tiles than waves, a latent that is no multiple of 512."""
+    return config(width=136, vocab=120, ff=100, layers=[dict(mixer=mixer(heads=37, dim=8, rot_dim=4, vdim=12, kv_rank=40, window=90)),
+                                                        dict(mixer=mixer(heads=12, dim=64, rot_dim=32, vdim=136, kv_rank=448, window=130))])
+
+
 def huge():
     """Past what the matrix-core attention kernels take: the general kernels."""
     return config(width=150, vocab=100, ff=90, layers=[dict(mixer=mixer(heads=3, dim=250, rot_dim=20, vdim=30, kv_rank=70, window=40)),

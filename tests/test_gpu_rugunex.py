@@ -11,13 +11,13 @@ import pytest
 
 import mlx_audio_swift_amd as mas
 from oracle import rugunex as orc
-from rugunex_util import config, huge, middle, mixer, no_branch, odd, rel_rms, row_rel_rms, standout, wide
+from rugunex_util import config, huge, many, middle, mixer, no_branch, odd, rel_rms, row_rel_rms, standout, wide
 from gpu_util import observe
 
 pytestmark = pytest.mark.gpu
 # relative rms error of the logits (mean taken off the reference); rows: of the worst row
 TOL = {"float32": 5e-6, "bfloat16": 1.2e-2}
-SHAPES = {"odd": odd, "wide": wide, "middle": middle, "huge": huge}
+SHAPES = {"odd": odd, "wide": wide, "middle": middle, "many": many, "huge": huge}
 ROOT = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
 
 
