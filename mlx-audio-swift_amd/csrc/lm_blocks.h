@@ -83,7 +83,6 @@ private:
     DevBuf<uint8_t> ph_, pact_, pq_, polat_, phead_;
     DevBuf<bf16_t> pkv_;
     std::map<int, DevBuf<uint8_t>> pattn_;
-    std::map<int, size_t> pattn_rows_;
     DevBuf<int32_t> pids_, pseq_, ppos_, pkey_, pwant_;
     DevBuf<LatentTile> ptiles_;
 

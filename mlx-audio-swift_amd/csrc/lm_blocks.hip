@@ -463,7 +463,6 @@ void LmBlocks::pass(const std::vector<PassEntry>& entries, const std::vector<int
         if (at.n < bytes) { at.alloc(bytes); at.zero(s); }                     // K padding columns: zero from here on
     }
     pids_.alloc(cap); pseq_.alloc(cap); ppos_.alloc(cap);
-    std::vector<int32_t> host;                                                 // residual taps
     size_t ei = 0, done_in_entry = 0, t0 = 0;
     while (t0 < total) {
         const size_t n = std::min(cap, total - t0);
@@ -519,13 +518,9 @@ void LmBlocks::pass(const std::vector<PassEntry>& entries, const std::vector<int
                 HIP_CHECK(hipMemcpyAsync(logits_out + (size_t)wo[k + j] * V, plog_.p + (size_t)j * Vpad, (size_t)V * 4, hipMemcpyDeviceToHost, s));
             HIP_CHECK(hipStreamSynchronize(s));
         }
-        if (last_rows && !last.empty()) {
-            // operand rows are batch rows: gather through a full-width row list (rows of sequences that did not end here keep row 0's place and are
-            // overwritten when theirs ends: every sequence of the call ends in exactly one chunk, so the rows are placed one sequence at a time)
-            for (auto& q : last) {
+        if (last_rows)                                                         // the stream of a request's last token becomes its batch row's
+            for (auto& q : last)
                 HIP_CHECK(hipMemcpyAsync(x_.p + (size_t)q.second * dp, px_.p + (size_t)q.first * dp, (size_t)dp * 4, hipMemcpyDeviceToDevice, s));
-            }
-        }
         HIP_CHECK(hipStreamSynchronize(s));                                    // (the host tables above are reused by the next chunk)
         t0 += n;
     }

@@ -1555,6 +1555,7 @@ static void run_generate_attempt(mis_tts* c, const int32_t* prompt_ids, const in
             HIP_CHECK(hipMemcpyAsync(out.tokens.data(), c->tokens_out.p, out.tokens.size() * 4, hipMemcpyDeviceToHost, s));
         }
         HIP_CHECK(hipStreamSynchronize(s));
+        if (c->blocks) HIP_CHECK(copy_now(c->blk_pos.data(), c->pos_next.p, (size_t)batch * 4, hipMemcpyDeviceToHost));     // rows stand behind what was generated
         if (collect_hidden) {                                // the graphs reference hid_count / hidden: never reuse them after this call
             destroy_graphs(c);
             c->graph_key = 0;

@@ -242,6 +242,10 @@ def test_greedy_generation(shape, compute, slack):
         assert len(a) == 40 and np.array_equal(a, b)
         margin, scale = greedy_margin(cfg, W, p, a)
         assert observe(f"greedy_margin_{compute}", float(margin.max() / scale), slack)
+    # the loop has run its layers on every generated id: the rows stand behind them
+    more = m.extend([(1, [int(first[1][0])])])
+    ref = orc.forward(cfg, W, list(prompts[1]) + [int(x) for x in again[1]] + [int(first[1][0])])[-1:]
+    check(more, ref, compute)
     # eager: the step function fed with the same ids chooses the same ones (float32: exactly)
     m.reset(1, 128)
     lg = m.extend([(0, prompts[1])])
