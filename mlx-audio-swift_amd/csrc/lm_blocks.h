@@ -6,15 +6,31 @@
 #include <memory>
 #include <set>
 #include "lm_latent.h"
+#include "lm_mixers.h"
 
 // ---- configuration
 struct LatentMixerSpec { int heads = 0, dim = 0, rot_dim = 0, vdim = 0, kv_rank = 0, window = 0; float scale = 1.0f; RotarySpec rot; };
-struct BlockSpec { LatentMixerSpec mix; int ff = 0 /* 0: no feed-forward */; int weights_of = -1; };
+struct GroupedMixerSpec { int heads = 0, kv_heads = 0, dim = 0, vdim = 0, window = 0, keep = 0; float scale = 1.0f; RotarySpec rot; };
+struct RecurMixerSpec { int width = 0, blocks = 0, conv = 0; };
+struct DecayMixerSpec { int heads = 0, dim = 0, vdim = 0; std::vector<float> decay; };
+// BLOCK_LATENT: one norm, mixer and feed-forward side by side, each with a layer scale.  The others: mixer, then feed-forward, each with a norm
+// before it and one behind it; BLOCK_DECAY mixes with `decay`, BLOCK_PARALLEL with left_scale * `grouped` + right_scale * `recur`.
+enum { BLOCK_LATENT = 0, BLOCK_DECAY = 1, BLOCK_PARALLEL = 2 };
+struct BlockSpec {
+    int kind = BLOCK_LATENT;
+    LatentMixerSpec mix; GroupedMixerSpec grouped; RecurMixerSpec recur; DecayMixerSpec decay;
+    float left_scale = 1.0f, right_scale = 1.0f;
+    int ff = 0 /* 0: no feed-forward */;
+    int weights_of = -1;        // run whose weights this one uses (-1: its own)
+    int index = 0;              // place in config.json's list: the tensors' prefix
+};
 struct BlockModelSpec {
     std::string architecture;
     int width = 0, vocab = 0;
     float eps = 1e-6f, logit_scale = 1.0f, softcap = 0.0f;
-    std::vector<BlockSpec> layers;
+    bool embed_norm = true;     // the embedding goes through a norm of its own
+    float norm_add = 0.0f;      // added to the weights of the norms over the width
+    std::vector<BlockSpec> layers;      // in the order they run; a layer that runs again is listed again, with its own cache or state
 };
 // architectures this engine serves, by config.json "architecture"
 bool block_architecture_known(const std::string& name);
@@ -25,6 +41,9 @@ struct PassEntry { int seq, pos0, n; };
 
 // Device state of the batch rows, owned by the engine
 struct BlockRows { const int32_t* ids; const uint8_t* active; int32_t *pos_cur, *pos_next; };
+
+int pad_k(int k);                // K of a GEMM operand
+GemmF32 gemm32(const void* X, int ldx, const bf16_t* W, float* out, int ldo, int M, int N, int K, int epi);
 
 class LmBlocks {
 public:
@@ -61,8 +80,16 @@ private:
         DevBuf<bf16_t> uk_t;            // packed per head [Rp / 16][np / 32]  (absorbed form)
         DevBuf<bf16_t> ukv;             // packed [(H np + H vp) / 16][Rp / 32] (expanded form; its value part serves the absorbed form too)
         DevBuf<bf16_t> wo, wdown;       // packed [dp / 16][Ko / 32], [dp / 16][ffp / 32]
+        // BLOCK_DECAY, BLOCK_PARALLEL (lm_blocks_mixed.hip).  w1 holds the mixer's input projections alone, wo both sides' output projections along K
+        DevBuf<bf16_t> norm1b, norm2, norm2b, wgu /* gate and up tiles in turn */, bias1, bias_o, wo_rows, mix_norm, qn, kn, sink, conv, conv_b, ra, ri, ra_b, ri_b;
+        DevBuf<float> decay, recur_c;
     };
-    struct Layer { LatentDims D; int owner, ffp, Nqkv, Ko, shares = 1, s1 = 1, s2 = 0, rope = 0; };
+    struct Layer {
+        LatentDims D; int owner, ffp, Nqkv, Ko, shares = 1, s1 = 1, s2 = 0, rope = 0;
+        int kind = BLOCK_LATENT, KR = 0 /* first operand column of the right side */;
+        int oq = 0, ok = 0, ov = 0, og = 0, oy = 0, ox = 0;      // columns of the input projections
+        GroupedDims A; RecurDims R; DecayDims S;
+    };
     std::vector<Layer> layers_;
     std::vector<std::unique_ptr<Weights>> w_;
     std::set<std::string> loaded_;
@@ -73,24 +100,43 @@ private:
 
     int batch_ = 0, Mpad_ = 0, Smax_ = 0, rope_len_ = 0;
     std::vector<std::unique_ptr<DevBuf<uint8_t>>> cache_;
+    std::vector<std::unique_ptr<DevBuf<float>>> state_;          // recurrent state (and convolution history) of a layer run
     // step buffers; bf16 ones hold float32 in the 32-bit mode (sized in bytes)
     DevBuf<float> x_, qkv_, part_, share_ml_, logits_;
     DevBuf<bf16_t> share_;
     DevBuf<uint8_t> h_, act_, q_, olat_;
-    std::map<int, DevBuf<uint8_t>> attn_;          // per H v: the columns up to the K padding stay zero
+    std::map<std::pair<int, int>, DevBuf<uint8_t>> attn_;        // per columns in use: those between and up to the K padding stay zero
     // pass buffers
     DevBuf<float> px_, pqkv_, plog_;
     DevBuf<uint8_t> ph_, pact_, pq_, polat_, phead_;
     DevBuf<bf16_t> pkv_;
-    std::map<int, DevBuf<uint8_t>> pattn_;
-    DevBuf<int32_t> pids_, pseq_, ppos_, pkey_, pwant_;
+    std::map<std::pair<int, int>, DevBuf<uint8_t>> pattn_;
+    DevBuf<int32_t> pids_, pseq_, ppos_, ppos0_, pkey_, pwant_;
     DevBuf<LatentTile> ptiles_;
+    DevBuf<RowSpan> pspans_;
+    // what the mixers of a step / a pass leave behind each other
+    struct MixBuffers { DevBuf<float> u, raw_r, raw_g, ss, gu, part; } mix_, pmix_;
+    // rows of one pass as the mixers see them
+    struct MixRows { RowTable rows; const int32_t* pos0; SpanTable spans; int M, n_spans; };
 
     int esz() const { return f32 ? 4 : 2; }
     const Weights& W(int li) const { return *w_[layers_[li].owner]; }
     void place(const bf16_t* src, int64_t N, int64_t K, int part1, int part2, int g_out, int off2, int Np, int Kp, hipStream_t s);
     Operand operand(void* p, int ld, int rows_padded, bool packed) const;
     LatentRows latent_rows(int li, const float* qkv, void* q, bool expanded, const RowTable& rows) const;
+    std::pair<int, int> columns(int li) const;
+    void norm_row(DevBuf<bf16_t>& dst, const bf16_t* src, int n, int padded, hipStream_t s);
+    void pack_rows(DevBuf<bf16_t>& dst, size_t total, int Np, int Kp, int tile0, int stride, hipStream_t s);
+    // BLOCK_DECAY, BLOCK_PARALLEL
+    void mixed_layer(int li);
+    void mixed_tensors(int li, std::vector<std::pair<std::string, std::vector<int64_t>>>& t) const;
+    void mixed_set(int li, const std::string& t, const bf16_t* src, const std::vector<int64_t>& shape, hipStream_t s);
+    double mixed_weight_bytes(int li) const;
+    void mixed_reset(int li, hipStream_t s);
+    void mixed_buffers(MixBuffers& b, int rows, hipStream_t s);
+    void mixer(int li, const float* proj, void* q, const Operand& out, const MixRows& r, MixBuffers& b, hipStream_t s);
+    void mixed_step_layer(int li, const BlockRows& r, hipStream_t s);
+    void mixed_pass_layer(int li, const MixRows& r, hipStream_t s);
     const bf16_t* norm_after(int li) const { return li + 1 < L ? W(li + 1).norm1.p : g_final_.p; }
     void step_layer(int li, const BlockRows& r, hipStream_t s);
     void pass_layer(int li, int M, const RowTable& rows, int n_tiles, int Mk, hipStream_t s);

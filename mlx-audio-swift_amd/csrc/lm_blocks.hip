@@ -7,13 +7,14 @@
 // launch -> x += ls1 sum + ls2 sum, norm for the next layer.  The residual stream, scores, norms and rotations are float32.
 // Prompt pass: rows = tokens of all requests, (sequence, position) per row; k_gemm_pf GEMMs, keys and values expanded from the latent
 // cache for the chunk's keys and the window before it, both projections added to the stream in their epilogues.
+// Layers that run one sublayer after the other (BLOCK_DECAY, BLOCK_PARALLEL): lm_blocks_mixed.hip.
 #include <math.h>
 #include <string.h>
 #include <algorithm>
 #include "lm_blocks.h"
 
 // ============================================================================ configuration
-bool block_architecture_known(const std::string& name) { return name == "Rugunex"; }
+bool block_architecture_known(const std::string& name) { return name == "Rugunex" || name == "Vamunex"; }
 
 static const JsonValue& need(const JsonValue& o, const char* key, const char* where) {
     const JsonValue* v = o.get(key);
@@ -51,33 +52,78 @@ static LatentMixerSpec parse_latent_mixer(const JsonValue& m) {
     MIS_REQUIRE(x.rot.dims >= 0 && x.rot.dims % 2 == 0 && x.rot.dims <= x.rot_dim && x.rot.base > 0, MIS_ERR_INVALID_INPUT, "latent attention: bad rotary sizes");
     return x;
 }
-BlockModelSpec parse_block_model(const JsonValue& j) {
-    MIS_REQUIRE(j.type == JsonValue::OBJ, MIS_ERR_INVALID_INPUT, "config.json is not an object");
-    BlockModelSpec sp;
-    const JsonValue& a = need(j, "architecture", "the model");
-    MIS_REQUIRE(a.type == JsonValue::STR && block_architecture_known(a.str), MIS_ERR_INVALID_INPUT, "unknown architecture '%s'", a.str.c_str());
-    sp.architecture = a.str;
-    sp.width = (int)need_num(j, "width", "the model");
-    sp.vocab = (int)need_num(j, "vocab", "the model");
-    sp.eps = (float)need_num(need(j, "norm", "the model"), "eps", "norm");
-    sp.logit_scale = (float)j.number_or("logit_scale", 1.0);
-    sp.softcap = (float)j.number_or("logit_softcap", 0.0);
-    MIS_REQUIRE(sp.width >= 1 && sp.width <= 16384 && sp.vocab >= 1, MIS_ERR_INVALID_INPUT, "bad model width or vocabulary");
-    const JsonValue& ls = need(j, "layers", "the model");
-    MIS_REQUIRE(ls.type == JsonValue::ARR && !ls.arr.empty(), MIS_ERR_INVALID_INPUT, "config.json: 'layers' is empty");
+static RotarySpec parse_rotary(const JsonValue& m) {
+    RotarySpec r;
+    const JsonValue* rot = m.get("rot");
+    if (!rot || rot->type != JsonValue::OBJ) return r;
+    r.dims = (int)need_num(*rot, "dims", "rot");
+    r.base = need_num(*rot, "base", "rot");
+    return r;
+}
+static GroupedMixerSpec parse_grouped_mixer(const JsonValue& m) {
+    GroupedMixerSpec x;
+    x.heads = (int)need_num(m, "heads", "mixer");
+    x.kv_heads = (int)need_num(m, "kv_heads", "mixer");
+    x.dim = (int)need_num(m, "dim", "mixer");
+    x.vdim = (int)need_num(m, "vdim", "mixer");
+    x.scale = (float)need_num(m, "scale", "mixer");
+    const JsonValue* mask = m.get("mask");
+    if (mask && mask->type == JsonValue::OBJ) {
+        x.window = (int)mask->number_or("size", 0);
+        x.keep = (int)mask->number_or("keep_first", 0);
+    }
+    x.rot = parse_rotary(m);
+    MIS_REQUIRE(x.heads >= 1 && x.kv_heads >= 1 && x.heads % x.kv_heads == 0 && x.dim >= 1 && x.vdim >= 1 && x.window >= 0 && x.keep >= 0, MIS_ERR_INVALID_INPUT,
+                "grouped attention: bad sizes");
+    MIS_REQUIRE(x.rot.dims >= 0 && x.rot.dims % 2 == 0 && x.rot.dims <= x.dim && x.rot.base > 0, MIS_ERR_INVALID_INPUT, "grouped attention: bad rotary sizes");
+    return x;
+}
+static RecurMixerSpec parse_recur_mixer(const JsonValue& m) {
+    RecurMixerSpec x;
+    x.width = (int)need_num(m, "width", "mixer");
+    x.blocks = (int)need_num(m, "blocks", "mixer");
+    x.conv = (int)need_num(m, "conv", "mixer");
+    MIS_REQUIRE(x.width >= 1 && x.blocks >= 1 && x.width % x.blocks == 0 && x.conv >= 1, MIS_ERR_INVALID_INPUT, "gated recurrence: bad sizes");
+    return x;
+}
+static DecayMixerSpec parse_decay_mixer(const JsonValue& m) {
+    DecayMixerSpec x;
+    x.heads = (int)need_num(m, "heads", "mixer");
+    x.dim = (int)need_num(m, "dim", "mixer");
+    x.vdim = (int)need_num(m, "vdim", "mixer");
+    const JsonValue& d = need(m, "decay", "mixer");
+    MIS_REQUIRE(x.heads >= 1 && x.dim >= 1 && x.vdim >= 1, MIS_ERR_INVALID_INPUT, "lightning attention: bad sizes");
+    MIS_REQUIRE(d.type == JsonValue::ARR && (int)d.arr.size() == x.heads, MIS_ERR_INVALID_INPUT, "lightning attention: 'decay' needs one number per head");
+    for (auto& v : d.arr) {
+        MIS_REQUIRE(v.type == JsonValue::NUM && v.num >= 0.0 && v.num <= 1.0, MIS_ERR_INVALID_INPUT, "lightning attention: 'decay' outside 0 .. 1");
+        x.decay.push_back((float)v.num);
+    }
+    return x;
+}
+// the feed-forward's width (0: none)
+static int parse_mlp(const JsonValue& layer, int i) {
+    const JsonValue* mlp = layer.get("mlp");
+    if (!mlp || mlp->type != JsonValue::OBJ) return 0;
+    const JsonValue* kind = mlp->get("kind");
+    MIS_REQUIRE(!kind || (kind->type == JsonValue::STR && kind->str == "dense"), MIS_ERR_INVALID_INPUT, "layer %d: unknown feed-forward kind", i);
+    const int ff = (int)need_num(*mlp, "ff", "mlp");
+    MIS_REQUIRE(ff >= 1, MIS_ERR_INVALID_INPUT, "layer %d: bad feed-forward size", i);
+    return ff;
+}
+static const std::string& layer_type(const JsonValue& e, int i) {
+    const JsonValue& type = need(e, "type", "a layer");
+    MIS_REQUIRE(type.type == JsonValue::STR, MIS_ERR_INVALID_INPUT, "layer %d: 'type' is not a string", i);
+    return type.str;
+}
+static void parse_rugunex_layers(const JsonValue& ls, BlockModelSpec& sp) {
     for (size_t i = 0; i < ls.arr.size(); ++i) {
         const JsonValue& e = ls.arr[i];
-        const JsonValue& type = need(e, "type", "a layer");
-        MIS_REQUIRE(type.type == JsonValue::STR && type.str == "latent_attention", MIS_ERR_INVALID_INPUT, "layer %d: unknown type '%s'", (int)i, type.str.c_str());
+        const std::string& type = layer_type(e, (int)i);
+        MIS_REQUIRE(type == "latent_attention", MIS_ERR_INVALID_INPUT, "layer %d: unknown type '%s'", (int)i, type.c_str());
         BlockSpec b;
+        b.index = (int)i;
         b.mix = parse_latent_mixer(need(e, "mixer", "a layer"));
-        const JsonValue* mlp = e.get("mlp");
-        if (mlp && mlp->type == JsonValue::OBJ) {
-            const JsonValue* kind = mlp->get("kind");
-            MIS_REQUIRE(!kind || (kind->type == JsonValue::STR && kind->str == "dense"), MIS_ERR_INVALID_INPUT, "layer %d: unknown feed-forward kind", (int)i);
-            b.ff = (int)need_num(*mlp, "ff", "mlp");
-            MIS_REQUIRE(b.ff >= 1, MIS_ERR_INVALID_INPUT, "layer %d: bad feed-forward size", (int)i);
-        }
+        b.ff = parse_mlp(e, (int)i);
         const JsonValue* wo = e.get("weights_of");
         if (!wo && e.get("mixer")) wo = e.get("mixer")->get("weights_of");
         if (wo && wo->type == JsonValue::NUM) {
@@ -96,25 +142,94 @@ BlockModelSpec parse_block_model(const JsonValue& j) {
                     MIS_ERR_INVALID_INPUT, "layer %d: sizes differ from those of the layer whose weights it uses", (int)i);
         sp.layers[i].weights_of = o;
     }
+}
+static void parse_vamunex_layers(const JsonValue& j, const JsonValue& ls, BlockModelSpec& sp) {
+    const int n = (int)ls.arr.size();
+    std::vector<BlockSpec> one;
+    for (int i = 0; i < n; ++i) {
+        const JsonValue& e = ls.arr[i];
+        const std::string& type = layer_type(e, i);
+        const JsonValue& m = need(e, "mixer", "a layer");
+        BlockSpec b;
+        b.index = i;
+        if (type == "lightning") {
+            b.kind = BLOCK_DECAY;
+            b.decay = parse_decay_mixer(m);
+        } else {
+            MIS_REQUIRE(type == "parallel", MIS_ERR_INVALID_INPUT, "layer %d: unknown type '%s'", i, type.c_str());
+            b.kind = BLOCK_PARALLEL;
+            b.grouped = parse_grouped_mixer(need(m, "left", "mixer"));
+            b.recur = parse_recur_mixer(need(m, "right", "mixer"));
+            b.left_scale = (float)need_num(m, "left_scale", "mixer");
+            b.right_scale = (float)need_num(m, "right_scale", "mixer");
+        }
+        b.ff = parse_mlp(e, i);
+        one.push_back(b);
+    }
+    int start = 0, stop = 0, times = 1;
+    if (const JsonValue* lp = j.get("loop"))
+        if (lp->type == JsonValue::OBJ) {
+            start = (int)need_num(*lp, "start", "loop"); stop = (int)need_num(*lp, "stop", "loop"); times = (int)need_num(*lp, "times", "loop");
+            MIS_REQUIRE(start >= 0 && start <= stop && stop <= n && times >= 1, MIS_ERR_INVALID_INPUT, "config.json: bad 'loop'");
+        }
+    std::vector<int> first(n, -1);
+    auto run = [&](int i) {
+        BlockSpec b = one[i];
+        b.weights_of = first[i];
+        if (first[i] < 0) first[i] = (int)sp.layers.size();
+        sp.layers.push_back(b);
+    };
+    for (int i = 0; i < start; ++i) run(i);
+    for (int t = 0; t < times; ++t) for (int i = start; i < stop; ++i) run(i);
+    for (int i = stop; i < n; ++i) run(i);
+}
+BlockModelSpec parse_block_model(const JsonValue& j) {
+    MIS_REQUIRE(j.type == JsonValue::OBJ, MIS_ERR_INVALID_INPUT, "config.json is not an object");
+    BlockModelSpec sp;
+    const JsonValue& a = need(j, "architecture", "the model");
+    MIS_REQUIRE(a.type == JsonValue::STR && block_architecture_known(a.str), MIS_ERR_INVALID_INPUT, "unknown architecture '%s'", a.str.c_str());
+    sp.architecture = a.str;
+    sp.width = (int)need_num(j, "width", "the model");
+    sp.vocab = (int)need_num(j, "vocab", "the model");
+    sp.eps = (float)need_num(need(j, "norm", "the model"), "eps", "norm");
+    MIS_REQUIRE(sp.width >= 1 && sp.width <= 16384 && sp.vocab >= 1, MIS_ERR_INVALID_INPUT, "bad model width or vocabulary");
+    const JsonValue& ls = need(j, "layers", "the model");
+    MIS_REQUIRE(ls.type == JsonValue::ARR && !ls.arr.empty(), MIS_ERR_INVALID_INPUT, "config.json: 'layers' is empty");
+    if (sp.architecture == "Vamunex") {
+        sp.embed_norm = false;
+        sp.norm_add = 1.0f;
+        parse_vamunex_layers(j, ls, sp);
+    } else {
+        sp.logit_scale = (float)j.number_or("logit_scale", 1.0);
+        sp.softcap = (float)j.number_or("logit_softcap", 0.0);
+        parse_rugunex_layers(ls, sp);
+    }
     return sp;
 }
 
-static int pad_k(int k) { return std::max(128, (int)round_up(k, 64)); }        // K of a GEMM operand (k_gemm_pf: whole 64-column steps, two at least)
+int pad_k(int k) { return std::max(128, (int)round_up(k, 64)); }        // K of a GEMM operand (k_gemm_pf: whole 64-column steps, two at least)
 
 LmBlocks::LmBlocks(const BlockModelSpec& sp, bool f32_) : spec(sp), f32(f32_) {
     d = sp.width; dp = pad_k(d); V = sp.vocab; Vpad = (int)round_up(V, 16); L = (int)sp.layers.size();
     for (int i = 0; i < L; ++i) {
         const BlockSpec& b = sp.layers[i];
         Layer l{};
-        l.D = latent_dims(b.mix.heads, b.mix.dim, b.mix.rot_dim, b.mix.vdim, b.mix.kv_rank, b.mix.window, b.mix.rot.dims, b.mix.scale, sp.eps);
+        l.kind = b.kind;
         l.owner = b.weights_of >= 0 ? b.weights_of : i;
         l.ffp = b.ff > 0 ? pad_k(b.ff) : 0;
+        const RotarySpec& rot = b.kind == BLOCK_PARALLEL ? b.grouped.rot : b.mix.rot;
+        for (l.rope = 0; l.rope < (int)ropes_.size() && !(ropes_[l.rope].spec == rot); ++l.rope) {}
+        if (l.rope == (int)ropes_.size()) { ropes_.emplace_back(); ropes_.back().spec = rot; }
+        w_.emplace_back(b.weights_of >= 0 ? nullptr : new Weights());
+        if (b.kind != BLOCK_LATENT) {
+            layers_.push_back(l);
+            mixed_layer(i);
+            continue;
+        }
+        l.D = latent_dims(b.mix.heads, b.mix.dim, b.mix.rot_dim, b.mix.vdim, b.mix.kv_rank, b.mix.window, b.mix.rot.dims, b.mix.scale, sp.eps);
         l.Nqkv = l.D.H * (l.D.np + l.D.rp) + l.D.Rp + l.D.rp;
         l.Ko = pad_k(l.D.H * l.D.v);
-        for (l.rope = 0; l.rope < (int)ropes_.size() && !(ropes_[l.rope].spec == b.mix.rot); ++l.rope) {}
-        if (l.rope == (int)ropes_.size()) { ropes_.emplace_back(); ropes_.back().spec = b.mix.rot; }
         layers_.push_back(l);
-        w_.emplace_back(b.weights_of >= 0 ? nullptr : new Weights());
     }
 }
 
@@ -144,9 +259,11 @@ void LmBlocks::place(const bf16_t* src, int64_t N, int64_t K, int part1, int par
 }
 
 std::vector<std::pair<std::string, std::vector<int64_t>>> LmBlocks::tensor_list() const {
-    std::vector<std::pair<std::string, std::vector<int64_t>>> t = {{"embed", {V, d}}, {"embed.norm", {d}}, {"final.norm", {d}}, {"head", {V, d}}};
+    std::vector<std::pair<std::string, std::vector<int64_t>>> t = {{"embed", {V, d}}, {"final.norm", {d}}, {"head", {V, d}}};
+    if (spec.embed_norm) t.push_back({"embed.norm", {d}});
     for (int i = 0; i < L; ++i) {
         if (layers_[i].owner != i) continue;
+        if (layers_[i].kind != BLOCK_LATENT) { mixed_tensors(i, t); continue; }
         const LatentDims& D = layers_[i].D;
         const std::string p = "l" + std::to_string(i) + ".";
         const int ff = spec.layers[i].ff;
@@ -167,24 +284,31 @@ std::vector<std::pair<std::string, std::vector<int64_t>>> LmBlocks::tensor_list(
     return t;
 }
 
+// a vector as one padded row
+void LmBlocks::norm_row(DevBuf<bf16_t>& dst, const bf16_t* src, int n, int padded, hipStream_t s) {
+    dst.alloc(padded);
+    hipLaunchKernelGGL(k_place_rows, dim3(cdiv(padded, 256)), dim3(256), 0, s, src, dst.p, 1, n, 1, 0, 1, 1, 1, padded);
+}
+// the placed rows into a packed matrix of `total` elements, n-tile t at tile0 + t stride
+void LmBlocks::pack_rows(DevBuf<bf16_t>& dst, size_t total, int Np, int Kp, int tile0, int stride, hipStream_t s) {
+    if (!dst.p) { dst.alloc(total); dst.zero(s); }
+    launch_pack_weight(place_.p, dst.p, Np, Kp, Np / 16, stride, tile0, s);
+}
 void LmBlocks::set_tensor(const std::string& name, const bf16_t* src, const std::vector<int64_t>& shape, hipStream_t s) {
     static const std::vector<int64_t> none;
     const std::vector<int64_t>* want = nullptr;
-    for (int i = 0; i < L; ++i)                                                // the second layer scale of a layer without feed-forward scales nothing
-        if (layers_[i].owner == i && !layers_[i].ffp && name == "l" + std::to_string(i) + ".ls2") return;
+    for (int i = 0; i < L; ++i) {                                              // what belongs to the feed-forward a layer does not have scales nothing
+        if (layers_[i].owner != i || layers_[i].ffp) continue;
+        const std::string p = "l" + std::to_string(spec.layers[i].index) + ".";
+        if (layers_[i].kind == BLOCK_LATENT ? name == p + "ls2" : name == p + "norm2" || name == p + "norm2b") return;
+    }
     const auto list = tensor_list();
     for (auto& t : list) if (t.first == name) want = &t.second;
     MIS_REQUIRE(want, MIS_ERR_INVALID_INPUT, "unexpected tensor %s", name.c_str());
     MIS_REQUIRE(*want == shape, MIS_ERR_INVALID_INPUT, "%s shape mismatch", name.c_str());
     const int64_t N = shape[0], K = shape.size() > 1 ? shape[1] : 1;
-    auto vec = [&](DevBuf<bf16_t>& dst, int padded) {                          // a vector as one padded row
-        dst.alloc(padded);
-        hipLaunchKernelGGL(k_place_rows, dim3(cdiv(padded, 256)), dim3(256), 0, s, src, dst.p, 1, (int)N, 1, 0, 1, 1, 1, padded);
-    };
-    auto pack = [&](DevBuf<bf16_t>& dst, size_t total, int Np, int Kp, int tile0) {
-        if (!dst.p) { dst.alloc(total); dst.zero(s); }
-        launch_pack_weight(place_.p, dst.p, Np, Kp, Np / 16, 1, tile0, s);
-    };
+    auto vec = [&](DevBuf<bf16_t>& dst, int padded) { norm_row(dst, src, (int)N, padded, s); };
+    auto pack = [&](DevBuf<bf16_t>& dst, size_t total, int Np, int Kp, int tile0) { pack_rows(dst, total, Np, Kp, tile0, 1, s); };
     if (name == "embed") { place(src, N, K, 1, 0, 1, 1, V, dp, s); emb_.alloc((size_t)V * dp); HIP_CHECK(hipMemcpyAsync(emb_.p, place_.p, (size_t)V * dp * 2, hipMemcpyDeviceToDevice, s)); }
     else if (name == "embed.norm") vec(g_embed_, dp);
     else if (name == "final.norm") vec(g_final_, dp);
@@ -193,7 +317,15 @@ void LmBlocks::set_tensor(const std::string& name, const bf16_t* src, const std:
         const size_t dot = name.find('.');
         const int li = atoi(name.substr(1, dot - 1).c_str());
         const std::string t = name.substr(dot + 1);
-        const Layer& l = layers_[li];
+        int run = 0;                                                            // the run that owns the layer's tensors
+        while (layers_[run].owner != run || spec.layers[run].index != li) ++run;
+        const Layer& l = layers_[run];
+        if (l.kind != BLOCK_LATENT) {
+            mixed_set(run, t, src, shape, s);
+            HIP_CHECK(hipGetLastError());
+            loaded_.insert(name);
+            return;
+        }
         const LatentDims& D = l.D;
         Weights& w = *w_[li];
         const int HQ = D.np + D.rp;
@@ -240,6 +372,7 @@ void LmBlocks::finalize() const {
 double LmBlocks::weight_bytes_per_step() const {
     double b = 2.0 * V * d;
     for (int i = 0; i < L; ++i) {
+        if (layers_[i].kind != BLOCK_LATENT) { b += mixed_weight_bytes(i); continue; }
         const LatentDims& D = layers_[i].D;
         b += 2.0 * ((double)D.H * (D.n + D.r) * d + (double)(D.R + D.r) * d + (double)D.H * (D.n + D.v) * D.R + (double)d * D.H * D.v + 2.0 * d * spec.layers[i].ff);
     }
@@ -247,7 +380,7 @@ double LmBlocks::weight_bytes_per_step() const {
 }
 double LmBlocks::cache_bytes_per_key() const {
     double b = 0;
-    for (auto& l : layers_) b += (double)(l.D.R + l.D.r) * esz();
+    for (auto& l : layers_) b += (l.kind == BLOCK_LATENT ? (double)(l.D.R + l.D.r) : (double)l.A.G * (l.A.D + l.A.E)) * esz();
     return b;
 }
 
@@ -267,14 +400,25 @@ void LmBlocks::reset(int batch, int Smax, hipStream_t s) {
         }
         rope_len_ = Smax;
     }
-    if (same) return;                                                          // (a cache row is written before it is read: nothing to clear)
-    cache_.resize(L);
+    if (same) return;                                                          // (a cache row is written before it is read, a state starts with position 0)
+    cache_.resize(L); state_.resize(L);
     size_t n_qkv = 0, n_act = 0, n_q = 0, n_ol = 0, n_share = 0, n_ml = 0, n_slab = 2;
     const int max_s = dp > 8192 ? 4 : 8;                                       // slabs the residual kernel takes
     for (int i = 0; i < L; ++i) {
         Layer& l = layers_[i];
         const LatentDims& D = l.D;
         if (!cache_[i]) cache_[i].reset(new DevBuf<uint8_t>());
+        if (!state_[i]) state_[i].reset(new DevBuf<float>());
+        if (l.kind != BLOCK_LATENT) {
+            mixed_reset(i, s);
+            n_qkv = std::max(n_qkv, (size_t)l.Nqkv); n_act = std::max(n_act, (size_t)l.ffp);
+            n_q = std::max(n_q, (size_t)l.A.H * l.A.Dp);
+            n_slab = std::max(n_slab, (size_t)std::max(l.s1, l.s2));
+            DevBuf<uint8_t>& at = attn_[columns(i)];
+            at.alloc((size_t)Mpad_ * l.Ko * esz());
+            at.zero(s);
+            continue;
+        }
         cache_[i]->alloc((size_t)batch * Smax * D.CW * esz());
         l.shares = !f32 && latent_decode_mfma_ok(D) ? latent_decode_shares(D, batch, Smax) : 0;
         l.s1 = 1; l.s2 = l.ffp ? 1 : 0;
@@ -285,7 +429,7 @@ void LmBlocks::reset(int batch, int Smax, hipStream_t s) {
         n_share = std::max(n_share, (size_t)l.shares * batch * D.H * D.Rp);
         n_ml = std::max(n_ml, (size_t)l.shares * batch * D.H * 2);
         n_slab = std::max(n_slab, (size_t)(l.s1 + l.s2));
-        DevBuf<uint8_t>& at = attn_[D.H * D.v];
+        DevBuf<uint8_t>& at = attn_[columns(i)];
         at.alloc((size_t)Mpad_ * l.Ko * esz());
         at.zero(s);
     }
@@ -295,9 +439,15 @@ void LmBlocks::reset(int batch, int Smax, hipStream_t s) {
     part_.alloc(n_slab * Mpad_ * dp);
     share_.alloc(n_share); share_ml_.alloc(n_ml);
     logits_.alloc((size_t)Mpad_ * Vpad);
+    mixed_buffers(mix_, Mpad_, s);
     x_.zero(s); h_.zero(s); qkv_.zero(s); act_.zero(s); q_.zero(s); olat_.zero(s); logits_.zero(s);
 }
 
+std::pair<int, int> LmBlocks::columns(int li) const {
+    const Layer& l = layers_[li];
+    if (l.kind == BLOCK_PARALLEL) return {l.A.H * l.A.E, l.R.W};
+    return {l.kind == BLOCK_DECAY ? l.S.H * l.S.E : l.D.H * l.D.v, 0};
+}
 Operand LmBlocks::operand(void* p, int ld, int rows_padded, bool packed) const {
     return Operand{p, f32 ? OPK_F32 : (packed ? OPK_PACKED : OPK_ROWS), ld, std::max(1, rows_padded / 16)};
 }
@@ -346,17 +496,17 @@ void LmBlocks::absorbed_attention(int li, const float* qkv, void* q, void* olat,
 }
 
 // ============================================================================ decode step
-static GemmF32 gemm32(const void* X, int ldx, const bf16_t* W, float* out, int ldo, int M, int N, int K, int epi) {
+GemmF32 gemm32(const void* X, int ldx, const bf16_t* W, float* out, int ldo, int M, int N, int K, int epi) {
     GemmF32 g{};
     g.X = (const float*)X; g.ldx = ldx; g.W = W; g.out = out; g.ldo = ldo; g.M = M; g.NT = N / 16; g.KT = K / 32; g.n_valid = N; g.epi = epi;
     return g;
 }
 void LmBlocks::step_layer(int li, const BlockRows& r, hipStream_t s) {
+    if (layers_[li].kind != BLOCK_LATENT) { mixed_step_layer(li, r, s); return; }
     const Layer& l = layers_[li];
-    const LatentDims& D = l.D;
     const Weights& w = W(li);
     RowTable rows; rows.pos = r.pos_cur; rows.on = r.active;
-    void* at = attn_[D.H * D.v].p;
+    void* at = attn_[columns(li)].p;
     if (f32) {
         launch_gemm_f32(gemm32(h_.p, dp, w.w1.p, qkv_.p, l.Nqkv, batch_, l.Nqkv, dp, F32_STORE), s);
         if (l.ffp) launch_gemm_f32(gemm32(h_.p, dp, w.w1.p + (size_t)l.Nqkv * dp, (float*)act_.p, l.ffp, batch_, l.ffp, dp, F32_RELU2), s);
@@ -380,7 +530,7 @@ void LmBlocks::step_layer(int li, const BlockRows& r, hipStream_t s) {
 }
 void LmBlocks::enqueue_step(const BlockRows& r, hipStream_t s) {
     launch_rows_embed_norm2(emb_.p, r.ids, V, g_embed_.p, W(0).norm1.p, x_.p, operand(h_.p, dp, Mpad_, true), d, dp, spec.eps, batch_, Mpad_, r.active, r.pos_cur,
-                            r.pos_next, s);
+                            r.pos_next, s, spec.norm_add);
     for (int li = 0; li < L; ++li) step_layer(li, r, s);
 }
 // operand rows -> float32 logits [rows][Vpad]
@@ -405,7 +555,7 @@ void LmBlocks::pass_layer(int li, int M, const RowTable& rows, int n_tiles, int 
     const Layer& l = layers_[li];
     const LatentDims& D = l.D;
     const Weights& w = W(li);
-    void* at = pattn_[D.H * D.v].p;
+    void* at = pattn_[columns(li)].p;
     if (f32) {
         launch_gemm_f32(gemm32(ph_.p, dp, w.w1.p, pqkv_.p, l.Nqkv, M, l.Nqkv, dp, F32_STORE), s);
         if (l.ffp) launch_gemm_f32(gemm32(ph_.p, dp, w.w1.p + (size_t)l.Nqkv * dp, (float*)pact_.p, l.ffp, M, l.ffp, dp, F32_RELU2), s);
@@ -444,38 +594,44 @@ void LmBlocks::pass(const std::vector<PassEntry>& entries, const std::vector<int
     int max_window = 0;
     bool all_keys = false, expanded = !f32;
     size_t n_qkv = 0, n_act = 1, n_q = 0, n_ol = 1, n_kv = 0;
+    bool latent = false;
     for (auto& l : layers_) {
+        n_qkv = std::max(n_qkv, (size_t)l.Nqkv); n_act = std::max(n_act, (size_t)l.ffp);
+        if (l.kind != BLOCK_LATENT) { n_q = std::max(n_q, (size_t)l.A.H * l.A.Dp); continue; }
+        latent = true;
         const bool ex = !f32 && latent_prefill_mfma_ok(l.D);
         expanded = expanded && ex;
         all_keys = all_keys || l.D.window <= 0;
         max_window = std::max(max_window, l.D.window);
-        n_qkv = std::max(n_qkv, (size_t)l.Nqkv); n_act = std::max(n_act, (size_t)l.ffp);
         n_q = std::max(n_q, (size_t)l.D.H * std::max(l.D.CW, l.D.DK)); n_ol = std::max(n_ol, (size_t)l.D.H * l.D.Rp);
         n_kv = std::max(n_kv, (size_t)l.D.H * (l.D.np + l.D.vp));
     }
     const size_t cap = std::min<size_t>(total, std::max(1, pass_rows));
     px_.alloc(cap * dp); ph_.alloc(cap * dp * esz()); pqkv_.alloc(cap * n_qkv); pact_.alloc(cap * n_act * esz());
     pq_.alloc(cap * n_q * esz());
-    if (!expanded) polat_.alloc(cap * n_ol * esz());
-    for (auto& l : layers_) {
-        DevBuf<uint8_t>& at = pattn_[l.D.H * l.D.v];
-        const size_t bytes = cap * l.Ko * esz();
+    if (latent && !expanded) polat_.alloc(cap * n_ol * esz());
+    mixed_buffers(pmix_, (int)cap, s);
+    for (int i = 0; i < L; ++i) {
+        DevBuf<uint8_t>& at = pattn_[columns(i)];
+        const size_t bytes = cap * layers_[i].Ko * esz();
         if (at.n < bytes) { at.alloc(bytes); at.zero(s); }                     // K padding columns: zero from here on
     }
-    pids_.alloc(cap); pseq_.alloc(cap); ppos_.alloc(cap);
+    pids_.alloc(cap); pseq_.alloc(cap); ppos_.alloc(cap); ppos0_.alloc(cap);
     size_t ei = 0, done_in_entry = 0, t0 = 0;
     while (t0 < total) {
         const size_t n = std::min(cap, total - t0);
-        std::vector<int32_t> seq(n), pos(n), keys;
+        std::vector<int32_t> seq(n), pos(n), pos0(n), keys;
         std::vector<LatentTile> tiles;
+        std::vector<RowSpan> spans;
         std::vector<std::pair<int32_t, int32_t>> last;                         // (row, sequence) of entries that end in this chunk
         size_t at = 0;
         while (at < n) {
             const PassEntry& e = entries[ei];
             const size_t take = std::min(n - at, (size_t)e.n - done_in_entry);
             const int p0 = e.pos0 + (int)done_in_entry;
-            for (size_t k = 0; k < take; ++k) { seq[at + k] = e.seq; pos[at + k] = p0 + (int)k; }
-            if (!f32) {
+            for (size_t k = 0; k < take; ++k) { seq[at + k] = e.seq; pos[at + k] = p0 + (int)k; pos0[at + k] = p0; }
+            spans.push_back(RowSpan{(int)at, (int)take, e.seq, p0});
+            if (!f32 && latent) {
                 const int kp0 = all_keys ? 0 : std::max(0, p0 - max_window + 1), krow0 = (int)keys.size();
                 for (int p = kp0; p < p0 + (int)take; ++p) keys.push_back(e.seq * Smax_ + p);
                 for (size_t q = 0; q < take; q += LATENT_QT)
@@ -487,17 +643,23 @@ void LmBlocks::pass(const std::vector<PassEntry>& entries, const std::vector<int
         HIP_CHECK(hipMemcpyAsync(pids_.p, tokens.data() + t0, n * 4, hipMemcpyHostToDevice, s));
         HIP_CHECK(hipMemcpyAsync(pseq_.p, seq.data(), n * 4, hipMemcpyHostToDevice, s));
         HIP_CHECK(hipMemcpyAsync(ppos_.p, pos.data(), n * 4, hipMemcpyHostToDevice, s));
-        if (!f32) {
+        HIP_CHECK(hipMemcpyAsync(ppos0_.p, pos0.data(), n * 4, hipMemcpyHostToDevice, s));
+        pspans_.alloc(spans.size());
+        HIP_CHECK(hipMemcpyAsync(pspans_.p, spans.data(), spans.size() * sizeof(RowSpan), hipMemcpyHostToDevice, s));
+        if (!f32 && latent) {
             pkey_.alloc(keys.size()); ptiles_.alloc(tiles.size());
             pkv_.alloc(keys.size() * n_kv);
             HIP_CHECK(hipMemcpyAsync(pkey_.p, keys.data(), keys.size() * 4, hipMemcpyHostToDevice, s));
             HIP_CHECK(hipMemcpyAsync(ptiles_.p, tiles.data(), tiles.size() * sizeof(LatentTile), hipMemcpyHostToDevice, s));
         }
         RowTable rows; rows.seq = pseq_.p; rows.pos = ppos_.p;
+        MixRows mr;
+        mr.rows = rows; mr.pos0 = ppos0_.p; mr.spans.span = pspans_.p; mr.M = (int)n; mr.n_spans = (int)spans.size();
         launch_rows_embed_norm2(emb_.p, pids_.p, V, g_embed_.p, W(0).norm1.p, px_.p, operand(ph_.p, dp, 0, false), d, dp, spec.eps, (int)n, (int)n, nullptr, nullptr,
-                                nullptr, s);
+                                nullptr, s, spec.norm_add);
         for (int li = 0; li < L; ++li) {
-            pass_layer(li, (int)n, rows, (int)tiles.size(), (int)keys.size(), s);
+            if (layers_[li].kind != BLOCK_LATENT) mixed_pass_layer(li, mr, s);
+            else pass_layer(li, (int)n, rows, (int)tiles.size(), (int)keys.size(), s);
             if (residual_out)
                 HIP_CHECK(hipMemcpy2DAsync(residual_out + ((size_t)li * total + t0) * d, (size_t)d * 4, px_.p, (size_t)dp * 4, (size_t)d * 4, n, hipMemcpyDeviceToHost, s));
         }
@@ -512,7 +674,7 @@ void LmBlocks::pass(const std::vector<PassEntry>& entries, const std::vector<int
             pwant_.alloc(512); phead_.alloc((size_t)slice * dp * esz()); plog_.alloc((size_t)slice * Vpad);
             HIP_CHECK(hipMemcpyAsync(pwant_.p, wr.data() + k, m * 4, hipMemcpyHostToDevice, s));
             if (packed) phead_.zero(s);
-            launch_gather_norm(px_.p, pwant_.p, g_final_.p, operand(phead_.p, dp, mp, packed), d, dp, spec.eps, m, s);
+            launch_gather_norm(px_.p, pwant_.p, g_final_.p, operand(phead_.p, dp, mp, packed), d, dp, spec.eps, m, s, spec.norm_add);
             head_rows(phead_.p, packed, m, mp, plog_.p, s);
             for (int j = 0; j < m; ++j)
                 HIP_CHECK(hipMemcpyAsync(logits_out + (size_t)wo[k + j] * V, plog_.p + (size_t)j * Vpad, (size_t)V * 4, hipMemcpyDeviceToHost, s));
@@ -524,7 +686,7 @@ void LmBlocks::pass(const std::vector<PassEntry>& entries, const std::vector<int
         HIP_CHECK(hipStreamSynchronize(s));                                    // (the host tables above are reused by the next chunk)
         t0 += n;
     }
-    if (last_rows) launch_gather_norm(x_.p, nullptr, g_final_.p, operand(h_.p, dp, Mpad_, true), d, dp, spec.eps, f32 ? batch_ : Mpad_, s);
+    if (last_rows) launch_gather_norm(x_.p, nullptr, g_final_.p, operand(h_.p, dp, Mpad_, true), d, dp, spec.eps, f32 ? batch_ : Mpad_, s, spec.norm_add);
     HIP_CHECK(hipGetLastError());
 }
 

@@ -10,7 +10,8 @@ __host__ __device__ __forceinline__ size_t xpk_index(int m, int k, int MT) {
 enum { EPI_PARTIAL = 0, EPI_BF16 = 1, EPI_SILU_MUL = 2, EPI_GELU_PACKED = 3, EPI_SILU_PACKED = 4,
        EPI_SPLIT_RELU2 = 5,      // tiles below GemmExtra::split: float32 sums; the others: T(relu(y)^2) in the packed layout (out2)
        EPI_SOFTCAP = 6,          // float32: cap tanh(scale y / cap) (cap <= 0: scale y)
-       EPI_DUAL = 7 };           // two products of one output width in one launch: slabs [0, s1) = X W^T, slabs [s1, S) = x2 w2^T (kt2 k-tiles)
+       EPI_DUAL = 7,           // two products of one output width in one launch: slabs [0, s1) = X W^T, slabs [s1, S) = x2 w2^T (kt2 k-tiles)
+       EPI_SWIGLU = 8 };         // EPI_SILU_MUL in float32 up to one rounding: T(silu(gate) up)
 struct GemmExtra {
     void* out2 = nullptr; int split = 0; float scale = 1.0f, cap = 0.0f;
     const bf16_t *w2 = nullptr, *x2 = nullptr; int kt2 = 0, s1 = 0;
@@ -62,7 +63,8 @@ enum { PF_F32 = 0, PF_RESID = 1, PF_SILU = 2,
        PF_SPLIT_RELU2 = 3,       // tiles below PfExtra::split: float32 [M][ldc]; the others: T(relu(y)^2) bf16 row-major [M][ld2] at out2
        PF_SCALED_ADD = 4,        // float32 C[M][ldc] += ls[n] * y
        PF_ROWS_BF16 = 5,         // bf16 row-major [M][ldc]; rows of X gathered: row m at X + xrow[m] * ldx
-       PF_SOFTCAP = 6 };         // float32 [M][ldc]: cap tanh(scale y / cap)
+       PF_SOFTCAP = 6,           // float32 [M][ldc]: cap tanh(scale y / cap)
+       PF_SWIGLU = 7 };          // PF_SILU in float32 up to one rounding
 struct PfExtra { int ldx = 0; const int32_t* xrow = nullptr; int ldc = 0; void* out2 = nullptr; int split = 0, ld2 = 0; const bf16_t* ls = nullptr; float scale = 1.0f, cap = 0.0f; };
 void launch_gemm_pf(int epi, const bf16_t* X, const bf16_t* Wp, void* C, int M, int N, int K, hipStream_t s, const PfExtra& ex = PfExtra());
 void launch_pf_embed_rmsnorm(const bf16_t* emb, const int32_t* prompt, const int32_t* lens, int Lmax, int t0, int Tc, int batch, int Mpad, int vocab,

@@ -709,7 +709,7 @@ __device__ __forceinline__ void gemm_epilogue(const f32x4_t (&acc)[R][MT], void*
                 *reinterpret_cast<uint2*>(o + off) = v;
             }
         }
-    } else {   // EPI_SILU_MUL: tile 2t = gate rows, 2t+1 = up rows  (LlamaTTS.swift:283)
+    } else {   // EPI_SILU_MUL, EPI_SWIGLU: tile 2t = gate rows, 2t+1 = up rows  (LlamaTTS.swift:283)
         bf16_t* o = reinterpret_cast<bf16_t*>(out);
 #pragma unroll
         for (int p = 0; p < R / 2; ++p) {                                  // tile pair p of the item: feature tile ntg * R / 2 + p
@@ -720,6 +720,11 @@ __device__ __forceinline__ void gemm_epilogue(const f32x4_t (&acc)[R][MT], void*
                 uint16_t res[4];
 #pragma unroll
                 for (int e = 0; e < 4; ++e) {
+                    if (EPI == EPI_SWIGLU) {
+                        const float gf = acc[2 * p][mt][e];
+                        res[e] = f32_to_bf16(gf / (1.0f + __expf(-gf)) * acc[2 * p + 1][mt][e]);
+                        continue;
+                    }
                     float g = bf16_round_f32(acc[2 * p][mt][e]);
                     float u = bf16_round_f32(acc[2 * p + 1][mt][e]);
                     float sg = bf16_round_f32(1.0f / (1.0f + __expf(-g)));     // T(sigmoid(g))
@@ -750,7 +755,7 @@ template <int MT, int R, int EPI, int KSB, int U>
 __global__ void __launch_bounds__((KSB == 1 ? 4 : KSB) * 64, 2) k_gemm_skinny(const bf16_t* __restrict__ Wp, const bf16_t* __restrict__ X,
                                                      void* __restrict__ out, int NT, int KT, int S, int n_items,
                                                      int N_out, int Mpad, const bf16_t* __restrict__ bias, GemmExtra ex) {
-    static_assert(EPI != EPI_SILU_MUL || (R & 1) == 0, "silu-mul epilogue pairs a gate tile with an up tile");
+    static_assert((EPI != EPI_SILU_MUL && EPI != EPI_SWIGLU) || (R & 1) == 0, "silu-mul epilogue pairs a gate tile with an up tile");
     // k-tiles per register buffer: 4 at R <= 2; 3 or 2 at four n-tiles per wave (4 would spill: 2 x 4 x (4 + 2) fragments + 32 accumulators)
     constexpr int GU = U;
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
@@ -912,8 +917,10 @@ static void launch_gemm_mt(int epi, int R, int ksb, int U, const bf16_t* Wp, con
     GEMM_CASE(EPI_BF16, 2, 4, 4)
     GEMM_CASE(EPI_SILU_MUL, 2, 1, 4)
     GEMM_CASE(EPI_SILU_MUL, 2, 4, 4)
+    GEMM_CASE(EPI_SWIGLU, 2, 4, 4)
     if constexpr (MT <= 2) {                       // four n-tiles per wave: 8 accumulator tiles, U <= 3 (no scratch up to 32 rows)
         GEMM_CASE(EPI_SILU_MUL, 4, 4, 3)
+        GEMM_CASE(EPI_SWIGLU, 4, 4, 3)
         GEMM_CASE(EPI_PARTIAL, 4, 4, 2)
         GEMM_CASE(EPI_PARTIAL, 4, 4, 3)
         GEMM_CASE(EPI_PARTIAL, 4, 2, 2)

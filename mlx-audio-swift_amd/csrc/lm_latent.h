@@ -26,16 +26,22 @@ void rotary_tables_host(const RotarySpec& r, int positions, std::vector<float>& 
 // ---- rows of a pass: row r belongs to sequence seq[r] (null: r) at position pos[r]; on (null: all) = 0 rows do nothing
 struct RowTable { const int32_t* seq = nullptr; const int32_t* pos = nullptr; const uint8_t* on = nullptr; };
 
-// x = rms(E[id]) * g_embed (float32 residual), operand = rms(x) * g_norm.  pos_cur / pos_next non-null: the decode step's position advance.
+// x = rms(E[id]) * g_embed (float32 residual; g_embed null: x = E[id]), operand = rms(x) * (g_norm + g_add).  pos_cur / pos_next non-null: the decode step's position advance.
 void launch_rows_embed_norm2(const bf16_t* emb, const int32_t* ids, int vocab, const bf16_t* g_embed, const bf16_t* g_norm, float* x, const Operand& h,
-                             int d, int dp, float eps, int n_rows, int rows, const uint8_t* on, int32_t* pos_cur, int32_t* pos_next, hipStream_t s);
+                             int d, int dp, float eps, int n_rows, int rows, const uint8_t* on, int32_t* pos_cur, int32_t* pos_next, hipStream_t s,
+                             float g_add = 0.0f);
 // x += ls1 * sum(slabs 0 .. s1 - 1) + ls2 * sum(slabs s1 .. s1 + s2 - 1); operand = rms(x) * g_norm.  Slabs [s1 + s2][slab_rows][dp] float32 (what an
 // EPI_DUAL launch writes), added in slab order; s2 = 0: one branch.
 struct ScaledSlabs { const float* p = nullptr; int s1 = 0, s2 = 0; const bf16_t *ls1 = nullptr, *ls2 = nullptr; };
 void launch_scaled_residual_norm(const ScaledSlabs& a, int slab_rows, float* x, const bf16_t* g_norm, const Operand& h, int d, int dp, float eps, int rows,
                                  hipStream_t s);
-// operand row i = rms(x[row_of[i]]) * g_norm (row_of null: i)
-void launch_gather_norm(const float* x, const int32_t* row_of, const bf16_t* g_norm, const Operand& h, int d, int dp, float eps, int rows, hipStream_t s);
+// operand row i = rms(x[row_of[i]]) * (g_norm + g_add) (row_of null: i)
+void launch_gather_norm(const float* x, const int32_t* row_of, const bf16_t* g_norm, const Operand& h, int d, int dp, float eps, int rows, hipStream_t s,
+                        float g_add = 0.0f);
+// block shape of the kernels that hold one row of the width per block
+int row_cpt(int dp);
+int row_threads(int dp, int cpt);
+void row_check(int dp);
 
 // ---- true-float32 GEMM on the packed bf16 weights (their values are exact in float32): out[m][n] = sum_k X[m][k] W[n][k], per head z
 enum { F32_STORE = 0, F32_RELU2 = 1, F32_ADD_SCALED = 2, F32_SOFTCAP = 3 };

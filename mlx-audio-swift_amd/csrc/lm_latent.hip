@@ -9,6 +9,7 @@
 //                       - (n + r + v) instead of (2 R + r) multiplications per (query, key, head).
 // Scores, the softmax and its weights are float32 in both; the weights enter the matrix cores as bf16 hi + lo pairs.
 #include "lm_latent.h"
+#include "lm_device.h"
 #include <math.h>
 
 // ============================================================================ rotary tables (host)
@@ -62,44 +63,12 @@ LatentDims latent_dims(int H, int n, int r, int v, int R, int window, int rot_di
     return D;
 }
 
-// ============================================================================ small helpers
-__device__ __forceinline__ float lat_block_sum(float v, float* red) {          // any block of whole waves; every thread gets the total
-    v = wave_sum_dpp(v);
-    if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = v;
-    __syncthreads();
-    const int nw = blockDim.x >> 6;
-    float t = 0.0f;
-    for (int i = 0; i < nw; ++i) t += red[i];
-    __syncthreads();
-    return t;
-}
-__device__ __forceinline__ void load4_bf16(const bf16_t* p, float (&o)[4]) {
-    const uint2 q = *reinterpret_cast<const uint2*>(p);
-    o[0] = bf16_to_f32((bf16_t)(q.x & 0xffffu)); o[1] = bf16_to_f32((bf16_t)(q.x >> 16));
-    o[2] = bf16_to_f32((bf16_t)(q.y & 0xffffu)); o[3] = bf16_to_f32((bf16_t)(q.y >> 16));
-}
-__device__ __forceinline__ uint2 pack4_bf16(const float (&v)[4]) {
-    return make_uint2((uint32_t)f32_to_bf16(v[0]) | ((uint32_t)f32_to_bf16(v[1]) << 16), (uint32_t)f32_to_bf16(v[2]) | ((uint32_t)f32_to_bf16(v[3]) << 16));
-}
-// four consecutive columns k .. k + 3 (k % 4 == 0) of operand row m
-__device__ __forceinline__ void operand_store4(const Operand& h, int m, int k, const float (&v)[4]) {
-    if (h.kind == OPK_F32) *reinterpret_cast<float4*>((float*)h.p + (size_t)m * h.ld + k) = make_float4(v[0], v[1], v[2], v[3]);
-    else {
-        bf16_t* o = (bf16_t*)h.p + (h.kind == OPK_PACKED ? xpk_index(m, k, h.MT) : (size_t)m * h.ld + k);
-        *reinterpret_cast<uint2*>(o) = pack4_bf16(v);
-    }
-}
-__device__ __forceinline__ void operand_store1(const Operand& h, int m, int k, float v) {
-    if (h.kind == OPK_F32) ((float*)h.p)[(size_t)m * h.ld + k] = v;
-    else ((bf16_t*)h.p)[h.kind == OPK_PACKED ? xpk_index(m, k, h.MT) : (size_t)m * h.ld + k] = f32_to_bf16(v);
-}
-
 // ============================================================================ embedding, residual + layer scale + norm
 // CPT groups of four columns per thread; columns of the width padding (d .. dp) hold zeros everywhere (weights, tables, stream)
 template <int CPT>
 __global__ void __launch_bounds__(1024) k_rows_embed_norm2(const bf16_t* __restrict__ emb, const int32_t* __restrict__ ids, int vocab,
                                                            const bf16_t* __restrict__ g_embed, const bf16_t* __restrict__ g_norm, float* __restrict__ x,
-                                                           Operand h, int d, int dp, float eps, int n_rows, const uint8_t* __restrict__ on,
+                                                           Operand h, int d, int dp, float eps, float g_add, int n_rows, const uint8_t* __restrict__ on,
                                                            int32_t* __restrict__ pos_cur, int32_t* __restrict__ pos_next) {
     __shared__ float red[16];
     const int m = blockIdx.x, tid = threadIdx.x, nth = blockDim.x, nc = dp >> 2;
@@ -115,7 +84,7 @@ __global__ void __launch_bounds__(1024) k_rows_embed_norm2(const bf16_t* __restr
     for (int g = 0; g < CPT; ++g) {
         const int c = tid + g * nth, cc = c < nc ? c : 0;
         load4_bf16(emb + (size_t)id * dp + 4 * cc, e[g]);
-        load4_bf16(g_embed + 4 * cc, ge[g]);
+        load4_bf16((g_embed ? g_embed : g_norm) + 4 * cc, ge[g]);
         load4_bf16(g_norm + 4 * cc, gn[g]);
 #pragma unroll
         for (int j = 0; j < 4; ++j) ss += c < nc ? e[g][j] * e[g][j] : 0.0f;
@@ -126,7 +95,7 @@ __global__ void __launch_bounds__(1024) k_rows_embed_norm2(const bf16_t* __restr
     for (int g = 0; g < CPT; ++g) {
         const int c = tid + g * nth;
 #pragma unroll
-        for (int j = 0; j < 4; ++j) { e[g][j] = e[g][j] * inv * ge[g][j]; s2 += c < nc ? e[g][j] * e[g][j] : 0.0f; }
+        for (int j = 0; j < 4; ++j) { if (g_embed) e[g][j] = e[g][j] * inv * ge[g][j]; s2 += c < nc ? e[g][j] * e[g][j] : 0.0f; }
         if (c < nc) *reinterpret_cast<float4*>(x + (size_t)m * dp + 4 * c) = make_float4(e[g][0], e[g][1], e[g][2], e[g][3]);
     }
     const float inv2 = 1.0f / sqrtf(lat_block_sum(s2, red) / (float)d + eps);
@@ -135,7 +104,7 @@ __global__ void __launch_bounds__(1024) k_rows_embed_norm2(const bf16_t* __restr
         const int c = tid + g * nth;
         float o[4];
 #pragma unroll
-        for (int j = 0; j < 4; ++j) o[j] = e[g][j] * inv2 * gn[g][j];
+        for (int j = 0; j < 4; ++j) o[j] = e[g][j] * inv2 * (gn[g][j] + g_add);
         if (c < nc) operand_store4(h, m, 4 * c, o);
     }
 }
@@ -143,7 +112,7 @@ __global__ void __launch_bounds__(1024) k_rows_embed_norm2(const bf16_t* __restr
 // SG >= s1 + s2 (clamped, unconditional loads: one round trip for everything the row needs); SG = 0: no slabs, the stream is only normed
 template <int CPT, int SG>
 __global__ void __launch_bounds__(1024) k_scaled_residual_norm(ScaledSlabs A, int slab_rows, float* __restrict__ x, const int32_t* __restrict__ row_of,
-                                                               const bf16_t* __restrict__ g_norm, Operand h, int d, int dp, float eps) {
+                                                               const bf16_t* __restrict__ g_norm, Operand h, int d, int dp, float eps, float g_add) {
     __shared__ float red[16];
     const int m = blockIdx.x, tid = threadIdx.x, nth = blockDim.x, nc = dp >> 2;
     const size_t xr = (size_t)(row_of ? row_of[m] : m) * dp;
@@ -191,29 +160,29 @@ __global__ void __launch_bounds__(1024) k_scaled_residual_norm(ScaledSlabs A, in
         const int c = tid + g * nth;
         float o[4];
 #pragma unroll
-        for (int j = 0; j < 4; ++j) o[j] = v[g][j] * inv * gn[g][j];
+        for (int j = 0; j < 4; ++j) o[j] = v[g][j] * inv * (gn[g][j] + g_add);
         if (c < nc) operand_store4(h, m, 4 * c, o);
     }
 }
 
-static int row_cpt(int dp) { const int nc = dp / 4; return nc <= 1024 ? (nc >= 512 ? 2 : 1) : (nc <= 2048 ? 2 : 4); }
-static int row_threads(int dp, int cpt) { return (int)round_up(cdiv(dp / 4, cpt), 64); }
-static void row_check(int dp) { MIS_REQUIRE(dp % 4 == 0 && dp <= 16384, MIS_ERR_INVALID_INPUT, "model width above 16384"); }
+int row_cpt(int dp) { const int nc = dp / 4; return nc <= 1024 ? (nc >= 512 ? 2 : 1) : (nc <= 2048 ? 2 : 4); }
+int row_threads(int dp, int cpt) { return (int)round_up(cdiv(dp / 4, cpt), 64); }
+void row_check(int dp) { MIS_REQUIRE(dp % 4 == 0 && dp <= 16384, MIS_ERR_INVALID_INPUT, "model width above 16384"); }
 
 void launch_rows_embed_norm2(const bf16_t* emb, const int32_t* ids, int vocab, const bf16_t* g_embed, const bf16_t* g_norm, float* x, const Operand& h,
-                             int d, int dp, float eps, int n_rows, int rows, const uint8_t* on, int32_t* pos_cur, int32_t* pos_next, hipStream_t s) {
+                             int d, int dp, float eps, int n_rows, int rows, const uint8_t* on, int32_t* pos_cur, int32_t* pos_next, hipStream_t s, float g_add) {
     row_check(dp);
     const int cpt = row_cpt(dp), nth = row_threads(dp, cpt);
-#define EMB2(C) hipLaunchKernelGGL((k_rows_embed_norm2<C>), dim3(rows), dim3(nth), 0, s, emb, ids, vocab, g_embed, g_norm, x, h, d, dp, eps, n_rows, on, pos_cur, pos_next)
+#define EMB2(C) hipLaunchKernelGGL((k_rows_embed_norm2<C>), dim3(rows), dim3(nth), 0, s, emb, ids, vocab, g_embed, g_norm, x, h, d, dp, eps, g_add, n_rows, on, pos_cur, pos_next)
     if (cpt == 1) EMB2(1); else if (cpt == 2) EMB2(2); else EMB2(4);
 #undef EMB2
 }
 static void residual_norm(const ScaledSlabs& a, int slab_rows, float* x, const int32_t* row_of, const bf16_t* g_norm, const Operand& h, int d, int dp,
-                          float eps, int rows, hipStream_t s) {
+                          float eps, float g_add, int rows, hipStream_t s) {
     row_check(dp);
     const int cpt = row_cpt(dp), nth = row_threads(dp, cpt), S = a.s1 + a.s2;
     MIS_REQUIRE(S <= (cpt == 4 ? 4 : 8), MIS_ERR_GENERATION_FAILED, "too many split-K slabs");
-#define RN(C, G) hipLaunchKernelGGL((k_scaled_residual_norm<C, G>), dim3(rows), dim3(nth), 0, s, a, slab_rows, x, row_of, g_norm, h, d, dp, eps)
+#define RN(C, G) hipLaunchKernelGGL((k_scaled_residual_norm<C, G>), dim3(rows), dim3(nth), 0, s, a, slab_rows, x, row_of, g_norm, h, d, dp, eps, g_add)
 #define RNC(C) do { if (S == 0) RN(C, 0); else if (S <= 2) RN(C, 2); else if (S <= 4) RN(C, 4); else RN(C, C == 4 ? 4 : 8); } while (0)
     if (cpt == 1) RNC(1); else if (cpt == 2) RNC(2); else RNC(4);
 #undef RNC
@@ -221,10 +190,10 @@ static void residual_norm(const ScaledSlabs& a, int slab_rows, float* x, const i
 }
 void launch_scaled_residual_norm(const ScaledSlabs& a, int slab_rows, float* x, const bf16_t* g_norm, const Operand& h, int d, int dp, float eps, int rows,
                                  hipStream_t s) {
-    residual_norm(a, slab_rows, x, nullptr, g_norm, h, d, dp, eps, rows, s);
+    residual_norm(a, slab_rows, x, nullptr, g_norm, h, d, dp, eps, 0.0f, rows, s);
 }
-void launch_gather_norm(const float* x, const int32_t* row_of, const bf16_t* g_norm, const Operand& h, int d, int dp, float eps, int rows, hipStream_t s) {
-    residual_norm(ScaledSlabs{}, 0, const_cast<float*>(x), row_of, g_norm, h, d, dp, eps, rows, s);
+void launch_gather_norm(const float* x, const int32_t* row_of, const bf16_t* g_norm, const Operand& h, int d, int dp, float eps, int rows, hipStream_t s, float g_add) {
+    residual_norm(ScaledSlabs{}, 0, const_cast<float*>(x), row_of, g_norm, h, d, dp, eps, g_add, rows, s);
 }
 
 // ============================================================================ float32 GEMM (v_mfma_f32_16x16x4_f32)
@@ -283,14 +252,6 @@ void launch_gemm_f32(const GemmF32& g, hipStream_t s) {
 }
 
 // ============================================================================ projections -> cache row and query rows
-__device__ __forceinline__ void put(float* p, float v) { *p = v; }
-__device__ __forceinline__ void put(bf16_t* p, float v) { *p = f32_to_bf16(v); }
-__device__ __forceinline__ float get(const float* p) { return *p; }
-__device__ __forceinline__ float get(const bf16_t* p) { return bf16_to_f32(*p); }
-
-__device__ __forceinline__ void put4(float* p, const float (&v)[4]) { *reinterpret_cast<float4*>(p) = make_float4(v[0], v[1], v[2], v[3]); }
-__device__ __forceinline__ void put4(bf16_t* p, const float (&v)[4]) { *reinterpret_cast<uint2*>(p) = pack4_bf16(v); }
-
 // columns j .. j + 3 (j % 4 == 0) of a rotary part: pairs (2 i, 2 i + 1) below rot_dims are turned, the others pass (padding columns hold zeros)
 __device__ __forceinline__ void rotary4(const float* src, int j, int rot_dims, const float* cs, const float* sn, float (&o)[4]) {
     const float4 t = *reinterpret_cast<const float4*>(src + j);
@@ -514,8 +475,6 @@ __global__ void __launch_bounds__(256) k_latent_attn_any(LatentDims D, LatentAtt
 #define LAD_KT 64                                  // key tile of the decode kernel
 #define LAD_VS 72
 #define LAD_PS 72                                  // LDS stride of a head's weights
-__device__ __forceinline__ void lds_barrier() { asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory"); }
-__device__ __forceinline__ bf16x8_t lds_frag(const bf16_t* p) { return *reinterpret_cast<const bf16x8_t*>(p); }
 // 4 keys x 8 columns -> column e: the four keys packed
 typedef uint32_t u32x4_t __attribute__((ext_vector_type(4)));
 __device__ __forceinline__ uint2 column_of(const u32x4_t (&r)[4], int e) {

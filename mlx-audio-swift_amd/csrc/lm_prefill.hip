@@ -184,7 +184,7 @@ __global__ void __launch_bounds__(256, 2) k_gemm_pf(PfGemmParams p) {
     for (int j = 0; j < 4; ++j) {
         const int m = m0 + wm * 64 + j * 16 + (lane & 15);
         if (m >= p.M) continue;
-        if (EPI == PF_SILU) {
+        if (EPI == PF_SILU || EPI == PF_SWIGLU) {
             bf16_t* act = reinterpret_cast<bf16_t*>(p.C);
             const int ff = p.N >> 1;
 #pragma unroll
@@ -194,6 +194,11 @@ __global__ void __launch_bounds__(256, 2) k_gemm_pf(PfGemmParams p) {
                 uint16_t res[4];
 #pragma unroll
                 for (int e = 0; e < 4; ++e) {
+                    if (EPI == PF_SWIGLU) {
+                        const float gf = acc[i][j][e];
+                        res[e] = f32_to_bf16(gf / (1.0f + __expf(-gf)) * acc[i + 1][j][e]);
+                        continue;
+                    }
                     const float g = bf16_round_f32(acc[i][j][e]);
                     const float u = bf16_round_f32(acc[i + 1][j][e]);
                     const float sg = bf16_round_f32(1.0f / (1.0f + __expf(-g)));
@@ -211,7 +216,7 @@ __global__ void __launch_bounds__(256, 2) k_gemm_pf(PfGemmParams p) {
                 const int tile = (n0 >> 4) + wn * 4 + i;
                 if (tile >= NT) continue;
                 const int n = tile * 16 + nl;
-                if constexpr (EPI >= PF_SPLIT_RELU2) {
+                if constexpr (EPI >= PF_SPLIT_RELU2 && EPI != PF_SWIGLU) {
                     float v[4] = {acc[i][j][0], acc[i][j][1], acc[i][j][2], acc[i][j][3]};
                     float* c32 = reinterpret_cast<float*>(p.C) + (size_t)m * p.ex.ldc + n;
                     if (EPI == PF_ROWS_BF16 || (EPI == PF_SPLIT_RELU2 && tile >= p.ex.split)) {
@@ -262,8 +267,8 @@ __global__ void __launch_bounds__(256, 2) k_gemm_pf(PfGemmParams p) {
 
 void launch_gemm_pf(int epi, const bf16_t* X, const bf16_t* Wp, void* C, int M, int N, int K, hipStream_t s, const PfExtra& ex) {
     MIS_REQUIRE(K % PF_BK == 0 && K >= 2 * PF_BK && N % 16 == 0 && M >= 1, MIS_ERR_GENERATION_FAILED, "prefill GEMM: K must be a multiple of 64");
-    MIS_REQUIRE(epi != PF_SILU || N % 32 == 0, MIS_ERR_GENERATION_FAILED, "prefill GEMM: gate / up tiles come in pairs");
-    MIS_REQUIRE(epi < PF_SPLIT_RELU2 || (ex.ldc % 4 == 0 && (epi != PF_ROWS_BF16 || (ex.xrow && ex.ldx % 8 == 0))), MIS_ERR_GENERATION_FAILED,
+    MIS_REQUIRE((epi != PF_SILU && epi != PF_SWIGLU) || N % 32 == 0, MIS_ERR_GENERATION_FAILED, "prefill GEMM: gate / up tiles come in pairs");
+    MIS_REQUIRE(epi < PF_SPLIT_RELU2 || epi == PF_SWIGLU || (ex.ldc % 4 == 0 && (epi != PF_ROWS_BF16 || (ex.xrow && ex.ldx % 8 == 0))), MIS_ERR_GENERATION_FAILED,
                 "prefill GEMM: bad row strides");
     PfGemmParams p{X, Wp, C, M, N, K, ex};
     // column tiles rounded up to the 8 XCDs: blocks are dealt to the XCDs by linear id, so that every row of tiles finds its weight tiles in the
@@ -277,6 +282,7 @@ void launch_gemm_pf(int epi, const bf16_t* X, const bf16_t* Wp, void* C, int M, 
     else if (epi == PF_SCALED_ADD) hipLaunchKernelGGL((k_gemm_pf<PF_SCALED_ADD>), grid, block, 0, s, p);
     else if (epi == PF_ROWS_BF16) hipLaunchKernelGGL((k_gemm_pf<PF_ROWS_BF16>), grid, block, 0, s, p);
     else if (epi == PF_SOFTCAP) hipLaunchKernelGGL((k_gemm_pf<PF_SOFTCAP>), grid, block, 0, s, p);
+    else if (epi == PF_SWIGLU) hipLaunchKernelGGL((k_gemm_pf<PF_SWIGLU>), grid, block, 0, s, p);
     else throw MisError(MIS_ERR_GENERATION_FAILED, "unknown prefill GEMM epilogue");
 }
 void launch_pf_embed_rmsnorm(const bf16_t* emb, const int32_t* prompt, const int32_t* lens, int Lmax, int t0, int Tc, int batch, int Mpad, int vocab,

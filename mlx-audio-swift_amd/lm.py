@@ -27,6 +27,7 @@ class BlockModelConfiguration:
     norm: dict = field(default_factory=lambda: {"eps": 1e-6})
     logit_scale: float = 1.0
     logit_softcap: float = 0.0
+    loop: dict | None = None            # {"start", "stop", "times"}: layers start .. stop - 1 run several times in a row
 
     @classmethod
     def from_dict(cls, d: dict) -> "BlockModelConfiguration":

@@ -9,7 +9,7 @@ from .generation import AudioGenerationError
 from .lm import BlockLanguageModel
 from .tts import LlamaTTSModel
 
-ARCHITECTURES = {"Rugunex": BlockLanguageModel}
+ARCHITECTURES = {"Rugunex": BlockLanguageModel, "Vamunex": BlockLanguageModel}
 MODEL_TYPES = {"llama": LlamaTTSModel, "qwen3": LlamaTTSModel, "orpheus": LlamaTTSModel}
 # classes whose engine has a true 32-bit mode
 FLOAT32 = {BlockLanguageModel}
