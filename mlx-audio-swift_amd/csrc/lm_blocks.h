@@ -113,11 +113,11 @@ private:
     std::map<std::pair<int, int>, DevBuf<uint8_t>> pattn_;
     DevBuf<int32_t> pids_, pseq_, ppos_, ppos0_, pkey_, pwant_;
     DevBuf<LatentTile> ptiles_;
-    DevBuf<RowSpan> pspans_;
+    DevBuf<RowSpan> pspans_, pqtiles_;
     // what the mixers of a step / a pass leave behind each other
     struct MixBuffers { DevBuf<float> u, raw_r, raw_g, ss, gu, part; } mix_, pmix_;
     // rows of one pass as the mixers see them
-    struct MixRows { RowTable rows; const int32_t* pos0; SpanTable spans; int M, n_spans; };
+    struct MixRows { RowTable rows; const int32_t* pos0; SpanTable spans; int M, n_spans; const RowSpan* tiles = nullptr; int n_tiles = 0; };
 
     int esz() const { return f32 ? 4 : 2; }
     const Weights& W(int li) const { return *w_[layers_[li].owner]; }

@@ -414,6 +414,7 @@ void LmBlocks::reset(int batch, int Smax, hipStream_t s) {
             n_qkv = std::max(n_qkv, (size_t)l.Nqkv); n_act = std::max(n_act, (size_t)l.ffp);
             n_q = std::max(n_q, (size_t)l.A.H * l.A.Dp);
             n_slab = std::max(n_slab, (size_t)std::max(l.s1, l.s2));
+            n_ml = std::max(n_ml, (size_t)l.shares * batch * l.A.H * 2);
             DevBuf<uint8_t>& at = attn_[columns(i)];
             at.alloc((size_t)Mpad_ * l.Ko * esz());
             at.zero(s);
@@ -622,7 +623,7 @@ void LmBlocks::pass(const std::vector<PassEntry>& entries, const std::vector<int
         const size_t n = std::min(cap, total - t0);
         std::vector<int32_t> seq(n), pos(n), pos0(n), keys;
         std::vector<LatentTile> tiles;
-        std::vector<RowSpan> spans;
+        std::vector<RowSpan> spans, qtiles;
         std::vector<std::pair<int32_t, int32_t>> last;                         // (row, sequence) of entries that end in this chunk
         size_t at = 0;
         while (at < n) {
@@ -631,6 +632,8 @@ void LmBlocks::pass(const std::vector<PassEntry>& entries, const std::vector<int
             const int p0 = e.pos0 + (int)done_in_entry;
             for (size_t k = 0; k < take; ++k) { seq[at + k] = e.seq; pos[at + k] = p0 + (int)k; pos0[at + k] = p0; }
             spans.push_back(RowSpan{(int)at, (int)take, e.seq, p0});
+            for (size_t q = 0; q < take; q += GROUPED_QT)
+                qtiles.push_back(RowSpan{(int)(at + q), (int)std::min<size_t>(GROUPED_QT, take - q), e.seq, p0 + (int)q});
             if (!f32 && latent) {
                 const int kp0 = all_keys ? 0 : std::max(0, p0 - max_window + 1), krow0 = (int)keys.size();
                 for (int p = kp0; p < p0 + (int)take; ++p) keys.push_back(e.seq * Smax_ + p);
@@ -646,6 +649,8 @@ void LmBlocks::pass(const std::vector<PassEntry>& entries, const std::vector<int
         HIP_CHECK(hipMemcpyAsync(ppos0_.p, pos0.data(), n * 4, hipMemcpyHostToDevice, s));
         pspans_.alloc(spans.size());
         HIP_CHECK(hipMemcpyAsync(pspans_.p, spans.data(), spans.size() * sizeof(RowSpan), hipMemcpyHostToDevice, s));
+        pqtiles_.alloc(qtiles.size());
+        HIP_CHECK(hipMemcpyAsync(pqtiles_.p, qtiles.data(), qtiles.size() * sizeof(RowSpan), hipMemcpyHostToDevice, s));
         if (!f32 && latent) {
             pkey_.alloc(keys.size()); ptiles_.alloc(tiles.size());
             pkv_.alloc(keys.size() * n_kv);
@@ -654,7 +659,7 @@ void LmBlocks::pass(const std::vector<PassEntry>& entries, const std::vector<int
         }
         RowTable rows; rows.seq = pseq_.p; rows.pos = ppos_.p;
         MixRows mr;
-        mr.rows = rows; mr.pos0 = ppos0_.p; mr.spans.span = pspans_.p; mr.M = (int)n; mr.n_spans = (int)spans.size();
+        mr.rows = rows; mr.pos0 = ppos0_.p; mr.spans.span = pspans_.p; mr.M = (int)n; mr.n_spans = (int)spans.size(); mr.tiles = pqtiles_.p; mr.n_tiles = (int)qtiles.size();
         launch_rows_embed_norm2(emb_.p, pids_.p, V, g_embed_.p, W(0).norm1.p, px_.p, operand(ph_.p, dp, 0, false), d, dp, spec.eps, (int)n, (int)n, nullptr, nullptr,
                                 nullptr, s, spec.norm_add);
         for (int li = 0; li < L; ++li) {

@@ -168,25 +168,27 @@ void LmBlocks::mixed_reset(int li, hipStream_t s) {
         if (l.ffp) l.s2 = std::min(max_s, gemm_choose_split(dp / 16 / 2, l.ffp / 32, 4, max_s));
     }
     if (l.kind == BLOCK_DECAY) { state_[li]->alloc((size_t)batch_ * l.S.H * l.S.D * l.S.Es); return; }
+    l.shares = !f32 && grouped_mfma_ok(l.A) ? grouped_decode_shares(l.A, batch_, Smax_) : 1;
     // a masked value still enters the matrix cores, times zero: it has to be a number
     cache_[li]->alloc((size_t)batch_ * l.A.G * Smax_ * (l.A.Dp + l.A.Ep) * esz());
     cache_[li]->zero(s);
     state_[li]->alloc((size_t)batch_ * (1 + l.R.taps) * l.R.W);
 }
 void LmBlocks::mixed_buffers(MixBuffers& b, int rows, hipStream_t s) {
-    size_t n_u = 0, n_raw = 0, n_ss = 0, n_ff = 0;
+    size_t n_u = 0, n_raw = 0, n_ss = 0, n_ff = 0, n_part = 0;
     bool mixed = false;
     for (auto& l : layers_) {
         if (l.kind == BLOCK_LATENT) continue;
         mixed = true;
         n_u = std::max(n_u, (size_t)l.R.B * l.R.np); n_raw = std::max(n_raw, (size_t)l.R.B * l.R.nt * 16);
         n_ss = std::max(n_ss, (size_t)l.S.H * l.S.ns); n_ff = std::max(n_ff, (size_t)l.ffp);
+        if (&b == &mix_ && l.shares > 1) n_part = std::max(n_part, (size_t)l.shares * batch_ * l.A.H * l.A.Ep);
     }
     if (!mixed) return;
     const bool grow = b.ss.n < rows * std::max<size_t>(n_ss, 1);
     b.u.alloc(rows * n_u); b.raw_r.alloc(rows * n_raw); b.raw_g.alloc(rows * n_raw); b.ss.alloc(rows * n_ss);
     if (f32) b.gu.alloc(rows * 2 * n_ff);
-    if (&b == &pmix_) b.part.alloc((size_t)rows * dp);
+    b.part.alloc(&b == &pmix_ ? (size_t)rows * dp : n_part);
     if (grow) b.ss.zero(s);
 }
 
@@ -208,10 +210,17 @@ void LmBlocks::mixer(int li, const float* proj, void* q, const Operand& out, con
     GroupedRows gr{};
     gr.proj = proj; gr.ld = l.Nqkv; gr.oq = l.oq; gr.ok = l.ok; gr.ov = l.ov; gr.bias = w.bias1.p; gr.qn = w.qn.p; gr.kn = w.kn.p;
     gr.rope_cos = ropes_[l.rope].cs.p; gr.rope_sin = ropes_[l.rope].sn.p; gr.rows = r.rows; gr.kc = kc; gr.vc = vc; gr.Smax = Smax_; gr.q = q; gr.f32 = f32;
-    launch_grouped_rows(A, gr, r.M, s);
     GroupedAttn ga{};
     ga.q = q; ga.kc = kc; ga.vc = vc; ga.Smax = Smax_; ga.sink = w.sink.p; ga.rows = r.rows; ga.out = out; ga.out_scale = spec.layers[li].left_scale; ga.f32 = f32;
-    launch_grouped_attn_any(A, ga, r.M, s);
+    if (!f32 && grouped_mfma_ok(A) && !r.spans.span) {
+        GroupedShares sh;
+        sh.S = l.shares; sh.part = b.part.p; sh.ml = share_ml_.p;
+        launch_grouped_attn_decode(A, gr, ga, sh, r.M, s);
+    } else {
+        launch_grouped_rows(A, gr, r.M, s);
+        if (!f32 && grouped_mfma_ok(A)) launch_grouped_attn_prefill(A, ga, r.tiles, r.n_tiles, s);
+        else launch_grouped_attn_any(A, ga, r.M, s);
+    }
     RecurParams p{};
     p.proj = proj; p.ld = l.Nqkv; p.oy = l.oy; p.ox = l.ox; p.bias = w.bias1.p; p.conv = w.conv.p; p.conv_b = w.conv_b.p; p.ra_b = w.ra_b.p; p.ri_b = w.ri_b.p;
     p.c = w.recur_c.p; p.rows = r.rows; p.pos0 = r.pos0; p.spans = r.spans; p.state = state_[li]->p; p.hist = state_[li]->p + (size_t)batch_ * R.W;

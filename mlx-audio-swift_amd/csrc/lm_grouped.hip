@@ -1,0 +1,412 @@
+// lm_grouped.hip - grouped attention of lm_mixers.h on the matrix cores (bf16): prompt tiles and decode shares over the fragment caches.
+//
+// Both kernels compute S^T = K q^T on 16 x 16 tiles (rows: keys, columns: queries - positions of one head in a prompt, heads of one group in a decode
+// step) and O^T = V^T P^T.  A pair of score tiles leaves a lane the weights of keys 4 q .. + 3 and 16 + 4 q .. + 3 of its column, and the value
+// fragments hold the keys in that order: the weights go from the accumulators into the next product without leaving the lane.  Scores and softmax are
+// float32, base 2; the weights enter as bf16 hi + lo.  The sink is a key-less term of the running sum: the sum starts with it.
+#include "lm_mixers.h"
+#include "lm_device.h"
+#include <math.h>
+
+#define GRP_LOG2E 1.4426950408889634f
+__device__ __forceinline__ float grp_exp2(float x) { return __builtin_amdgcn_exp2f(x); }
+__device__ __forceinline__ bool grp_sees(const GroupedDims& D, int pos, int key) {
+    return (key <= pos) & ((D.window <= 0) | (pos - key < D.window) | (key < D.keep));
+}
+// steps of 32 keys that a query (a range of queries) may see: [0, kept) and [s0, s1]
+struct GrpSteps { int kept, s0, s1; __device__ int count() const { return kept + s1 - s0 + 1; } __device__ int at(int i) const { return i < kept ? i : s0 + i - kept; } };
+__device__ __forceinline__ GrpSteps grp_steps(const GroupedDims& D, int pos_lo, int pos_hi) {
+    GrpSteps r;
+    r.s0 = D.window > 0 ? max(0, pos_lo - D.window + 1) >> 5 : 0;
+    r.s1 = pos_hi >> 5;
+    r.kept = min((D.keep + 31) >> 5, r.s0);
+    return r;
+}
+// weights of a pair of score tiles -> bf16 hi and lo fragments
+__device__ __forceinline__ void grp_split(const float (&w)[8], bf16x8_t& hi, bf16x8_t& lo) {
+#pragma unroll
+    for (int j = 0; j < 8; ++j) {
+        const bf16_t h = f32_to_bf16(w[j]);
+        hi[j] = (short)h;
+        lo[j] = (short)f32_to_bf16(w[j] - bf16_to_f32(h));
+    }
+}
+
+// ============================================================================ prompt pass
+// Block = up to 64 queries of one request and up to NW / 2 heads of one group; a wave = 32 queries of one head.  The 32 keys of a step - KT pairs of key
+// fragments and VT value fragments, contiguous in the caches - come into LDS by DMA, two buffers, one barrier per step.
+// EXACT: the heads have KT and VT tiles, not fewer (no guards in the loop)
+template <int KT, int VT, bool EXACT>
+__global__ void __launch_bounds__(256, (KT <= 4 && VT <= 8) ? 2 : 1) k_grouped_attn_prefill(GroupedDims D, GroupedAttn p, const RowSpan* __restrict__ tiles, int ipb) {
+    __shared__ __attribute__((aligned(1024))) bf16_t buf[2][(2 * KT + VT) * 512];
+    const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, nw = blockDim.x >> 6, li = lane & 15, lq = lane >> 4;
+    const RowSpan t = tiles[blockIdx.x];
+    const int g = blockIdx.y, R = D.H / D.G, kt_n = EXACT ? KT : D.Dp >> 5, vt_n = EXACT ? VT : D.Ep >> 4;
+    const int item = blockIdx.z * ipb + wave, hd = g * R + min(item >> 1, R - 1), q0 = (item & 1) * 32;
+    const bool live = item < 2 * R && q0 < t.n;                                // (a wave without queries only helps to stage)
+    const int nq = min(32, t.n - q0), p_lo = t.pos0 + q0, p_hi = p_lo + nq - 1;
+    const GrpSteps st = grp_steps(D, t.pos0, t.pos0 + t.n - 1);
+    const bf16_t* kc = (const bf16_t*)p.kc + ((size_t)t.seq * D.G + g) * p.Smax * D.Dp;
+    const bf16_t* vc = (const bf16_t*)p.vc + ((size_t)t.seq * D.G + g) * p.Smax * D.Ep;
+    auto stage = [&](int b, int s) {
+        const bf16_t *ks = kc + (size_t)s * 32 * D.Dp, *vs = vc + (size_t)s * 32 * D.Ep;
+        for (int f = wave; f < 2 * kt_n + vt_n; f += nw) {
+            const bf16_t* src = f < 2 * kt_n ? ks + (size_t)f * 512 : vs + (size_t)(f - 2 * kt_n) * 512;
+            __builtin_amdgcn_global_load_lds((const __attribute__((address_space(1))) void*)(src + lane * 8),
+                                             (__attribute__((address_space(3))) void*)&buf[b][(f < 2 * kt_n ? f : 2 * KT + f - 2 * kt_n) * 512], 16, 0, 0);
+        }
+    };
+    stage(0, st.at(0));
+    bf16x8_t q[2][KT];
+    int pos[2];
+#pragma unroll
+    for (int c = 0; c < 2; ++c) {
+        const int r = live ? min(c * 16 + li, nq - 1) : 0;
+        pos[c] = p_lo + c * 16 + li;
+        const bf16_t* qr = (const bf16_t*)p.q + ((size_t)(live ? t.row0 + q0 + r : t.row0) * D.H + hd) * D.Dp + lq * 8;
+#pragma unroll
+        for (int k = 0; k < KT; ++k) q[c][k] = *reinterpret_cast<const bf16x8_t*>(qr + min(k, kt_n - 1) * 32);
+    }
+    f32x4_t o[2][VT];
+#pragma unroll
+    for (int c = 0; c < 2; ++c)
+#pragma unroll
+        for (int v = 0; v < VT; ++v) o[c][v] = (f32x4_t){0.f, 0.f, 0.f, 0.f};
+    const float sc = D.scale * GRP_LOG2E, sink = bf16_to_f32(p.sink[hd]) * GRP_LOG2E;
+    float mx[2] = {sink, sink}, ls[2] = {lq == 0 ? 1.0f : 0.0f, lq == 0 ? 1.0f : 0.0f};      // ls: this lane's keys only
+    const int n = st.count();
+    for (int i = 0; i < n; ++i) {
+        __syncthreads();                                                       // step i has landed; the other buffer is free
+        if (i + 1 < n) stage((i + 1) & 1, st.at(i + 1));
+        const int k0 = st.at(i) * 32;
+        if (!live || k0 > p_hi) continue;                                      // (wave-uniform)
+        if (D.window > 0 && p_lo - (k0 + 31) >= D.window && k0 >= D.keep) continue;
+        const bf16_t* b = buf[i & 1];
+        f32x4_t s[2][2];
+#pragma unroll
+        for (int c = 0; c < 2; ++c) s[c][0] = s[c][1] = (f32x4_t){0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int k = 0; k < KT; ++k) {
+            if (k >= kt_n) continue;
+            const bf16x8_t a0 = lds_frag(b + (size_t)k * 512 + lane * 8), a1 = lds_frag(b + (size_t)(kt_n + k) * 512 + lane * 8);
+#pragma unroll
+            for (int c = 0; c < 2; ++c) {
+                s[c][0] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a0, q[c][k], s[c][0], 0, 0, 0);
+                s[c][1] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a1, q[c][k], s[c][1], 0, 0, 0);
+            }
+        }
+        const bool all = k0 + 31 <= p_lo && (D.window <= 0 || p_hi - k0 < D.window || k0 + 31 < D.keep);
+        bf16x8_t ph[2], pl[2];
+#pragma unroll
+        for (int c = 0; c < 2; ++c) {
+            float w[8], tm = -INFINITY;
+#pragma unroll
+            for (int h = 0; h < 2; ++h)
+#pragma unroll
+                for (int e = 0; e < 4; ++e) {
+                    w[h * 4 + e] = s[c][h][e] * sc;
+                    if (!all && !grp_sees(D, pos[c], k0 + h * 16 + lq * 4 + e)) w[h * 4 + e] = -INFINITY;
+                    tm = fmaxf(tm, w[h * 4 + e]);
+                }
+            tm = fmaxf(tm, __shfl_xor(tm, 16, 64));
+            tm = fmaxf(tm, __shfl_xor(tm, 32, 64));
+            if (__any(tm > mx[c])) {
+                const float mn = fmaxf(mx[c], tm), alpha = grp_exp2(mx[c] - mn);
+                mx[c] = mn;
+                ls[c] *= alpha;
+#pragma unroll
+                for (int v = 0; v < VT; ++v) o[c][v] *= alpha;
+            }
+            float add = 0.0f;
+#pragma unroll
+            for (int j = 0; j < 8; ++j) { w[j] = grp_exp2(w[j] - mx[c]); add += w[j]; }
+            ls[c] += add;
+            grp_split(w, ph[c], pl[c]);
+        }
+#pragma unroll
+        for (int v = 0; v < VT; ++v) {
+            if (v >= vt_n) continue;
+            const bf16x8_t a = lds_frag(b + (size_t)(2 * KT + v) * 512 + lane * 8);
+#pragma unroll
+            for (int c = 0; c < 2; ++c) {
+                o[c][v] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, ph[c], o[c][v], 0, 0, 0);
+                o[c][v] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, pl[c], o[c][v], 0, 0, 0);
+            }
+        }
+    }
+    if (!live) return;
+#pragma unroll
+    for (int c = 0; c < 2; ++c) {
+        float l = ls[c];
+        l += __shfl_xor(l, 16, 64);
+        l += __shfl_xor(l, 32, 64);
+        const float r = p.out_scale / l;
+        if (c * 16 + li >= nq) continue;
+        const int m = t.row0 + q0 + c * 16 + li;
+#pragma unroll
+        for (int v = 0; v < VT; ++v) {
+            const int col = v * 16 + lq * 4;
+            const float x[4] = {o[c][v][0] * r, o[c][v][1] * r, o[c][v][2] * r, o[c][v][3] * r};
+            if ((D.E & 3) == 0) { if (col < D.E) operand_store4(p.out, m, hd * D.E + col, x); }
+            else {
+#pragma unroll
+                for (int e = 0; e < 4; ++e) if (col + e < D.E) operand_store1(p.out, m, hd * D.E + col + e, x[e]);
+            }
+        }
+    }
+}
+bool grouped_mfma_ok(const GroupedDims& D) { return D.Dp <= 256 && D.Ep <= 256; }
+void launch_grouped_attn_prefill(const GroupedDims& D, const GroupedAttn& p, const RowSpan* tiles, int n_tiles, hipStream_t s) {
+    MIS_REQUIRE(grouped_mfma_ok(D) && !p.f32 && p.Smax % 32 == 0 && p.out.kind == OPK_ROWS && p.out.ld % 4 == 0, MIS_ERR_GENERATION_FAILED, "grouped attention: bad layout");
+    const int items = 2 * (D.H / D.G);
+    const int ipb = items % 4 == 0 ? 4 : (items % 3 == 0 ? 3 : (items <= 4 ? items : 4));     // waves per block
+    const dim3 grid(n_tiles, D.G, cdiv(items, ipb)), block(64 * ipb);
+    const int kt = D.Dp / 32, vt = D.Ep / 16;
+#define GRP_PF(K, V, X) hipLaunchKernelGGL((k_grouped_attn_prefill<K, V, X>), grid, block, 0, s, D, p, tiles, ipb)
+    if (kt == 2 && vt == 4) GRP_PF(2, 4, true);
+    else if (kt == 4 && vt == 8) GRP_PF(4, 8, true);
+    else if (kt <= 2 && vt <= 4) GRP_PF(2, 4, false);
+    else if (kt <= 4 && vt <= 8) GRP_PF(4, 8, false);
+    else GRP_PF(8, 16, false);
+#undef GRP_PF
+}
+
+// ============================================================================ decode step
+// Block = one row, up to 16 heads of one group, one share of the row's steps; its four waves take the share's steps in turn, each with its own running
+// softmax, and meet in LDS.  The block norms and rotates its heads' queries itself; the current token's key and value never come from the cache: its
+// score and value join when the waves meet (last share), the sink with the first share.  The last share's block of a group's first head tile also
+// appends the token to the caches - for the NEXT step.
+struct GrpDecodeLds { float q[16][260]; float k[260], v[260]; float m[4][16], l[4][16], self[16]; };
+template <int KT, int VT, bool EXACT>
+__global__ void __launch_bounds__(256, (KT <= 4 && VT <= 8) ? 2 : 1) k_grouped_attn_decode(GroupedDims D, GroupedRows r, GroupedAttn p, GroupedShares sh, int rows) {
+    __shared__ GrpDecodeLds L;
+    __shared__ float acc[2][16][VT * 16 + 4];
+    const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, li = lane & 15, lq = lane >> 4;
+    const int m = blockIdx.x % rows, sp = blockIdx.x / rows, g = blockIdx.y, R = D.H / D.G, kt_n = EXACT ? KT : D.Dp >> 5, vt_n = EXACT ? VT : D.Ep >> 4;
+    const int a0 = blockIdx.z * 16, na = min(16, R - a0), h0 = g * R + a0;     // heads h0 .. h0 + na - 1
+    if (r.rows.on && !r.rows.on[m]) return;                                    // block-uniform
+    const int pos = r.rows.pos[m], half = D.rot >> 1;
+    const GrpSteps st = grp_steps(D, pos, pos);
+    const int n = st.count(), per = (n + sh.S - 1) / sh.S, i0 = min(sp * per, n), i1 = min(i0 + per, n);
+    const bool first = sp == 0, last = sp == sh.S - 1;
+    const bf16_t* kc = (const bf16_t*)p.kc + ((size_t)m * D.G + g) * p.Smax * D.Dp;
+    const bf16_t* vc = (const bf16_t*)p.vc + ((size_t)m * D.G + g) * p.Smax * D.Ep;
+    // ---- the wave's first keys are requested before anything else
+    bf16x8_t ka[2][KT], va[VT];
+    auto fetch_k = [&](int s) {
+        const bf16_t* ks = kc + (size_t)s * 32 * D.Dp + lane * 8;
+#pragma unroll
+        for (int k = 0; k < KT; ++k) {
+            ka[0][k] = __builtin_nontemporal_load(reinterpret_cast<const bf16x8_t*>(ks + (size_t)min(k, kt_n - 1) * 512));
+            ka[1][k] = __builtin_nontemporal_load(reinterpret_cast<const bf16x8_t*>(ks + (size_t)(kt_n + min(k, kt_n - 1)) * 512));
+        }
+    };
+    auto fetch_v = [&](int s) {
+        const bf16_t* vs = vc + (size_t)s * 32 * D.Ep + lane * 8;
+#pragma unroll
+        for (int v = 0; v < VT; ++v) va[v] = __builtin_nontemporal_load(reinterpret_cast<const bf16x8_t*>(vs + (size_t)min(v, vt_n - 1) * 512));
+    };
+    if (i0 + wave < i1) { fetch_k(st.at(i0 + wave)); fetch_v(st.at(i0 + wave)); }
+    __builtin_amdgcn_sched_barrier(0);
+    // ---- queries (and, last share, the token's key and value): bias, norm, rotation
+    const float *cs = r.rope_cos + (size_t)pos * half, *sn = r.rope_sin + (size_t)pos * half;
+    const float* row = r.proj + (size_t)m * r.ld;
+    for (int a = wave; a < na + (last ? 2 : 0); a += 4) {
+        if (a == na + 1) {                                                     // value
+            const int o = r.ov + g * D.E;
+            for (int i = lane; i < D.Ep; i += 64) L.v[i] = i < D.E ? bf16_round_f32(row[o + i] + bf16_to_f32(r.bias[o + i])) : 0.0f;
+            continue;
+        }
+        const bool is_q = a < na;
+        const int o = is_q ? r.oq + (h0 + a) * D.D : r.ok + g * D.D;
+        const bf16_t* w = is_q ? r.qn : r.kn;
+        float x[4], ss = 0.0f;                                                 // D <= 256: four dimensions a lane
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+            const int i = lane + 64 * j;
+            x[j] = i < D.D ? row[o + i] + bf16_to_f32(r.bias[o + i]) : 0.0f;
+            ss += x[j] * x[j];
+        }
+        const float inv = 1.0f / sqrtf(wave_sum(ss) / (float)D.D + D.eps);
+        float* dst = is_q ? L.q[a] : L.k;
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+            const int i = lane + 64 * j;
+            if (i < D.Dp) dst[i] = i < D.D ? x[j] * inv * bf16_to_f32(w[i]) : 0.0f;
+        }
+    }
+    for (int i = threadIdx.x + na * 260; i < 16 * 260; i += 256) L.q[0][i] = 0.0f;           // columns past the heads
+    __syncthreads();
+    for (int t = threadIdx.x; t < (na + (last ? 1 : 0)) * half; t += 256) {    // rotation in place: a pair per thread
+        const int a = t / half, i = t - a * half;
+        float* x = a < na ? L.q[a] : L.k;
+        const float c = cs[i], s = sn[i], u = x[i], v = x[i + half];
+        x[i] = u * c - v * s;
+        x[i + half] = v * c + u * s;
+    }
+    __syncthreads();
+    if (last) {
+        if (a0 == 0) {
+            bf16_t *kd = (bf16_t*)r.kc + ((size_t)m * D.G + g) * p.Smax * D.Dp, *vd = (bf16_t*)r.vc + ((size_t)m * D.G + g) * p.Smax * D.Ep;
+            for (int i = threadIdx.x; i < D.Dp; i += 256)
+                kd[((size_t)(pos >> 4) * kt_n + (i >> 5)) * 512 + (((i & 31) >> 3) * 16 + (pos & 15)) * 8 + (i & 7)] = f32_to_bf16(L.k[i]);
+            for (int i = threadIdx.x; i < D.Ep; i += 256)
+                vd[((size_t)(pos >> 5) * vt_n + (i >> 4)) * 512 + (((pos & 15) >> 2) * 16 + (i & 15)) * 8 + ((pos >> 4) & 1) * 4 + (pos & 3)] = f32_to_bf16(L.v[i]);
+        }
+        for (int a = wave; a < na; a += 4) {                                   // score of the token with itself, on the values the cache will hold
+            float d = 0.0f;
+            for (int i = lane; i < D.D; i += 64) d += bf16_round_f32(L.q[a][i]) * bf16_round_f32(L.k[i]);
+            d = wave_sum(d);
+            if (lane == 0) L.self[a] = d * D.scale * GRP_LOG2E;
+        }
+    }
+    bf16x8_t q[KT];
+#pragma unroll
+    for (int k = 0; k < KT; ++k) {
+        const float* x = &L.q[li][min(k, kt_n - 1) * 32 + lq * 8];
+#pragma unroll
+        for (int e = 0; e < 8; ++e) q[k][e] = (short)f32_to_bf16(x[e]);
+    }
+    f32x4_t o[VT];
+#pragma unroll
+    for (int v = 0; v < VT; ++v) o[v] = (f32x4_t){0.f, 0.f, 0.f, 0.f};
+    const float sc = D.scale * GRP_LOG2E;
+    float mx = -1e30f, ls = 0.0f;
+    for (int i = i0 + wave; i < i1; i += 4) {
+        const int k0 = st.at(i) * 32;
+        f32x4_t s0 = (f32x4_t){0.f, 0.f, 0.f, 0.f}, s1 = s0;
+#pragma unroll
+        for (int k = 0; k < KT; ++k) {
+            if (k >= kt_n) continue;
+            s0 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(ka[0][k], q[k], s0, 0, 0, 0);
+            s1 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(ka[1][k], q[k], s1, 0, 0, 0);
+        }
+        if (i + 4 < i1) fetch_k(st.at(i + 4));
+        __builtin_amdgcn_sched_barrier(0);
+        float w[8], tm = -1e30f;
+#pragma unroll
+        for (int j = 0; j < 8; ++j) {
+            const int key = k0 + (j >> 2) * 16 + lq * 4 + (j & 3);
+            const bool on = key != pos && grp_sees(D, pos, key);
+            w[j] = on ? (j < 4 ? s0[j & 3] : s1[j & 3]) * sc : -INFINITY;
+            tm = fmaxf(tm, w[j]);
+        }
+        tm = fmaxf(tm, __shfl_xor(tm, 16, 64));
+        tm = fmaxf(tm, __shfl_xor(tm, 32, 64));
+        if (__any(tm > mx)) {
+            const float mn = fmaxf(mx, tm), alpha = grp_exp2(mx - mn);
+            mx = mn;
+            ls *= alpha;
+#pragma unroll
+            for (int v = 0; v < VT; ++v) o[v] *= alpha;
+        }
+        float add = 0.0f;
+#pragma unroll
+        for (int j = 0; j < 8; ++j) { w[j] = grp_exp2(w[j] - mx); add += w[j]; }
+        ls += add;
+        bf16x8_t ph, pl;
+        grp_split(w, ph, pl);
+#pragma unroll
+        for (int v = 0; v < VT; ++v) {
+            if (v >= vt_n) continue;
+            o[v] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(va[v], ph, o[v], 0, 0, 0);
+            o[v] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(va[v], pl, o[v], 0, 0, 0);
+        }
+        if (i + 4 < i1) fetch_v(st.at(i + 4));
+        __builtin_amdgcn_sched_barrier(0);
+    }
+    // ---- the waves meet: common maximum (with the sink and the token itself), sums, values
+    ls += __shfl_xor(ls, 16, 64);
+    ls += __shfl_xor(ls, 32, 64);
+    if (lq == 0) { L.m[wave][li] = mx; L.l[wave][li] = ls; }
+    __syncthreads();
+    const int hd = h0 + min(li, na - 1);
+    float M = fmaxf(fmaxf(L.m[0][li], L.m[1][li]), fmaxf(L.m[2][li], L.m[3][li]));
+    const float sink = first ? bf16_to_f32(p.sink[hd]) * GRP_LOG2E : -1e30f, self = last && li < na ? L.self[li] : -1e30f;
+    M = fmaxf(M, fmaxf(sink, self));
+    float T = (L.l[0][li] * grp_exp2(L.m[0][li] - M) + L.l[1][li] * grp_exp2(L.m[1][li] - M)) + (L.l[2][li] * grp_exp2(L.m[2][li] - M) + L.l[3][li] * grp_exp2(L.m[3][li] - M));
+    const float ps = last && li < na ? grp_exp2(self - M) : 0.0f;
+    T += (first ? grp_exp2(sink - M) : 0.0f) + ps;
+    const float f = grp_exp2(mx - M);
+#pragma unroll
+    for (int rd = 0; rd < 2; ++rd) {                                           // waves 1, 3 hand over to 0, 2; then 2 to 0
+        if (rd == 0 ? (wave & 1) : wave == 2) {
+            float (*d)[VT * 16 + 4] = acc[rd == 0 ? wave >> 1 : 0];
+#pragma unroll
+            for (int v = 0; v < VT; ++v)
+#pragma unroll
+                for (int e = 0; e < 4; ++e) d[li][v * 16 + lq * 4 + e] = rd == 0 ? o[v][e] * f : o[v][e];
+        }
+        __syncthreads();
+        if (rd == 0 ? !(wave & 1) : wave == 0) {
+            float (*d)[VT * 16 + 4] = acc[rd == 0 ? wave >> 1 : 0];
+#pragma unroll
+            for (int v = 0; v < VT; ++v)
+#pragma unroll
+                for (int e = 0; e < 4; ++e) o[v][e] = (rd == 0 ? o[v][e] * f : o[v][e]) + d[li][v * 16 + lq * 4 + e];
+        }
+        __syncthreads();
+    }
+    if (wave != 0 || li >= na) return;
+    const float inv = sh.S == 1 ? p.out_scale / T : 1.0f;
+    float* part = sh.S == 1 ? nullptr : sh.part + (((size_t)sp * rows + m) * D.H + hd) * D.Ep;
+#pragma unroll
+    for (int v = 0; v < VT; ++v) {
+        const int col = v * 16 + lq * 4;
+        if (v >= vt_n) continue;
+        float x[4];
+#pragma unroll
+        for (int e = 0; e < 4; ++e) x[e] = (o[v][e] + (last ? ps * L.v[col + e] : 0.0f)) * inv;
+        if (part) *reinterpret_cast<float4*>(part + col) = make_float4(x[0], x[1], x[2], x[3]);
+        else if ((D.E & 3) == 0) { if (col < D.E) operand_store4(p.out, m, hd * D.E + col, x); }
+        else {
+#pragma unroll
+            for (int e = 0; e < 4; ++e) if (col + e < D.E) operand_store1(p.out, m, hd * D.E + col + e, x[e]);
+        }
+    }
+    if (part && lq == 0) {
+        float* ml = sh.ml + (((size_t)sp * rows + m) * D.H + hd) * 2;
+        *reinterpret_cast<float2*>(ml) = make_float2(M, T);
+    }
+}
+// shares of a head -> operand: one wave per (row, head)
+__global__ void __launch_bounds__(256) k_grouped_shares(GroupedDims D, GroupedShares sh, Operand out, float out_scale, const uint8_t* __restrict__ on, int rows) {
+    const int lane = threadIdx.x & 63, item = blockIdx.x * 4 + (threadIdx.x >> 6);
+    if (item >= rows * D.H) return;
+    const int m = item / D.H, hd = item - m * D.H;
+    if (on && !on[m]) return;
+    const float2* ml = reinterpret_cast<const float2*>(sh.ml);
+    float M = -1e30f, T = 0.0f;
+    for (int s = 0; s < sh.S; ++s) M = fmaxf(M, ml[((size_t)s * rows + m) * D.H + hd].x);
+    for (int s = 0; s < sh.S; ++s) { const float2 t = ml[((size_t)s * rows + m) * D.H + hd]; T += t.y * grp_exp2(t.x - M); }
+    const float inv = out_scale / T;
+    for (int i = lane; i < D.E; i += 64) {
+        float a = 0.0f;
+        for (int s = 0; s < sh.S; ++s) {
+            const size_t at = ((size_t)s * rows + m) * D.H + hd;
+            a += sh.part[at * D.Ep + i] * grp_exp2(ml[at].x - M);
+        }
+        operand_store1(out, m, hd * D.E + i, a * inv);
+    }
+}
+int grouped_decode_shares(const GroupedDims& D, int rows, int Smax) {
+    const int keys = D.window > 0 ? std::min(Smax, D.window + D.keep + 32) : Smax, steps = cdiv(keys, 32);
+    const int blocks = rows * D.G * cdiv(D.H / D.G, 16);
+    int S = 1;
+    while (S < 32 && blocks * S < 512 && steps / (S + 1) >= 8) ++S;            // two steps a wave at least
+    return S;
+}
+void launch_grouped_attn_decode(const GroupedDims& D, const GroupedRows& r, const GroupedAttn& p, const GroupedShares& sh, int rows, hipStream_t s) {
+    MIS_REQUIRE(grouped_mfma_ok(D) && !p.f32 && p.Smax % 32 == 0 && sh.S >= 1 && (sh.S == 1 || (sh.part && sh.ml)) && !r.rows.seq, MIS_ERR_GENERATION_FAILED,
+                "grouped attention: bad layout");
+    const dim3 grid(rows * sh.S, D.G, cdiv(D.H / D.G, 16)), block(256);
+    const int kt = D.Dp / 32, vt = D.Ep / 16;
+#define GRP_DEC(K, V, X) hipLaunchKernelGGL((k_grouped_attn_decode<K, V, X>), grid, block, 0, s, D, r, p, sh, rows)
+    if (kt == 2 && vt == 4) GRP_DEC(2, 4, true);
+    else if (kt == 4 && vt == 8) GRP_DEC(4, 8, true);
+    else if (kt <= 2 && vt <= 4) GRP_DEC(2, 4, false);
+    else if (kt <= 4 && vt <= 8) GRP_DEC(4, 8, false);
+    else GRP_DEC(8, 16, false);
+#undef GRP_DEC
+    if (sh.S > 1) hipLaunchKernelGGL(k_grouped_shares, dim3(cdiv((int64_t)rows * D.H, 4)), dim3(256), 0, s, D, sh, p.out, p.out_scale, r.rows.on, rows);
+}

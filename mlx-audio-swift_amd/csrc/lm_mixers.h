@@ -49,7 +49,16 @@ struct GroupedAttn {
     Operand out; float out_scale;           // head a at columns a E ..
     int f32;
 };
+// any sizes, either element type; the cache holds the rows already
 void launch_grouped_attn_any(const GroupedDims& D, const GroupedAttn& p, int rows, hipStream_t s);
+// matrix cores, bf16 (lm_grouped.hip)
+bool grouped_mfma_ok(const GroupedDims& D);
+#define GROUPED_QT 64           // queries of one request per prompt tile
+void launch_grouped_attn_prefill(const GroupedDims& D, const GroupedAttn& p, const RowSpan* tiles, int n_tiles, hipStream_t s);
+// decode: queries, cache rows, attention and (more than one share) the shares' sum; p.q is not used
+struct GroupedShares { int S = 1; float *part = nullptr, *ml = nullptr; };      // part [S][rows][H][Ep], ml [S][rows][H][2]
+int grouped_decode_shares(const GroupedDims& D, int rows, int Smax);
+void launch_grouped_attn_decode(const GroupedDims& D, const GroupedRows& r, const GroupedAttn& p, const GroupedShares& sh, int rows, hipStream_t s);
 
 // ---- gated linear recurrence: u = conv(x);  r, g = sigmoid(block-diagonal products of u);  S = a S + sqrt(1 - a^2) g u, a = exp(-c r)
 struct RecurDims {
