@@ -82,7 +82,7 @@ private:
         DevBuf<bf16_t> wo, wdown;       // packed [dp / 16][Ko / 32], [dp / 16][ffp / 32]
         // BLOCK_DECAY, BLOCK_PARALLEL (lm_blocks_mixed.hip).  w1 holds the mixer's input projections alone, wo both sides' output projections along K
         DevBuf<bf16_t> norm1b, norm2, norm2b, wgu /* gate and up tiles in turn */, bias1, bias_o, wo_rows, mix_norm, qn, kn, sink, conv, conv_b, ra, ri, ra_b, ri_b;
-        DevBuf<float> decay, recur_c;
+        DevBuf<float> decay, recur_c, conv32 /* launch_conv_tables */;
     };
     struct Layer {
         LatentDims D; int owner, ffp, Nqkv, Ko, shares = 1, s1 = 1, s2 = 0, rope = 0;
@@ -93,6 +93,7 @@ private:
     std::vector<Layer> layers_;
     std::vector<std::unique_ptr<Weights>> w_;
     std::set<std::string> loaded_;
+    std::set<int> x_bias_set_;          // layers whose recurrence has its input bias
     DevBuf<bf16_t> emb_, g_embed_, g_final_, head_;
     struct Rope { RotarySpec spec; DevBuf<float> cs, sn; };
     std::deque<Rope> ropes_;
@@ -114,10 +115,11 @@ private:
     DevBuf<int32_t> pids_, pseq_, ppos_, ppos0_, pkey_, pwant_;
     DevBuf<LatentTile> ptiles_;
     DevBuf<RowSpan> pspans_, pqtiles_;
+    DevBuf<RecurChunk> pchunks_;
     // what the mixers of a step / a pass leave behind each other
     struct MixBuffers { DevBuf<float> u, raw_r, raw_g, ss, gu, part; } mix_, pmix_;
     // rows of one pass as the mixers see them
-    struct MixRows { RowTable rows; const int32_t* pos0; SpanTable spans; int M, n_spans; const RowSpan* tiles = nullptr; int n_tiles = 0; };
+    struct MixRows { RowTable rows; const int32_t* pos0; SpanTable spans; int M, n_spans; const RowSpan* tiles = nullptr; int n_tiles = 0; const RecurChunk* chunks = nullptr; int n_chunks = 0; };
 
     int esz() const { return f32 ? 4 : 2; }
     const Weights& W(int li) const { return *w_[layers_[li].owner]; }

@@ -624,6 +624,7 @@ void LmBlocks::pass(const std::vector<PassEntry>& entries, const std::vector<int
         std::vector<int32_t> seq(n), pos(n), pos0(n), keys;
         std::vector<LatentTile> tiles;
         std::vector<RowSpan> spans, qtiles;
+        std::vector<RecurChunk> chunks;
         std::vector<std::pair<int32_t, int32_t>> last;                         // (row, sequence) of entries that end in this chunk
         size_t at = 0;
         while (at < n) {
@@ -632,6 +633,9 @@ void LmBlocks::pass(const std::vector<PassEntry>& entries, const std::vector<int
             const int p0 = e.pos0 + (int)done_in_entry;
             for (size_t k = 0; k < take; ++k) { seq[at + k] = e.seq; pos[at + k] = p0 + (int)k; pos0[at + k] = p0; }
             spans.push_back(RowSpan{(int)at, (int)take, e.seq, p0});
+            for (size_t q = 0; q < take; q += RECUR_CHUNK)
+                chunks.push_back(RecurChunk{RowSpan{(int)(at + q), (int)std::min<size_t>(RECUR_CHUNK, take - q), e.seq, p0 + (int)q}, (int)spans.size() - 1, p0,
+                                            (int)(q / RECUR_CHUNK), q + RECUR_CHUNK >= take ? 1 : 0});
             for (size_t q = 0; q < take; q += GROUPED_QT)
                 qtiles.push_back(RowSpan{(int)(at + q), (int)std::min<size_t>(GROUPED_QT, take - q), e.seq, p0 + (int)q});
             if (!f32 && latent) {
@@ -651,6 +655,8 @@ void LmBlocks::pass(const std::vector<PassEntry>& entries, const std::vector<int
         HIP_CHECK(hipMemcpyAsync(pspans_.p, spans.data(), spans.size() * sizeof(RowSpan), hipMemcpyHostToDevice, s));
         pqtiles_.alloc(qtiles.size());
         HIP_CHECK(hipMemcpyAsync(pqtiles_.p, qtiles.data(), qtiles.size() * sizeof(RowSpan), hipMemcpyHostToDevice, s));
+        pchunks_.alloc(chunks.size());
+        HIP_CHECK(hipMemcpyAsync(pchunks_.p, chunks.data(), chunks.size() * sizeof(RecurChunk), hipMemcpyHostToDevice, s));
         if (!f32 && latent) {
             pkey_.alloc(keys.size()); ptiles_.alloc(tiles.size());
             pkv_.alloc(keys.size() * n_kv);
@@ -660,6 +666,7 @@ void LmBlocks::pass(const std::vector<PassEntry>& entries, const std::vector<int
         RowTable rows; rows.seq = pseq_.p; rows.pos = ppos_.p;
         MixRows mr;
         mr.rows = rows; mr.pos0 = ppos0_.p; mr.spans.span = pspans_.p; mr.M = (int)n; mr.n_spans = (int)spans.size(); mr.tiles = pqtiles_.p; mr.n_tiles = (int)qtiles.size();
+        mr.chunks = pchunks_.p; mr.n_chunks = (int)chunks.size();
         launch_rows_embed_norm2(emb_.p, pids_.p, V, g_embed_.p, W(0).norm1.p, px_.p, operand(ph_.p, dp, 0, false), d, dp, spec.eps, (int)n, (int)n, nullptr, nullptr,
                                 nullptr, s, spec.norm_add);
         for (int li = 0; li < L; ++li) {

@@ -127,7 +127,7 @@ void LmBlocks::mixed_set(int li, const std::string& t, const bf16_t* src, const 
     else if (is("mix.left.k.b")) bias(l.ok);
     else if (is("mix.left.v.b")) bias(l.ov);
     else if (is("mix.right.y.b")) bias(l.oy);
-    else if (is("mix.right.x.b")) bias(l.ox);
+    else if (is("mix.right.x.b")) { bias(l.ox); x_bias_set_.insert(li); }
     else if (is("mix.o") || is("mix.left.o")) output(0);
     else if (is("mix.right.o")) output(l.KR);
     else if (is("mix.left.o.b")) norm_row(w.bias_o, src, N, dp, s);
@@ -143,6 +143,11 @@ void LmBlocks::mixed_set(int li, const std::string& t, const bf16_t* src, const 
     else if (is("mix.right.ri.b")) plain(w.ri_b);
     else if (is("mix.right.lam")) { w.recur_c.alloc(N); launch_softplus_scaled(src, w.recur_c.p, N, 8.0f, s); }
     else throw MisError(MIS_ERR_INVALID_INPUT, "unexpected tensor " + t);
+    if (l.kind == BLOCK_PARALLEL && !w.conv32.p && w.conv.p && w.conv_b.p && x_bias_set_.count(li)) {
+        const RecurDims& R = l.R;
+        w.conv32.alloc((size_t)(R.taps + 2) * R.W);
+        launch_conv_tables(w.conv.p, w.conv_b.p, w.bias1.p + l.ox, w.conv32.p, w.conv32.p + (size_t)R.taps * R.W, w.conv32.p + (size_t)(R.taps + 1) * R.W, R.W, R.taps, s);
+    }
     if (l.kind == BLOCK_DECAY && !w.decay.p) {
         const std::vector<float>& c = spec.layers[li].decay.decay;
         w.decay.alloc(c.size());
@@ -180,7 +185,8 @@ void LmBlocks::mixed_buffers(MixBuffers& b, int rows, hipStream_t s) {
     for (auto& l : layers_) {
         if (l.kind == BLOCK_LATENT) continue;
         mixed = true;
-        n_u = std::max(n_u, (size_t)l.R.B * l.R.np); n_raw = std::max(n_raw, (size_t)l.R.B * l.R.nt * 16);
+        if (f32) { n_u = std::max(n_u, (size_t)l.R.B * l.R.np); n_raw = std::max(n_raw, (size_t)l.R.B * l.R.nt * 16); }
+        else if (&b == &pmix_) n_u = n_raw = std::max(n_u, (size_t)l.R.W);      // local states, decays, carried states
         n_ss = std::max(n_ss, (size_t)l.S.H * l.S.ns); n_ff = std::max(n_ff, (size_t)l.ffp);
         if (&b == &mix_ && l.shares > 1) n_part = std::max(n_part, (size_t)l.shares * batch_ * l.A.H * l.A.Ep);
     }
@@ -200,7 +206,9 @@ void LmBlocks::mixer(int li, const float* proj, void* q, const Operand& out, con
         DecayParams p{};
         p.proj = proj; p.ld = l.Nqkv; p.oq = l.oq; p.ok = l.ok; p.ov = l.ov; p.og = l.og;
         p.decay = w.decay.p; p.norm = w.mix_norm.p; p.spans = r.spans; p.state = state_[li]->p; p.out = out; p.ss = b.ss.p;
-        launch_decay_any(l.S, p, r.n_spans, s);
+        if (f32 || !decay_mfma_ok(l.S)) launch_decay_any(l.S, p, r.n_spans, s);
+        else if (!r.spans.span) launch_decay_step(l.S, p, r.M, s);
+        else { p.act = reinterpret_cast<const bf16_t*>(proj); launch_decay_prefill(l.S, p, r.n_spans, s); }
         return;
     }
     const GroupedDims& A = l.A;
@@ -225,6 +233,12 @@ void LmBlocks::mixer(int li, const float* proj, void* q, const Operand& out, con
     p.proj = proj; p.ld = l.Nqkv; p.oy = l.oy; p.ox = l.ox; p.bias = w.bias1.p; p.conv = w.conv.p; p.conv_b = w.conv_b.p; p.ra_b = w.ra_b.p; p.ri_b = w.ri_b.p;
     p.c = w.recur_c.p; p.rows = r.rows; p.pos0 = r.pos0; p.spans = r.spans; p.state = state_[li]->p; p.hist = state_[li]->p + (size_t)batch_ * R.W;
     p.out = out; p.col0 = l.KR; p.out_scale = spec.layers[li].right_scale;
+    if (!f32) {
+        p.ra = w.ra.p; p.ri = w.ri.p; p.conv_t = w.conv32.p; p.conv_b32 = w.conv32.p + (size_t)R.taps * R.W; p.bias_x = p.conv_b32 + R.W;
+        if (!r.spans.span) launch_recur_step(R, p, r.M, s);
+        else launch_recur_prefill(R, p, r.chunks, r.n_chunks, b.u.p, b.raw_r.p, b.raw_g.p, s);
+        return;
+    }
     launch_conv_rows(R, p, b.u.p, r.M, s);
     GemmF32 g{};
     g.X = b.u.p; g.ldx = R.B * R.np; g.xz = R.np; g.wz = (size_t)R.nt * 16 * R.np; g.ldo = R.B * R.nt * 16; g.oz = R.nt * 16;
@@ -290,7 +304,10 @@ void LmBlocks::mixed_pass_layer(int li, const MixRows& r, hipStream_t s) {
         else launch_gemm_pf(PF_F32, (const bf16_t*)X, Wp, out, M, N, K, s);
     };
     const Operand h = operand(ph_.p, dp, 0, false);
-    product(ph_.p, w.w1.p, pqkv_.p, l.Nqkv, dp);
+    if (!f32 && l.kind == BLOCK_DECAY && decay_mfma_ok(l.S)) {
+        PfExtra ex; ex.ldc = l.Nqkv; ex.split = l.og / 16;
+        launch_gemm_pf(PF_ACT_ROWS, (const bf16_t*)ph_.p, w.w1.p, pqkv_.p, M, l.Nqkv, dp, s, ex);
+    } else product(ph_.p, w.w1.p, pqkv_.p, l.Nqkv, dp);
     mixer(li, pqkv_.p, pq_.p, operand(at, l.Ko, 0, false), r, pmix_, s);
     product(at, w.wo.p, pmix_.part.p, dp, l.Ko);
     const SublayerOut y1 = mixer_out(pmix_.part.p, 1, l.kind == BLOCK_DECAY, l.S, pmix_.ss.p, w.bias_o.p, spec.layers[li].left_scale);

@@ -64,7 +64,8 @@ enum { PF_F32 = 0, PF_RESID = 1, PF_SILU = 2,
        PF_SCALED_ADD = 4,        // float32 C[M][ldc] += ls[n] * y
        PF_ROWS_BF16 = 5,         // bf16 row-major [M][ldc]; rows of X gathered: row m at X + xrow[m] * ldx
        PF_SOFTCAP = 6,           // float32 [M][ldc]: cap tanh(scale y / cap)
-       PF_SWIGLU = 7 };          // PF_SILU in float32 up to one rounding
+       PF_SWIGLU = 7,            // PF_SILU in float32 up to one rounding
+       PF_ACT_ROWS = 8 };        // bf16 row-major [M][ldc]: T(silu(y)) in the tiles below PfExtra::split, T(sigmoid(y)) in the others
 struct PfExtra { int ldx = 0; const int32_t* xrow = nullptr; int ldc = 0; void* out2 = nullptr; int split = 0, ld2 = 0; const bf16_t* ls = nullptr; float scale = 1.0f, cap = 0.0f; };
 void launch_gemm_pf(int epi, const bf16_t* X, const bf16_t* Wp, void* C, int M, int N, int K, hipStream_t s, const PfExtra& ex = PfExtra());
 void launch_pf_embed_rmsnorm(const bf16_t* emb, const int32_t* prompt, const int32_t* lens, int Lmax, int t0, int Tc, int batch, int Mpad, int vocab,

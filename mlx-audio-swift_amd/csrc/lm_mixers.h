@@ -70,6 +70,8 @@ struct RecurParams {
     const float* proj; int ld, oy, ox;
     const bf16_t* bias;         // [ld]
     const bf16_t *conv, *conv_b, *ra_b, *ri_b;
+    const bf16_t *ra, *ri;      // packed per block [B][nt][np / 32][64][8]
+    const float *conv_t, *conv_b32, *bias_x;        // [taps][W], [W], [W]: the same values in float32, channels side by side
     const float* c;             // [W] 8 softplus(lam)
     RowTable rows; const int32_t* pos0;     // pos0: first position of the row's span (null: the row's own)
     SpanTable spans;
@@ -81,6 +83,14 @@ struct RecurParams {
 void launch_conv_rows(const RecurDims& D, const RecurParams& p, float* u, int rows, hipStream_t s);
 // raw products [rows][B][nt 16] -> recurrence along every span, times gelu of the other branch; leaves state and history behind the span
 void launch_gated_scan_any(const RecurDims& D, const RecurParams& p, const float* u, const float* raw_r, const float* raw_g, int spans, hipStream_t s);
+// matrix cores, bf16 (lm_recurrent.hip).  Decode: convolution, gates, state, operand in one launch; at most 64 rows
+void launch_recur_step(const RecurDims& D, const RecurParams& p, int rows, hipStream_t s);
+// prompt: spans in chunks of RECUR_CHUNK rows (only the last of a span may be shorter)
+#define RECUR_CHUNK 64
+struct RecurChunk { RowSpan rows; int32_t span, span_pos0, index, last; };      // index: in the span; last: of the span
+void launch_recur_prefill(const RecurDims& D, const RecurParams& p, const RecurChunk* chunks, int n_chunks, float* loc, float* dec, float* carry0, hipStream_t s);
+// float32 copies [taps][W], [W], [W] of the convolution's weights and bias and of the input's bias
+void launch_conv_tables(const bf16_t* conv, const bf16_t* conv_b, const bf16_t* bias_x, float* conv_t, float* conv_b32, float* bias_x32, int W, int taps, hipStream_t s);
 void launch_softplus_scaled(const bf16_t* lam, float* out, int n, float scale, hipStream_t s);
 
 // ---- attention with a decayed outer-product state, per head: S = c S + k v^T, o = S^T q
@@ -88,6 +98,7 @@ struct DecayDims { int H, D, E, Es, ns; };              // Es: row stride of the
 DecayDims decay_dims(int H, int D, int E);
 struct DecayParams {
     const float* proj; int ld, oq, ok, ov, og;          // raw projections; q, k, v go through silu, the gate through a sigmoid
+    const bf16_t* act;          // prompt on the matrix cores, instead of proj: silu(q, k, v), sigmoid(gate)
     const float* decay;         // [H]
     const bf16_t* norm;         // [H E]
     SpanTable spans;
@@ -95,4 +106,9 @@ struct DecayParams {
     Operand out;                // o * norm * sigmoid(gate), not yet divided by the row's root mean square
     float* ss;                  // [rows][H ns] sums of squares of o
 };
+// any sizes, either element type
 void launch_decay_any(const DecayDims& D, const DecayParams& p, int spans, hipStream_t s);
+// bf16 (lm_recurrent.hip)
+bool decay_mfma_ok(const DecayDims& D);
+void launch_decay_step(const DecayDims& D, const DecayParams& p, int rows, hipStream_t s);
+void launch_decay_prefill(const DecayDims& D, const DecayParams& p, int spans, hipStream_t s);

@@ -219,7 +219,15 @@ __global__ void __launch_bounds__(256, 2) k_gemm_pf(PfGemmParams p) {
                 if constexpr (EPI >= PF_SPLIT_RELU2 && EPI != PF_SWIGLU) {
                     float v[4] = {acc[i][j][0], acc[i][j][1], acc[i][j][2], acc[i][j][3]};
                     float* c32 = reinterpret_cast<float*>(p.C) + (size_t)m * p.ex.ldc + n;
-                    if (EPI == PF_ROWS_BF16 || (EPI == PF_SPLIT_RELU2 && tile >= p.ex.split)) {
+                    if (EPI == PF_ACT_ROWS) {
+#pragma unroll
+                        for (int e = 0; e < 4; ++e) {
+                            const float sg = 1.0f / (1.0f + __expf(-v[e]));
+                            v[e] = tile < p.ex.split ? v[e] * sg : sg;
+                        }
+                        *reinterpret_cast<uint2*>(reinterpret_cast<bf16_t*>(p.C) + (size_t)m * p.ex.ldc + n) =
+                            make_uint2((uint32_t)f32_to_bf16(v[0]) | ((uint32_t)f32_to_bf16(v[1]) << 16), (uint32_t)f32_to_bf16(v[2]) | ((uint32_t)f32_to_bf16(v[3]) << 16));
+                    } else if (EPI == PF_ROWS_BF16 || (EPI == PF_SPLIT_RELU2 && tile >= p.ex.split)) {
                         uint16_t res[4];
 #pragma unroll
                         for (int e = 0; e < 4; ++e) {
@@ -283,6 +291,7 @@ void launch_gemm_pf(int epi, const bf16_t* X, const bf16_t* Wp, void* C, int M, 
     else if (epi == PF_ROWS_BF16) hipLaunchKernelGGL((k_gemm_pf<PF_ROWS_BF16>), grid, block, 0, s, p);
     else if (epi == PF_SOFTCAP) hipLaunchKernelGGL((k_gemm_pf<PF_SOFTCAP>), grid, block, 0, s, p);
     else if (epi == PF_SWIGLU) hipLaunchKernelGGL((k_gemm_pf<PF_SWIGLU>), grid, block, 0, s, p);
+    else if (epi == PF_ACT_ROWS) hipLaunchKernelGGL((k_gemm_pf<PF_ACT_ROWS>), grid, block, 0, s, p);
     else throw MisError(MIS_ERR_GENERATION_FAILED, "unknown prefill GEMM epilogue");
 }
 void launch_pf_embed_rmsnorm(const bf16_t* emb, const int32_t* prompt, const int32_t* lens, int Lmax, int t0, int Tc, int batch, int Mpad, int vocab,
