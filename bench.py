@@ -361,19 +361,30 @@ def latent_config(z, window):
                 layers=[dict(type="latent_attention", mixer=mx, mlp=dict(kind="dense", ff=z["ff"]))] * z["layers"])
 
 
+def vamunex_config(z, window):
+    """Parallel and lightning layers in turn, at the Llama chain's weight count per layer: half the attention heads beside a recurrence of half the
+    width, or half as many lightning heads (five projections instead of four narrower ones)."""
+    H, G, D, w = z["heads"] // 2, z["kv_heads"] // 2, z["dim"], z["width"]
+    mlp = dict(kind="dense", ff=z["ff"])
+    left = dict(heads=H, kv_heads=G, dim=D, vdim=z["vdim"], scale=D ** -0.5, mask=dict(size=window, keep_first=4), rot=dict(base=500000.0, dims=D))
+    par = dict(type="parallel", mixer=dict(left=left, right=dict(width=w // 2, blocks=max(1, w // 512), conv=4), left_scale=1.0, right_scale=1.0), mlp=mlp)
+    lit = dict(type="lightning", mixer=dict(heads=H, dim=D, vdim=z["vdim"], decay=[1.0 - 2.0 ** (-1 - 7.0 * a / H) for a in range(H)]), mlp=mlp)
+    return dict(architecture="Vamunex", width=w, vocab=z["vocab"], norm=dict(eps=1e-6), layers=[par, lit] * (z["layers"] // 2))
+
+
 def latent_lm_bench(args):
-    """--latent-lm: prefill and decode throughput of the Rugunex design (random weights) beside the Llama chain at equal size; one JSON line per
-    (size, batch, prompt).  Greedy generation through the same loop for both; prefill and decode are timed by the engine with HIP events."""
+    """--latent-lm, --vamunex-lm: prefill and decode throughput of a layer-list design (random weights) beside the Llama chain at equal size; one JSON
+    line per (size, batch, prompt).  Greedy generation through the same loop for all; prefill and decode are timed by the engine with HIP events."""
     import ctypes as C
     import mlx_audio_swift_amd as mas
     L = mas._lib.lib()
-    window, new = args.latent_window, args.latent_new
-    cases = [tuple(int(x) for x in c.split("x")) for c in args.latent_cases.split(",")]
-    for name in args.latent_sizes.split(","):
+    window, new = args.lm_window, args.lm_new
+    cases = [tuple(int(x) for x in c.split("x")) for c in args.lm_cases.split(",")]
+    for name in args.lm_sizes.split(","):
         z = LATENT_SIZES[name]
-        for kind in args.latent_models.split(","):
-            if kind == "rugunex":
-                m = mas.BlockLanguageModel.synthetic(latent_config(z, window))
+        for kind in (args.lm_models or ("vamunex,llama" if args.vamunex_lm else "rugunex,llama")).split(","):
+            if kind in ("rugunex", "vamunex"):
+                m = mas.BlockLanguageModel.synthetic((latent_config if kind == "rugunex" else vamunex_config)(z, window))
             else:
                 m = mas.LlamaTTSModel.synthetic(mas.LlamaTTSConfiguration(
                     hidden_size=z["width"], num_hidden_layers=z["layers"], intermediate_size=z["ff"], num_attention_heads=z["heads"],
@@ -392,8 +403,8 @@ def latent_lm_bench(args):
                     if it >= args.warmup:
                         cur = (t["prefill_ms"], t["decode_ms"] / t["steps"])
                         best = cur if best is None else (min(best[0], cur[0]), min(best[1], cur[1]))
-                print(json.dumps({"bench": "latent-lm", "size": name, "model": kind, "batch": batch, "prompt": prompt, "new_tokens": new,
-                                  "window": window if kind == "rugunex" else None, "prefill_ms": round(best[0], 3),
+                print(json.dumps({"bench": "vamunex-lm" if args.vamunex_lm else "latent-lm", "size": name, "model": kind, "batch": batch, "prompt": prompt, "new_tokens": new,
+                                  "window": None if kind == "llama" else window, "prefill_ms": round(best[0], 3),
                                   "prefill_tokens_per_s": round(batch * prompt / best[0] * 1e3), "decode_step_ms": round(best[1], 4),
                                   "decode_tokens_per_s": round(batch / best[1] * 1e3), "dtype": "bf16", "data": "synthetic"}), flush=True)
             m.close()
@@ -407,13 +418,14 @@ def main():
     ap.add_argument("--no-cpu-baseline", action="store_true")
     ap.add_argument("--no-secondary", action="store_true", help="skip the secondary configurations (Whisper / Soprano / Qwen3-TTS) after the timed region")
     ap.add_argument("--latent-lm", action="store_true", help="instead of the headline workload: the Rugunex design beside the Llama chain at equal size")
-    ap.add_argument("--latent-sizes", default="3b,small")
-    ap.add_argument("--latent-cases", default="1x512,32x512,4x2048", help="batch x prompt, comma separated")
-    ap.add_argument("--latent-models", default="rugunex,llama")
-    ap.add_argument("--latent-window", type=int, default=4096)
-    ap.add_argument("--latent-new", type=int, default=128)
+    ap.add_argument("--vamunex-lm", action="store_true", help="instead of the headline workload: the Vamunex design beside the Llama chain at equal size")
+    ap.add_argument("--lm-sizes", "--latent-sizes", default="3b,small")
+    ap.add_argument("--lm-cases", "--latent-cases", default="1x512,32x512,4x2048", help="batch x prompt, comma separated")
+    ap.add_argument("--lm-models", "--latent-models", default=None, help="of rugunex, vamunex, llama")
+    ap.add_argument("--lm-window", "--latent-window", type=int, default=4096)
+    ap.add_argument("--lm-new", "--latent-new", type=int, default=128)
     args = ap.parse_args()
-    if args.latent_lm:
+    if args.latent_lm or args.vamunex_lm:
         latent_lm_bench(args)
         return
     if args.gpus > 1 and "WORLD_SIZE" not in os.environ:

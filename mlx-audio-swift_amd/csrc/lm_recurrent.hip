@@ -5,9 +5,19 @@
 #include "lm_device.h"
 #include <math.h>
 
-__device__ __forceinline__ float rec_sigmoid(float z) { return 1.0f / (1.0f + expf(-z)); }
-__device__ __forceinline__ float rec_silu(float z) { return z / (1.0f + __expf(-z)); }
-__device__ __forceinline__ float rec_gelu_tanh(float z) { return 0.5f * z * (1.0f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z))); }
+// float32 on the hardware's base-2 exponential, reciprocal and square root (each within an ulp or two)
+#define REC_LOG2E 1.4426950408889634f
+__device__ __forceinline__ float rec_exp(float z) { return __builtin_amdgcn_exp2f(z * REC_LOG2E); }
+__device__ __forceinline__ float rec_sigmoid(float z) { return __builtin_amdgcn_rcpf(1.0f + rec_exp(-z)); }
+__device__ __forceinline__ float rec_silu(float z) { return z * rec_sigmoid(z); }
+// 0.5 (1 + tanh y) = sigmoid(2 y)
+__device__ __forceinline__ float rec_gelu_tanh(float z) { return z * rec_sigmoid(1.5957691216057308f * (z + 0.044715f * z * z * z)); }
+// sqrt(1 - a^2) for a = e^la, la <= 0: near la = 0 by the series of 1 - e^t, which the difference would cancel away
+__device__ __forceinline__ float rec_complement(float a, float la) {
+    const float t = 2.0f * la;
+    const float series = -t * (1.0f + t * (0.5f + t * (0.16666667f + t * (0.041666667f + t * (0.0083333333f + t * 0.0013888889f)))));
+    return __builtin_amdgcn_sqrtf(t > -0.25f ? series : 1.0f - a * a);
+}
 __device__ __forceinline__ uint32_t rec_pair(float a, float b) { return (uint32_t)f32_to_bf16(a) | ((uint32_t)f32_to_bf16(b) << 16); }
 
 // ============================================================================ gated linear recurrence: gates
@@ -28,7 +38,8 @@ __device__ __forceinline__ void rec_scan_step(float& a, float& b) {
     b += a * pb;
     a *= pa;
 }
-template <int MT, bool DECODE>
+// VEC: a block's channels are a multiple of 4
+template <int MT, bool DECODE, bool VEC>
 __global__ void __launch_bounds__(256, 2) k_recur_gates(RecurDims D, RecurParams p, const RecurChunk* __restrict__ chunks, float* __restrict__ loc, float* __restrict__ dec,
                                                         float* __restrict__ carry0, int rows) {
     __shared__ __attribute__((aligned(16))) bf16_t us[REC_KC / 32][2][MT][512];
@@ -39,7 +50,6 @@ __global__ void __launch_bounds__(256, 2) k_recur_gates(RecurDims D, RecurParams
     RecurChunk c{};
     if (!DECODE) c = chunks[blockIdx.x];
     const int m0 = DECODE ? 0 : c.rows.row0, nrows = DECODE ? rows : c.rows.n;
-    const bool vec = (D.n & 3) == 0;
     const int grp = tid & 15, r0 = tid >> 4;                                   // staging: 8 channels, rows r0, r0 + 16, ..
     f32x4_t ar[MT], ag[MT];
 #pragma unroll
@@ -59,38 +69,33 @@ __global__ void __launch_bounds__(256, 2) k_recur_gates(RecurDims D, RecurParams
         const int i0 = kc * REC_KC + grp * 8;                                  // channel inside the block
 #pragma unroll
         for (int t = 0; t < MT; ++t) {
-            const int r = t * 16 + r0, m = m0 + r;
-            f32x8_t u = (f32x8_t){0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
-            bool on = r < nrows && i0 < D.n;
-            if (DECODE && on) on = !p.rows.on || p.rows.on[m];
-            if (on) {
-                const int seq = DECODE ? m : c.rows.seq, pos = DECODE ? p.rows.pos[m] : c.rows.pos0 + r, pos0 = DECODE ? pos : c.span_pos0;
-                const int ch = ch0 + i0;
-                auto load8 = [&](const float* q) {
-                    f32x8_t x;
-                    if (vec) {
-                        const f32x4_t x0 = *reinterpret_cast<const f32x4_t*>(q);
-                        f32x4_t x1 = (f32x4_t){0.f, 0.f, 0.f, 0.f};
-                        if (i0 + 4 < D.n) x1 = *reinterpret_cast<const f32x4_t*>(q + 4);
-                        x = __builtin_shufflevector(x0, x1, 0, 1, 2, 3, 4, 5, 6, 7);
-                    } else {
+            const int r = t * 16 + r0;
+            // clamped places, no branches: channels past the block and rows past the end are dropped behind the sum
+            const int mc = m0 + min(r, nrows - 1), seq = DECODE ? mc : c.rows.seq, pos = DECODE ? p.rows.pos[mc] : c.rows.pos0 + min(r, nrows - 1);
+            const int pos0 = DECODE ? pos : c.span_pos0;
+            auto load8 = [&](const float* q) {
+                f32x8_t x;
+                if constexpr (VEC) {
+                    const int a0 = min(i0, D.n - 4), a1 = min(i0 + 4, D.n - 4);
+                    x = __builtin_shufflevector(*reinterpret_cast<const f32x4_t*>(q + ch0 + a0), *reinterpret_cast<const f32x4_t*>(q + ch0 + a1), 0, 1, 2, 3, 4, 5, 6, 7);
+                } else {
 #pragma unroll
-                        for (int j = 0; j < 8; ++j) x[j] = i0 + j < D.n ? q[j] : 0.0f;
-                    }
-                    return x;
-                };
-                const f32x8_t xb = load8(p.bias_x + ch);
-                u = load8(p.conv_b32 + ch);
-                for (int i = 0; i < D.taps; ++i) {
-                    const int q = pos - i;
-                    if (q < 0) break;
-                    const bool here = q >= pos0;                               // this pass's rows, or what earlier ones left
-                    const f32x8_t w = load8(p.conv_t + (size_t)(D.taps - 1 - i) * D.W + ch);
-                    const f32x8_t x = load8(here ? p.proj + (size_t)(m - i) * p.ld + p.ox + ch : p.hist + ((size_t)seq * D.taps + q % D.taps) * D.W + ch);
-#pragma unroll
-                    for (int j = 0; j < 8; ++j) u[j] += w[j] * (here ? x[j] + xb[j] : x[j]);
+                    for (int j = 0; j < 8; ++j) x[j] = q[ch0 + min(i0 + j, D.n - 1)];
                 }
+                return x;
+            };
+            const f32x8_t xb = load8(p.bias_x);
+            f32x8_t u = load8(p.conv_b32);
+            for (int i = 0; i < D.taps; ++i) {
+                const int q = pos - i;
+                const bool here = q >= pos0;                                   // this pass's rows, or what earlier ones left
+                const f32x8_t w = load8(p.conv_t + (size_t)(D.taps - 1 - i) * D.W);
+                const f32x8_t x = load8(here ? p.proj + (size_t)(mc - i) * p.ld + p.ox : p.hist + ((size_t)seq * D.taps + max(q, 0) % D.taps) * D.W);
+#pragma unroll
+                for (int j = 0; j < 8; ++j) u[j] += q < 0 ? 0.0f : w[j] * (here ? x[j] + xb[j] : x[j]);
             }
+#pragma unroll
+            for (int j = 0; j < 8; ++j) u[j] = r < nrows && i0 + j < D.n ? u[j] : 0.0f;
             bf16x8_t hi, lo;
 #pragma unroll
             for (int j = 0; j < 8; ++j) {
@@ -139,8 +144,8 @@ __global__ void __launch_bounds__(256, 2) k_recur_gates(RecurDims D, RecurParams
             const int sh = 16 * (e & 1);
             const float u = bf16_to_f32((bf16_t)((hw[e >> 1] >> sh) & 0xffffu)) + bf16_to_f32((bf16_t)((lw[e >> 1] >> sh) & 0xffffu));
             const float la = -cf[e] * rec_sigmoid(ar[t][e] + rb[e]);
-            a[e] = expf(la);
-            x[e] = sqrtf(-expm1f(2.0f * la)) * rec_sigmoid(ag[t][e] + gb[e]) * u;
+            a[e] = rec_exp(la);
+            x[e] = rec_complement(a[e], la) * rec_sigmoid(ag[t][e] + gb[e]) * u;
         }
         if (DECODE) {
             if (r >= rows || (p.rows.on && !p.rows.on[m])) continue;
@@ -178,7 +183,7 @@ __global__ void __launch_bounds__(256, 2) k_recur_gates(RecurDims D, RecurParams
             }
             if (!on) continue;
             float *lp = loc + (size_t)m * D.W + ch, *dp = dec + (size_t)m * D.W + ch;
-            if (nv == 4 && vec) {
+            if (VEC) {
                 *reinterpret_cast<float4*>(lp) = make_float4(B[0], B[1], B[2], B[3]);
                 *reinterpret_cast<float4*>(dp) = make_float4(A[0], A[1], A[2], A[3]);
             } else {
@@ -194,10 +199,13 @@ void launch_recur_step(const RecurDims& D, const RecurParams& p, int rows, hipSt
     MIS_REQUIRE(rows <= 64 && !p.rows.seq, MIS_ERR_GENERATION_FAILED, "recurrent step: more than 64 rows");
     const dim3 grid(1, D.B * cdiv(D.nt, 4)), block(256);
     switch (cdiv(rows, 16)) {
-        case 1: hipLaunchKernelGGL((k_recur_gates<1, true>), grid, block, 0, s, D, p, nullptr, nullptr, nullptr, nullptr, rows); break;
-        case 2: hipLaunchKernelGGL((k_recur_gates<2, true>), grid, block, 0, s, D, p, nullptr, nullptr, nullptr, nullptr, rows); break;
-        case 3: hipLaunchKernelGGL((k_recur_gates<3, true>), grid, block, 0, s, D, p, nullptr, nullptr, nullptr, nullptr, rows); break;
-        default: hipLaunchKernelGGL((k_recur_gates<4, true>), grid, block, 0, s, D, p, nullptr, nullptr, nullptr, nullptr, rows); break;
+#define REC_STEP(T) do { if (D.n % 4 == 0) hipLaunchKernelGGL((k_recur_gates<T, true, true>), grid, block, 0, s, D, p, nullptr, nullptr, nullptr, nullptr, rows);      \
+        else hipLaunchKernelGGL((k_recur_gates<T, true, false>), grid, block, 0, s, D, p, nullptr, nullptr, nullptr, nullptr, rows); } while (0)
+        case 1: REC_STEP(1); break;
+        case 2: REC_STEP(2); break;
+        case 3: REC_STEP(3); break;
+        default: REC_STEP(4); break;
+#undef REC_STEP
     }
 }
 // chunk: state = loc + dec * (state before the chunk), times the other branch; the chunks before it in the span give that state
@@ -208,6 +216,7 @@ __global__ void __launch_bounds__(256) k_recur_apply(RecurDims D, RecurParams p,
     if (ch >= D.W) return;
     float h = carry0[(size_t)c.span * D.W + ch];
     const int first = c.rows.row0 - c.index * RECUR_CHUNK;
+#pragma unroll 8
     for (int k = 0; k < c.index; ++k) {
         const size_t e = ((size_t)first + k * RECUR_CHUNK + RECUR_CHUNK - 1) * D.W + ch;
         h = dec[e] * h + loc[e];
@@ -215,6 +224,7 @@ __global__ void __launch_bounds__(256) k_recur_apply(RecurDims D, RecurParams p,
     const float yb = bf16_to_f32(p.bias[p.oy + ch]);
     const int t1 = min((part + 1) * (RECUR_CHUNK / 4), c.rows.n);
     float S = h;
+#pragma unroll 4
     for (int t = part * (RECUR_CHUNK / 4); t < t1; ++t) {
         const size_t m = c.rows.row0 + t;
         S = dec[m * D.W + ch] * h + loc[m * D.W + ch];
@@ -228,7 +238,9 @@ __global__ void __launch_bounds__(256) k_recur_apply(RecurDims D, RecurParams p,
     }
 }
 void launch_recur_prefill(const RecurDims& D, const RecurParams& p, const RecurChunk* chunks, int n_chunks, float* loc, float* dec, float* carry0, hipStream_t s) {
-    hipLaunchKernelGGL((k_recur_gates<RECUR_CHUNK / 16, false>), dim3(n_chunks, D.B * cdiv(D.nt, 4)), dim3(256), 0, s, D, p, chunks, loc, dec, carry0, 0);
+    const dim3 grid(n_chunks, D.B * cdiv(D.nt, 4));
+    if (D.n % 4 == 0) hipLaunchKernelGGL((k_recur_gates<RECUR_CHUNK / 16, false, true>), grid, dim3(256), 0, s, D, p, chunks, loc, dec, carry0, 0);
+    else hipLaunchKernelGGL((k_recur_gates<RECUR_CHUNK / 16, false, false>), grid, dim3(256), 0, s, D, p, chunks, loc, dec, carry0, 0);
     hipLaunchKernelGGL(k_recur_apply, dim3(n_chunks, cdiv(D.W, 64)), dim3(256), 0, s, D, p, chunks, loc, dec, carry0);
 }
 
@@ -311,7 +323,8 @@ void launch_decay_step(const DecayDims& D, const DecayParams& p, int rows, hipSt
 // q, k, v and the gate come as bf16 behind their activation (the projection's epilogue), everything that carries a decay is hi + lo.  The next chunk's
 // rows are in flight meanwhile.
 #define DCP_C 64
-template <int DT>
+// VEC: the heads' sizes are multiples of 4
+template <int DT, bool VEC>
 __global__ void __launch_bounds__(256, DT <= 4 ? 2 : 1) k_decay_prefill(DecayDims D, DecayParams p) {
     constexpr int DP = DT * 32, QS = DP + 8, TS = DCP_C + 8, NQ = (DP / 4 * 16 + 255) / 256;
     extern __shared__ __attribute__((aligned(16))) uint8_t lds[];
@@ -319,55 +332,52 @@ __global__ void __launch_bounds__(256, DT <= 4 ? 2 : 1) k_decay_prefill(DecayDim
     bf16_t* sk = sq + DCP_C * QS;                                              // [64][QS] keys
     bf16_t* st = sk + DCP_C * QS;                                              // [DP][TS] keys, transposed
     bf16_t* sv = st + DP * TS;                                                 // [64][TS] values, transposed
-    float* pw = reinterpret_cast<float*>(sv + 64 * TS);                        // [65] c^i
+    float* pw = reinterpret_cast<float*>(sv + 64 * TS) + DCP_C;                // c^i for i = 0 .. 64, zero for i = -64 .. -1 (pairs out of order)
     float* ssq = pw + 68;                                                      // [4][64]
     const int hd = blockIdx.x / D.ns, sl = blockIdx.x - hd * D.ns, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, li = lane & 15, lq = lane >> 4;
     const RowSpan sp = p.spans.span[blockIdx.y];
     const float dc = p.decay[hd];
-    if (tid <= DCP_C) pw[tid] = powf(dc, (float)tid);
-    const bool vq = (D.D & 3) == 0, vv = (D.E & 3) == 0;
+    if (tid <= 2 * DCP_C) pw[tid - DCP_C] = tid < DCP_C ? 0.0f : powf(dc, (float)(tid - DCP_C));
     float* state = p.state + ((size_t)sp.seq * D.H + hd) * D.D * D.Es + sl * 64 + wave * 16 + li;
     f32x4_t S[2 * DT];
 #pragma unroll
-    for (int t = 0; t < 2 * DT; ++t)
+    for (int t = 0; t < 2 * DT; ++t) S[t] = (f32x4_t){0.f, 0.f, 0.f, 0.f};
+    if (sp.pos0 > 0) {                                                         // (dimensions past the head meet zero queries and keys)
 #pragma unroll
-        for (int e = 0; e < 4; ++e) {
-            const int d = t * 16 + lq * 4 + e;
-            S[t][e] = sp.pos0 > 0 && d < D.D ? state[(size_t)d * D.Es] : 0.0f;
-        }
+        for (int t = 0; t < 2 * DT; ++t)
+#pragma unroll
+            for (int e = 0; e < 4; ++e) S[t][e] = state[(size_t)min(t * 16 + lq * 4 + e, D.D - 1) * D.Es];
+    }
     float nrm[4];                                                              // norm weights of this wave's outputs
 #pragma unroll
     for (int e = 0; e < 4; ++e) nrm[e] = bf16_to_f32(p.norm[hd * D.E + min(sl * 64 + wave * 16 + lq * 4 + e, D.E - 1)]);
     // an item of the staging: 4 tokens x 4 columns
+    // an unconditional load of a clamped place each (behind a branch every load would be waited for alone); `only` drops what lies outside
     uint2 rq[NQ][4], rk[NQ][4], rv[4];
-    auto load4 = [&](const bf16_t* q, int col, int limit, bool vec) {
-        uint2 x = make_uint2(0, 0);
-        if (vec) { if (col < limit) x = *reinterpret_cast<const uint2*>(q + col); }
-        else {
-            if (col < limit) x.x = q[col];
-            if (col + 1 < limit) x.x |= (uint32_t)q[col + 1] << 16;
-            if (col + 2 < limit) x.y = q[col + 2];
-            if (col + 3 < limit) x.y |= (uint32_t)q[col + 3] << 16;
-        }
-        return x;
+    auto load4 = [&](const bf16_t* q, int col, int limit) {
+        if constexpr (VEC) return *reinterpret_cast<const uint2*>(q + min(col, limit - 4));
+        else return make_uint2(q[min(col, limit - 1)] | (uint32_t)q[min(col + 1, limit - 1)] << 16, q[min(col + 2, limit - 1)] | (uint32_t)q[min(col + 3, limit - 1)] << 16);
     };
-    auto fetch = [&](int c0) {                                                 // (columns past the sizes and tokens past the span: zeros)
+    auto only = [&](uint2 x, int col, int limit, bool on) {
+        if (!on) return make_uint2(0, 0);
+        if constexpr (VEC) return col < limit ? x : make_uint2(0, 0);
+        else return make_uint2((col < limit ? x.x & 0xffffu : 0) | (col + 1 < limit ? x.x & 0xffff0000u : 0), (col + 2 < limit ? x.y & 0xffffu : 0) | (col + 3 < limit ? x.y & 0xffff0000u : 0));
+    };
+    auto fetch = [&](int c0) {
         const int n = sp.n - c0;
 #pragma unroll
         for (int i = 0; i < NQ; ++i) {
             const int it = tid + 256 * i, t4 = it / (DP / 4) * 4, col = (it % (DP / 4)) * 4;
 #pragma unroll
             for (int j = 0; j < 4; ++j) {
-                const int lim = t4 + j < n && t4 < DCP_C ? D.D : 0;
                 const bf16_t* row = p.act + (size_t)(sp.row0 + c0 + min(t4 + j, n - 1)) * p.ld;
-                rq[i][j] = load4(row + p.oq + hd * D.D, col, lim, vq);
-                rk[i][j] = load4(row + p.ok + hd * D.D, col, lim, vq);
+                rq[i][j] = load4(row + p.oq + hd * D.D, col, D.D);
+                rk[i][j] = load4(row + p.ok + hd * D.D, col, D.D);
             }
         }
         const int t4 = (tid >> 4) * 4, col = (tid & 15) * 4;
 #pragma unroll
-        for (int j = 0; j < 4; ++j)
-            rv[j] = load4(p.act + (size_t)(sp.row0 + c0 + min(t4 + j, n - 1)) * p.ld + p.ov + hd * D.E, sl * 64 + col, t4 + j < n ? D.E : 0, vv);
+        for (int j = 0; j < 4; ++j) rv[j] = load4(p.act + (size_t)(sp.row0 + c0 + min(t4 + j, n - 1)) * p.ld + p.ov + hd * D.E, sl * 64 + col, D.E);
     };
     // 4 tokens x 4 columns -> column rows of 4 tokens
     auto turn = [&](const uint2 (&r)[4], bf16_t* dst) {
@@ -387,11 +397,15 @@ __global__ void __launch_bounds__(256, DT <= 4 ? 2 : 1) k_decay_prefill(DecayDim
             if (t4 >= DCP_C) continue;
 #pragma unroll
             for (int j = 0; j < 4; ++j) {
+                rq[i][j] = only(rq[i][j], col, D.D, t4 + j < n);
+                rk[i][j] = only(rk[i][j], col, D.D, t4 + j < n);
                 *reinterpret_cast<uint2*>(sq + (t4 + j) * QS + col) = rq[i][j];
                 *reinterpret_cast<uint2*>(sk + (t4 + j) * QS + col) = rk[i][j];
             }
             turn(rk[i], st + col * TS + t4);
         }
+#pragma unroll
+        for (int j = 0; j < 4; ++j) rv[j] = only(rv[j], sl * 64 + (tid & 15) * 4, D.E, (tid >> 4) * 4 + j < n);
         turn(rv, sv + ((tid & 15) * 4) * TS + (tid >> 4) * 4);
         if (c0 + DCP_C < sp.n) fetch(c0 + DCP_C);
         const int vc = sl * 64 + wave * 16 + lq * 4;
@@ -414,16 +428,16 @@ __global__ void __launch_bounds__(256, DT <= 4 ? 2 : 1) k_decay_prefill(DecayDim
         const bf16_t* vr = sv + (wave * 16 + li) * TS + lq * 4;
 #pragma unroll 1
         for (int qt = 0; qt * 16 < n; ++qt) {
-            const uint2 gate = load4(p.act + (size_t)(sp.row0 + c0 + min(qt * 16 + li, n - 1)) * p.ld + p.og + hd * D.E, vc, D.E, vv);
+            const uint2 gate = load4(p.act + (size_t)(sp.row0 + c0 + min(qt * 16 + li, n - 1)) * p.ld + p.og + hd * D.E, vc, D.E);
             const bf16_t* qr = sq + (qt * 16 + li) * QS;
-            f32x4_t o = (f32x4_t){0.f, 0.f, 0.f, 0.f};
+            f32x4_t o = (f32x4_t){0.f, 0.f, 0.f, 0.f}, ol = o;
 #pragma unroll
             for (int k = 0; k < DT; ++k) {
                 const bf16x8_t q = two(qr + k * 32 + lq * 4, qr + k * 32 + 16 + lq * 4);
                 o = __builtin_amdgcn_mfma_f32_16x16x32_bf16(sh[k], q, o, 0, 0, 0);
-                o = __builtin_amdgcn_mfma_f32_16x16x32_bf16(sl_[k], q, o, 0, 0, 0);
+                ol = __builtin_amdgcn_mfma_f32_16x16x32_bf16(sl_[k], q, ol, 0, 0, 0);
             }
-            o *= pw[qt * 16 + li + 1];
+            o = (o + ol) * pw[qt * 16 + li + 1];
             bf16x8_t q[DT];
 #pragma unroll
             for (int k = 0; k < DT; ++k) q[k] = lds_frag(qr + k * 32 + lq * 8);
@@ -434,13 +448,13 @@ __global__ void __launch_bounds__(256, DT <= 4 ? 2 : 1) k_decay_prefill(DecayDim
 #pragma unroll
                 for (int k = 0; k < DT; ++k) {
                     a0 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(lds_frag(k0 + k * 32), q[k], a0, 0, 0, 0);
-                    if (kp * 2 + 1 <= qt) a1 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(lds_frag(k1 + k * 32), q[k], a1, 0, 0, 0);
+                    a1 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(lds_frag(k1 + k * 32), q[k], a1, 0, 0, 0);
                 }
                 bf16x8_t ph, pl;
 #pragma unroll
                 for (int j = 0; j < 8; ++j) {
                     const int d = qt * 16 + li - (kp * 32 + (j >> 2) * 16 + lq * 4 + (j & 3));
-                    const float x = d >= 0 ? (j < 4 ? a0[j & 3] : a1[j & 3]) * pw[max(d, 0)] : 0.0f;
+                    const float x = (j < 4 ? a0[j & 3] : a1[j & 3]) * pw[d];
                     const bf16_t h = f32_to_bf16(x);
                     ph[j] = (short)h;
                     pl[j] = (short)f32_to_bf16(x - bf16_to_f32(h));
@@ -462,10 +476,11 @@ __global__ void __launch_bounds__(256, DT <= 4 ? 2 : 1) k_decay_prefill(DecayDim
                 float x[4];
 #pragma unroll
                 for (int e = 0; e < 4; ++e) x[e] = vc + e < D.E ? o[e] * nrm[e] * g[e] : 0.0f;
-                if (vv) { if (vc < D.E) operand_store4(p.out, (int)m, hd * D.E + vc, x); }
+                bf16_t* dst = (bf16_t*)p.out.p + m * p.out.ld + hd * D.E + vc;
+                if constexpr (VEC) { if (vc < D.E) *reinterpret_cast<uint2*>(dst) = pack4_bf16(x); }
                 else {
 #pragma unroll
-                    for (int e = 0; e < 4; ++e) if (vc + e < D.E) operand_store1(p.out, (int)m, hd * D.E + vc + e, x[e]);
+                    for (int e = 0; e < 4; ++e) if (vc + e < D.E) dst[e] = f32_to_bf16(x[e]);
                 }
             }
         }
@@ -506,11 +521,14 @@ __global__ void __launch_bounds__(256, DT <= 4 ? 2 : 1) k_decay_prefill(DecayDim
 void launch_decay_prefill(const DecayDims& D, const DecayParams& p, int spans, hipStream_t s) {
     MIS_REQUIRE(decay_mfma_ok(D) && p.spans.span && p.out.kind == OPK_ROWS && p.out.ld % 4 == 0, MIS_ERR_GENERATION_FAILED, "decayed state prompt: bad layout");
     const dim3 grid(D.H * D.ns, spans), block(256);
-#define DCP(T) do { const size_t lds = (size_t)(2 * DCP_C * (T * 32 + 8) + T * 32 * (DCP_C + 8) + 64 * (DCP_C + 8)) * 2 + (68 + 256) * 4;        \
-        static const hipError_t attr = hipFuncSetAttribute(reinterpret_cast<const void*>(&k_decay_prefill<T>), hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024); \
+    const bool vec = D.D % 4 == 0 && D.E % 4 == 0;
+#define DCP(T) do { if (vec) DCPV(T, true); else DCPV(T, false); } while (0)
+#define DCPV(T, V) do { const size_t lds = (size_t)(2 * DCP_C * (T * 32 + 8) + T * 32 * (DCP_C + 8) + 64 * (DCP_C + 8)) * 2 + (DCP_C + 68 + 256) * 4;        \
+        static const hipError_t attr = hipFuncSetAttribute(reinterpret_cast<const void*>(&k_decay_prefill<T, V>), hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024); \
         HIP_CHECK(attr);                                                                                                                           \
-        hipLaunchKernelGGL((k_decay_prefill<T>), grid, block, lds, s, D, p); } while (0)
+        hipLaunchKernelGGL((k_decay_prefill<T, V>), grid, block, lds, s, D, p); } while (0)
     const int t = cdiv(D.D, 32);
     if (t == 1) DCP(1); else if (t == 2) DCP(2); else if (t <= 4) DCP(4); else DCP(8);
 #undef DCP
+#undef DCPV
 }
