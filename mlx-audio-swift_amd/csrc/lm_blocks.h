@@ -116,10 +116,11 @@ private:
     DevBuf<LatentTile> ptiles_;
     DevBuf<RowSpan> pspans_, pqtiles_;
     DevBuf<RecurChunk> pchunks_;
+    DevBuf<DecaySegment> psegs_;
     // what the mixers of a step / a pass leave behind each other
-    struct MixBuffers { DevBuf<float> u, raw_r, raw_g, ss, gu, part; } mix_, pmix_;
+    struct MixBuffers { DevBuf<float> u, raw_r, raw_g, ss, gu, part, ends; } mix_, pmix_;
     // rows of one pass as the mixers see them
-    struct MixRows { RowTable rows; const int32_t* pos0; SpanTable spans; int M, n_spans; const RowSpan* tiles = nullptr; int n_tiles = 0; const RecurChunk* chunks = nullptr; int n_chunks = 0; };
+    struct MixRows { RowTable rows; const int32_t* pos0; SpanTable spans; int M, n_spans; const RowSpan* tiles = nullptr; int n_tiles = 0; const RecurChunk* chunks = nullptr; int n_chunks = 0; const DecaySegment* segs = nullptr; int n_segs = 0; };
 
     int esz() const { return f32 ? 4 : 2; }
     const Weights& W(int li) const { return *w_[layers_[li].owner]; }
@@ -127,6 +128,12 @@ private:
     Operand operand(void* p, int ld, int rows_padded, bool packed) const;
     LatentRows latent_rows(int li, const float* qkv, void* q, bool expanded, const RowTable& rows) const;
     std::pair<int, int> columns(int li) const;
+    const Layer* widest_decay() const {              // the layer with the largest decayed state (null: none)
+        const Layer* w = nullptr;
+        for (auto& l : layers_)
+            if (l.kind == BLOCK_DECAY && (!w || (size_t)l.S.H * l.S.D * l.S.Es > (size_t)w->S.H * w->S.D * w->S.Es)) w = &l;
+        return w;
+    }
     void norm_row(DevBuf<bf16_t>& dst, const bf16_t* src, int n, int padded, hipStream_t s);
     void pack_rows(DevBuf<bf16_t>& dst, size_t total, int Np, int Kp, int tile0, int stride, hipStream_t s);
     // BLOCK_DECAY, BLOCK_PARALLEL

@@ -647,6 +647,16 @@ void LmBlocks::pass(const std::vector<PassEntry>& entries, const std::vector<int
             at += take; done_in_entry += take;
             if (done_in_entry == (size_t)e.n) { last.push_back({(int)at - 1, e.seq}); ++ei; done_in_entry = 0; }
         }
+        std::vector<DecaySegment> segs;
+        if (const Layer* big = widest_decay()) {
+            const int len = decay_segment_rows(big->S, (int)n, (int)spans.size());
+            for (auto& sp : spans)
+                for (int at2 = 0, k = 0, count = cdiv(sp.n, len); at2 < sp.n; at2 += len, ++k)
+                    segs.push_back(DecaySegment{RowSpan{sp.row0 + at2, std::min(len, sp.n - at2), sp.seq, sp.pos0 + at2}, k, count, len, sp.pos0});
+            psegs_.alloc(segs.size());
+            HIP_CHECK(hipMemcpyAsync(psegs_.p, segs.data(), segs.size() * sizeof(DecaySegment), hipMemcpyHostToDevice, s));
+            if (!f32 && segs.size() > spans.size()) pmix_.ends.alloc(segs.size() * big->S.H * big->S.D * big->S.Es);
+        }
         HIP_CHECK(hipMemcpyAsync(pids_.p, tokens.data() + t0, n * 4, hipMemcpyHostToDevice, s));
         HIP_CHECK(hipMemcpyAsync(pseq_.p, seq.data(), n * 4, hipMemcpyHostToDevice, s));
         HIP_CHECK(hipMemcpyAsync(ppos_.p, pos.data(), n * 4, hipMemcpyHostToDevice, s));
@@ -666,7 +676,7 @@ void LmBlocks::pass(const std::vector<PassEntry>& entries, const std::vector<int
         RowTable rows; rows.seq = pseq_.p; rows.pos = ppos_.p;
         MixRows mr;
         mr.rows = rows; mr.pos0 = ppos0_.p; mr.spans.span = pspans_.p; mr.M = (int)n; mr.n_spans = (int)spans.size(); mr.tiles = pqtiles_.p; mr.n_tiles = (int)qtiles.size();
-        mr.chunks = pchunks_.p; mr.n_chunks = (int)chunks.size();
+        mr.chunks = pchunks_.p; mr.n_chunks = (int)chunks.size(); mr.segs = psegs_.p; mr.n_segs = (int)segs.size();
         launch_rows_embed_norm2(emb_.p, pids_.p, V, g_embed_.p, W(0).norm1.p, px_.p, operand(ph_.p, dp, 0, false), d, dp, spec.eps, (int)n, (int)n, nullptr, nullptr,
                                 nullptr, s, spec.norm_add);
         for (int li = 0; li < L; ++li) {

@@ -208,7 +208,7 @@ void LmBlocks::mixer(int li, const float* proj, void* q, const Operand& out, con
         p.decay = w.decay.p; p.norm = w.mix_norm.p; p.spans = r.spans; p.state = state_[li]->p; p.out = out; p.ss = b.ss.p;
         if (f32 || !decay_mfma_ok(l.S)) launch_decay_any(l.S, p, r.n_spans, s);
         else if (!r.spans.span) launch_decay_step(l.S, p, r.M, s);
-        else { p.act = reinterpret_cast<const bf16_t*>(proj); launch_decay_prefill(l.S, p, r.n_spans, s); }
+        else { p.act = reinterpret_cast<const bf16_t*>(proj); launch_decay_prefill(l.S, p, r.segs, r.n_segs, r.n_segs > r.n_spans, b.ends.p, s); }
         return;
     }
     const GroupedDims& A = l.A;
@@ -220,22 +220,23 @@ void LmBlocks::mixer(int li, const float* proj, void* q, const Operand& out, con
     gr.rope_cos = ropes_[l.rope].cs.p; gr.rope_sin = ropes_[l.rope].sn.p; gr.rows = r.rows; gr.kc = kc; gr.vc = vc; gr.Smax = Smax_; gr.q = q; gr.f32 = f32;
     GroupedAttn ga{};
     ga.q = q; ga.kc = kc; ga.vc = vc; ga.Smax = Smax_; ga.sink = w.sink.p; ga.rows = r.rows; ga.out = out; ga.out_scale = spec.layers[li].left_scale; ga.f32 = f32;
-    if (!f32 && grouped_mfma_ok(A) && !r.spans.span) {
-        GroupedShares sh;
-        sh.S = l.shares; sh.part = b.part.p; sh.ml = share_ml_.p;
-        launch_grouped_attn_decode(A, gr, ga, sh, r.M, s);
-    } else {
-        launch_grouped_rows(A, gr, r.M, s);
-        if (!f32 && grouped_mfma_ok(A)) launch_grouped_attn_prefill(A, ga, r.tiles, r.n_tiles, s);
-        else launch_grouped_attn_any(A, ga, r.M, s);
-    }
     RecurParams p{};
     p.proj = proj; p.ld = l.Nqkv; p.oy = l.oy; p.ox = l.ox; p.bias = w.bias1.p; p.conv = w.conv.p; p.conv_b = w.conv_b.p; p.ra_b = w.ra_b.p; p.ri_b = w.ri_b.p;
     p.c = w.recur_c.p; p.rows = r.rows; p.pos0 = r.pos0; p.spans = r.spans; p.state = state_[li]->p; p.hist = state_[li]->p + (size_t)batch_ * R.W;
     p.out = out; p.col0 = l.KR; p.out_scale = spec.layers[li].right_scale;
+    const bool mfma = !f32 && grouped_mfma_ok(A), step = !r.spans.span;
+    if (!f32) { p.ra = w.ra.p; p.ri = w.ri.p; p.conv_t = w.conv32.p; p.conv_b32 = w.conv32.p + (size_t)R.taps * R.W; p.bias_x = p.conv_b32 + R.W; }
+    if (mfma && step) {                                                        // both sides in one launch
+        GroupedShares sh;
+        sh.S = l.shares; sh.part = b.part.p; sh.ml = share_ml_.p;
+        launch_grouped_attn_decode(A, gr, ga, sh, &R, &p, r.M, s);
+        return;
+    }
+    launch_grouped_rows(A, gr, r.M, s);
+    if (mfma) launch_grouped_attn_prefill(A, ga, r.tiles, r.n_tiles, s);
+    else launch_grouped_attn_any(A, ga, r.M, s);
     if (!f32) {
-        p.ra = w.ra.p; p.ri = w.ri.p; p.conv_t = w.conv32.p; p.conv_b32 = w.conv32.p + (size_t)R.taps * R.W; p.bias_x = p.conv_b32 + R.W;
-        if (!r.spans.span) launch_recur_step(R, p, r.M, s);
+        if (step) launch_recur_step(R, p, r.M, s);
         else launch_recur_prefill(R, p, r.chunks, r.n_chunks, b.u.p, b.raw_r.p, b.raw_g.p, s);
         return;
     }
@@ -266,7 +267,8 @@ void LmBlocks::mixed_step_layer(int li, const BlockRows& r, hipStream_t s) {
     const int rows = f32 ? batch_ : Mpad_;
     auto skinny = [&](const bf16_t* Wp, const void* X, float* out, int NT, int KT, int S, int N) {
         const bool wide = S == 1 && Mpad_ <= 32 && NT / 4 >= 192;              // four n-tiles per wave where the launch still fills the chip
-        launch_gemm_skinny(EPI_PARTIAL, wide ? 4 : 2, wide ? 2 : 4, Wp, (const bf16_t*)X, out, NT, KT, S, N, Mpad_, s, nullptr, wide ? 2 : 4);
+        const int R = wide ? 4 : (S == 1 && NT / 2 < 256 && getenv("TRY_R1") ? 1 : 2);
+        launch_gemm_skinny(EPI_PARTIAL, R, wide || (R == 2 && KT >= 64 && Mpad_ <= 32 && getenv("TRY_K2")) ? 2 : 4, Wp, (const bf16_t*)X, out, NT, KT, S, N, Mpad_, s, nullptr, wide ? 2 : 4);
     };
     if (f32) launch_gemm_f32(gemm32(h_.p, dp, w.w1.p, qkv_.p, l.Nqkv, batch_, l.Nqkv, dp, F32_STORE), s);
     else skinny(w.w1.p, h_.p, qkv_.p, l.Nqkv / 16, dp / 32, 1, l.Nqkv);

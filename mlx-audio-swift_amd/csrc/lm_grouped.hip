@@ -6,6 +6,7 @@
 // float32, base 2; the weights enter as bf16 hi + lo.  The sink is a key-less term of the running sum: the sum starts with it.
 #include "lm_mixers.h"
 #include "lm_device.h"
+#include "lm_recurrent.h"
 #include <math.h>
 
 #define GRP_LOG2E 1.4426950408889634f
@@ -176,14 +177,14 @@ void launch_grouped_attn_prefill(const GroupedDims& D, const GroupedAttn& p, con
 // softmax, and meet in LDS.  The block norms and rotates its heads' queries itself; the current token's key and value never come from the cache: its
 // score and value join when the waves meet (last share), the sink with the first share.  The last share's block of a group's first head tile also
 // appends the token to the caches - for the NEXT step.
-struct GrpDecodeLds { float q[16][260]; float k[260], v[260]; float m[4][16], l[4][16], self[16]; };
+template <int VT>
+struct GrpDecodeLds { float q[16][260]; float k[260], v[260]; float m[4][16], l[4][16], self[16]; float acc[2][16][VT * 16 + 4]; };
 template <int KT, int VT, bool EXACT>
-__global__ void __launch_bounds__(256, (KT <= 4 && VT <= 8) ? 2 : 1) k_grouped_attn_decode(GroupedDims D, GroupedRows r, GroupedAttn p, GroupedShares sh, int rows) {
-    __shared__ GrpDecodeLds L;
-    __shared__ float acc[2][16][VT * 16 + 4];
+__device__ __forceinline__ void grouped_decode_block(const GroupedDims& D, const GroupedRows& r, const GroupedAttn& p, const GroupedShares& sh, int rows, int bx, int g, int bz,
+                                                     GrpDecodeLds<VT>& L) {
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, li = lane & 15, lq = lane >> 4;
-    const int m = blockIdx.x % rows, sp = blockIdx.x / rows, g = blockIdx.y, R = D.H / D.G, kt_n = EXACT ? KT : D.Dp >> 5, vt_n = EXACT ? VT : D.Ep >> 4;
-    const int a0 = blockIdx.z * 16, na = min(16, R - a0), h0 = g * R + a0;     // heads h0 .. h0 + na - 1
+    const int m = bx % rows, sp = bx / rows, R = D.H / D.G, kt_n = EXACT ? KT : D.Dp >> 5, vt_n = EXACT ? VT : D.Ep >> 4;
+    const int a0 = bz * 16, na = min(16, R - a0), h0 = g * R + a0;             // heads h0 .. h0 + na - 1
     if (r.rows.on && !r.rows.on[m]) return;                                    // block-uniform
     const int pos = r.rows.pos[m], half = D.rot >> 1;
     const GrpSteps st = grp_steps(D, pos, pos);
@@ -191,7 +192,7 @@ __global__ void __launch_bounds__(256, (KT <= 4 && VT <= 8) ? 2 : 1) k_grouped_a
     const bool first = sp == 0, last = sp == sh.S - 1;
     const bf16_t* kc = (const bf16_t*)p.kc + ((size_t)m * D.G + g) * p.Smax * D.Dp;
     const bf16_t* vc = (const bf16_t*)p.vc + ((size_t)m * D.G + g) * p.Smax * D.Ep;
-    // ---- the wave's first keys are requested before anything else
+    float (*acc)[16][VT * 16 + 4] = L.acc;
     bf16x8_t ka[2][KT], va[VT];
     auto fetch_k = [&](int s) {
         const bf16_t* ks = kc + (size_t)s * 32 * D.Dp + lane * 8;
@@ -206,44 +207,51 @@ __global__ void __launch_bounds__(256, (KT <= 4 && VT <= 8) ? 2 : 1) k_grouped_a
 #pragma unroll
         for (int v = 0; v < VT; ++v) va[v] = __builtin_nontemporal_load(reinterpret_cast<const bf16x8_t*>(vs + (size_t)min(v, vt_n - 1) * 512));
     };
-    if (i0 + wave < i1) { fetch_k(st.at(i0 + wave)); fetch_v(st.at(i0 + wave)); }
-    __builtin_amdgcn_sched_barrier(0);
-    // ---- queries (and, last share, the token's key and value): bias, norm, rotation
+    // ---- queries (and, last share, the token's key and value): bias, norm, rotation; a wave per vector.  Its projections are requested before the wave's
+    // first keys (loads return in order)
     const float *cs = r.rope_cos + (size_t)pos * half, *sn = r.rope_sin + (size_t)pos * half;
     const float* row = r.proj + (size_t)m * r.ld;
-    for (int a = wave; a < na + (last ? 2 : 0); a += 4) {
-        if (a == na + 1) {                                                     // value
-            const int o = r.ov + g * D.E;
-            for (int i = lane; i < D.Ep; i += 64) L.v[i] = i < D.E ? bf16_round_f32(row[o + i] + bf16_to_f32(r.bias[o + i])) : 0.0f;
-            continue;
-        }
-        const bool is_q = a < na;
-        const int o = is_q ? r.oq + (h0 + a) * D.D : r.ok + g * D.D;
-        const bf16_t* w = is_q ? r.qn : r.kn;
-        float x[4], ss = 0.0f;                                                 // D <= 256: four dimensions a lane
+    const int n_vec = na + (last ? 2 : 0);                                     // heads, key, value
+    float x[4], xb[4], xw[4];                                                  // sizes <= 256: four dimensions a lane
+    auto load_vec = [&](int a) {
+        const int o = a < na ? r.oq + (h0 + a) * D.D : (a == na ? r.ok + g * D.D : r.ov + g * D.E), size = a <= na ? D.D : D.E;
+        const bf16_t* w = a < na ? r.qn : r.kn;
 #pragma unroll
         for (int j = 0; j < 4; ++j) {
-            const int i = lane + 64 * j;
-            x[j] = i < D.D ? row[o + i] + bf16_to_f32(r.bias[o + i]) : 0.0f;
+            const int i = min(lane + 64 * j, size - 1);
+            x[j] = row[o + i]; xb[j] = bf16_to_f32(r.bias[o + i]); xw[j] = bf16_to_f32(w[min(i, D.D - 1)]);
+        }
+    };
+    if (wave < n_vec) load_vec(wave);
+    __builtin_amdgcn_sched_barrier(0);
+    if (i0 + wave < i1) { fetch_k(st.at(i0 + wave)); fetch_v(st.at(i0 + wave)); }
+    __builtin_amdgcn_sched_barrier(0);
+    for (int a = wave; a < n_vec; a += 4) {
+        if (a != wave) load_vec(a);
+        const int size = a <= na ? D.D : D.E;
+        float ss = 0.0f;
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+            x[j] = lane + 64 * j < size ? x[j] + xb[j] : 0.0f;
             ss += x[j] * x[j];
         }
-        const float inv = 1.0f / sqrtf(wave_sum(ss) / (float)D.D + D.eps);
-        float* dst = is_q ? L.q[a] : L.k;
+        if (a == na + 1) {                                                     // value
 #pragma unroll
-        for (int j = 0; j < 4; ++j) {
-            const int i = lane + 64 * j;
-            if (i < D.Dp) dst[i] = i < D.D ? x[j] * inv * bf16_to_f32(w[i]) : 0.0f;
+            for (int j = 0; j < 4; ++j) if (lane + 64 * j < D.Ep) L.v[lane + 64 * j] = bf16_round_f32(x[j]);
+            continue;
+        }
+        const float inv = 1.0f / sqrtf(wave_sum_dpp(ss) / (float)D.D + D.eps);
+        float* dst = a < na ? L.q[a] : L.k;
+#pragma unroll
+        for (int j = 0; j < 4; ++j) if (lane + 64 * j < D.Dp) dst[lane + 64 * j] = x[j] * inv * xw[j];
+        __builtin_amdgcn_wave_barrier();                                       // (one wave's LDS accesses stay in order)
+        for (int i = lane; i < half; i += 64) {                                // rotation in place, a pair per lane
+            const float c = cs[i], s = sn[i], u = dst[i], v = dst[i + half];
+            dst[i] = u * c - v * s;
+            dst[i + half] = v * c + u * s;
         }
     }
     for (int i = threadIdx.x + na * 260; i < 16 * 260; i += 256) L.q[0][i] = 0.0f;           // columns past the heads
-    __syncthreads();
-    for (int t = threadIdx.x; t < (na + (last ? 1 : 0)) * half; t += 256) {    // rotation in place: a pair per thread
-        const int a = t / half, i = t - a * half;
-        float* x = a < na ? L.q[a] : L.k;
-        const float c = cs[i], s = sn[i], u = x[i], v = x[i + half];
-        x[i] = u * c - v * s;
-        x[i + half] = v * c + u * s;
-    }
     __syncthreads();
     if (last) {
         if (a0 == 0) {
@@ -369,6 +377,18 @@ __global__ void __launch_bounds__(256, (KT <= 4 && VT <= 8) ? 2 : 1) k_grouped_a
         *reinterpret_cast<float2*>(ml) = make_float2(M, T);
     }
 }
+// One launch of a decode step: attention blocks, then (RECUR) the blocks of a gated recurrence that reads the same projections
+template <int KT, int VT, bool EXACT, int RECUR>
+__global__ void __launch_bounds__(256, (KT <= 4 && VT <= 8) ? 2 : 1) k_grouped_attn_decode(GroupedDims D, GroupedRows r, GroupedAttn p, GroupedShares sh, int rows, int nz,
+                                                                                           RecurDims RD, RecurParams rp) {
+    __shared__ union { GrpDecodeLds<VT> attn; RecurStepLds recur; } L;
+    const int n_attn = rows * sh.S * D.G * nz;
+    int b = blockIdx.x;
+    if (RECUR && b >= n_attn) { recur_step_block<RECUR == 2>(RD, rp, rows, b - n_attn, L.recur); return; }
+    const int bx = b % (rows * sh.S);
+    b /= rows * sh.S;
+    grouped_decode_block<KT, VT, EXACT>(D, r, p, sh, rows, bx, b % D.G, b / D.G, L.attn);
+}
 // shares of a head -> operand: one wave per (row, head)
 __global__ void __launch_bounds__(256) k_grouped_shares(GroupedDims D, GroupedShares sh, Operand out, float out_scale, const uint8_t* __restrict__ on, int rows) {
     const int lane = threadIdx.x & 63, item = blockIdx.x * 4 + (threadIdx.x >> 6);
@@ -396,17 +416,23 @@ int grouped_decode_shares(const GroupedDims& D, int rows, int Smax) {
     while (S < 32 && blocks * S < 512 && steps / (S + 1) >= 8) ++S;            // two steps a wave at least
     return S;
 }
-void launch_grouped_attn_decode(const GroupedDims& D, const GroupedRows& r, const GroupedAttn& p, const GroupedShares& sh, int rows, hipStream_t s) {
-    MIS_REQUIRE(grouped_mfma_ok(D) && !p.f32 && p.Smax % 32 == 0 && sh.S >= 1 && (sh.S == 1 || (sh.part && sh.ml)) && !r.rows.seq, MIS_ERR_GENERATION_FAILED,
-                "grouped attention: bad layout");
-    const dim3 grid(rows * sh.S, D.G, cdiv(D.H / D.G, 16)), block(256);
-    const int kt = D.Dp / 32, vt = D.Ep / 16;
-#define GRP_DEC(K, V, X) hipLaunchKernelGGL((k_grouped_attn_decode<K, V, X>), grid, block, 0, s, D, r, p, sh, rows)
-    if (kt == 2 && vt == 4) GRP_DEC(2, 4, true);
-    else if (kt == 4 && vt == 8) GRP_DEC(4, 8, true);
-    else if (kt <= 2 && vt <= 4) GRP_DEC(2, 4, false);
-    else if (kt <= 4 && vt <= 8) GRP_DEC(4, 8, false);
-    else GRP_DEC(8, 16, false);
+void launch_grouped_attn_decode(const GroupedDims& D, const GroupedRows& r, const GroupedAttn& p, const GroupedShares& sh, const RecurDims* RD, const RecurParams* rp, int rows,
+                                hipStream_t s) {
+    MIS_REQUIRE(grouped_mfma_ok(D) && !p.f32 && p.Smax % 32 == 0 && sh.S >= 1 && (sh.S == 1 || (sh.part && sh.ml)) && !r.rows.seq && D.rot % 2 == 0 && D.rot <= D.D,
+                MIS_ERR_GENERATION_FAILED, "grouped attention: bad layout");
+    MIS_REQUIRE(!RD || (rp && rp->rows.pos && !rp->rows.seq), MIS_ERR_GENERATION_FAILED, "gated recurrence step: bad layout");
+    const int nz = cdiv(D.H / D.G, 16), kt = D.Dp / 32, vt = D.Ep / 16;
+    const dim3 grid(rows * sh.S * D.G * nz + (RD ? recur_step_blocks(*RD, rows) : 0)), block(256);
+    const RecurDims rd = RD ? *RD : RecurDims{};
+    const RecurParams rpp = RD ? *rp : RecurParams{};
+#define GRP_DEC(K, V, X, C) hipLaunchKernelGGL((k_grouped_attn_decode<K, V, X, C>), grid, block, 0, s, D, r, p, sh, rows, nz, rd, rpp)
+#define GRP_DECR(K, V, X) do { if (!RD) GRP_DEC(K, V, X, 0); else if (RD->n % 4) GRP_DEC(K, V, X, 1); else GRP_DEC(K, V, X, 2); } while (0)
+    if (kt == 2 && vt == 4) GRP_DECR(2, 4, true);
+    else if (kt == 4 && vt == 8) GRP_DECR(4, 8, true);
+    else if (kt <= 2 && vt <= 4) GRP_DECR(2, 4, false);
+    else if (kt <= 4 && vt <= 8) GRP_DECR(4, 8, false);
+    else GRP_DECR(8, 16, false);
+#undef GRP_DECR
 #undef GRP_DEC
     if (sh.S > 1) hipLaunchKernelGGL(k_grouped_shares, dim3(cdiv((int64_t)rows * D.H, 4)), dim3(256), 0, s, D, sh, p.out, p.out_scale, r.rows.on, rows);
 }

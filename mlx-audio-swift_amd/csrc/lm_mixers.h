@@ -55,11 +55,6 @@ void launch_grouped_attn_any(const GroupedDims& D, const GroupedAttn& p, int row
 bool grouped_mfma_ok(const GroupedDims& D);
 #define GROUPED_QT 64           // queries of one request per prompt tile
 void launch_grouped_attn_prefill(const GroupedDims& D, const GroupedAttn& p, const RowSpan* tiles, int n_tiles, hipStream_t s);
-// decode: queries, cache rows, attention and (more than one share) the shares' sum; p.q is not used
-struct GroupedShares { int S = 1; float *part = nullptr, *ml = nullptr; };      // part [S][rows][H][Ep], ml [S][rows][H][2]
-int grouped_decode_shares(const GroupedDims& D, int rows, int Smax);
-void launch_grouped_attn_decode(const GroupedDims& D, const GroupedRows& r, const GroupedAttn& p, const GroupedShares& sh, int rows, hipStream_t s);
-
 // ---- gated linear recurrence: u = conv(x);  r, g = sigmoid(block-diagonal products of u);  S = a S + sqrt(1 - a^2) g u, a = exp(-c r)
 struct RecurDims {
     int W, B, n, taps;          // channels, blocks, channels per block, convolution taps
@@ -83,7 +78,7 @@ struct RecurParams {
 void launch_conv_rows(const RecurDims& D, const RecurParams& p, float* u, int rows, hipStream_t s);
 // raw products [rows][B][nt 16] -> recurrence along every span, times gelu of the other branch; leaves state and history behind the span
 void launch_gated_scan_any(const RecurDims& D, const RecurParams& p, const float* u, const float* raw_r, const float* raw_g, int spans, hipStream_t s);
-// matrix cores, bf16 (lm_recurrent.hip).  Decode: convolution, gates, state, operand in one launch; at most 64 rows
+// matrix cores, bf16 (lm_recurrent.hip).  Decode: convolution, gates, state, operand in one launch
 void launch_recur_step(const RecurDims& D, const RecurParams& p, int rows, hipStream_t s);
 // prompt: spans in chunks of RECUR_CHUNK rows (only the last of a span may be shorter)
 #define RECUR_CHUNK 64
@@ -92,6 +87,13 @@ void launch_recur_prefill(const RecurDims& D, const RecurParams& p, const RecurC
 // float32 copies [taps][W], [W], [W] of the convolution's weights and bias and of the input's bias
 void launch_conv_tables(const bf16_t* conv, const bf16_t* conv_b, const bf16_t* bias_x, float* conv_t, float* conv_b32, float* bias_x32, int W, int taps, hipStream_t s);
 void launch_softplus_scaled(const bf16_t* lam, float* out, int n, float scale, hipStream_t s);
+
+// ---- grouped attention, decode: queries, cache rows, attention and (more than one share) the shares' sum; p.q is not used.  RD, rp non-null: a gated
+// recurrence on the same projections advances in the same launch
+struct GroupedShares { int S = 1; float *part = nullptr, *ml = nullptr; };      // part [S][rows][H][Ep], ml [S][rows][H][2]
+int grouped_decode_shares(const GroupedDims& D, int rows, int Smax);
+void launch_grouped_attn_decode(const GroupedDims& D, const GroupedRows& r, const GroupedAttn& p, const GroupedShares& sh, const RecurDims* RD, const RecurParams* rp, int rows,
+                                hipStream_t s);
 
 // ---- attention with a decayed outer-product state, per head: S = c S + k v^T, o = S^T q
 struct DecayDims { int H, D, E, Es, ns; };              // Es: row stride of the state (E % 64), ns: column slices of 64
@@ -111,4 +113,8 @@ void launch_decay_any(const DecayDims& D, const DecayParams& p, int spans, hipSt
 // bf16 (lm_recurrent.hip)
 bool decay_mfma_ok(const DecayDims& D);
 void launch_decay_step(const DecayDims& D, const DecayParams& p, int rows, hipStream_t s);
-void launch_decay_prefill(const DecayDims& D, const DecayParams& p, int spans, hipStream_t s);
+// segment index of count of one request's rows in this pass, all but the last `length` rows long (a multiple of 64); a request's segments follow each
+// other in the table.  cut: some request has more than one; ends: [n_segs][H][D][Es]
+struct DecaySegment { RowSpan rows; int32_t index, count, length, span_pos0; };
+int decay_segment_rows(const DecayDims& D, int rows, int spans);       // length to cut `rows` rows of `spans` requests into
+void launch_decay_prefill(const DecayDims& D, const DecayParams& p, const DecaySegment* segs, int n_segs, bool cut, float* ends, hipStream_t s);

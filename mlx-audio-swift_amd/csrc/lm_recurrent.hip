@@ -3,31 +3,17 @@
 // float32 values that enter a product do so as bf16 hi + lo pairs.
 #include "lm_mixers.h"
 #include "lm_device.h"
+#include "lm_recurrent.h"
 #include <math.h>
 
-// float32 on the hardware's base-2 exponential, reciprocal and square root (each within an ulp or two)
-#define REC_LOG2E 1.4426950408889634f
-__device__ __forceinline__ float rec_exp(float z) { return __builtin_amdgcn_exp2f(z * REC_LOG2E); }
-__device__ __forceinline__ float rec_sigmoid(float z) { return __builtin_amdgcn_rcpf(1.0f + rec_exp(-z)); }
-__device__ __forceinline__ float rec_silu(float z) { return z * rec_sigmoid(z); }
-// 0.5 (1 + tanh y) = sigmoid(2 y)
-__device__ __forceinline__ float rec_gelu_tanh(float z) { return z * rec_sigmoid(1.5957691216057308f * (z + 0.044715f * z * z * z)); }
-// sqrt(1 - a^2) for a = e^la, la <= 0: near la = 0 by the series of 1 - e^t, which the difference would cancel away
-__device__ __forceinline__ float rec_complement(float a, float la) {
-    const float t = 2.0f * la;
-    const float series = -t * (1.0f + t * (0.5f + t * (0.16666667f + t * (0.041666667f + t * (0.0083333333f + t * 0.0013888889f)))));
-    return __builtin_amdgcn_sqrtf(t > -0.25f ? series : 1.0f - a * a);
-}
 __device__ __forceinline__ uint32_t rec_pair(float a, float b) { return (uint32_t)f32_to_bf16(a) | ((uint32_t)f32_to_bf16(b) << 16); }
 
 // ============================================================================ gated linear recurrence: gates
-// Block = 64 output channels of one block of channels (a wave: one 16-row tile of both gate matrices) x MT 16-row tiles of rows: the batch rows of a
-// decode step or 64 consecutive tokens of one request.  The convolution's outputs u of 128 channels at a time come into LDS as hi and lo fragments; the
-// channels the block's own outputs belong to come last and stay for the epilogue.
-// Decode: the epilogue advances the state and writes the operand.  Prompt: it scans the 64 tokens - 16 on the lanes of a DPP row, the tiles one after
-// the other - and leaves, per token, the state reached from zero (loc) and the product of the decays (dec) since the chunk's start.
+// Block = 64 output channels of one block of channels (a wave: one 16-row tile of both gate matrices) x 64 consecutive tokens of one request (decode
+// steps: recur_step_block).  The convolution's outputs u of 128 channels at a time come into LDS as hi and lo fragments; the
+// channels the block's own outputs belong to come last and stay for the epilogue, which scans the 64 tokens - 16 on the lanes of a DPP row, the tiles one
+// after the other - and leaves, per token, the state reached from zero (loc) and the product of the decays (dec) since the chunk's start.
 #define REC_KC 128
-typedef float f32x8_t __attribute__((ext_vector_type(8)));
 template <int S>
 __device__ __forceinline__ float rec_shr(float v, float before) {              // lane i of a row of 16: v of lane i - S; the first S lanes: before
     return __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(__builtin_bit_cast(int, before), __builtin_bit_cast(int, v), 0x110 | S, 0xF, 0xF, false));
@@ -39,17 +25,17 @@ __device__ __forceinline__ void rec_scan_step(float& a, float& b) {
     a *= pa;
 }
 // VEC: a block's channels are a multiple of 4
-template <int MT, bool DECODE, bool VEC>
+template <bool VEC>
 __global__ void __launch_bounds__(256, 2) k_recur_gates(RecurDims D, RecurParams p, const RecurChunk* __restrict__ chunks, float* __restrict__ loc, float* __restrict__ dec,
-                                                        float* __restrict__ carry0, int rows) {
+                                                        float* __restrict__ carry0) {
+    constexpr int MT = RECUR_CHUNK / 16;
     __shared__ __attribute__((aligned(16))) bf16_t us[REC_KC / 32][2][MT][512];
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, li = lane & 15, lq = lane >> 4;
     const int slices = (D.nt + 3) >> 2, b = blockIdx.y / slices, sl = blockIdx.y - b * slices;
     const int tile = sl * 4 + wave, KT = D.np >> 5;
     const int ch0 = b * D.n;                                                   // first channel of the block
-    RecurChunk c{};
-    if (!DECODE) c = chunks[blockIdx.x];
-    const int m0 = DECODE ? 0 : c.rows.row0, nrows = DECODE ? rows : c.rows.n;
+    const RecurChunk c = chunks[blockIdx.x];
+    const int m0 = c.rows.row0, nrows = c.rows.n;
     const int grp = tid & 15, r0 = tid >> 4;                                   // staging: 8 channels, rows r0, r0 + 16, ..
     f32x4_t ar[MT], ag[MT];
 #pragma unroll
@@ -71,8 +57,7 @@ __global__ void __launch_bounds__(256, 2) k_recur_gates(RecurDims D, RecurParams
         for (int t = 0; t < MT; ++t) {
             const int r = t * 16 + r0;
             // clamped places, no branches: channels past the block and rows past the end are dropped behind the sum
-            const int mc = m0 + min(r, nrows - 1), seq = DECODE ? mc : c.rows.seq, pos = DECODE ? p.rows.pos[mc] : c.rows.pos0 + min(r, nrows - 1);
-            const int pos0 = DECODE ? pos : c.span_pos0;
+            const int mc = m0 + min(r, nrows - 1), pos = c.rows.pos0 + min(r, nrows - 1);
             auto load8 = [&](const float* q) {
                 f32x8_t x;
                 if constexpr (VEC) {
@@ -88,9 +73,9 @@ __global__ void __launch_bounds__(256, 2) k_recur_gates(RecurDims D, RecurParams
             f32x8_t u = load8(p.conv_b32);
             for (int i = 0; i < D.taps; ++i) {
                 const int q = pos - i;
-                const bool here = q >= pos0;                                   // this pass's rows, or what earlier ones left
+                const bool here = q >= c.span_pos0;                                   // this pass's rows, or what earlier ones left
                 const f32x8_t w = load8(p.conv_t + (size_t)(D.taps - 1 - i) * D.W);
-                const f32x8_t x = load8(here ? p.proj + (size_t)(mc - i) * p.ld + p.ox : p.hist + ((size_t)seq * D.taps + max(q, 0) % D.taps) * D.W);
+                const f32x8_t x = load8(here ? p.proj + (size_t)(mc - i) * p.ld + p.ox : p.hist + ((size_t)c.rows.seq * D.taps + max(q, 0) % D.taps) * D.W);
 #pragma unroll
                 for (int j = 0; j < 8; ++j) u[j] += q < 0 ? 0.0f : w[j] * (here ? x[j] + xb[j] : x[j]);
             }
@@ -147,66 +132,42 @@ __global__ void __launch_bounds__(256, 2) k_recur_gates(RecurDims D, RecurParams
             a[e] = rec_exp(la);
             x[e] = rec_complement(a[e], la) * rec_sigmoid(ag[t][e] + gb[e]) * u;
         }
-        if (DECODE) {
-            if (r >= rows || (p.rows.on && !p.rows.on[m])) continue;
-            const int pos = p.rows.pos[m];
-            float o[4];
+        const bool on = r < nrows;
+        float A[4], B[4];
 #pragma unroll
-            for (int e = 0; e < 4; ++e) {
-                if (e >= nv) { o[e] = 0.0f; continue; }
-                float* sp = p.state + (size_t)m * D.W + ch + e;
-                const float S = pos == 0 ? x[e] : a[e] * *sp + x[e];
-                *sp = S;
-                const float* pr = p.proj + (size_t)m * p.ld;
-                o[e] = S * rec_gelu_tanh(pr[p.oy + ch + e] + bf16_to_f32(p.bias[p.oy + ch + e])) * p.out_scale;
-                p.hist[((size_t)m * D.taps + pos % D.taps) * D.W + ch + e] = pr[p.ox + ch + e] + p.bias_x[ch + e];      // (a slot no row reads in this step)
-            }
-            if (nv == 4 && ((p.col0 + ch) & 3) == 0) operand_store4(p.out, m, p.col0 + ch, o);
-            else {
-#pragma unroll
-                for (int e = 0; e < 4; ++e) if (e < nv) operand_store1(p.out, m, p.col0 + ch + e, o[e]);
-            }
+        for (int e = 0; e < 4; ++e) {
+            float pa = on ? a[e] : 1.0f, pb = on ? x[e] : 0.0f;
+            rec_scan_step<1>(pa, pb);
+            rec_scan_step<2>(pa, pb);
+            rec_scan_step<4>(pa, pb);
+            rec_scan_step<8>(pa, pb);
+            B[e] = pb + pa * cb[e];
+            A[e] = pa * ca[e];
+            ca[e] = __shfl(A[e], lane | 15, 64);
+            cb[e] = __shfl(B[e], lane | 15, 64);
+        }
+        if (!on) continue;
+        float *lp = loc + (size_t)m * D.W + ch, *dp = dec + (size_t)m * D.W + ch;
+        if (VEC) {
+            *reinterpret_cast<float4*>(lp) = make_float4(B[0], B[1], B[2], B[3]);
+            *reinterpret_cast<float4*>(dp) = make_float4(A[0], A[1], A[2], A[3]);
         } else {
-            const bool on = r < nrows;
-            float A[4], B[4];
 #pragma unroll
-            for (int e = 0; e < 4; ++e) {
-                float pa = on ? a[e] : 1.0f, pb = on ? x[e] : 0.0f;
-                rec_scan_step<1>(pa, pb);
-                rec_scan_step<2>(pa, pb);
-                rec_scan_step<4>(pa, pb);
-                rec_scan_step<8>(pa, pb);
-                B[e] = pb + pa * cb[e];
-                A[e] = pa * ca[e];
-                ca[e] = __shfl(A[e], lane | 15, 64);
-                cb[e] = __shfl(B[e], lane | 15, 64);
-            }
-            if (!on) continue;
-            float *lp = loc + (size_t)m * D.W + ch, *dp = dec + (size_t)m * D.W + ch;
-            if (VEC) {
-                *reinterpret_cast<float4*>(lp) = make_float4(B[0], B[1], B[2], B[3]);
-                *reinterpret_cast<float4*>(dp) = make_float4(A[0], A[1], A[2], A[3]);
-            } else {
-#pragma unroll
-                for (int e = 0; e < 4; ++e) if (e < nv) { lp[e] = B[e]; dp[e] = A[e]; }
-            }
+            for (int e = 0; e < 4; ++e) if (e < nv) { lp[e] = B[e]; dp[e] = A[e]; }
         }
     }
-    if (!DECODE && c.index == 0 && li == 0)                                    // what the span starts from (its last chunk overwrites the state)
+    if (c.index == 0 && li == 0)                                               // what the span starts from (its last chunk overwrites the state)
         for (int e = 0; e < nv; ++e) carry0[(size_t)c.span * D.W + ch + e] = c.span_pos0 == 0 ? 0.0f : p.state[(size_t)c.rows.seq * D.W + ch + e];
 }
+template <bool VEC>
+__global__ void __launch_bounds__(256) k_recur_step(RecurDims D, RecurParams p, int rows) {
+    __shared__ RecurStepLds L;
+    recur_step_block<VEC>(D, p, rows, blockIdx.x, L);
+}
 void launch_recur_step(const RecurDims& D, const RecurParams& p, int rows, hipStream_t s) {
-    MIS_REQUIRE(rows <= 64 && !p.rows.seq, MIS_ERR_GENERATION_FAILED, "recurrent step: more than 64 rows");
-    const dim3 grid(1, D.B * cdiv(D.nt, 4)), block(256);
-    switch (cdiv(rows, 16)) {
-#define REC_STEP(T) do { if (D.n % 4 == 0) hipLaunchKernelGGL((k_recur_gates<T, true, true>), grid, block, 0, s, D, p, nullptr, nullptr, nullptr, nullptr, rows);      \
-        else hipLaunchKernelGGL((k_recur_gates<T, true, false>), grid, block, 0, s, D, p, nullptr, nullptr, nullptr, nullptr, rows); } while (0)
-        case 1: REC_STEP(1); break;
-        case 2: REC_STEP(2); break;
-        case 3: REC_STEP(3); break;
-        default: REC_STEP(4); break;
-#undef REC_STEP
-    }
+    MIS_REQUIRE(p.rows.pos && !p.rows.seq, MIS_ERR_GENERATION_FAILED, "gated recurrence step: bad layout");
+    if (D.n % 4 == 0) hipLaunchKernelGGL((k_recur_step<true>), dim3(recur_step_blocks(D, rows)), dim3(256), 0, s, D, p, rows);
+    else hipLaunchKernelGGL((k_recur_step<false>), dim3(recur_step_blocks(D, rows)), dim3(256), 0, s, D, p, rows);
 }
 // chunk: state = loc + dec * (state before the chunk), times the other branch; the chunks before it in the span give that state
 __global__ void __launch_bounds__(256) k_recur_apply(RecurDims D, RecurParams p, const RecurChunk* __restrict__ chunks, const float* __restrict__ loc,
@@ -239,8 +200,8 @@ __global__ void __launch_bounds__(256) k_recur_apply(RecurDims D, RecurParams p,
 }
 void launch_recur_prefill(const RecurDims& D, const RecurParams& p, const RecurChunk* chunks, int n_chunks, float* loc, float* dec, float* carry0, hipStream_t s) {
     const dim3 grid(n_chunks, D.B * cdiv(D.nt, 4));
-    if (D.n % 4 == 0) hipLaunchKernelGGL((k_recur_gates<RECUR_CHUNK / 16, false, true>), grid, dim3(256), 0, s, D, p, chunks, loc, dec, carry0, 0);
-    else hipLaunchKernelGGL((k_recur_gates<RECUR_CHUNK / 16, false, false>), grid, dim3(256), 0, s, D, p, chunks, loc, dec, carry0, 0);
+    if (D.n % 4 == 0) hipLaunchKernelGGL((k_recur_gates<true>), grid, dim3(256), 0, s, D, p, chunks, loc, dec, carry0);
+    else hipLaunchKernelGGL((k_recur_gates<false>), grid, dim3(256), 0, s, D, p, chunks, loc, dec, carry0);
     hipLaunchKernelGGL(k_recur_apply, dim3(n_chunks, cdiv(D.W, 64)), dim3(256), 0, s, D, p, chunks, loc, dec, carry0);
 }
 
@@ -322,10 +283,13 @@ void launch_decay_step(const DecayDims& D, const DecayParams& p, int rows, hipSt
 // hi + lo), the queries are read in that order; the pair weights go into the next product the same way (see lm_grouped.hip), keys in that order.
 // q, k, v and the gate come as bf16 behind their activation (the projection's epilogue), everything that carries a decay is hi + lo.  The next chunk's
 // rows are in flight meanwhile.
+// A long request is cut into segments that run beside each other: a first launch (ENDS) takes every segment but the last from a zero state - the first one
+// from the request's - to its end and leaves that state; the second starts segment i from the ends before it, E_0 c^(..) + .. + E_{i - 1}.  The slot of
+// the last segment's end holds the state the request came with (the last segment overwrites it).
 #define DCP_C 64
 // VEC: the heads' sizes are multiples of 4
-template <int DT, bool VEC>
-__global__ void __launch_bounds__(256, DT <= 4 ? 2 : 1) k_decay_prefill(DecayDims D, DecayParams p) {
+template <int DT, bool VEC, bool ENDS>
+__global__ void __launch_bounds__(256, DT <= 4 ? 2 : 1) k_decay_prefill(DecayDims D, DecayParams p, const DecaySegment* __restrict__ segs, float* __restrict__ ends) {
     constexpr int DP = DT * 32, QS = DP + 8, TS = DCP_C + 8, NQ = (DP / 4 * 16 + 255) / 256;
     extern __shared__ __attribute__((aligned(16))) uint8_t lds[];
     bf16_t* sq = reinterpret_cast<bf16_t*>(lds);                               // [64][QS] queries
@@ -335,18 +299,42 @@ __global__ void __launch_bounds__(256, DT <= 4 ? 2 : 1) k_decay_prefill(DecayDim
     float* pw = reinterpret_cast<float*>(sv + 64 * TS) + DCP_C;                // c^i for i = 0 .. 64, zero for i = -64 .. -1 (pairs out of order)
     float* ssq = pw + 68;                                                      // [4][64]
     const int hd = blockIdx.x / D.ns, sl = blockIdx.x - hd * D.ns, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, li = lane & 15, lq = lane >> 4;
-    const RowSpan sp = p.spans.span[blockIdx.y];
+    const DecaySegment sg = segs[blockIdx.y];
+    const RowSpan sp = sg.rows;
+    const bool last = sg.index == sg.count - 1;
+    if (ENDS && sg.count == 1) return;
     const float dc = p.decay[hd];
     if (tid <= 2 * DCP_C) pw[tid - DCP_C] = tid < DCP_C ? 0.0f : powf(dc, (float)(tid - DCP_C));
     float* state = p.state + ((size_t)sp.seq * D.H + hd) * D.D * D.Es + sl * 64 + wave * 16 + li;
     f32x4_t S[2 * DT];
 #pragma unroll
     for (int t = 0; t < 2 * DT; ++t) S[t] = (f32x4_t){0.f, 0.f, 0.f, 0.f};
-    if (sp.pos0 > 0) {                                                         // (dimensions past the head meet zero queries and keys)
+    // (dimensions past the head meet zero queries and keys)
+    const size_t slot = (size_t)D.H * D.D * D.Es;                              // a segment's end
+    float* end = ends + (size_t)blockIdx.y * slot + (size_t)hd * D.D * D.Es + sl * 64 + wave * 16 + li;
+    auto load_state = [&](const float* src, float scale) {                     // S = scale S + state
 #pragma unroll
         for (int t = 0; t < 2 * DT; ++t)
 #pragma unroll
-            for (int e = 0; e < 4; ++e) S[t][e] = state[(size_t)min(t * 16 + lq * 4 + e, D.D - 1) * D.Es];
+            for (int e = 0; e < 4; ++e) S[t][e] = scale * S[t][e] + src[(size_t)min(t * 16 + lq * 4 + e, D.D - 1) * D.Es];
+    };
+    auto store_state = [&](float* dst) {
+#pragma unroll
+        for (int t = 0; t < 2 * DT; ++t)
+#pragma unroll
+            for (int e = 0; e < 4; ++e) {
+                const int d = t * 16 + lq * 4 + e;
+                if (d < D.D) dst[(size_t)d * D.Es] = S[t][e];
+            }
+    };
+    if (ENDS) {
+        if (sg.span_pos0 > 0 && (sg.index == 0 || last)) load_state(state, 0.0f);
+        if (last) { store_state(end); return; }                                // the state the request came with
+    } else if (sg.count == 1) { if (sp.pos0 > 0) load_state(state, 0.0f); }
+    else if (sg.index == 0) { if (sp.pos0 > 0) load_state(end + (size_t)(sg.count - 1) * slot, 0.0f); }
+    else {
+        const float cs = powf(dc, (float)sg.length);
+        for (int k = 0; k < sg.index; ++k) load_state(end - (size_t)(sg.index - k) * slot, cs);
     }
     float nrm[4];                                                              // norm weights of this wave's outputs
 #pragma unroll
@@ -371,7 +359,7 @@ __global__ void __launch_bounds__(256, DT <= 4 ? 2 : 1) k_decay_prefill(DecayDim
 #pragma unroll
             for (int j = 0; j < 4; ++j) {
                 const bf16_t* row = p.act + (size_t)(sp.row0 + c0 + min(t4 + j, n - 1)) * p.ld;
-                rq[i][j] = load4(row + p.oq + hd * D.D, col, D.D);
+                if (!ENDS) rq[i][j] = load4(row + p.oq + hd * D.D, col, D.D);
                 rk[i][j] = load4(row + p.ok + hd * D.D, col, D.D);
             }
         }
@@ -397,8 +385,9 @@ __global__ void __launch_bounds__(256, DT <= 4 ? 2 : 1) k_decay_prefill(DecayDim
             if (t4 >= DCP_C) continue;
 #pragma unroll
             for (int j = 0; j < 4; ++j) {
-                rq[i][j] = only(rq[i][j], col, D.D, t4 + j < n);
                 rk[i][j] = only(rk[i][j], col, D.D, t4 + j < n);
+                if (ENDS) continue;
+                rq[i][j] = only(rq[i][j], col, D.D, t4 + j < n);
                 *reinterpret_cast<uint2*>(sq + (t4 + j) * QS + col) = rq[i][j];
                 *reinterpret_cast<uint2*>(sk + (t4 + j) * QS + col) = rk[i][j];
             }
@@ -415,72 +404,74 @@ __global__ void __launch_bounds__(256, DT <= 4 ? 2 : 1) k_decay_prefill(DecayDim
             const uint4 z = make_uint4(x.x, x.y, y.x, y.y);
             return __builtin_bit_cast(bf16x8_t, z);
         };
-        bf16x8_t sh[DT], sl_[DT];
-#pragma unroll
-        for (int k = 0; k < DT; ++k)
-#pragma unroll
-            for (int j = 0; j < 8; ++j) {
-                const float x = S[2 * k + (j >> 2)][j & 3];
-                const bf16_t h = f32_to_bf16(x);
-                sh[k][j] = (short)h;
-                sl_[k][j] = (short)f32_to_bf16(x - bf16_to_f32(h));
-            }
         const bf16_t* vr = sv + (wave * 16 + li) * TS + lq * 4;
-#pragma unroll 1
-        for (int qt = 0; qt * 16 < n; ++qt) {
-            const uint2 gate = load4(p.act + (size_t)(sp.row0 + c0 + min(qt * 16 + li, n - 1)) * p.ld + p.og + hd * D.E, vc, D.E);
-            const bf16_t* qr = sq + (qt * 16 + li) * QS;
-            f32x4_t o = (f32x4_t){0.f, 0.f, 0.f, 0.f}, ol = o;
+        if constexpr (!ENDS) {
+            bf16x8_t sh[DT], sl_[DT];
 #pragma unroll
-            for (int k = 0; k < DT; ++k) {
-                const bf16x8_t q = two(qr + k * 32 + lq * 4, qr + k * 32 + 16 + lq * 4);
-                o = __builtin_amdgcn_mfma_f32_16x16x32_bf16(sh[k], q, o, 0, 0, 0);
-                ol = __builtin_amdgcn_mfma_f32_16x16x32_bf16(sl_[k], q, ol, 0, 0, 0);
-            }
-            o = (o + ol) * pw[qt * 16 + li + 1];
-            bf16x8_t q[DT];
-#pragma unroll
-            for (int k = 0; k < DT; ++k) q[k] = lds_frag(qr + k * 32 + lq * 8);
-#pragma unroll 1
-            for (int kp = 0; kp <= qt / 2; ++kp) {
-                f32x4_t a0 = (f32x4_t){0.f, 0.f, 0.f, 0.f}, a1 = a0;
-                const bf16_t *k0 = sk + (kp * 32 + li) * QS + lq * 8, *k1 = k0 + 16 * QS;
-#pragma unroll
-                for (int k = 0; k < DT; ++k) {
-                    a0 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(lds_frag(k0 + k * 32), q[k], a0, 0, 0, 0);
-                    a1 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(lds_frag(k1 + k * 32), q[k], a1, 0, 0, 0);
-                }
-                bf16x8_t ph, pl;
+            for (int k = 0; k < DT; ++k)
 #pragma unroll
                 for (int j = 0; j < 8; ++j) {
-                    const int d = qt * 16 + li - (kp * 32 + (j >> 2) * 16 + lq * 4 + (j & 3));
-                    const float x = (j < 4 ? a0[j & 3] : a1[j & 3]) * pw[d];
+                    const float x = S[2 * k + (j >> 2)][j & 3];
                     const bf16_t h = f32_to_bf16(x);
-                    ph[j] = (short)h;
-                    pl[j] = (short)f32_to_bf16(x - bf16_to_f32(h));
+                    sh[k][j] = (short)h;
+                    sl_[k][j] = (short)f32_to_bf16(x - bf16_to_f32(h));
                 }
-                const bf16x8_t v = two(vr + kp * 32, vr + kp * 32 + 16);
-                o = __builtin_amdgcn_mfma_f32_16x16x32_bf16(v, ph, o, 0, 0, 0);
-                o = __builtin_amdgcn_mfma_f32_16x16x32_bf16(v, pl, o, 0, 0, 0);
-            }
-            // rows of o: value columns, columns: tokens
-            const int t = qt * 16 + li;
-            float ss = (o[0] * o[0] + o[1] * o[1]) + (o[2] * o[2] + o[3] * o[3]);
-            ss += __shfl_xor(ss, 16, 64);
-            ss += __shfl_xor(ss, 32, 64);
-            if (lq == 0) ssq[wave * 64 + t] = ss;
-            if (t < n) {
-                const float g[4] = {bf16_to_f32((bf16_t)(gate.x & 0xffffu)), bf16_to_f32((bf16_t)(gate.x >> 16)), bf16_to_f32((bf16_t)(gate.y & 0xffffu)),
-                                    bf16_to_f32((bf16_t)(gate.y >> 16))};
-                const size_t m = sp.row0 + c0 + t;
-                float x[4];
+#pragma unroll 1
+            for (int qt = 0; qt * 16 < n; ++qt) {
+                const uint2 gate = load4(p.act + (size_t)(sp.row0 + c0 + min(qt * 16 + li, n - 1)) * p.ld + p.og + hd * D.E, vc, D.E);
+                const bf16_t* qr = sq + (qt * 16 + li) * QS;
+                f32x4_t o = (f32x4_t){0.f, 0.f, 0.f, 0.f}, ol = o;
 #pragma unroll
-                for (int e = 0; e < 4; ++e) x[e] = vc + e < D.E ? o[e] * nrm[e] * g[e] : 0.0f;
-                bf16_t* dst = (bf16_t*)p.out.p + m * p.out.ld + hd * D.E + vc;
-                if constexpr (VEC) { if (vc < D.E) *reinterpret_cast<uint2*>(dst) = pack4_bf16(x); }
-                else {
+                for (int k = 0; k < DT; ++k) {
+                    const bf16x8_t q = two(qr + k * 32 + lq * 4, qr + k * 32 + 16 + lq * 4);
+                    o = __builtin_amdgcn_mfma_f32_16x16x32_bf16(sh[k], q, o, 0, 0, 0);
+                    ol = __builtin_amdgcn_mfma_f32_16x16x32_bf16(sl_[k], q, ol, 0, 0, 0);
+                }
+                o = (o + ol) * pw[qt * 16 + li + 1];
+                bf16x8_t q[DT];
 #pragma unroll
-                    for (int e = 0; e < 4; ++e) if (vc + e < D.E) dst[e] = f32_to_bf16(x[e]);
+                for (int k = 0; k < DT; ++k) q[k] = lds_frag(qr + k * 32 + lq * 8);
+#pragma unroll 1
+                for (int kp = 0; kp <= qt / 2; ++kp) {
+                    f32x4_t a0 = (f32x4_t){0.f, 0.f, 0.f, 0.f}, a1 = a0;
+                    const bf16_t *k0 = sk + (kp * 32 + li) * QS + lq * 8, *k1 = k0 + 16 * QS;
+#pragma unroll
+                    for (int k = 0; k < DT; ++k) {
+                        a0 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(lds_frag(k0 + k * 32), q[k], a0, 0, 0, 0);
+                        a1 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(lds_frag(k1 + k * 32), q[k], a1, 0, 0, 0);
+                    }
+                    bf16x8_t ph, pl;
+#pragma unroll
+                    for (int j = 0; j < 8; ++j) {
+                        const int d = qt * 16 + li - (kp * 32 + (j >> 2) * 16 + lq * 4 + (j & 3));
+                        const float x = (j < 4 ? a0[j & 3] : a1[j & 3]) * pw[d];
+                        const bf16_t h = f32_to_bf16(x);
+                        ph[j] = (short)h;
+                        pl[j] = (short)f32_to_bf16(x - bf16_to_f32(h));
+                    }
+                    const bf16x8_t v = two(vr + kp * 32, vr + kp * 32 + 16);
+                    o = __builtin_amdgcn_mfma_f32_16x16x32_bf16(v, ph, o, 0, 0, 0);
+                    o = __builtin_amdgcn_mfma_f32_16x16x32_bf16(v, pl, o, 0, 0, 0);
+                }
+                // rows of o: value columns, columns: tokens
+                const int t = qt * 16 + li;
+                float ss = (o[0] * o[0] + o[1] * o[1]) + (o[2] * o[2] + o[3] * o[3]);
+                ss += __shfl_xor(ss, 16, 64);
+                ss += __shfl_xor(ss, 32, 64);
+                if (lq == 0) ssq[wave * 64 + t] = ss;
+                if (t < n) {
+                    const float g[4] = {bf16_to_f32((bf16_t)(gate.x & 0xffffu)), bf16_to_f32((bf16_t)(gate.x >> 16)), bf16_to_f32((bf16_t)(gate.y & 0xffffu)),
+                                        bf16_to_f32((bf16_t)(gate.y >> 16))};
+                    const size_t m = sp.row0 + c0 + t;
+                    float x[4];
+#pragma unroll
+                    for (int e = 0; e < 4; ++e) x[e] = vc + e < D.E ? o[e] * nrm[e] * g[e] : 0.0f;
+                    bf16_t* dst = (bf16_t*)p.out.p + m * p.out.ld + hd * D.E + vc;
+                    if constexpr (VEC) { if (vc < D.E) *reinterpret_cast<uint2*>(dst) = pack4_bf16(x); }
+                    else {
+#pragma unroll
+                        for (int e = 0; e < 4; ++e) if (vc + e < D.E) dst[e] = f32_to_bf16(x[e]);
+                    }
                 }
             }
         }
@@ -507,28 +498,32 @@ __global__ void __launch_bounds__(256, DT <= 4 ? 2 : 1) k_decay_prefill(DecayDim
                 S[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(k, vl, S[t], 0, 0, 0);
             }
         }
+        if (ENDS) continue;
         __syncthreads();
         if (tid < n) p.ss[(size_t)(sp.row0 + c0 + tid) * D.H * D.ns + hd * D.ns + sl] = (ssq[tid] + ssq[64 + tid]) + (ssq[128 + tid] + ssq[192 + tid]);
     }
-#pragma unroll
-    for (int t = 0; t < 2 * DT; ++t)
-#pragma unroll
-        for (int e = 0; e < 4; ++e) {
-            const int d = t * 16 + lq * 4 + e;
-            if (d < D.D) state[(size_t)d * D.Es] = S[t][e];
-        }
+    if (ENDS) store_state(end);
+    else if (last) store_state(state);
 }
-void launch_decay_prefill(const DecayDims& D, const DecayParams& p, int spans, hipStream_t s) {
-    MIS_REQUIRE(decay_mfma_ok(D) && p.spans.span && p.out.kind == OPK_ROWS && p.out.ld % 4 == 0, MIS_ERR_GENERATION_FAILED, "decayed state prompt: bad layout");
-    const dim3 grid(D.H * D.ns, spans), block(256);
+int decay_segment_rows(const DecayDims& D, int rows, int spans) {
+    const int per = cdiv(rows, spans), blocks = D.H * D.ns * spans;            // segments of at least eight chunks, until the launch fills the chip
+    const int segs = std::max(1, std::min(per / (8 * DCP_C), cdiv(384, blocks)));
+    return (int)round_up(cdiv(per, segs), DCP_C);
+}
+void launch_decay_prefill(const DecayDims& D, const DecayParams& p, const DecaySegment* segs, int n_segs, bool cut, float* ends, hipStream_t s) {
+    MIS_REQUIRE(decay_mfma_ok(D) && p.act && segs && (!cut || ends) && p.out.kind == OPK_ROWS && p.out.ld % 4 == 0, MIS_ERR_GENERATION_FAILED, "decayed state prompt: bad layout");
+    const dim3 grid(D.H * D.ns, n_segs), block(256);
     const bool vec = D.D % 4 == 0 && D.E % 4 == 0;
 #define DCP(T) do { if (vec) DCPV(T, true); else DCPV(T, false); } while (0)
-#define DCPV(T, V) do { const size_t lds = (size_t)(2 * DCP_C * (T * 32 + 8) + T * 32 * (DCP_C + 8) + 64 * (DCP_C + 8)) * 2 + (DCP_C + 68 + 256) * 4;        \
-        static const hipError_t attr = hipFuncSetAttribute(reinterpret_cast<const void*>(&k_decay_prefill<T, V>), hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024); \
-        HIP_CHECK(attr);                                                                                                                           \
-        hipLaunchKernelGGL((k_decay_prefill<T, V>), grid, block, lds, s, D, p); } while (0)
+#define DCPV(T, V) do { if (cut) DCPE(T, V, true); DCPE(T, V, false); } while (0)
+#define DCPE(T, V, X) do {                                                                                                                               \
+        const size_t lds = (size_t)(2 * DCP_C * (T * 32 + 8) + T * 32 * (DCP_C + 8) + 64 * (DCP_C + 8)) * 2 + (DCP_C + 68 + 256) * 4;                       \
+        static const hipError_t attr = hipFuncSetAttribute(reinterpret_cast<const void*>(&k_decay_prefill<T, V, X>), hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024); \
+        HIP_CHECK(attr);                                                                                                                                   \
+        hipLaunchKernelGGL((k_decay_prefill<T, V, X>), grid, block, lds, s, D, p, segs, ends); } while (0)
     const int t = cdiv(D.D, 32);
     if (t == 1) DCP(1); else if (t == 2) DCP(2); else if (t <= 4) DCP(4); else DCP(8);
 #undef DCP
 #undef DCPV
+#undef DCPE
 }

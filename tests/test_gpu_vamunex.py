@@ -277,6 +277,24 @@ def test_recurrent_memory_reaches_far(compute):
 
 
 @both
+def test_long_prompts_in_segments(compute):
+    """Prompts long enough to be cut into segments that run beside each other, from the start and behind earlier tokens, one and several requests."""
+    cfg = config([lightning(heads=2, dim=24, vdim=40, decay=[0.9995, 0.97], mlp=None), parallel(left(heads=2, kv_heads=1, window=30), right(32, 2, 2), mlp=None),
+                  lightning(heads=1, dim=64, vdim=64, decay=[1.0], mlp=None)], width=64, vocab=50)
+    W, m = build(cfg, compute)
+    seqs = [tokens(n, 50, 70 + n) for n in (2300, 1090, 40)]
+    refs = [orc.forward(cfg, W, t) for t in seqs]
+    m.reset(1, 2304)
+    for cut in ([2300], [130, 2170], [1300, 900, 1]):
+        m.reset(1, 2304)
+        got = run_all(m, seqs[0], cut)
+        check(got, refs[0], compute, "segments")
+    m.reset(3, 2304)
+    got = m.extend([(b, t) for b, t in enumerate(seqs)], [list(range(len(t))) for t in seqs])
+    check(got, np.concatenate(refs), compute, "segments")
+
+
+@both
 def test_convolution_across_portions(compute):
     """A convolution longer than the portions: its inputs come from several of them."""
     cfg = one_side(config([parallel(left(window=4), right(48, 3, 7), mlp=None)], width=64, vocab=50), "right")
