@@ -232,7 +232,8 @@ void LmBlocks::mixer(int li, const float* proj, void* q, const Operand& out, con
         launch_grouped_attn_decode(A, gr, ga, sh, &R, &p, r.M, s);
         return;
     }
-    launch_grouped_rows(A, gr, r.M, s);
+    if (mfma) launch_grouped_rows_prefill(A, gr, r.tiles, r.n_tiles, r.M, s);
+    else launch_grouped_rows(A, gr, r.M, s);
     if (mfma) launch_grouped_attn_prefill(A, ga, r.tiles, r.n_tiles, s);
     else launch_grouped_attn_any(A, ga, r.M, s);
     if (!f32) {
@@ -267,8 +268,8 @@ void LmBlocks::mixed_step_layer(int li, const BlockRows& r, hipStream_t s) {
     const int rows = f32 ? batch_ : Mpad_;
     auto skinny = [&](const bf16_t* Wp, const void* X, float* out, int NT, int KT, int S, int N) {
         const bool wide = S == 1 && Mpad_ <= 32 && NT / 4 >= 192;              // four n-tiles per wave where the launch still fills the chip
-        const int R = wide ? 4 : (S == 1 && NT / 2 < 256 && getenv("TRY_R1") ? 1 : 2);
-        launch_gemm_skinny(EPI_PARTIAL, R, wide || (R == 2 && KT >= 64 && Mpad_ <= 32 && getenv("TRY_K2")) ? 2 : 4, Wp, (const bf16_t*)X, out, NT, KT, S, N, Mpad_, s, nullptr, wide ? 2 : 4);
+        const bool pairs = wide || (KT >= 64 && Mpad_ <= 32);                  // two waves per item instead of four
+        launch_gemm_skinny(EPI_PARTIAL, wide ? 4 : 2, pairs ? 2 : 4, Wp, (const bf16_t*)X, out, NT, KT, S, N, Mpad_, s, nullptr, wide ? 2 : 4);
     };
     if (f32) launch_gemm_f32(gemm32(h_.p, dp, w.w1.p, qkv_.p, l.Nqkv, batch_, l.Nqkv, dp, F32_STORE), s);
     else skinny(w.w1.p, h_.p, qkv_.p, l.Nqkv / 16, dp / 32, 1, l.Nqkv);

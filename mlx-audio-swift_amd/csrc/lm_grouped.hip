@@ -156,6 +156,78 @@ __global__ void __launch_bounds__(256, (KT <= 4 && VT <= 8) ? 2 : 1) k_grouped_a
         }
     }
 }
+// Projections of a pass -> query rows and caches.  Queries and keys: LPV lanes a vector, four dimensions a lane.  Values (the blocks behind n_qk): four
+// positions x four columns a thread, whole groups of four positions as one store each.
+__global__ void __launch_bounds__(256) k_grouped_rows_prefill(GroupedDims D, GroupedRows p, const RowSpan* __restrict__ tiles, int rows, int n_qk, int LPV, int vblocks) {
+    const int tid = threadIdx.x;
+    if ((int)blockIdx.x < n_qk) {
+        const int vec = (blockIdx.x * 256 + tid) / LPV, l = tid & (LPV - 1), HG = D.H + D.G, m = min(vec / HG, rows - 1), a = vec % HG;
+        const bool is_q = a < D.H, on = vec < rows * HG, in = 4 * l < D.D;
+        const int o = is_q ? p.oq + a * D.D : p.ok + (a - D.H) * D.D, i = 4 * l, ic = in ? i : 0, half = D.rot >> 1;
+        const int pos = p.rows.pos[m], seq = p.rows.seq ? p.rows.seq[m] : m;
+        const float4 x4 = *reinterpret_cast<const float4*>(p.proj + (size_t)m * p.ld + o + ic);
+        float b[4], w[4], x[4] = {x4.x, x4.y, x4.z, x4.w};
+        load4_bf16(p.bias + o + ic, b);
+        load4_bf16((is_q ? p.qn : p.kn) + ic, w);
+        const bool lowp = i < half, turn = i < D.rot;
+        const int ri = turn ? (lowp ? i : i - half) : 0;
+        float4 c = make_float4(1.f, 1.f, 1.f, 1.f), s = make_float4(0.f, 0.f, 0.f, 0.f);
+        if (half) { c = *reinterpret_cast<const float4*>(p.rope_cos + (size_t)pos * half + ri); s = *reinterpret_cast<const float4*>(p.rope_sin + (size_t)pos * half + ri); }
+        float ss = 0.0f;
+#pragma unroll
+        for (int e = 0; e < 4; ++e) { x[e] = in ? x[e] + b[e] : 0.0f; ss += x[e] * x[e]; }
+        for (int d = LPV >> 1; d > 0; d >>= 1) ss += __shfl_xor(ss, d, 64);
+        const float inv = 1.0f / sqrtf(ss / (float)D.D + D.eps);
+        const float cv[4] = {c.x, c.y, c.z, c.w}, sv[4] = {s.x, s.y, s.z, s.w};
+        const int other = (tid & 63) + (turn ? (lowp ? half >> 2 : -(half >> 2)) : 0);
+        float v[4];
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+            x[e] *= inv * w[e];
+            const float y = __shfl(x[e], other, 64);
+            v[e] = turn ? (lowp ? x[e] * cv[e] - y * sv[e] : x[e] * cv[e] + y * sv[e]) : x[e];
+        }
+        if (!on || i >= D.Dp) return;
+        bf16_t* dst = is_q ? (bf16_t*)p.q + ((size_t)m * D.H + a) * D.Dp + i
+                           : (bf16_t*)p.kc + ((((size_t)seq * D.G + a - D.H) * (p.Smax >> 4) + (pos >> 4)) * (D.Dp >> 5) + (i >> 5)) * 512 + (((i & 31) >> 3) * 16 + (pos & 15)) * 8 + (i & 7);
+        *reinterpret_cast<uint2*>(dst) = pack4_bf16(v);
+        return;
+    }
+    const int vb = blockIdx.x - n_qk, tile = vb / vblocks, e4 = D.E >> 2, it = (vb - tile * vblocks) * 256 + tid;
+    const RowSpan t = tiles[tile];
+    const int col = (it % e4) * 4, g = (it / e4) % D.G, p4 = (t.pos0 & ~3) + 4 * (it / (e4 * D.G));
+    if (p4 >= t.pos0 + t.n) return;
+    float x[4][4], b[4];
+    load4_bf16(p.bias + p.ov + g * D.E + col, b);
+#pragma unroll
+    for (int k = 0; k < 4; ++k) {
+        const int q = min(max(p4 + k, t.pos0), t.pos0 + t.n - 1);
+        const float4 f = *reinterpret_cast<const float4*>(p.proj + (size_t)(t.row0 + q - t.pos0) * p.ld + p.ov + g * D.E + col);
+        x[k][0] = f.x + b[0]; x[k][1] = f.y + b[1]; x[k][2] = f.z + b[2]; x[k][3] = f.w + b[3];
+    }
+    const bool whole = p4 >= t.pos0 && p4 + 3 < t.pos0 + t.n;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+        const int i = col + e;
+        bf16_t* dst = (bf16_t*)p.vc + ((((size_t)t.seq * D.G + g) * (p.Smax >> 5) + (p4 >> 5)) * (D.Ep >> 4) + (i >> 4)) * 512 + (((p4 & 15) >> 2) * 16 + (i & 15)) * 8 +
+                      ((p4 >> 4) & 1) * 4;
+        const float v[4] = {x[0][e], x[1][e], x[2][e], x[3][e]};
+        if (whole) *reinterpret_cast<uint2*>(dst) = pack4_bf16(v);
+        else
+#pragma unroll
+            for (int k = 0; k < 4; ++k)
+                if (p4 + k >= t.pos0 && p4 + k < t.pos0 + t.n) dst[k] = f32_to_bf16(v[k]);
+    }
+}
+void launch_grouped_rows_prefill(const GroupedDims& D, const GroupedRows& p, const RowSpan* tiles, int n_tiles, int rows, hipStream_t s) {
+    if (D.D % 4 || D.E % 4 || D.rot % 8 || D.Dp > 256 || p.f32 || p.rows.on) { launch_grouped_rows(D, p, rows, s); return; }
+    MIS_REQUIRE(p.rows.pos && p.Smax % 32 == 0 && D.rot <= D.D && D.H % D.G == 0 && p.ld % 4 == 0, MIS_ERR_GENERATION_FAILED, "grouped attention: bad layout");
+    int lpv = 8;
+    while (lpv * 4 < D.Dp) lpv *= 2;
+    const int n_qk = cdiv((int64_t)rows * (D.H + D.G) * lpv, 256), vblocks = cdiv((int64_t)(GROUPED_QT / 4 + 1) * D.G * (D.E / 4), 256);
+    hipLaunchKernelGGL(k_grouped_rows_prefill, dim3(n_qk + n_tiles * vblocks), dim3(256), 0, s, D, p, tiles, rows, n_qk, lpv, vblocks);
+}
+
 bool grouped_mfma_ok(const GroupedDims& D) { return D.Dp <= 256 && D.Ep <= 256; }
 void launch_grouped_attn_prefill(const GroupedDims& D, const GroupedAttn& p, const RowSpan* tiles, int n_tiles, hipStream_t s) {
     MIS_REQUIRE(grouped_mfma_ok(D) && !p.f32 && p.Smax % 32 == 0 && p.out.kind == OPK_ROWS && p.out.ld % 4 == 0, MIS_ERR_GENERATION_FAILED, "grouped attention: bad layout");
@@ -185,8 +257,8 @@ __device__ __forceinline__ void grouped_decode_block(const GroupedDims& D, const
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, li = lane & 15, lq = lane >> 4;
     const int m = bx % rows, sp = bx / rows, R = D.H / D.G, kt_n = EXACT ? KT : D.Dp >> 5, vt_n = EXACT ? VT : D.Ep >> 4;
     const int a0 = bz * 16, na = min(16, R - a0), h0 = g * R + a0;             // heads h0 .. h0 + na - 1
-    if (r.rows.on && !r.rows.on[m]) return;                                    // block-uniform
     const int pos = r.rows.pos[m], half = D.rot >> 1;
+    if (r.rows.on && !r.rows.on[m]) return;                                    // block-uniform
     const GrpSteps st = grp_steps(D, pos, pos);
     const int n = st.count(), per = (n + sh.S - 1) / sh.S, i0 = min(sp * per, n), i1 = min(i0 + per, n);
     const bool first = sp == 0, last = sp == sh.S - 1;
@@ -223,6 +295,10 @@ __device__ __forceinline__ void grouped_decode_block(const GroupedDims& D, const
         }
     };
     if (wave < n_vec) load_vec(wave);
+    float rc[2], rs[2];                                                        // half <= 128: two pairs a lane
+#pragma unroll
+    for (int j = 0; j < 2; ++j) { const int i = min(lane + 64 * j, max(half - 1, 0)); rc[j] = cs[i]; rs[j] = sn[i]; }
+    const float sink_raw = bf16_to_f32(p.sink[h0 + min(li, na - 1)]);
     __builtin_amdgcn_sched_barrier(0);
     if (i0 + wave < i1) { fetch_k(st.at(i0 + wave)); fetch_v(st.at(i0 + wave)); }
     __builtin_amdgcn_sched_barrier(0);
@@ -245,10 +321,13 @@ __device__ __forceinline__ void grouped_decode_block(const GroupedDims& D, const
 #pragma unroll
         for (int j = 0; j < 4; ++j) if (lane + 64 * j < D.Dp) dst[lane + 64 * j] = x[j] * inv * xw[j];
         __builtin_amdgcn_wave_barrier();                                       // (one wave's LDS accesses stay in order)
-        for (int i = lane; i < half; i += 64) {                                // rotation in place, a pair per lane
-            const float c = cs[i], s = sn[i], u = dst[i], v = dst[i + half];
-            dst[i] = u * c - v * s;
-            dst[i + half] = v * c + u * s;
+#pragma unroll
+        for (int j = 0; j < 2; ++j) {                                          // rotation in place
+            const int i = lane + 64 * j;
+            if (i >= half) continue;
+            const float u = dst[i], v = dst[i + half];
+            dst[i] = u * rc[j] - v * rs[j];
+            dst[i + half] = v * rc[j] + u * rs[j];
         }
     }
     for (int i = threadIdx.x + na * 260; i < 16 * 260; i += 256) L.q[0][i] = 0.0f;           // columns past the heads
@@ -330,7 +409,7 @@ __device__ __forceinline__ void grouped_decode_block(const GroupedDims& D, const
     __syncthreads();
     const int hd = h0 + min(li, na - 1);
     float M = fmaxf(fmaxf(L.m[0][li], L.m[1][li]), fmaxf(L.m[2][li], L.m[3][li]));
-    const float sink = first ? bf16_to_f32(p.sink[hd]) * GRP_LOG2E : -1e30f, self = last && li < na ? L.self[li] : -1e30f;
+    const float sink = first ? sink_raw * GRP_LOG2E : -1e30f, self = last && li < na ? L.self[li] : -1e30f;
     M = fmaxf(M, fmaxf(sink, self));
     float T = (L.l[0][li] * grp_exp2(L.m[0][li] - M) + L.l[1][li] * grp_exp2(L.m[1][li] - M)) + (L.l[2][li] * grp_exp2(L.m[2][li] - M) + L.l[3][li] * grp_exp2(L.m[3][li] - M));
     const float ps = last && li < na ? grp_exp2(self - M) : 0.0f;
@@ -413,7 +492,7 @@ int grouped_decode_shares(const GroupedDims& D, int rows, int Smax) {
     const int keys = D.window > 0 ? std::min(Smax, D.window + D.keep + 32) : Smax, steps = cdiv(keys, 32);
     const int blocks = rows * D.G * cdiv(D.H / D.G, 16);
     int S = 1;
-    while (S < 32 && blocks * S < 512 && steps / (S + 1) >= 8) ++S;            // two steps a wave at least
+    while (S < 32 && blocks * S < 256 && steps / (S + 1) >= 8) ++S;            // two steps a wave at least
     return S;
 }
 void launch_grouped_attn_decode(const GroupedDims& D, const GroupedRows& r, const GroupedAttn& p, const GroupedShares& sh, const RecurDims* RD, const RecurParams* rp, int rows,

@@ -54,6 +54,8 @@ void launch_grouped_attn_any(const GroupedDims& D, const GroupedAttn& p, int row
 // matrix cores, bf16 (lm_grouped.hip)
 bool grouped_mfma_ok(const GroupedDims& D);
 #define GROUPED_QT 64           // queries of one request per prompt tile
+// launch_grouped_rows for the rows of a prompt pass (bf16)
+void launch_grouped_rows_prefill(const GroupedDims& D, const GroupedRows& p, const RowSpan* tiles, int n_tiles, int rows, hipStream_t s);
 void launch_grouped_attn_prefill(const GroupedDims& D, const GroupedAttn& p, const RowSpan* tiles, int n_tiles, hipStream_t s);
 // ---- gated linear recurrence: u = conv(x);  r, g = sigmoid(block-diagonal products of u);  S = a S + sqrt(1 - a^2) g u, a = exp(-c r)
 struct RecurDims {

@@ -24,8 +24,8 @@ __device__ __forceinline__ void rec_scan_step(float& a, float& b) {
     b += a * pb;
     a *= pa;
 }
-// VEC: a block's channels are a multiple of 4
-template <bool VEC>
+// VEC: a block's channels are a multiple of 4.  TAPS4: at most four taps - a thread's four tokens follow each other and share the inputs they reach back to
+template <bool VEC, bool TAPS4>
 __global__ void __launch_bounds__(256, 2) k_recur_gates(RecurDims D, RecurParams p, const RecurChunk* __restrict__ chunks, float* __restrict__ loc, float* __restrict__ dec,
                                                         float* __restrict__ carry0) {
     constexpr int MT = RECUR_CHUNK / 16;
@@ -36,7 +36,7 @@ __global__ void __launch_bounds__(256, 2) k_recur_gates(RecurDims D, RecurParams
     const int ch0 = b * D.n;                                                   // first channel of the block
     const RecurChunk c = chunks[blockIdx.x];
     const int m0 = c.rows.row0, nrows = c.rows.n;
-    const int grp = tid & 15, r0 = tid >> 4;                                   // staging: 8 channels, rows r0, r0 + 16, ..
+    const int grp = tid & 15, r0 = tid >> 4;                                   // staging: 8 channels, rows 4 r0 .. + 3
     f32x4_t ar[MT], ag[MT];
 #pragma unroll
     for (int t = 0; t < MT; ++t) ar[t] = ag[t] = (f32x4_t){0.f, 0.f, 0.f, 0.f};
@@ -53,44 +53,66 @@ __global__ void __launch_bounds__(256, 2) k_recur_gates(RecurDims D, RecurParams
         }
         if (cc) __syncthreads();
         const int i0 = kc * REC_KC + grp * 8;                                  // channel inside the block
+        // clamped places, no branches: channels past the block and rows past the end are dropped behind the sum
+        auto load8 = [&](const float* v) {
+            f32x8_t x;
+            if constexpr (VEC) {
+                const int a0 = min(i0, D.n - 4), a1 = min(i0 + 4, D.n - 4);
+                x = __builtin_shufflevector(*reinterpret_cast<const f32x4_t*>(v + ch0 + a0), *reinterpret_cast<const f32x4_t*>(v + ch0 + a1), 0, 1, 2, 3, 4, 5, 6, 7);
+            } else {
 #pragma unroll
-        for (int t = 0; t < MT; ++t) {
-            const int r = t * 16 + r0;
-            // clamped places, no branches: channels past the block and rows past the end are dropped behind the sum
-            const int mc = m0 + min(r, nrows - 1), pos = c.rows.pos0 + min(r, nrows - 1);
-            auto load8 = [&](const float* q) {
-                f32x8_t x;
-                if constexpr (VEC) {
-                    const int a0 = min(i0, D.n - 4), a1 = min(i0 + 4, D.n - 4);
-                    x = __builtin_shufflevector(*reinterpret_cast<const f32x4_t*>(q + ch0 + a0), *reinterpret_cast<const f32x4_t*>(q + ch0 + a1), 0, 1, 2, 3, 4, 5, 6, 7);
-                } else {
+                for (int j = 0; j < 8; ++j) x[j] = v[ch0 + min(i0 + j, D.n - 1)];
+            }
+            return x;
+        };
+        const f32x8_t xb = load8(p.bias_x), u0 = load8(p.conv_b32);
+        auto input = [&](int r) {                                              // of the convolution at row r of the chunk (below 0: before it)
+            const int at = min(r, nrows - 1), q = c.rows.pos0 + at;
+            const bool here = q >= c.span_pos0;                                // this pass's rows, or what earlier ones left
+            f32x8_t x = load8(here ? p.proj + (size_t)(m0 + at) * p.ld + p.ox : p.hist + ((size_t)c.rows.seq * D.taps + max(q, 0) % D.taps) * D.W);
+            if (here) x += xb;
 #pragma unroll
-                    for (int j = 0; j < 8; ++j) x[j] = q[ch0 + min(i0 + j, D.n - 1)];
-                }
-                return x;
-            };
-            const f32x8_t xb = load8(p.bias_x);
-            f32x8_t u = load8(p.conv_b32);
-            for (int i = 0; i < D.taps; ++i) {
-                const int q = pos - i;
-                const bool here = q >= c.span_pos0;                                   // this pass's rows, or what earlier ones left
-                const f32x8_t w = load8(p.conv_t + (size_t)(D.taps - 1 - i) * D.W);
-                const f32x8_t x = load8(here ? p.proj + (size_t)(mc - i) * p.ld + p.ox : p.hist + ((size_t)c.rows.seq * D.taps + max(q, 0) % D.taps) * D.W);
+            for (int j = 0; j < 8; ++j) x[j] = q < 0 ? 0.0f : x[j];
+            return x;
+        };
+        f32x8_t u[MT];
 #pragma unroll
-                for (int j = 0; j < 8; ++j) u[j] += q < 0 ? 0.0f : w[j] * (here ? x[j] + xb[j] : x[j]);
+        for (int t = 0; t < MT; ++t) u[t] = u0;
+        if constexpr (TAPS4) {
+            f32x8_t w[4];
+#pragma unroll
+            for (int i = 0; i < 4; ++i) {
+                w[i] = load8(p.conv_t + (size_t)max(D.taps - 1 - i, 0) * D.W);
+                if (i >= D.taps) w[i] = (f32x8_t){0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
             }
 #pragma unroll
-            for (int j = 0; j < 8; ++j) u[j] = r < nrows && i0 + j < D.n ? u[j] : 0.0f;
+            for (int k = 0; k < MT + 3; ++k) {                                 // row r0 MT + k - 3 is what tap t - (k - 3) of token t reads
+                const f32x8_t x = input(r0 * MT + k - 3);
+#pragma unroll
+                for (int t = 0; t < MT; ++t)
+                    if (t - (k - 3) >= 0 && t - (k - 3) < 4) u[t] += w[t - (k - 3)] * x;
+            }
+        } else {
+            for (int i = 0; i < D.taps; ++i) {
+                const f32x8_t w = load8(p.conv_t + (size_t)(D.taps - 1 - i) * D.W);
+#pragma unroll
+                for (int t = 0; t < MT; ++t) u[t] += w * input(r0 * MT + t - i);
+            }
+        }
+#pragma unroll
+        for (int t = 0; t < MT; ++t) {
+            const int r = r0 * MT + t;
             bf16x8_t hi, lo;
 #pragma unroll
             for (int j = 0; j < 8; ++j) {
-                const bf16_t h = f32_to_bf16(u[j]);
+                const float v = r < nrows && i0 + j < D.n ? u[t][j] : 0.0f;
+                const bf16_t h = f32_to_bf16(v);
                 hi[j] = (short)h;
-                lo[j] = (short)f32_to_bf16(u[j] - bf16_to_f32(h));
+                lo[j] = (short)f32_to_bf16(v - bf16_to_f32(h));
             }
-            const int kt = grp >> 2, at = ((grp & 3) * 16 + r0) * 8;
-            *reinterpret_cast<bf16x8_t*>(&us[kt][0][t][at]) = hi;
-            *reinterpret_cast<bf16x8_t*>(&us[kt][1][t][at]) = lo;
+            const int kt = grp >> 2, at = ((grp & 3) * 16 + (r & 15)) * 8;
+            *reinterpret_cast<bf16x8_t*>(&us[kt][0][r >> 4][at]) = hi;
+            *reinterpret_cast<bf16x8_t*>(&us[kt][1][r >> 4][at]) = lo;
         }
         __syncthreads();
 #pragma unroll
@@ -200,8 +222,10 @@ __global__ void __launch_bounds__(256) k_recur_apply(RecurDims D, RecurParams p,
 }
 void launch_recur_prefill(const RecurDims& D, const RecurParams& p, const RecurChunk* chunks, int n_chunks, float* loc, float* dec, float* carry0, hipStream_t s) {
     const dim3 grid(n_chunks, D.B * cdiv(D.nt, 4));
-    if (D.n % 4 == 0) hipLaunchKernelGGL((k_recur_gates<true>), grid, dim3(256), 0, s, D, p, chunks, loc, dec, carry0);
-    else hipLaunchKernelGGL((k_recur_gates<false>), grid, dim3(256), 0, s, D, p, chunks, loc, dec, carry0);
+#define REC_GATES(V, T) hipLaunchKernelGGL((k_recur_gates<V, T>), grid, dim3(256), 0, s, D, p, chunks, loc, dec, carry0)
+    if (D.n % 4 == 0) { if (D.taps <= 4) REC_GATES(true, true); else REC_GATES(true, false); }
+    else { if (D.taps <= 4) REC_GATES(false, true); else REC_GATES(false, false); }
+#undef REC_GATES
     hipLaunchKernelGGL(k_recur_apply, dim3(n_chunks, cdiv(D.W, 64)), dim3(256), 0, s, D, p, chunks, loc, dec, carry0);
 }
 
@@ -225,13 +249,13 @@ __global__ void __launch_bounds__(256) k_decay_step(DecayDims D, DecayParams p) 
     __shared__ float sq[DR * 16], sk[DR * 16];
     __shared__ float red[16][68];
     const int hd = blockIdx.x / D.ns, sl = blockIdx.x - hd * D.ns, m = blockIdx.y, tid = threadIdx.x, c4 = (tid & 15) * 4, dg = tid >> 4;
-    if (p.spans.on && !p.spans.on[m]) return;
     const bool fresh = p.spans.pos[m] == 0;
     float* state = p.state + ((size_t)m * D.H + hd) * D.D * D.Es + sl * 64 + c4;
     f32x4_t S[DR];
 #pragma unroll
     for (int j = 0; j < DR; ++j) S[j] = __builtin_nontemporal_load(reinterpret_cast<const f32x4_t*>(state + (size_t)min(dg + 16 * j, D.D - 1) * D.Es));
     __builtin_amdgcn_sched_barrier(0);
+    if (p.spans.on && !p.spans.on[m]) return;
     const float* row = p.proj + (size_t)m * p.ld;
     for (int i = tid; i < DR * 16; i += 256) {
         sq[i] = i < D.D ? rec_silu(row[p.oq + hd * D.D + i]) : 0.0f;
