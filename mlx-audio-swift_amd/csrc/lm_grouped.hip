@@ -245,12 +245,13 @@ void launch_grouped_attn_prefill(const GroupedDims& D, const GroupedAttn& p, con
 }
 
 // ============================================================================ decode step
-// Block = one row, up to 16 heads of one group, one share of the row's steps; its four waves take the share's steps in turn, each with its own running
-// softmax, and meet in LDS.  The block norms and rotates its heads' queries itself; the current token's key and value never come from the cache: its
+// Block = one row, up to 16 heads of one group, one share of the row's steps; its eight waves take the share's steps in turn, each with its own running
+// softmax, and meet in LDS once.  The block norms and rotates its heads' queries itself; the current token's key and value never come from the cache: its
 // score and value join when the waves meet (last share), the sink with the first share.  The last share's block of a group's first head tile also
 // appends the token to the caches - for the NEXT step.
+#define GRP_NW 8
 template <int VT>
-struct GrpDecodeLds { float q[16][260]; float k[260], v[260]; float m[4][16], l[4][16], self[16]; float acc[2][16][VT * 16 + 4]; };
+struct GrpDecodeLds { float q[16][260]; float k[260], v[260]; float m[GRP_NW][16], l[GRP_NW][16], self[16]; float acc[GRP_NW][16][VT * 16 + 4]; };
 template <int KT, int VT, bool EXACT>
 __device__ __forceinline__ void grouped_decode_block(const GroupedDims& D, const GroupedRows& r, const GroupedAttn& p, const GroupedShares& sh, int rows, int bx, int g, int bz,
                                                      GrpDecodeLds<VT>& L) {
@@ -264,7 +265,6 @@ __device__ __forceinline__ void grouped_decode_block(const GroupedDims& D, const
     const bool first = sp == 0, last = sp == sh.S - 1;
     const bf16_t* kc = (const bf16_t*)p.kc + ((size_t)m * D.G + g) * p.Smax * D.Dp;
     const bf16_t* vc = (const bf16_t*)p.vc + ((size_t)m * D.G + g) * p.Smax * D.Ep;
-    float (*acc)[16][VT * 16 + 4] = L.acc;
     bf16x8_t ka[2][KT], va[VT];
     auto fetch_k = [&](int s) {
         const bf16_t* ks = kc + (size_t)s * 32 * D.Dp + lane * 8;
@@ -298,11 +298,10 @@ __device__ __forceinline__ void grouped_decode_block(const GroupedDims& D, const
     float rc[2], rs[2];                                                        // half <= 128: two pairs a lane
 #pragma unroll
     for (int j = 0; j < 2; ++j) { const int i = min(lane + 64 * j, max(half - 1, 0)); rc[j] = cs[i]; rs[j] = sn[i]; }
-    const float sink_raw = bf16_to_f32(p.sink[h0 + min(li, na - 1)]);
     __builtin_amdgcn_sched_barrier(0);
     if (i0 + wave < i1) { fetch_k(st.at(i0 + wave)); fetch_v(st.at(i0 + wave)); }
     __builtin_amdgcn_sched_barrier(0);
-    for (int a = wave; a < n_vec; a += 4) {
+    for (int a = wave; a < n_vec; a += GRP_NW) {
         if (a != wave) load_vec(a);
         const int size = a <= na ? D.D : D.E;
         float ss = 0.0f;
@@ -330,20 +329,20 @@ __device__ __forceinline__ void grouped_decode_block(const GroupedDims& D, const
             dst[i + half] = v * rc[j] + u * rs[j];
         }
     }
-    for (int i = threadIdx.x + na * 260; i < 16 * 260; i += 256) L.q[0][i] = 0.0f;           // columns past the heads
+    for (int i = threadIdx.x + na * 260; i < 16 * 260; i += 64 * GRP_NW) L.q[0][i] = 0.0f;           // columns past the heads
     __syncthreads();
     if (last) {
         if (a0 == 0) {
             bf16_t *kd = (bf16_t*)r.kc + ((size_t)m * D.G + g) * p.Smax * D.Dp, *vd = (bf16_t*)r.vc + ((size_t)m * D.G + g) * p.Smax * D.Ep;
-            for (int i = threadIdx.x; i < D.Dp; i += 256)
+            for (int i = threadIdx.x; i < D.Dp; i += 64 * GRP_NW)
                 kd[((size_t)(pos >> 4) * kt_n + (i >> 5)) * 512 + (((i & 31) >> 3) * 16 + (pos & 15)) * 8 + (i & 7)] = f32_to_bf16(L.k[i]);
-            for (int i = threadIdx.x; i < D.Ep; i += 256)
+            for (int i = threadIdx.x; i < D.Ep; i += 64 * GRP_NW)
                 vd[((size_t)(pos >> 5) * vt_n + (i >> 4)) * 512 + (((pos & 15) >> 2) * 16 + (i & 15)) * 8 + ((pos >> 4) & 1) * 4 + (pos & 3)] = f32_to_bf16(L.v[i]);
         }
-        for (int a = wave; a < na; a += 4) {                                   // score of the token with itself, on the values the cache will hold
+        for (int a = wave; a < na; a += GRP_NW) {                              // score of the token with itself, on the values the cache will hold
             float d = 0.0f;
             for (int i = lane; i < D.D; i += 64) d += bf16_round_f32(L.q[a][i]) * bf16_round_f32(L.k[i]);
-            d = wave_sum(d);
+            d = wave_sum_dpp(d);
             if (lane == 0) L.self[a] = d * D.scale * GRP_LOG2E;
         }
     }
@@ -359,7 +358,7 @@ __device__ __forceinline__ void grouped_decode_block(const GroupedDims& D, const
     for (int v = 0; v < VT; ++v) o[v] = (f32x4_t){0.f, 0.f, 0.f, 0.f};
     const float sc = D.scale * GRP_LOG2E;
     float mx = -1e30f, ls = 0.0f;
-    for (int i = i0 + wave; i < i1; i += 4) {
+    for (int i = i0 + wave; i < i1; i += GRP_NW) {
         const int k0 = st.at(i) * 32;
         f32x4_t s0 = (f32x4_t){0.f, 0.f, 0.f, 0.f}, s1 = s0;
 #pragma unroll
@@ -368,7 +367,7 @@ __device__ __forceinline__ void grouped_decode_block(const GroupedDims& D, const
             s0 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(ka[0][k], q[k], s0, 0, 0, 0);
             s1 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(ka[1][k], q[k], s1, 0, 0, 0);
         }
-        if (i + 4 < i1) fetch_k(st.at(i + 4));
+        if (i + GRP_NW < i1) fetch_k(st.at(i + GRP_NW));
         __builtin_amdgcn_sched_barrier(0);
         float w[8], tm = -1e30f;
 #pragma unroll
@@ -399,74 +398,59 @@ __device__ __forceinline__ void grouped_decode_block(const GroupedDims& D, const
             o[v] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(va[v], ph, o[v], 0, 0, 0);
             o[v] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(va[v], pl, o[v], 0, 0, 0);
         }
-        if (i + 4 < i1) fetch_v(st.at(i + 4));
+        if (i + GRP_NW < i1) fetch_v(st.at(i + GRP_NW));
         __builtin_amdgcn_sched_barrier(0);
     }
-    // ---- the waves meet: common maximum (with the sink and the token itself), sums, values
+    // ---- the waves meet: common maximum (with the sink and the token itself), sums, values; a thread per head and four columns
     ls += __shfl_xor(ls, 16, 64);
     ls += __shfl_xor(ls, 32, 64);
     if (lq == 0) { L.m[wave][li] = mx; L.l[wave][li] = ls; }
+#pragma unroll
+    for (int v = 0; v < VT; ++v) *reinterpret_cast<f32x4_t*>(&L.acc[wave][li][v * 16 + lq * 4]) = o[v];
     __syncthreads();
-    const int hd = h0 + min(li, na - 1);
-    float M = fmaxf(fmaxf(L.m[0][li], L.m[1][li]), fmaxf(L.m[2][li], L.m[3][li]));
-    const float sink = first ? sink_raw * GRP_LOG2E : -1e30f, self = last && li < na ? L.self[li] : -1e30f;
-    M = fmaxf(M, fmaxf(sink, self));
-    float T = (L.l[0][li] * grp_exp2(L.m[0][li] - M) + L.l[1][li] * grp_exp2(L.m[1][li] - M)) + (L.l[2][li] * grp_exp2(L.m[2][li] - M) + L.l[3][li] * grp_exp2(L.m[3][li] - M));
-    const float ps = last && li < na ? grp_exp2(self - M) : 0.0f;
-    T += (first ? grp_exp2(sink - M) : 0.0f) + ps;
-    const float f = grp_exp2(mx - M);
+    const int c4 = D.Ep >> 2;
+    for (int t = threadIdx.x; t < na * c4; t += 64 * GRP_NW) {
+        const int a = t / c4, col = (t - a * c4) * 4, hd = h0 + a;
+        const float sink = first ? bf16_to_f32(p.sink[hd]) * GRP_LOG2E : -1e30f, self = last ? L.self[a] : -1e30f;
+        float M = fmaxf(sink, self);
 #pragma unroll
-    for (int rd = 0; rd < 2; ++rd) {                                           // waves 1, 3 hand over to 0, 2; then 2 to 0
-        if (rd == 0 ? (wave & 1) : wave == 2) {
-            float (*d)[VT * 16 + 4] = acc[rd == 0 ? wave >> 1 : 0];
+        for (int w = 0; w < GRP_NW; ++w) M = fmaxf(M, L.m[w][a]);
+        const float ps = last ? grp_exp2(self - M) : 0.0f;
+        float T = (first ? grp_exp2(sink - M) : 0.0f) + ps;
+        f32x4_t x = (f32x4_t){0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-            for (int v = 0; v < VT; ++v)
-#pragma unroll
-                for (int e = 0; e < 4; ++e) d[li][v * 16 + lq * 4 + e] = rd == 0 ? o[v][e] * f : o[v][e];
+        for (int w = 0; w < GRP_NW; ++w) {
+            const float f = grp_exp2(L.m[w][a] - M);
+            T += f * L.l[w][a];
+            x += f * *reinterpret_cast<const f32x4_t*>(&L.acc[w][a][col]);
         }
-        __syncthreads();
-        if (rd == 0 ? !(wave & 1) : wave == 0) {
-            float (*d)[VT * 16 + 4] = acc[rd == 0 ? wave >> 1 : 0];
-#pragma unroll
-            for (int v = 0; v < VT; ++v)
-#pragma unroll
-                for (int e = 0; e < 4; ++e) o[v][e] = (rd == 0 ? o[v][e] * f : o[v][e]) + d[li][v * 16 + lq * 4 + e];
+        if (last) x += ps * *reinterpret_cast<const f32x4_t*>(&L.v[col]);
+        if (sh.S > 1) {
+            const size_t at = ((size_t)sp * rows + m) * D.H + hd;
+            *reinterpret_cast<f32x4_t*>(sh.part + at * D.Ep + col) = x;
+            if (col == 0) *reinterpret_cast<float2*>(sh.ml + at * 2) = make_float2(M, T);
+            continue;
         }
-        __syncthreads();
-    }
-    if (wave != 0 || li >= na) return;
-    const float inv = sh.S == 1 ? p.out_scale / T : 1.0f;
-    float* part = sh.S == 1 ? nullptr : sh.part + (((size_t)sp * rows + m) * D.H + hd) * D.Ep;
-#pragma unroll
-    for (int v = 0; v < VT; ++v) {
-        const int col = v * 16 + lq * 4;
-        if (v >= vt_n) continue;
-        float x[4];
-#pragma unroll
-        for (int e = 0; e < 4; ++e) x[e] = (o[v][e] + (last ? ps * L.v[col + e] : 0.0f)) * inv;
-        if (part) *reinterpret_cast<float4*>(part + col) = make_float4(x[0], x[1], x[2], x[3]);
-        else if ((D.E & 3) == 0) { if (col < D.E) operand_store4(p.out, m, hd * D.E + col, x); }
+        x *= p.out_scale / T;
+        const float y[4] = {x[0], x[1], x[2], x[3]};
+        if ((D.E & 3) == 0) { if (col < D.E) operand_store4(p.out, m, hd * D.E + col, y); }
         else {
 #pragma unroll
-            for (int e = 0; e < 4; ++e) if (col + e < D.E) operand_store1(p.out, m, hd * D.E + col + e, x[e]);
+            for (int e = 0; e < 4; ++e) if (col + e < D.E) operand_store1(p.out, m, hd * D.E + col + e, y[e]);
         }
-    }
-    if (part && lq == 0) {
-        float* ml = sh.ml + (((size_t)sp * rows + m) * D.H + hd) * 2;
-        *reinterpret_cast<float2*>(ml) = make_float2(M, T);
     }
 }
 // One launch of a decode step: attention blocks, then (RECUR) the blocks of a gated recurrence that reads the same projections
 template <int KT, int VT, bool EXACT, int RECUR>
-__global__ void __launch_bounds__(256, (KT <= 4 && VT <= 8) ? 2 : 1) k_grouped_attn_decode(GroupedDims D, GroupedRows r, GroupedAttn p, GroupedShares sh, int rows, int nz,
-                                                                                           RecurDims RD, RecurParams rp) {
-    __shared__ union { GrpDecodeLds<VT> attn; RecurStepLds recur; } L;
+__global__ void __launch_bounds__(64 * GRP_NW, 2) k_grouped_attn_decode(GroupedDims D, GroupedRows r, GroupedAttn p, GroupedShares sh, int rows, int nz, RecurDims RD,
+                                                                        RecurParams rp) {
+    extern __shared__ __attribute__((aligned(16))) uint8_t lds[];
     const int n_attn = rows * sh.S * D.G * nz;
     int b = blockIdx.x;
-    if (RECUR && b >= n_attn) { recur_step_block<RECUR == 2>(RD, rp, rows, b - n_attn, L.recur); return; }
+    if (RECUR && b >= n_attn) { recur_step_block<RECUR == 2, GRP_NW / 4>(RD, rp, rows, b - n_attn, *reinterpret_cast<RecurStepLds<GRP_NW / 4>*>(lds)); return; }
     const int bx = b % (rows * sh.S);
     b /= rows * sh.S;
-    grouped_decode_block<KT, VT, EXACT>(D, r, p, sh, rows, bx, b % D.G, b / D.G, L.attn);
+    grouped_decode_block<KT, VT, EXACT>(D, r, p, sh, rows, bx, b % D.G, b / D.G, *reinterpret_cast<GrpDecodeLds<VT>*>(lds));
 }
 // shares of a head -> operand: one wave per (row, head)
 __global__ void __launch_bounds__(256) k_grouped_shares(GroupedDims D, GroupedShares sh, Operand out, float out_scale, const uint8_t* __restrict__ on, int rows) {
@@ -474,25 +458,22 @@ __global__ void __launch_bounds__(256) k_grouped_shares(GroupedDims D, GroupedSh
     if (item >= rows * D.H) return;
     const int m = item / D.H, hd = item - m * D.H;
     if (on && !on[m]) return;
-    const float2* ml = reinterpret_cast<const float2*>(sh.ml);
-    float M = -1e30f, T = 0.0f;
-    for (int s = 0; s < sh.S; ++s) M = fmaxf(M, ml[((size_t)s * rows + m) * D.H + hd].x);
-    for (int s = 0; s < sh.S; ++s) { const float2 t = ml[((size_t)s * rows + m) * D.H + hd]; T += t.y * grp_exp2(t.x - M); }
-    const float inv = out_scale / T;
-    for (int i = lane; i < D.E; i += 64) {
+    const size_t step = (size_t)rows * D.H, at = (size_t)m * D.H + hd;
+    const float2 mine = *reinterpret_cast<const float2*>(sh.ml + (at + min(lane, sh.S - 1) * step) * 2);       // a share per lane
+    const float M = wave_max(mine.x), f = lane < sh.S ? grp_exp2(mine.x - M) : 0.0f, inv = out_scale / wave_sum_dpp(f * mine.y);
+    for (int i = lane; i < D.Ep; i += 64) {
         float a = 0.0f;
-        for (int s = 0; s < sh.S; ++s) {
-            const size_t at = ((size_t)s * rows + m) * D.H + hd;
-            a += sh.part[at * D.Ep + i] * grp_exp2(ml[at].x - M);
-        }
-        operand_store1(out, m, hd * D.E + i, a * inv);
+#pragma unroll 4
+        for (int s = 0; s < sh.S; ++s) a += sh.part[(at + s * step) * D.Ep + i] * __shfl(f, s, 64);
+        if (i < D.E) operand_store1(out, m, hd * D.E + i, a * inv);
     }
 }
 int grouped_decode_shares(const GroupedDims& D, int rows, int Smax) {
     const int keys = D.window > 0 ? std::min(Smax, D.window + D.keep + 32) : Smax, steps = cdiv(keys, 32);
     const int blocks = rows * D.G * cdiv(D.H / D.G, 16);
     int S = 1;
-    while (S < 32 && blocks * S < 256 && steps / (S + 1) >= 8) ++S;            // two steps a wave at least
+    if (steps <= 24) return 1;                                                 // three steps a wave: no second launch
+    while (S < 32 && blocks * (S + 1) <= 256 && steps / S > GRP_NW) ++S;
     return S;
 }
 void launch_grouped_attn_decode(const GroupedDims& D, const GroupedRows& r, const GroupedAttn& p, const GroupedShares& sh, const RecurDims* RD, const RecurParams* rp, int rows,
@@ -501,10 +482,14 @@ void launch_grouped_attn_decode(const GroupedDims& D, const GroupedRows& r, cons
                 MIS_ERR_GENERATION_FAILED, "grouped attention: bad layout");
     MIS_REQUIRE(!RD || (rp && rp->rows.pos && !rp->rows.seq), MIS_ERR_GENERATION_FAILED, "gated recurrence step: bad layout");
     const int nz = cdiv(D.H / D.G, 16), kt = D.Dp / 32, vt = D.Ep / 16;
-    const dim3 grid(rows * sh.S * D.G * nz + (RD ? recur_step_blocks(*RD, rows) : 0)), block(256);
+    const dim3 grid(rows * sh.S * D.G * nz + (RD ? recur_step_blocks(*RD, rows, GRP_NW / 4) : 0)), block(64 * GRP_NW);
     const RecurDims rd = RD ? *RD : RecurDims{};
     const RecurParams rpp = RD ? *rp : RecurParams{};
-#define GRP_DEC(K, V, X, C) hipLaunchKernelGGL((k_grouped_attn_decode<K, V, X, C>), grid, block, 0, s, D, r, p, sh, rows, nz, rd, rpp)
+#define GRP_DEC(K, V, X, C) do {                                                                                                                         \
+        const size_t lds = std::max(sizeof(GrpDecodeLds<V>), sizeof(RecurStepLds<GRP_NW / 4>));                                                            \
+        static const hipError_t attr = hipFuncSetAttribute(reinterpret_cast<const void*>(&k_grouped_attn_decode<K, V, X, C>), hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024); \
+        HIP_CHECK(attr);                                                                                                                                   \
+        hipLaunchKernelGGL((k_grouped_attn_decode<K, V, X, C>), grid, block, lds, s, D, r, p, sh, rows, nz, rd, rpp); } while (0)
 #define GRP_DECR(K, V, X) do { if (!RD) GRP_DEC(K, V, X, 0); else if (RD->n % 4) GRP_DEC(K, V, X, 1); else GRP_DEC(K, V, X, 2); } while (0)
     if (kt == 2 && vt == 4) GRP_DECR(2, 4, true);
     else if (kt == 4 && vt == 8) GRP_DECR(4, 8, true);

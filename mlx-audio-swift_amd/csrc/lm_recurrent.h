@@ -21,17 +21,21 @@ typedef float f32x8_t __attribute__((ext_vector_type(8)));
 // ---- decode step of the gated recurrence: block = 16 output channels of a block of channels, 16 rows; its four waves share the products' columns.  A wave
 // computes the convolution outputs its columns need straight into hi and lo fragments (lane: 8 channels of a row); the waves' sums meet in LDS, then a
 // thread finishes one (row, channel): gates, state, the other branch.
-struct RecurStepLds { float red[4][2][64][4]; };
-__host__ __device__ static inline int recur_step_blocks(const RecurDims& D, int rows) { return D.B * D.nt * ((rows + 15) / 16); }
+// (PARTS: such tiles per block, four waves each.)
+template <int PARTS>
+struct RecurStepLds { float red[PARTS][4][2][64][4]; };
+static inline int recur_step_blocks(const RecurDims& D, int rows, int parts) { return cdiv((int64_t)D.B * D.nt * ((rows + 15) / 16), parts); }
 // VEC: a block's channels are a multiple of 4
-template <bool VEC>
-__device__ __forceinline__ void recur_step_block(const RecurDims& D, const RecurParams& p, int rows, int bi, RecurStepLds& L) {
-    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, li = lane & 15, lq = lane >> 4;
+template <bool VEC, int PARTS>
+__device__ __forceinline__ void recur_step_block(const RecurDims& D, const RecurParams& p, int rows, int block, RecurStepLds<PARTS>& lds) {
+    const int tid = threadIdx.x & 255, part = threadIdx.x >> 8, lane = tid & 63, wave = tid >> 6, li = lane & 15, lq = lane >> 4;
+    const int tiles = D.B * D.nt * ((rows + 15) / 16), want = block * PARTS + part, bi = min(want, tiles - 1);
+    auto& red = lds.red[part];
     const int mt = bi / (D.B * D.nt), t = bi - mt * D.B * D.nt, b = t / D.nt, tile = t - b * D.nt, ch0 = b * D.n, KT = D.np >> 5;
     // ---- what the finishing thread needs, requested first
     const int fm = mt * 16 + (tid >> 4), fi = tile * 16 + (tid & 15), fmc = min(fm, rows - 1), ch = ch0 + min(fi, D.n - 1);
     const int pos_f = p.rows.pos[fmc];
-    const bool on = fm < rows && fi < D.n && (!p.rows.on || p.rows.on[fmc]);
+    const bool on = want < tiles && fm < rows && fi < D.n && (!p.rows.on || p.rows.on[fmc]);
     const float* prow = p.proj + (size_t)fmc * p.ld;
     float* sp = p.state + (size_t)fmc * D.W + ch;
     const float s_old = *sp, x_now = prow[p.ox + ch] + p.bias_x[ch], y_raw = prow[p.oy + ch] + bf16_to_f32(p.bias[p.oy + ch]);
@@ -82,14 +86,14 @@ __device__ __forceinline__ void recur_step_block(const RecurDims& D, const Recur
         ag = __builtin_amdgcn_mfma_f32_16x16x32_bf16(fg, hi, ag, 0, 0, 0);
         bg = __builtin_amdgcn_mfma_f32_16x16x32_bf16(fg, lo, bg, 0, 0, 0);
     }
-    *reinterpret_cast<f32x4_t*>(L.red[wave][0][lane]) = ar + br;
-    *reinterpret_cast<f32x4_t*>(L.red[wave][1][lane]) = ag + bg;
+    *reinterpret_cast<f32x4_t*>(red[wave][0][lane]) = ar + br;
+    *reinterpret_cast<f32x4_t*>(red[wave][1][lane]) = ag + bg;
     __syncthreads();
     if (!on) return;
     // ---- one (row, channel) per thread: accumulator row = channel, column = row
     const int at = ((tid & 15) >> 2) * 16 + (tid >> 4), e = tid & 3;
-    const float zr = (L.red[0][0][at][e] + L.red[1][0][at][e]) + (L.red[2][0][at][e] + L.red[3][0][at][e]);
-    const float zg = (L.red[0][1][at][e] + L.red[1][1][at][e]) + (L.red[2][1][at][e] + L.red[3][1][at][e]);
+    const float zr = (red[0][0][at][e] + red[1][0][at][e]) + (red[2][0][at][e] + red[3][0][at][e]);
+    const float zg = (red[0][1][at][e] + red[1][1][at][e]) + (red[2][1][at][e] + red[3][1][at][e]);
     const float la = -cf * rec_sigmoid(zr + rb), a = rec_exp(la);
     const float in = rec_complement(a, la) * rec_sigmoid(zg + gb) * u_own;
     const float S = pos_f == 0 ? in : a * s_old + in;

@@ -183,13 +183,13 @@ __global__ void __launch_bounds__(256, 2) k_recur_gates(RecurDims D, RecurParams
 }
 template <bool VEC>
 __global__ void __launch_bounds__(256) k_recur_step(RecurDims D, RecurParams p, int rows) {
-    __shared__ RecurStepLds L;
-    recur_step_block<VEC>(D, p, rows, blockIdx.x, L);
+    __shared__ RecurStepLds<1> L;
+    recur_step_block<VEC, 1>(D, p, rows, blockIdx.x, L);
 }
 void launch_recur_step(const RecurDims& D, const RecurParams& p, int rows, hipStream_t s) {
     MIS_REQUIRE(p.rows.pos && !p.rows.seq, MIS_ERR_GENERATION_FAILED, "gated recurrence step: bad layout");
-    if (D.n % 4 == 0) hipLaunchKernelGGL((k_recur_step<true>), dim3(recur_step_blocks(D, rows)), dim3(256), 0, s, D, p, rows);
-    else hipLaunchKernelGGL((k_recur_step<false>), dim3(recur_step_blocks(D, rows)), dim3(256), 0, s, D, p, rows);
+    if (D.n % 4 == 0) hipLaunchKernelGGL((k_recur_step<true>), dim3(recur_step_blocks(D, rows, 1)), dim3(256), 0, s, D, p, rows);
+    else hipLaunchKernelGGL((k_recur_step<false>), dim3(recur_step_blocks(D, rows, 1)), dim3(256), 0, s, D, p, rows);
 }
 // chunk: state = loc + dec * (state before the chunk), times the other branch; the chunks before it in the span give that state
 __global__ void __launch_bounds__(256) k_recur_apply(RecurDims D, RecurParams p, const RecurChunk* __restrict__ chunks, const float* __restrict__ loc,
