@@ -238,7 +238,9 @@ mis_status mis_lm_prefill(mis_tts*, const int32_t* prompt_ids, const int32_t* pr
 mis_status mis_lm_forward(mis_tts*, const int32_t* ids, const uint8_t* active, float* logits_out);
 /* ---- language models by architecture.  config.json with an "architecture" entry describes the model layer by layer ("layers": per layer the
  * mixer with its sizes, the feed-forward, optionally another layer whose tensors it shares); the engine serves "Rugunex" (parallel blocks
- * with layer scale, latent attention under a sliding window, squared-ReLU feed-forward).  The handle is the mis_tts of this section: rows,
+ * with layer scale, latent attention under a sliding window, squared-ReLU feed-forward) and "Vamunex" (a norm before and behind each sublayer;
+ * lightning attention, or grouped attention under a sliding window with kept first tokens and a sink beside a gated linear recurrence; a range of
+ * layers may run several times, each run is a layer of its own to mis_lm_num_layers and residual_out).  The handle is the mis_tts of this section: rows,
  * caches, mis_lm_reset / prefill / forward, the sampler and the generate loop are shared. */
 enum { MIS_COMPUTE_BF16 = 0, MIS_COMPUTE_F32 = 1 };  /* MIS_COMPUTE_F32: every product and activation in float32 */
 /* chosen by config.json; directories without "architecture" load as the Llama family (bf16 only, no codec) */
