@@ -34,14 +34,14 @@ __device__ __forceinline__ void grp_split(const float (&w)[8], bf16x8_t& hi, bf1
 }
 
 // ============================================================================ prompt pass
-// Block = up to 64 queries of one request and up to NW / 2 heads of one group; a wave = 32 queries of one head.  The 32 keys of a step - KT pairs of key
+// Block = up to 64 queries of one request and up to four heads of one group; a wave = 32 queries of one head.  The 32 keys of a step - KT pairs of key
 // fragments and VT value fragments, contiguous in the caches - come into LDS by DMA, two buffers, one barrier per step.
 // EXACT: the heads have KT and VT tiles, not fewer (no guards in the loop)
 template <int KT, int VT, bool EXACT>
-__global__ void __launch_bounds__(256, (KT <= 4 && VT <= 8) ? 2 : 1) k_grouped_attn_prefill(GroupedDims D, GroupedAttn p, const RowSpan* __restrict__ tiles, int ipb) {
+__global__ void __launch_bounds__(512, 2) k_grouped_attn_prefill(GroupedDims D, GroupedAttn p, const RowSpan* __restrict__ tiles, int ipb) {
     __shared__ __attribute__((aligned(1024))) bf16_t buf[2][(2 * KT + VT) * 512];
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, nw = blockDim.x >> 6, li = lane & 15, lq = lane >> 4;
-    const RowSpan t = tiles[blockIdx.x];
+    const RowSpan t = tiles[gridDim.x - 1 - blockIdx.x];                       // (a request's last queries see the most keys: they start first)
     const int g = blockIdx.y, R = D.H / D.G, kt_n = EXACT ? KT : D.Dp >> 5, vt_n = EXACT ? VT : D.Ep >> 4;
     const int item = blockIdx.z * ipb + wave, hd = g * R + min(item >> 1, R - 1), q0 = (item & 1) * 32;
     const bool live = item < 2 * R && q0 < t.n;                                // (a wave without queries only helps to stage)
@@ -232,7 +232,8 @@ bool grouped_mfma_ok(const GroupedDims& D) { return D.Dp <= 256 && D.Ep <= 256; 
 void launch_grouped_attn_prefill(const GroupedDims& D, const GroupedAttn& p, const RowSpan* tiles, int n_tiles, hipStream_t s) {
     MIS_REQUIRE(grouped_mfma_ok(D) && !p.f32 && p.Smax % 32 == 0 && p.out.kind == OPK_ROWS && p.out.ld % 4 == 0, MIS_ERR_GENERATION_FAILED, "grouped attention: bad layout");
     const int items = 2 * (D.H / D.G);
-    const int ipb = items % 4 == 0 ? 4 : (items % 3 == 0 ? 3 : (items <= 4 ? items : 4));     // waves per block
+    int ipb = std::min(items, 8);                                              // waves per block: they share the staged keys
+    while (items > 8 && ipb > 4 && items % ipb) --ipb;
     const dim3 grid(n_tiles, D.G, cdiv(items, ipb)), block(64 * ipb);
     const int kt = D.Dp / 32, vt = D.Ep / 16;
 #define GRP_PF(K, V, X) hipLaunchKernelGGL((k_grouped_attn_prefill<K, V, X>), grid, block, 0, s, D, p, tiles, ipb)
