@@ -451,14 +451,17 @@ def test_directory_and_commands(tmp_path):
     out.mkdir()
     steps = [{"step": 0, "entries": [{"id": "x", "tokens": t[:20].tolist(), "want": [3, 19]}, {"id": "y", "tokens": t[:4].tolist(), "want": []}], "end": []},
              {"step": 1, "entries": [{"id": "y", "tokens": [int(t[4])], "want": [0]}, {"id": "x", "tokens": [int(t[20])], "want": [0]}], "end": ["y"]},
-             {"step": 2, "entries": [{"id": "x", "tokens": [int(t[21])], "want": []}], "end": ["x"]},
-             {"step": 3, "entries": [{"id": "z", "tokens": t[:9].tolist(), "want": [8]}], "end": ["z"]}]
-    r = subprocess.run([sys.executable, os.path.join(ROOT, "bin", "trace_run"), "--model", d, "--dtype", "float32", "--out", str(out), "--max-tokens", "40"],
+             {"step": 2, "entries": [{"id": "x", "tokens": [int(t[21])], "want": []}], "end": []}]
+    steps += [{"step": k, "entries": [{"id": "x", "tokens": [int(t[19 + k])], "want": [0]}], "end": ["x"] if k == 6 else []} for k in (3, 4, 5, 6)]
+    steps += [{"step": 7, "entries": [{"id": "z", "tokens": t[:9].tolist(), "want": [8]}], "end": ["z"]}]
+    r = subprocess.run([sys.executable, os.path.join(ROOT, "bin", "trace_run"), "--model", d, "--dtype", "float32", "--out", str(out), "--max-tokens", "26"],
                        input="\n".join(json.dumps(s) for s in steps) + "\n", capture_output=True, text=True, timeout=100)
     assert r.returncode == 0, r.stderr[-2000:]
-    assert [x for x in r.stdout.splitlines() if x.startswith("done")] == ["done 0", "done 1", "done 2", "done 3"]
-    got = {i: np.fromfile(out / f"{i}.f32", "<f4").reshape(-1, cfg["vocab"]) for i in (0, 1, 3)}
+    assert [x for x in r.stdout.splitlines() if x.startswith("done")] == [f"done {k}" for k in range(8)]
+    got = {i: np.fromfile(out / f"{i}.f32", "<f4").reshape(-1, cfg["vocab"]) for i in (0, 1, 3, 4, 5, 6, 7)}
     assert not (out / "2.f32").exists()
     check(got[0], ref[[3, 19]], "float32")
     check(got[1], ref[[4, 20]], "float32")
-    check(got[3], ref[[8]], "float32")
+    for k in (3, 4, 5, 6):                                                      # the one that is left holds as much as both did
+        check(got[k], ref[[19 + k]], "float32")
+    check(got[7], ref[[8]], "float32")
